@@ -255,6 +255,30 @@ MI355X_API mi355x_status mi355x_add(const float* a, const float* b, float* out, 
  * index of each row's largest value, into device memory. */
 MI355X_API mi355x_status mi355x_argmax(const float* logits, int64_t rows, int64_t n, int32_t* out, void* stream);
 
+/* ---- model handles --------------------------------------------------------------
+ * What every decoder behind a handle takes, whichever *_create made it
+ * (mi355x_llama_create, mi355x_stack_create): tensors by the names of the model's
+ * file, then mi355x_model_finalize, then calls. batch sequences go in lockstep. */
+MI355X_API mi355x_status mi355x_model_destroy(void* model);
+MI355X_API mi355x_status mi355x_model_set_tensor(void* model, const char* name, int dtype, const void* host_data, int64_t n_elems);
+/* Checks the tensors and allocates caches, states (zeroed) and the activations of
+ * calls of up to max_tokens tokens per sequence. */
+MI355X_API mi355x_status mi355x_model_finalize(void* model, int64_t max_tokens);
+/* Empties caches and states: the next call starts new sequences. */
+MI355X_API mi355x_status mi355x_model_reset(void* model);
+MI355X_API int64_t mi355x_model_cache_len(void* model);
+/* Runs tokens [batch, n], which follow the positions that are held, and copies to
+ * the host the logits of the last token [batch, vocab], or of every token
+ * [batch, n, vocab] if all. */
+MI355X_API mi355x_status mi355x_model_logits(void* model, const int32_t* tokens, int64_t n, int all, float* logits_host);
+/* The same for the n_want rows b * n + t that want lists (possibly none), in that
+ * order: [n_want, vocab]. */
+MI355X_API mi355x_status mi355x_model_logits_at(void* model, const int32_t* tokens, int64_t n, const int64_t* want, int64_t n_want, float* logits_host);
+/* Greedy generation: prompt [batch, n_prompt], then n_new tokens a sequence into
+ * out_tokens [batch, n_new]. seconds, if not NULL, gets the device time of the
+ * prompt pass (with the first token) and of the n_new - 1 decoding steps. */
+MI355X_API mi355x_status mi355x_model_generate(void* model, const int32_t* prompt, int64_t n_prompt, int64_t n_new, int32_t* out_tokens, double* seconds);
+
 /* ---- the decoder: llm.Model, its caches and the greedy loop ------------------
  * (llm/model.go:216-455; nn/transformer.go:348-423;
  * examples/llama/generate.go:44-53,162-202). Weights keep their block dtypes on
@@ -304,6 +328,43 @@ MI355X_API mi355x_status mi355x_llama_logits(void* model, const int32_t* tokens,
  * out_tokens [batch, n_new]. seconds, if not NULL, gets the device time of the
  * prompt pass (with the first token) and of the n_new - 1 decoding steps. */
 MI355X_API mi355x_status mi355x_llama_generate(void* model, const int32_t* prompt, int64_t n_prompt, int64_t n_new, int32_t* out_tokens, double* seconds);
+
+/* ---- the mixer stack ------------------------------------------------------------
+ * A decoder whose layers are a list of mixers with sizes of their own, beside the
+ * reference's architectures (which have no counterpart of it): norms in groups
+ * before and after every sublayer, a short causal convolution in front of every
+ * mixer, an average over all earlier layers' results behind every layer, and the
+ * embedding table as output matrix. A handle takes the mi355x_model_* calls;
+ * tensors have the names of the model's file (embed, l0.norm1, l0.mix.q, ...) and
+ * are bfloat16. */
+enum { MI355X_MIXER_LATENT = 1, MI355X_MIXER_MLSTM = 2, MI355X_MIXER_LIGHTNING = 3 };
+
+typedef struct mi355x_stack_layer {
+    int32_t mixer;    /* MI355X_MIXER_* */
+    int32_t heads;
+    int32_t dim;      /* features of a query and key (latent attention: of their part without positions) */
+    int32_t vdim;     /* features of a value */
+    int32_t rot_dim;  /* latent attention: rotated features of a query and key, interleaved pairs */
+    int32_t kv_rank;  /* latent attention: size of the latent */
+    int32_t ff;       /* rows of the feed-forward's up matrix (squared ReLU), 0: no feed-forward */
+    int32_t reserved;
+    double scale;     /* latent attention: of the scores */
+    double rot_base;
+    double gate_cap;  /* mLSTM: soft cap of its two gates */
+    const double* decay; /* lightning attention: [heads] */
+} mi355x_stack_layer;
+
+typedef struct mi355x_stack_config {
+    int32_t width, vocab, layers;
+    int32_t context;      /* capacity of the caches, in positions */
+    int32_t batch;
+    int32_t taps;         /* of the causal convolutions */
+    int32_t norm_groups;
+    int32_t dtype;        /* MI355X_BF16: prompts on the bfloat16 matrix cores; MI355X_F32: float32 throughout */
+    double eps;
+} mi355x_stack_config;
+
+MI355X_API mi355x_status mi355x_stack_create(const mi355x_stack_config* cfg, const mi355x_stack_layer* layers, void** model);
 
 /* ---- the reference's operator interface for this path ---------------------------
  * backend.Backend and backend.Batcher (backend/backend.go:141-171,

@@ -1,10 +1,14 @@
 """Builds libmimir_mi355x.so, the gfx950 code of this package, with hipcc.
 
-The library is built in-tree (mimir_amd/lib/) ahead of time; nothing compiles
-at run time. `python -m mimir_amd.build` rebuilds it.
+The library is built in-tree (mimir_amd/lib/) ahead of time. `python -m
+mimir_amd.build` rebuilds it; with the name of a part (PARTS) it compiles that
+part's sources alone, into a library of their own with the same entry points.
+ensure() does the same if nothing is built yet, for commands that are run from a
+fresh checkout.
 """
 from __future__ import annotations
 
+import fcntl
 import os
 import subprocess
 import sys
@@ -23,8 +27,21 @@ FLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-fvisibility=h
          "-Wno-unknown-warning-option", "-ffp-contract=on"] + DEVICE_FLAGS
 
 
-def sources() -> list[str]:
+# Sources that make a library of their own: what the decoders of one kind need.
+PARTS = {
+    "stack": ("runtime", "decoder", "stack", "residual_ops", "linear_recurrence", "attention_latent", "gemv_float", "gemm_float", "gemm_bf16",
+              "decode_ops"),
+}
+
+
+def sources(part: str | None = None) -> list[str]:
+    if part is not None:
+        return [os.path.join(CSRC, f + ".hip") for f in PARTS[part]]
     return sorted(os.path.join(CSRC, f) for f in os.listdir(CSRC) if f.endswith(".hip"))
+
+
+def lib_path(part: str | None = None) -> str:
+    return LIB_PATH if part is None else os.path.join(LIB_DIR, f"libmimir_mi355x_{part}.so")
 
 
 def _compile(src: str) -> str:
@@ -54,23 +71,40 @@ def build_probe() -> list[str]:
     return outs
 
 
-def build(verbose: bool = False) -> str:
-    """Compiles every .hip source for gfx950 and links the shared library."""
+def build(verbose: bool = False, part: str | None = None) -> str:
+    """Compiles every .hip source (or a part's) for gfx950 and links the shared library."""
     os.makedirs(OBJ_DIR, exist_ok=True)
-    srcs = sources()
+    srcs = sources(part)
     with ThreadPoolExecutor(max_workers=min(8, len(srcs))) as ex:
         objs = list(ex.map(_compile, srcs))
-    tmp = LIB_PATH + ".tmp"
+    out = lib_path(part)
+    tmp = out + ".tmp"
     cmd = ["hipcc", "-shared", "-fPIC", f"--offload-arch={ARCH}", "-o", tmp, *objs]
+    if part is not None:  # a reference into another part's sources shows here and not when the library is loaded
+        cmd.append("-Wl,-z,defs")
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError(f"link failed:\n{r.stderr[-4000:]}")
-    os.replace(tmp, LIB_PATH)
-    build_probe()
+    os.replace(tmp, out)
+    if part is None:
+        build_probe()
     if verbose:
-        print(f"built {LIB_PATH} from {len(srcs)} sources", file=sys.stderr)
-    return LIB_PATH
+        print(f"built {out} from {len(srcs)} sources", file=sys.stderr)
+    return out
+
+
+def ensure(part: str | None = None) -> None:
+    """Builds the library, or the part of it that is asked for, if neither is there. One process builds at a time."""
+    def there():
+        return os.path.exists(LIB_PATH) or (part is not None and os.path.exists(lib_path(part)))
+    if there():
+        return
+    os.makedirs(LIB_DIR, exist_ok=True)
+    with open(os.path.join(LIB_DIR, "build.lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        if not there():
+            build(part=part)
 
 
 if __name__ == "__main__":
-    build(verbose=True)
+    build(verbose=True, part=sys.argv[1] if len(sys.argv) > 1 else None)

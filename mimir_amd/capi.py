@@ -49,6 +49,15 @@ SYMBOLS = {
     "mi355x_swiglu": (C.c_uint32, [_vp, _vp, _vp, _i64, _i64, _i64, _vp]),
     "mi355x_add": (C.c_uint32, [_vp, _vp, _vp, _i64, _vp]),
     "mi355x_argmax": (C.c_uint32, [_vp, _i64, _i64, _vp, _vp]),
+    "mi355x_model_destroy": (C.c_uint32, [_vp]),
+    "mi355x_model_set_tensor": (C.c_uint32, [_vp, C.c_char_p, _int, _vp, _i64]),
+    "mi355x_model_finalize": (C.c_uint32, [_vp, _i64]),
+    "mi355x_model_reset": (C.c_uint32, [_vp]),
+    "mi355x_model_cache_len": (_i64, [_vp]),
+    "mi355x_model_logits": (C.c_uint32, [_vp, _vp, _i64, _int, _vp]),
+    "mi355x_model_logits_at": (C.c_uint32, [_vp, _vp, _i64, _vp, _i64, _vp]),
+    "mi355x_model_generate": (C.c_uint32, [_vp, _vp, _i64, _i64, _vp, _vp]),
+    "mi355x_stack_create": (C.c_uint32, [_vp, _vp, C.POINTER(_vp)]),
     "mi355x_llama_create": (C.c_uint32, [_vp, C.POINTER(_vp)]),
     "mi355x_llama_destroy": (C.c_uint32, [_vp]),
     "mi355x_llama_set_tensor": (C.c_uint32, [_vp, C.c_char_p, _int, _vp, _i64]),
@@ -90,6 +99,20 @@ class LlamaConfig(C.Structure):
                                           "interleaved", "cache_dtype", "batch")] + [(n, C.c_double) for n in ("rope_base", "rope_scale", "eps")]
 
 
+MIXER_LATENT, MIXER_MLSTM, MIXER_LIGHTNING = 1, 2, 3
+
+
+class StackConfig(C.Structure):
+    """mi355x_stack_config."""
+    _fields_ = [(n, C.c_int32) for n in ("width", "vocab", "layers", "context", "batch", "taps", "norm_groups", "dtype")] + [("eps", C.c_double)]
+
+
+class StackLayer(C.Structure):
+    """mi355x_stack_layer."""
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "dim", "vdim", "rot_dim", "kv_rank", "ff", "reserved")] + \
+               [(n, C.c_double) for n in ("scale", "rot_base", "gate_cap")] + [("decay", C.POINTER(C.c_double))]
+
+
 class AttentionDesc(C.Structure):
     """mi355x_attention_desc."""
     _fields_ = [(n, C.c_void_p) for n in ("q", "k", "v", "mask", "out", "lse")] + \
@@ -105,26 +128,38 @@ class Mi355xError(RuntimeError):
 
 
 _lib = None
+_lib_part = None  # the part that _lib holds, None: all of it
 
 
-def load() -> C.CDLL:
-    """Loads the library and declares every symbol; raises if it is not built."""
-    global _lib
-    if _lib is None:
-        path = os.environ.get("MIMIR_MI355X_LIB") or LIB_PATH  # as the reference's loaders take a path from the environment
-        if not os.path.exists(path):
-            raise FileNotFoundError(f"{path} is not built: run `python -m mimir_amd.build`")
-        lib = C.CDLL(path)
-        for name, (res, args) in SYMBOLS.items():
+def load(part: str | None = None) -> C.CDLL:
+    """Loads the library and declares every symbol; raises if it is not built. With `part` (a name of
+    mimir_amd.build.PARTS) the library of that part alone will do where the whole one is not built: it
+    exports the entry points of the part's sources."""
+    global _lib, _lib_part
+    if _lib is not None and (_lib_part is None or _lib_part == part):
+        return _lib
+    path = os.environ.get("MIMIR_MI355X_LIB") or LIB_PATH  # as the reference's loaders take a path from the environment
+    whole = os.path.exists(path)
+    if not whole and part is not None:
+        path = os.path.join(HERE, "lib", f"libmimir_mi355x_{part}.so")
+    if not os.path.exists(path):
+        raise FileNotFoundError(f"{path} is not built: run `python -m mimir_amd.build{' ' + part if part else ''}`")
+    lib = C.CDLL(path)
+    for name, (res, args) in SYMBOLS.items():
+        try:
             fn = getattr(lib, name)  # AttributeError if the symbol is missing
-            fn.restype, fn.argtypes = res, args
-        _lib = lib
+        except AttributeError:
+            if whole:
+                raise
+            continue
+        fn.restype, fn.argtypes = res, args
+    _lib, _lib_part = lib, (None if whole else part)
     return _lib
 
 
 def last_error() -> str:
     buf = C.create_string_buffer(1024)
-    load().mi355x_last_error(buf, 1024)
+    (_lib or load()).mi355x_last_error(buf, 1024)
     return buf.value.decode(errors="replace")
 
 

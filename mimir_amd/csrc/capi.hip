@@ -6,7 +6,6 @@
 
 #include <hip/hip_runtime.h>
 
-#include <cstdarg>
 #include <cstdio>
 #include <cstring>
 #include <map>
@@ -15,68 +14,12 @@
 #include <string>
 
 #include "kernels.h"
+#include "runtime.h"
+
+using namespace mimir;
 
 namespace {
 
-thread_local std::string g_last_error;
-
-mi355x_status fail(mi355x_status code, const char* fmt, ...) {
-    char buf[512];
-    va_list ap;
-    va_start(ap, fmt);
-    vsnprintf(buf, sizeof buf, fmt, ap);
-    va_end(ap);
-    g_last_error = buf;
-    return code;
-}
-
-mi355x_status hip_fail(hipError_t e, const char* what) {
-    return fail((mi355x_status)e, "mi355x: %s: %s", what, hipGetErrorName(e));
-}
-
-#define HIP_TRY(expr, what)                         \
-    do {                                            \
-        hipError_t e_ = (expr);                     \
-        if (e_ != hipSuccess) return hip_fail(e_, what); \
-    } while (0)
-
-constexpr int kMaxDevices = 16;
-
-// The converted activations of mi355x_qgemv_noalloc: a fixed block in the code object's own
-// device memory, so that the entry point allocates nothing. Every device the library runs on
-// holds its own copy at its own address (DeviceState::fixed, looked up when the device's state
-// is created); in host code the array's name is only a handle for that lookup, never an address.
-constexpr size_t kNoallocScratchBytes = (size_t)1 << 20;
-static __device__ __align__(256) unsigned char g_noalloc_scratch[kNoallocScratchBytes];
-
-// Scratch memory of the entry points that need some beyond their arguments (converted activations,
-// partial results and tickets of split attention and argmax, float32 copies of qgemm_bf16's general
-// route). One set per device and stream: calls on different streams never share a block, calls on one
-// stream are ordered by it. A block that has become too small is replaced by a larger one and kept
-// aside: work already queued, and HIP graphs a caller has instantiated over an entry point, may still
-// read and write it, tickets included (a graph keeps the block it was recorded with and stays valid).
-// Growth at least doubles a block, so what is kept aside stays below the size of the live block.
-// mi355x_stream_release frees everything a stream holds, live and kept aside.
-struct ScratchBlock {
-    void* p = nullptr;
-    size_t bytes = 0;
-};
-struct StreamScratch {
-    ScratchBlock act, attn, attn_flags, gemm, argmax;
-    std::vector<void*> retired;  // outgrown blocks
-};
-
-// Per-device state: the error word kernels OR bits into, read back at sync.
-struct DeviceState {
-    bool ready = false;
-    uint32_t* err_dev = nullptr;
-    uint32_t* err_host = nullptr;  // pinned
-    std::map<void*, StreamScratch> scratch;  // by stream handle
-    void* fixed = nullptr;                   // this device's copy of g_noalloc_scratch
-};
-
-std::mutex g_mu;
-DeviceState g_dev[kMaxDevices];
 std::atomic<int> g_tune_q4_live[5] = {{0}, {0}, {0}, {0}, {0}};
 // A call's own copy of the launch-plan overrides, so that one call sees one plan.
 struct TuneQ4 {
@@ -97,51 +40,11 @@ std::atomic<int> g_tune_gemm{0};  // 1: qgemm_bf16 always takes its general rout
 std::atomic<int> g_tune_gemm_f16{0};  // 1: the Q4_0 matrix-core product with weights rounded to binary16
 std::atomic<int> g_tune_attn{0};  // 1: the general kernels also for one query position
 }
-thread_local char t_last_kernel[160] = "";
-thread_local std::vector<hipEvent_t> t_events;
-thread_local size_t t_events_used = 0;
 namespace mimir {
-void set_llama_step_mode(int mode);  // llm.hip
+void set_llama_step_mode(int mode);  // decoder.hip
 void set_llama_rows_off(int v);      // llm.hip
-void note_kernel(const char* fmt, ...) {
-    va_list ap;
-    va_start(ap, fmt);
-    vsnprintf(t_last_kernel, sizeof t_last_kernel, fmt, ap);
-    va_end(ap);
-}
-bool next_timing_events(hipEvent_t* start, hipEvent_t* stop) {
-    if (t_events_used + 2 > t_events.size()) return false;
-    *start = t_events[t_events_used];
-    *stop = t_events[t_events_used + 1];
-    t_events_used += 2;
-    return true;
-}
 }
 namespace {
-
-mi355x_status current_state(DeviceState** out) {
-    int dev = 0;
-    HIP_TRY(hipGetDevice(&dev), "hipGetDevice");
-    if (dev < 0 || dev >= kMaxDevices) return fail(MI355X_ERR_INTERNAL, "mi355x: device %d out of range", dev);
-    std::lock_guard<std::mutex> lock(g_mu);
-    DeviceState& s = g_dev[dev];
-    if (!s.ready) {
-        hipDeviceProp_t prop;
-        HIP_TRY(hipGetDeviceProperties(&prop, dev), "hipGetDeviceProperties");
-        if (strncmp(prop.gcnArchName, "gfx950", 6) != 0)
-            return fail(MI355X_ERR_INTERNAL, "mi355x: device %d is %s; this library holds gfx950 code only", dev, prop.gcnArchName);
-        // the lookup first: if it fails nothing has been allocated that a later call would allocate again
-        HIP_TRY(hipGetSymbolAddress(&s.fixed, HIP_SYMBOL(g_noalloc_scratch)), "hipGetSymbolAddress(fixed scratch)");
-        if (!s.err_dev) {
-            HIP_TRY(hipMalloc((void**)&s.err_dev, 256), "hipMalloc(error word)");
-            HIP_TRY(hipMemset(s.err_dev, 0, 256), "hipMemset(error word)");
-        }
-        if (!s.err_host) HIP_TRY(hipHostMalloc((void**)&s.err_host, 256, hipHostMallocDefault), "hipHostMalloc(error word)");
-        s.ready = true;
-    }
-    *out = &s;
-    return MI355X_OK;
-}
 
 // Returns the calling stream's block `which` of the current device, at least `bytes` long (at least `floor`
 // when it has to be allocated); the first `zero_prefix` bytes of a new block are zeroed (tickets).
@@ -159,14 +62,14 @@ mi355x_status stream_scratch(void* stream, ScratchBlock StreamScratch::*which, s
         if (want < 2 * b.bytes) want = 2 * b.bytes;
         void* p = nullptr;
         hipError_t e = hipMalloc(&p, want);
-        if (e != hipSuccess) return fail((mi355x_status)e, "mi355x: hipMalloc(%s scratch, %zu bytes): %s", what, want, hipGetErrorName(e));
+        if (e != hipSuccess) return capi_fail((mi355x_status)e, "mi355x: hipMalloc(%s scratch, %zu bytes): %s", what, want, hipGetErrorName(e));
         if (zero_prefix) {
             // on the calling stream, so that the zeros are in place before the first kernel that takes a ticket there
             // (never under capture: the allocation above fails first)
             e = hipMemsetAsync(p, 0, zero_prefix < want ? zero_prefix : want, (hipStream_t)stream);
             if (e != hipSuccess) {
                 (void)hipFree(p);  // nothing has seen it yet
-                return fail((mi355x_status)e, "mi355x: hipMemset(%s tickets): %s", what, hipGetErrorName(e));
+                return capi_fail((mi355x_status)e, "mi355x: hipMemset(%s tickets): %s", what, hipGetErrorName(e));
             }
         }
         if (b.p) mine.retired.push_back(b.p);
@@ -190,7 +93,7 @@ struct ActSource {
 mi355x_status act_for(const ActSource& src, size_t bytes, void** out) {
     if (!src.fixed) return act_scratch(src.stream, bytes, out);
     if (bytes > src.fixed_bytes)
-        return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_noalloc: the converted activations take %zu bytes, the fixed scratch holds %zu", bytes, src.fixed_bytes);
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_noalloc: the converted activations take %zu bytes, the fixed scratch holds %zu", bytes, src.fixed_bytes);
     *out = src.fixed;
     return MI355X_OK;
 }
@@ -210,111 +113,22 @@ mi355x_status argmax_scratch(void* stream, size_t bytes, void** out) {
 
 }  // namespace
 
-// For the other host files of the library.
-namespace mimir {
-mi355x_status capi_fail(mi355x_status code, const char* fmt, ...) {
-    char buf[512];
-    va_list ap;
-    va_start(ap, fmt);
-    vsnprintf(buf, sizeof buf, fmt, ap);
-    va_end(ap);
-    g_last_error = buf;
-    return code;
-}
-uint32_t* device_error_word() {
-    DeviceState* s;
-    return current_state(&s) == MI355X_OK ? s->err_dev : nullptr;
-}
-}  // namespace mimir
-
 extern "C" {
-
-mi355x_status mi355x_init(int device) {
-    int n = 0;
-    HIP_TRY(hipGetDeviceCount(&n), "hipGetDeviceCount");
-    if (device < 0 || device >= n) return fail(MI355X_ERR_INTERNAL, "mi355x: device %d of %d", device, n);
-    HIP_TRY(hipSetDevice(device), "hipSetDevice");
-    DeviceState* s;
-    return current_state(&s);
-}
-
-size_t mi355x_last_error(char* buf, size_t n) {
-    if (buf && n) {
-        size_t c = g_last_error.size() < n - 1 ? g_last_error.size() : n - 1;
-        memcpy(buf, g_last_error.data(), c);
-        buf[c] = 0;
-    }
-    return g_last_error.size();
-}
-
-int mi355x_block_size(int dtype) { return mimir::block_size(dtype); }
-int mi355x_block_bytes(int dtype) { return mimir::block_bytes(dtype); }
-
-int64_t mi355x_bytes(int dtype, int64_t n) {
-    int bs = mimir::block_size(dtype), bb = mimir::block_bytes(dtype);
-    if (bb == 0 || n < 0 || n % bs != 0 || n / bs > INT64_MAX / bb) return -1;
-    return n / bs * bb;
-}
-
-mi355x_status mi355x_alloc(void** out, size_t bytes) {
-    if (!out) return fail(MI355X_ERR_INTERNAL, "mi355x: alloc: null result pointer");
-    *out = nullptr;
-    // at least 4 bytes, as the reference's Alloc (backend/rocm/rocm_linux.go:220-240)
-    hipError_t e = hipMalloc(out, bytes < 4 ? 4 : bytes);
-    if (e != hipSuccess) return hip_fail(e, "hipMalloc");
-    return MI355X_OK;
-}
-
-mi355x_status mi355x_free(void* ptr) {
-    if (!ptr) return MI355X_OK;
-    HIP_TRY(hipFree(ptr), "hipFree");
-    return MI355X_OK;
-}
-
-mi355x_status mi355x_upload(void* dst, const void* src, size_t bytes, void* stream) {
-    if (bytes == 0) return MI355X_OK;
-    if (!dst || !src) return fail(MI355X_ERR_INTERNAL, "mi355x: upload: null pointer");
-    HIP_TRY(hipMemcpyAsync(dst, src, bytes, hipMemcpyHostToDevice, (hipStream_t)stream), "hipMemcpyAsync(H2D)");
-    return MI355X_OK;
-}
-
-mi355x_status mi355x_download(void* dst, const void* src, size_t bytes, void* stream) {
-    if (bytes == 0) return MI355X_OK;
-    if (!dst || !src) return fail(MI355X_ERR_INTERNAL, "mi355x: download: null pointer");
-    HIP_TRY(hipMemcpyAsync(dst, src, bytes, hipMemcpyDeviceToHost, (hipStream_t)stream), "hipMemcpyAsync(D2H)");
-    HIP_TRY(hipStreamSynchronize((hipStream_t)stream), "hipStreamSynchronize");
-    return MI355X_OK;
-}
-
-mi355x_status mi355x_sync(void* stream) {
-    DeviceState* s;
-    if (mi355x_status st = current_state(&s)) return st;
-    HIP_TRY(hipMemcpyAsync(s->err_host, s->err_dev, 4, hipMemcpyDeviceToHost, (hipStream_t)stream), "hipMemcpyAsync(error word)");
-    HIP_TRY(hipStreamSynchronize((hipStream_t)stream), "hipStreamSynchronize");
-    uint32_t bits = *s->err_host;
-    if (bits) {
-        HIP_TRY(hipMemsetAsync(s->err_dev, 0, 4, (hipStream_t)stream), "hipMemsetAsync(error word)");
-        HIP_TRY(hipStreamSynchronize((hipStream_t)stream), "hipStreamSynchronize");
-        if (bits & mimir::kErrIndex) return fail(MI355X_ERR_INDEX, "mi355x: a gather read an index out of range");
-        return fail(MI355X_ERR_INTERNAL, "mi355x: device error bits %#x", bits);
-    }
-    return MI355X_OK;
-}
 
 // Tensor.MatMulT with bfloat16 activations (tensor/quant.go:45-48): float32
 // product, one rounding to the output's dtype.
 mi355x_status mi355x_qgemm_bf16(int dtype, const void* W, const void* X, void* Y, int64_t M, int64_t N, int64_t K, int64_t x_row_stride,
                                 int out_dtype, void* stream) {
-    if (!mimir::is_quantized(dtype)) return fail(MI355X_ERR_DTYPE, "mi355x: qgemm_bf16 by weights of dtype %d", dtype);
-    if (out_dtype != MI355X_BF16 && out_dtype != MI355X_F32) return fail(MI355X_ERR_DTYPE, "mi355x: qgemm_bf16 into dtype %d", out_dtype);
+    if (!mimir::is_quantized(dtype)) return capi_fail(MI355X_ERR_DTYPE, "mi355x: qgemm_bf16 by weights of dtype %d", dtype);
+    if (out_dtype != MI355X_BF16 && out_dtype != MI355X_F32) return capi_fail(MI355X_ERR_DTYPE, "mi355x: qgemm_bf16 into dtype %d", out_dtype);
     if (M < 0 || N < 0 || K < 0 || K % mimir::block_size(dtype) != 0)
-        return fail(MI355X_ERR_INTERNAL, "mi355x: qgemm_bf16 of [%lld, %lld] by [%lld, %lld] in blocks of %d", (long long)M, (long long)K,
+        return capi_fail(MI355X_ERR_INTERNAL, "mi355x: qgemm_bf16 of [%lld, %lld] by [%lld, %lld] in blocks of %d", (long long)M, (long long)K,
                     (long long)N, (long long)K, mimir::block_size(dtype));
     if (M == 0 || N == 0) return MI355X_OK;
-    if (!W || !X || !Y) return fail(MI355X_ERR_INTERNAL, "mi355x: qgemm_bf16: null pointer");
+    if (!W || !X || !Y) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: qgemm_bf16: null pointer");
     if (M > 65535 || N > (int64_t)1 << 24 || K > (int64_t)1 << 24)
-        return fail(MI355X_ERR_SHAPE, "mi355x: qgemm_bf16 of %lld rows by [%lld, %lld]: too large", (long long)M, (long long)N, (long long)K);
-    if (M > 1 && x_row_stride < K) return fail(MI355X_ERR_SHAPE, "mi355x: qgemm_bf16: rows of x %lld apart overlap (K = %lld)", (long long)x_row_stride, (long long)K);
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemm_bf16 of %lld rows by [%lld, %lld]: too large", (long long)M, (long long)N, (long long)K);
+    if (M > 1 && x_row_stride < K) return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemm_bf16: rows of x %lld apart overlap (K = %lld)", (long long)x_row_stride, (long long)K);
     hipStream_t st = (hipStream_t)stream;
     const bool f32 = out_dtype == MI355X_F32;
     if (K == 0) {
@@ -375,18 +189,18 @@ mi355x_status mi355x_qgemm_bf16(int dtype, const void* W, const void* X, void* Y
 static mi355x_status qgemv_impl(int dtype, const void* W, const float* x, float* y, int64_t M, int64_t N, int64_t K, int64_t x_row_stride,
                                 void* stream, const ActSource& src) {
     const TuneQ4 g_tune_q4;  // this call's copy of the launch-plan overrides
-    if (!mimir::is_quantized(dtype)) return fail(MI355X_ERR_DTYPE, "mi355x: qgemv by weights of dtype %d", dtype);
+    if (!mimir::is_quantized(dtype)) return capi_fail(MI355X_ERR_DTYPE, "mi355x: qgemv by weights of dtype %d", dtype);
     int bs = mimir::block_size(dtype);
     if (M < 0 || N < 0 || K < 0 || K % bs != 0)
-        return fail(MI355X_ERR_INTERNAL, "mi355x: qgemv of [%lld, %lld] by [%lld, %lld] in blocks of %d", (long long)M,
+        return capi_fail(MI355X_ERR_INTERNAL, "mi355x: qgemv of [%lld, %lld] by [%lld, %lld] in blocks of %d", (long long)M,
                     (long long)K, (long long)N, (long long)K, bs);
     if (M == 0 || N == 0) return MI355X_OK;
-    if (!W || !x || !y) return fail(MI355X_ERR_INTERNAL, "mi355x: qgemv: null pointer");
+    if (!W || !x || !y) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: qgemv: null pointer");
     if (M > 65535 || N > (int64_t)1 << 30 || K > (int64_t)1 << 30)
-        return fail(MI355X_ERR_SHAPE, "mi355x: qgemv of %lld rows by [%lld, %lld]: too large", (long long)M, (long long)N,
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv of %lld rows by [%lld, %lld]: too large", (long long)M, (long long)N,
                     (long long)K);
     if (M > 1 && x_row_stride < K && x_row_stride != 0)
-        return fail(MI355X_ERR_SHAPE, "mi355x: qgemv: rows of x %lld apart overlap (K = %lld)", (long long)x_row_stride, (long long)K);
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv: rows of x %lld apart overlap (K = %lld)", (long long)x_row_stride, (long long)K);
     if (K == 0) {  // an empty sum: zeros (backend/cpu/qmatmul.go:336-339)
         HIP_TRY(mimir::fill_u32(y, 0, M * N, (hipStream_t)stream), "launch fill");
         return MI355X_OK;
@@ -449,7 +263,7 @@ static mi355x_status qgemv_impl(int dtype, const void* W, const float* x, float*
         HIP_TRY(mimir::qgemv_q4_0(a, g_tune_q4, (hipStream_t)stream), "launch qgemv_q4_0");
         return MI355X_OK;
     case MI355X_Q8_0: {
-        if (!mimir::q8_act_fits(K)) return fail(MI355X_ERR_SHAPE, "mi355x: qgemv by q8_0 with K = %lld: rows longer than 57344 are not supported", (long long)K);
+        if (!mimir::q8_act_fits(K)) return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv by q8_0 with K = %lld: rows longer than 57344 are not supported", (long long)K);
         // Small products in one launch (a.act stays null: every workgroup rounds x for itself); this kernel does not
         // request its weights ahead of that, so on large ones a conversion launch of its own is the faster (measured).
         if (M <= kConvertInProductRows && N * K <= (int64_t)24 << 20 && ((uintptr_t)x & 15) == 0 && (M == 1 || x_row_stride % 4 == 0)) {
@@ -487,7 +301,7 @@ static mi355x_status qgemv_impl(int dtype, const void* W, const float* x, float*
         return MI355X_OK;
     }
     default:
-        return fail(MI355X_ERR_DTYPE, "mi355x: qgemv by weights of dtype %d", dtype);
+        return capi_fail(MI355X_ERR_DTYPE, "mi355x: qgemv by weights of dtype %d", dtype);
     }
 }
 
@@ -507,7 +321,7 @@ mi355x_status mi355x_qgemv_noalloc(int dtype, const void* W, const float* x, flo
         std::lock_guard<std::mutex> lock(g_mu);
         if (g_dev[dev].ready) fixed = g_dev[dev].fixed;
     }
-    if (!fixed) return fail(MI355X_ERR_INTERNAL, "mi355x: qgemv_noalloc: call mi355x_init(%d) first (creating the device's state allocates)", dev);
+    if (!fixed) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: qgemv_noalloc: call mi355x_init(%d) first (creating the device's state allocates)", dev);
     return qgemv_impl(dtype, W, x, y, M, N, K, x_row_stride, stream, ActSource{stream, fixed, kNoallocScratchBytes});
 }
 
@@ -521,9 +335,9 @@ size_t mi355x_act_bytes(int dtype, int64_t K) {
 
 mi355x_status mi355x_convert_act(int dtype, const float* x, int64_t M, int64_t K, int64_t x_row_stride, void* act, void* stream) {
     if (mi355x_act_bytes(dtype, K) == 0 || M < 0 || M > 65535)
-        return fail(MI355X_ERR_SHAPE, "mi355x: convert activations [%lld, %lld] for weights of dtype %d", (long long)M, (long long)K, dtype);
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: convert activations [%lld, %lld] for weights of dtype %d", (long long)M, (long long)K, dtype);
     if (M == 0) return MI355X_OK;
-    if (!x || !act || ((uintptr_t)act & 15)) return fail(MI355X_ERR_INTERNAL, "mi355x: convert activations: null or misaligned pointer");
+    if (!x || !act || ((uintptr_t)act & 15)) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: convert activations: null or misaligned pointer");
     if (dtype == MI355X_Q4_0)
         HIP_TRY(mimir::q4_0_convert_act(x, M, K, x_row_stride, act, (hipStream_t)stream), "launch q4_0_convert_act");
     else if (dtype == MI355X_Q8_0)
@@ -536,23 +350,23 @@ mi355x_status mi355x_convert_act(int dtype, const float* x, int64_t M, int64_t K
 mi355x_status mi355x_qgemv_act(int dtype, const void* W, const void* act, float* y, int64_t M, int64_t N, int64_t K, void* stream) {
     const TuneQ4 g_tune_q4;  // this call's copy of the launch-plan overrides
     if (M < 0 || N < 0 || K <= 0 || M > 65535 || N > (int64_t)1 << 30)
-        return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act of %lld rows by [%lld, %lld]", (long long)M, (long long)N, (long long)K);
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act of %lld rows by [%lld, %lld]", (long long)M, (long long)N, (long long)K);
     if (M == 0 || N == 0) return MI355X_OK;
-    if (!W || !act || !y || ((uintptr_t)act & 15)) return fail(MI355X_ERR_INTERNAL, "mi355x: qgemv_act: null or misaligned pointer");
+    if (!W || !act || !y || ((uintptr_t)act & 15)) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: qgemv_act: null or misaligned pointer");
     mimir::QGemvArgs a{W, nullptr, act, y, M, N, K, 0, 0};
     if (dtype == MI355X_Q4_0) {
         if (!mimir::q4_0_fixed_point_ok(W, K))
-            return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act by q4_0 needs K a multiple of 64 up to 20928 and W dword aligned (K = %lld)", (long long)K);
+            return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act by q4_0 needs K a multiple of 64 up to 20928 and W dword aligned (K = %lld)", (long long)K);
         HIP_TRY(mimir::qgemv_q4_0_act(a, g_tune_q4, (hipStream_t)stream), "launch qgemv_q4_0_act");
     } else if (dtype == MI355X_Q8_0) {
         if (K % 32 != 0 || !mimir::q8_act_fits(K))
-            return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act by q8_0 needs K a multiple of 32 up to 57344 (K = %lld)", (long long)K);
+            return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act by q8_0 needs K a multiple of 32 up to 57344 (K = %lld)", (long long)K);
         HIP_TRY(mimir::qgemv_q8_0_act(a, g_tune_q4, (hipStream_t)stream), "launch qgemv_q8_0_act");
     } else if (dtype == MI355X_Q4_K || dtype == MI355X_Q6_K) {
-        if (K % 256 != 0) return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act by a K-quant needs K a multiple of 256 (K = %lld)", (long long)K);
+        if (K % 256 != 0) return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act by a K-quant needs K a multiple of 256 (K = %lld)", (long long)K);
         HIP_TRY(mimir::qgemv_kquant_act(dtype, a, (hipStream_t)stream), "launch qgemv_kquant_act");
     } else {
-        return fail(MI355X_ERR_DTYPE, "mi355x: qgemv_act by dtype %d", dtype);
+        return capi_fail(MI355X_ERR_DTYPE, "mi355x: qgemv_act by dtype %d", dtype);
     }
     return MI355X_OK;
 }
@@ -560,18 +374,18 @@ mi355x_status mi355x_qgemv_act(int dtype, const void* W, const void* act, float*
 // The fused products of a decoding step. The reference fuses the same ones on
 // its CPU path by concatenating weights (fusedFor, llm/decode.go:240-266).
 static mi355x_status fused_args_ok(const char* what, int dtype, const void* act, const float* y, int64_t M, int64_t K) {
-    if (dtype != MI355X_Q4_0) return fail(MI355X_ERR_DTYPE, "mi355x: %s by weights of dtype %d (q4_0 only)", what, dtype);
-    if (M < 0 || M > 65535 || K <= 0) return fail(MI355X_ERR_SHAPE, "mi355x: %s of [%lld, %lld]", what, (long long)M, (long long)K);
-    if (!act || !y || ((uintptr_t)act & 15)) return fail(MI355X_ERR_INTERNAL, "mi355x: %s: null or misaligned pointer", what);
+    if (dtype != MI355X_Q4_0) return capi_fail(MI355X_ERR_DTYPE, "mi355x: %s by weights of dtype %d (q4_0 only)", what, dtype);
+    if (M < 0 || M > 65535 || K <= 0) return capi_fail(MI355X_ERR_SHAPE, "mi355x: %s of [%lld, %lld]", what, (long long)M, (long long)K);
+    if (!act || !y || ((uintptr_t)act & 15)) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: %s: null or misaligned pointer", what);
     return MI355X_OK;
 }
 
 mi355x_status mi355x_qgemv_act_add(int dtype, const void* W, const void* act, const float* resid, float* y, int64_t M, int64_t N, int64_t K, void* stream) {
     const TuneQ4 g_tune_q4;  // this call's copy of the launch-plan overrides
     if (mi355x_status st = fused_args_ok("qgemv_act_add", dtype, act, y, M, K)) return st;
-    if (N < 0 || N > (int64_t)1 << 30) return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_add of %lld rows", (long long)N);
+    if (N < 0 || N > (int64_t)1 << 30) return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_add of %lld rows", (long long)N);
     if (M == 0 || N == 0) return MI355X_OK;
-    if (!W || !resid || !mimir::q4_0_fixed_point_ok(W, K)) return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_add needs K a multiple of 64 up to 20928 and W dword aligned");
+    if (!W || !resid || !mimir::q4_0_fixed_point_ok(W, K)) return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_add needs K a multiple of 64 up to 20928 and W dword aligned");
     mimir::QGemvArgs a{W, nullptr, act, y, M, N, K, 0, 0};
     a.resid = resid;
     HIP_TRY(mimir::qgemv_q4_0_act(a, g_tune_q4, (hipStream_t)stream), "launch qgemv_q4_0_act");
@@ -585,12 +399,12 @@ mi355x_status mi355x_qgemv_act_multi(int dtype, const void* W0, const void* W1, 
     const void* W[3] = {W0, W1, W2};
     const int64_t n[3] = {n0, n1, n2};
     for (int i = 0; i < 3; i++) {
-        if (n[i] < 0 || n[i] > (int64_t)1 << 28) return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_multi: matrix %d of %lld rows", i, (long long)n[i]);
+        if (n[i] < 0 || n[i] > (int64_t)1 << 28) return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_multi: matrix %d of %lld rows", i, (long long)n[i]);
         if (n[i] > 0 && (!W[i] || !mimir::q4_0_fixed_point_ok(W[i], K)))
-            return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_multi needs K a multiple of 64 up to 20928 and every W dword aligned");
+            return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_multi needs K a multiple of 64 up to 20928 and every W dword aligned");
     }
-    if (n0 == 0 && (n1 > 0 || n2 > 0)) return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_multi: the first matrix is empty");
-    if (n1 == 0 && n2 > 0) return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_multi: the second matrix is empty");
+    if (n0 == 0 && (n1 > 0 || n2 > 0)) return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_multi: the first matrix is empty");
+    if (n1 == 0 && n2 > 0) return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_multi: the second matrix is empty");
     if (M == 0 || n0 + n1 + n2 == 0) return MI355X_OK;
     HIP_TRY(mimir::qgemv_q4_0_act_multi(W, n, act, y, M, K, g_tune_q4, (hipStream_t)stream), "launch qgemv_q4_0_act_multi");
     return MI355X_OK;
@@ -599,32 +413,32 @@ mi355x_status mi355x_qgemv_act_multi(int dtype, const void* W0, const void* W1, 
 mi355x_status mi355x_qgemv_act_swiglu(int dtype, const void* gate, const void* up, const void* act, float* y, int64_t M, int64_t N, int64_t K, void* stream) {
     const TuneQ4 g_tune_q4;  // this call's copy of the launch-plan overrides
     if (mi355x_status st = fused_args_ok("qgemv_act_swiglu", dtype, act, y, M, K)) return st;
-    if (N < 0 || N > (int64_t)1 << 28) return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_swiglu of %lld rows", (long long)N);
+    if (N < 0 || N > (int64_t)1 << 28) return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_swiglu of %lld rows", (long long)N);
     if (M == 0 || N == 0) return MI355X_OK;
     if (!gate || !up || !mimir::q4_0_fixed_point_ok(gate, K) || !mimir::q4_0_fixed_point_ok(up, K))
-        return fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_swiglu needs K a multiple of 64 up to 20928 and both W dword aligned");
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: qgemv_act_swiglu needs K a multiple of 64 up to 20928 and both W dword aligned");
     HIP_TRY(mimir::qgemv_q4_0_act_swiglu(gate, up, act, y, M, N, K, g_tune_q4, (hipStream_t)stream), "launch qgemv_q4_0_act_swiglu");
     return MI355X_OK;
 }
 
 mi355x_status mi355x_dequant(int dtype, const void* W, int64_t first, int64_t n, void* out, int out_dtype, void* stream) {
-    if (!mimir::is_quantized(dtype)) return fail(MI355X_ERR_DTYPE, "mi355x: dequantize dtype %d", dtype);
+    if (!mimir::is_quantized(dtype)) return capi_fail(MI355X_ERR_DTYPE, "mi355x: dequantize dtype %d", dtype);
     if (out_dtype != MI355X_F32 && out_dtype != MI355X_BF16 && out_dtype != MI355X_F16)
-        return fail(MI355X_ERR_DTYPE, "mi355x: dequantize into dtype %d", out_dtype);  // backend/cpu/quant.go:288-290
-    if (first < 0 || n < 0) return fail(MI355X_ERR_INTERNAL, "mi355x: dequantize elements [%lld, +%lld)", (long long)first, (long long)n);
+        return capi_fail(MI355X_ERR_DTYPE, "mi355x: dequantize into dtype %d", out_dtype);  // backend/cpu/quant.go:288-290
+    if (first < 0 || n < 0) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: dequantize elements [%lld, +%lld)", (long long)first, (long long)n);
     if (n == 0) return MI355X_OK;
-    if (!W || !out) return fail(MI355X_ERR_INTERNAL, "mi355x: dequantize: null pointer");
+    if (!W || !out) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: dequantize: null pointer");
     HIP_TRY(mimir::dequantize(dtype, W, first, n, out, out_dtype, (hipStream_t)stream), "launch dequantize");
     return MI355X_OK;
 }
 
 mi355x_status mi355x_gather_rows(int dtype, const void* table, int64_t rows, int64_t K, const int32_t* idx, int64_t n,
                                  float* out, void* stream) {
-    if (!mimir::is_quantized(dtype)) return fail(MI355X_ERR_DTYPE, "mi355x: gather from dtype %d", dtype);
+    if (!mimir::is_quantized(dtype)) return capi_fail(MI355X_ERR_DTYPE, "mi355x: gather from dtype %d", dtype);
     if (rows < 0 || K < 0 || n < 0 || K % mimir::block_size(dtype) != 0 || n > 65535)
-        return fail(MI355X_ERR_SHAPE, "mi355x: gather %lld rows of [%lld, %lld]", (long long)n, (long long)rows, (long long)K);
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: gather %lld rows of [%lld, %lld]", (long long)n, (long long)rows, (long long)K);
     if (n == 0 || K == 0) return MI355X_OK;
-    if (!table || !idx || !out) return fail(MI355X_ERR_INTERNAL, "mi355x: gather: null pointer");
+    if (!table || !idx || !out) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: gather: null pointer");
     DeviceState* s;
     if (mi355x_status st = current_state(&s)) return st;
     HIP_TRY(mimir::gather_rows(dtype, table, rows, K, idx, n, out, s->err_dev, (hipStream_t)stream), "launch gather_rows");
@@ -632,9 +446,9 @@ mi355x_status mi355x_gather_rows(int dtype, const void* table, int64_t rows, int
 }
 
 mi355x_status mi355x_rmsnorm(const float* x, const float* w, float* y, int64_t rows, int64_t d, double eps, void* stream) {
-    if (rows < 0 || d < 0 || rows > INT32_MAX || d > INT32_MAX) return fail(MI355X_ERR_SHAPE, "mi355x: rmsnorm of [%lld, %lld]", (long long)rows, (long long)d);
+    if (rows < 0 || d < 0 || rows > INT32_MAX || d > INT32_MAX) return capi_fail(MI355X_ERR_SHAPE, "mi355x: rmsnorm of [%lld, %lld]", (long long)rows, (long long)d);
     if (rows == 0 || d == 0) return MI355X_OK;
-    if (!x || !y) return fail(MI355X_ERR_INTERNAL, "mi355x: rmsnorm: null pointer");
+    if (!x || !y) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: rmsnorm: null pointer");
     HIP_TRY(mimir::rmsnorm(x, w, y, rows, d, eps, (hipStream_t)stream), "launch rmsnorm");
     return MI355X_OK;
 }
@@ -645,10 +459,10 @@ mi355x_status mi355x_rope(const float* x, float* y, int64_t rows, int64_t S, int
     // nn/transformer.go:229-231
     if (rows < 0 || S < 0 || head_dim <= 0 || rope_dim <= 0 || rope_dim % 2 != 0 || rope_dim > head_dim || offset < 0 ||
         offset + S > table_len)
-        return fail(MI355X_ERR_SHAPE, "mi355x: rotary embedding of %d of %d features at positions [%lld, %lld) of a table of %lld",
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: rotary embedding of %d of %d features at positions [%lld, %lld) of a table of %lld",
                     rope_dim, head_dim, (long long)offset, (long long)(offset + S), (long long)table_len);
     if (rows == 0 || S == 0) return MI355X_OK;
-    if (!x || !y || !cos_table || !sin_table) return fail(MI355X_ERR_INTERNAL, "mi355x: rope: null pointer");
+    if (!x || !y || !cos_table || !sin_table) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: rope: null pointer");
     HIP_TRY(mimir::rope(x, y, rows, S, head_dim, rope_dim, interleaved, x_row_stride, x_pos_stride, y_row_stride, y_pos_stride,
                         cos_table, sin_table, offset, (hipStream_t)stream), "launch rope");
     return MI355X_OK;
@@ -657,12 +471,12 @@ mi355x_status mi355x_rope(const float* x, float* y, int64_t rows, int64_t S, int
 mi355x_status mi355x_kv_write(const float* src, void* cache, int cache_dtype, int64_t B, int heads, int64_t S, int dim,
                               int64_t capacity, int64_t pos, int64_t src_b_stride, int64_t src_h_stride, int64_t src_p_stride,
                               void* stream) {
-    if (cache_dtype != MI355X_F32 && cache_dtype != MI355X_F16) return fail(MI355X_ERR_DTYPE, "mi355x: KV cache of dtype %d", cache_dtype);
+    if (cache_dtype != MI355X_F32 && cache_dtype != MI355X_F16) return capi_fail(MI355X_ERR_DTYPE, "mi355x: KV cache of dtype %d", cache_dtype);
     // nn/transformer.go:405-411
     if (B < 0 || heads <= 0 || S < 0 || dim <= 0 || pos < 0 || pos + S > capacity)
-        return fail(MI355X_ERR_SHAPE, "mi355x: write %lld positions at %lld to a cache of %lld", (long long)S, (long long)pos, (long long)capacity);
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: write %lld positions at %lld to a cache of %lld", (long long)S, (long long)pos, (long long)capacity);
     if (B == 0 || S == 0) return MI355X_OK;
-    if (!src || !cache) return fail(MI355X_ERR_INTERNAL, "mi355x: kv_write: null pointer");
+    if (!src || !cache) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: kv_write: null pointer");
     HIP_TRY(mimir::kv_write(src, cache, cache_dtype, B, heads, S, dim, capacity, pos, src_b_stride, src_h_stride, src_p_stride,
                             (hipStream_t)stream), "launch kv_write");
     return MI355X_OK;
@@ -672,15 +486,15 @@ mi355x_status mi355x_attention(const float* q, const int64_t* q_strides, const v
                                const int64_t* v_strides, int kv_dtype, const float* mask, const int64_t* mask_strides, float* out,
                                const int64_t* out_strides, float* lse, int64_t B, int H, int HK, int64_t Q, int64_t K, int D, int DV, double scale,
                                int causal, int64_t causal_offset, void* stream) {
-    if (kv_dtype != MI355X_F32 && kv_dtype != MI355X_F16) return fail(MI355X_ERR_DTYPE, "mi355x: attention over keys of dtype %d", kv_dtype);
+    if (kv_dtype != MI355X_F32 && kv_dtype != MI355X_F16) return capi_fail(MI355X_ERR_DTYPE, "mi355x: attention over keys of dtype %d", kv_dtype);
     // backend/attention.go:36-62
     if (B < 0 || Q < 0 || K < 0 || H <= 0 || HK <= 0 || H % HK != 0 || D <= 0 || D > 256 || DV <= 0 || DV > 256)
-        return fail(MI355X_ERR_SHAPE, "mi355x: attention of %d heads on %d key heads of %d features and values of %d (at most 256)", H, HK, D, DV);
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: attention of %d heads on %d key heads of %d features and values of %d (at most 256)", H, HK, D, DV);
     if (B == 0 || Q == 0) return MI355X_OK;
     if (B * Q > 65535 || (int64_t)HK * ((H / HK + 3) / 4) > 65535)
-        return fail(MI355X_ERR_SHAPE, "mi355x: attention of %lld query rows: too many for one launch", (long long)(B * Q));
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: attention of %lld query rows: too many for one launch", (long long)(B * Q));
     if (!q || !out || !q_strides || !out_strides || (K > 0 && (!k || !v || !k_strides || !v_strides)) || (mask && !mask_strides))
-        return fail(MI355X_ERR_INTERNAL, "mi355x: attention: null pointer");
+        return capi_fail(MI355X_ERR_INTERNAL, "mi355x: attention: null pointer");
     mimir::AttnArgs a;
     a.q = q; a.k = k; a.v = v; a.kv_dtype = kv_dtype; a.out = out; a.lse = lse;
     for (int i = 0; i < 3; i++) {
@@ -722,31 +536,31 @@ mi355x_status mi355x_attention(const float* q, const int64_t* q_strides, const v
 }
 
 mi355x_status mi355x_attention_d(const mi355x_attention_desc* d, void* stream) {
-    if (!d) return fail(MI355X_ERR_INTERNAL, "mi355x: attention_d: null descriptor");
+    if (!d) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: attention_d: null descriptor");
     return mi355x_attention(d->q, d->q_strides, d->k, d->k_strides, d->v, d->v_strides, d->kv_dtype, d->mask, d->mask_strides, d->out, d->out_strides, d->lse,
                             d->B, d->H, d->HK, d->Q, d->K, d->D, d->DV, d->scale, d->causal, d->causal_offset, stream);
 }
 
 mi355x_status mi355x_swiglu(const float* gate, const float* up, float* out, int64_t rows, int64_t n, int64_t in_row_stride, void* stream) {
-    if (rows < 0 || n < 0) return fail(MI355X_ERR_SHAPE, "mi355x: swiglu of [%lld, %lld]", (long long)rows, (long long)n);
+    if (rows < 0 || n < 0) return capi_fail(MI355X_ERR_SHAPE, "mi355x: swiglu of [%lld, %lld]", (long long)rows, (long long)n);
     if (rows == 0 || n == 0) return MI355X_OK;
-    if (!gate || !up || !out) return fail(MI355X_ERR_INTERNAL, "mi355x: swiglu: null pointer");
+    if (!gate || !up || !out) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: swiglu: null pointer");
     HIP_TRY(mimir::swiglu(gate, up, out, rows, n, in_row_stride, (hipStream_t)stream), "launch swiglu");
     return MI355X_OK;
 }
 
 mi355x_status mi355x_add(const float* a, const float* b, float* out, int64_t n, void* stream) {
-    if (n < 0) return fail(MI355X_ERR_SHAPE, "mi355x: add of %lld elements", (long long)n);
+    if (n < 0) return capi_fail(MI355X_ERR_SHAPE, "mi355x: add of %lld elements", (long long)n);
     if (n == 0) return MI355X_OK;
-    if (!a || !b || !out) return fail(MI355X_ERR_INTERNAL, "mi355x: add: null pointer");
+    if (!a || !b || !out) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: add: null pointer");
     HIP_TRY(mimir::add(a, b, out, n, (hipStream_t)stream), "launch add");
     return MI355X_OK;
 }
 
 mi355x_status mi355x_argmax(const float* logits, int64_t rows, int64_t n, int32_t* out, void* stream) {
-    if (rows < 0 || n <= 0 || n > INT32_MAX || rows > 65535) return fail(MI355X_ERR_SHAPE, "mi355x: argmax of [%lld, %lld]", (long long)rows, (long long)n);
+    if (rows < 0 || n <= 0 || n > INT32_MAX || rows > 65535) return capi_fail(MI355X_ERR_SHAPE, "mi355x: argmax of [%lld, %lld]", (long long)rows, (long long)n);
     if (rows == 0) return MI355X_OK;
-    if (!logits || !out) return fail(MI355X_ERR_INTERNAL, "mi355x: argmax: null pointer");
+    if (!logits || !out) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: argmax: null pointer");
     void* ws = nullptr;
     if (rows <= 1024)
         if (mi355x_status st = argmax_scratch(stream, mimir::argmax_workspace_bytes(1024), &ws)) return st;
@@ -884,13 +698,13 @@ mi355x_status mi355x_tune(const char* key, int value) {
         mimir::set_llama_step_mode(value);
         return MI355X_OK;
     }
-    return fail(MI355X_ERR_INTERNAL, "mi355x: unknown tuning key %s", key ? key : "(null)");
+    return capi_fail(MI355X_ERR_INTERNAL, "mi355x: unknown tuning key %s", key ? key : "(null)");
 }
 
 // Per-launch timing of the fixed-point Q4_0 kernel: between timed_begin and
 // timed_end every such launch of this thread carries its own pair of events.
 mi355x_status mi355x_timed_begin(int max_launches) {
-    if (max_launches <= 0 || max_launches > (1 << 20) || !t_events.empty()) return fail(MI355X_ERR_INTERNAL, "mi355x: timed_begin(%d)", max_launches);
+    if (max_launches <= 0 || max_launches > (1 << 20) || !t_events.empty()) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: timed_begin(%d)", max_launches);
     t_events.resize(2 * (size_t)max_launches);
     for (auto& e : t_events) HIP_TRY(hipEventCreate(&e), "hipEventCreate");
     t_events_used = 0;
@@ -898,7 +712,7 @@ mi355x_status mi355x_timed_begin(int max_launches) {
 }
 
 mi355x_status mi355x_timed_end(float* ms_each, int* n_launches) {
-    if (!ms_each || !n_launches) return fail(MI355X_ERR_INTERNAL, "mi355x: timed_end: null pointer");
+    if (!ms_each || !n_launches) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: timed_end: null pointer");
     hipError_t e = hipDeviceSynchronize();
     size_t n = t_events_used / 2;
     for (size_t i = 0; i < n && e == hipSuccess; i++) e = hipEventElapsedTime(&ms_each[i], t_events[2 * i], t_events[2 * i + 1]);
@@ -920,14 +734,14 @@ mi355x_status mi355x_gemv_stamps(void* stamps) {
 
 // The kernel (name and template arguments) that the calling thread's latest Q4_0 product (one row of x, or prompt-sized) launched.
 mi355x_status mi355x_last_kernel(char* buf, size_t n) {
-    if (!buf || n == 0) return fail(MI355X_ERR_INTERNAL, "mi355x: last_kernel: no buffer");
+    if (!buf || n == 0) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: last_kernel: no buffer");
     snprintf(buf, n, "%s", t_last_kernel);
     return MI355X_OK;
 }
 
 mi355x_status mi355x_stream_read(const void* p, size_t bytes, float* scratch, int grid, int threads, void* stream) {
     if (!p || !scratch || grid <= 0 || threads <= 0 || threads > 1024 || threads % 64 != 0 || ((uintptr_t)p & 15))
-        return fail(MI355X_ERR_INTERNAL, "mi355x: stream_read: bad arguments");
+        return capi_fail(MI355X_ERR_INTERNAL, "mi355x: stream_read: bad arguments");
     HIP_TRY(mimir::stream_read(p, bytes, scratch, grid, threads, (hipStream_t)stream), "launch stream_read");
     return MI355X_OK;
 }

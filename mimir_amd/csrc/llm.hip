@@ -25,51 +25,14 @@
 #include <string>
 #include <vector>
 
+#include "decoder.h"
 #include "kernels.h"
 
 namespace mimir {
 
-mi355x_status capi_fail(mi355x_status code, const char* fmt, ...);  // capi.hip
-
 namespace {
 
-#define LLM_HIP(expr, what)                                                          \
-    do {                                                                             \
-        hipError_t e_ = (expr);                                                      \
-        if (e_ != hipSuccess) return capi_fail((mi355x_status)e_, "mi355x: llama: %s: %s", what, hipGetErrorName(e_)); \
-    } while (0)
-
-struct DevBuf {
-    void* p = nullptr;
-    size_t bytes = 0;
-    bool view = false;  // p points into another buffer's memory
-    ~DevBuf() { release(); }
-    void release() {
-        if (p && !view) (void)hipFree(p);
-        p = nullptr;
-        view = false;
-    }
-    hipError_t alloc(size_t n) {
-        release();
-        bytes = n;
-        return hipMalloc(&p, n < 4 ? 4 : n);
-    }
-    void point_at(void* q, size_t n) {
-        release();
-        p = q;
-        bytes = n;
-        view = true;
-    }
-    template <typename T>
-    T* as() const { return (T*)p; }
-};
-
-struct Weight {
-    int dtype = 0;
-    int64_t n = 0, k = 0;
-    DevBuf buf;
-    bool set() const { return buf.p != nullptr; }
-};
+#define LLM_HIP(expr, what) DECODER_HIP(expr, "llama", what)
 
 // The form of converted activations a weight's product reads.
 // kActFx: Q4_0 by many rows of x, on the int8 matrix cores; kActFxPairs: the same product through the binary16 ones
@@ -86,43 +49,36 @@ struct Block {
     bool biased() const { return q_bias.set(); }
 };
 
-struct Model {
+struct Model : Decoder {
     mi355x_llama_config c{};
     Weight embed, norm, output;
     bool tied = false;
     std::vector<Block> blocks;
     std::vector<float> rope_factors;
-    bool ready = false;
 
     DevBuf cos_t, sin_t;                 // [context, rope_dim/2]
     DevBuf attn_flags;                   // decode attention's (value, flag) slots: zero between launches
     std::vector<DevBuf> keys, values;    // per block: [batch, kv_heads, context, head_dim]
-    int64_t cache_len = 0;
 
     // activations of up to max_rows rows (batch x tokens of one call)
-    int64_t max_rows = 0;
-    DevBuf x, h, q, k, v, a, o, gate, up, s, xlast, hlast, logits, act[kActClasses], act2, tokens_dev, next_tok;
+    DevBuf x, h, q, k, v, a, o, gate, up, s, xlast, hlast, act[kActClasses], act2;
     DevBuf fx_panel;  // the workspace of the fixed-point Q4_0 product of a prompt's rows in its binary16 form: the largest matrix's
-    hipStream_t stream = nullptr;
 
-    // The decoding step as a fixed run of launches that read the position from
-    // the device: state = {position, steps taken}; record holds the tokens
-    // chosen so far, [max_new, batch]. `fast` says the blocks qualify (Q4_0
-    // linears that the fixed-point kernel takes); step_graph replays the run.
+    // `fast` says the blocks qualify for the step of fused launches (Q4_0 linears that the fixed-point kernel takes).
     bool fast = false;
-    DevBuf state, record, qkv, gu, argmax_ws;  // gu: gate|up of a step, [batch, 2 hidden]
+    DevBuf qkv, gu;  // gu: gate|up of a step, [batch, 2 hidden]
     // `rows`: a fast model with two to sixty-four sequences, whose step reads every weight once per eight of them
     // (step_rows): the sequences' activations converted together, and the two shares of K of the output and
     // down projections, [2, batch, embed].
     bool rows = false;
     DevBuf rows_act, rows_act2, parts;
-    hipGraphExec_t step_graph = nullptr;
-    int graph_rows = 0;  // which step the graph holds: 0 step_fast or step_any, 1 step_rows, 2 step_rows without its riders
 
-    ~Model() {
-        if (step_graph) (void)hipGraphExecDestroy(step_graph);
-        if (stream) (void)hipStreamDestroy(stream);
-    }
+    mi355x_status set_tensor(const char* tensor, int dtype, const void* host, int64_t n_elems) override;
+    mi355x_status finalize(int64_t max_tokens) override;
+    mi355x_status forward(int64_t s) override;
+    mi355x_status head(const int64_t* rows, int64_t n) override;
+    mi355x_status step() override;
+    int step_variant() const override;
 };
 
 // panel_bytes: what the model holds as workspace for the fixed-point product's binary16 form (0: that form is not taken)
@@ -207,8 +163,6 @@ mi355x_status embed_rows(Model& m, const int32_t* idx_dev, int64_t rows, float* 
 }
 
 }  // namespace
-
-uint32_t* device_error_word();  // capi.hip
 
 // One pass of s tokens per sequence over the blocks (llm/model.go:391-437),
 // tokens already on the device at m.tokens_dev [batch, s]. Leaves the final
@@ -577,17 +531,33 @@ static mi355x_status head(Model& m, const float* xin, int64_t rows, int64_t row_
     return linear(m, w, hl, m.logits.as<float>(), rows);
 }
 
+mi355x_status Model::forward(int64_t s) { return mimir::forward(*this, s); }
+
+// Rows an equal distance apart (all of a call's, or the last of each sequence) in one run; others one by one.
+mi355x_status Model::head(const int64_t* rows_of, int64_t n) {
+    if (n <= 0) return MI355X_OK;
+    const int64_t apart = n > 1 ? rows_of[1] - rows_of[0] : 1;
+    for (int64_t i = 1; i < n; i++)
+        if (rows_of[i] - rows_of[i - 1] != apart || apart <= 0) {
+            if (n > max_rows) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: llama: %lld rows of logits", (long long)n);
+            for (int64_t r = 0; r < n; r++)  // gathered in o, which no pass is using now
+                LLM_HIP(hipMemcpyAsync(o.as<float>() + r * c.embed, x.as<float>() + rows_of[r] * c.embed, (size_t)c.embed * 4, hipMemcpyDeviceToDevice, stream), "gather rows");
+            return mimir::head(*this, o.as<float>(), n, c.embed);
+        }
+    return mimir::head(*this, x.as<float>() + rows_of[0] * c.embed, n, apart * c.embed);
+}
+
+mi355x_status Model::step() {
+    if (mi355x_status st = rows && !g_llama_rows_off ? step_rows(*this) : fast ? step_fast(*this) : step_any(*this)) return st;
+    return mimir::head(*this, x.as<float>(), c.batch, c.embed);
+}
+
+// 0 step_fast or step_any, 1 step_rows, more: step_rows without its riders
+int Model::step_variant() const { return rows && !g_llama_rows_off ? 1 + g_llama_rows_plain : 0; }
+
 }  // namespace mimir
 
 using mimir::Model;
-
-// How mi355x_llama_generate runs its decoding steps: 0 the fused launches
-// replayed as a graph where the model qualifies, 1 the same launches issued one
-// by one, 2 the general per-operator path.
-static std::atomic<int> g_llama_step_mode{0};
-namespace mimir {
-void set_llama_step_mode(int mode) { g_llama_step_mode = mode; }
-}
 
 extern "C" {
 
@@ -604,22 +574,17 @@ mi355x_status mi355x_llama_create(const mi355x_llama_config* cfg, void** out) {
     if (c.cache_dtype != MI355X_F32 && c.cache_dtype != MI355X_F16) return capi_fail(MI355X_ERR_DTYPE, "mi355x: llama: KV cache of dtype %d", c.cache_dtype);
     auto m = std::make_unique<Model>();
     m->c = c;
+    m->name = "llama"; m->vocab = c.vocab; m->context = c.context; m->batch = c.batch;
     m->blocks.resize(c.layers);
-    *out = m.release();
+    *out = (Decoder*)m.release();
     return MI355X_OK;
 }
 
-mi355x_status mi355x_llama_destroy(void* model) {
-    delete (Model*)model;
-    return MI355X_OK;
-}
+}  // extern "C"
 
 // Names are llama.cpp's, as the reference reads them (llm/model.go:268-310).
-mi355x_status mi355x_llama_set_tensor(void* model, const char* name, int dtype, const void* host, int64_t n_elems) {
-    using namespace mimir;
-    Model* m = (Model*)model;
-    if (!m || !name || !host) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: llama_set_tensor: null pointer");
-    const auto& c = m->c;
+mi355x_status mimir::Model::set_tensor(const char* name, int dtype, const void* host, int64_t n_elems) {
+    Model* m = this;
     const int64_t qd = (int64_t)c.heads * c.head_dim, kvd = (int64_t)c.kv_heads * c.head_dim;
     Weight* w = nullptr;
     int64_t n = 0, k = 0;
@@ -660,10 +625,12 @@ mi355x_status mi355x_llama_set_tensor(void* model, const char* name, int dtype, 
     return MI355X_OK;
 }
 
+extern "C" {
+
 // Divisors of each pair's frequency (rope_freqs.weight, llm/model.go:318-346).
 mi355x_status mi355x_llama_set_rope_factors(void* model, const float* factors, int32_t n) {
     using namespace mimir;
-    Model* m = (Model*)model;
+    Model* m = (Model*)(mimir::Decoder*)model;
     if (!m || (n > 0 && !factors)) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: llama_set_rope_factors: null pointer");
     if (n != 0 && n != m->c.rope_dim / 2) return capi_fail(MI355X_ERR_SHAPE, "mi355x: llama: %d rope frequency factors, want %d", n, m->c.rope_dim / 2);
     for (int i = 0; i < n; i++)
@@ -673,14 +640,13 @@ mi355x_status mi355x_llama_set_rope_factors(void* model, const float* factors, i
     return MI355X_OK;
 }
 
+}  // extern "C"
+
 // Checks that every tensor is there, builds the rotary table and allocates
 // the caches and the activations of calls of up to max_tokens tokens per
 // sequence.
-mi355x_status mi355x_llama_finalize(void* model, int64_t max_tokens) {
-    using namespace mimir;
-    Model* m = (Model*)model;
-    if (!m || max_tokens <= 0) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: llama_finalize: bad arguments");
-    const auto& c = m->c;
+mi355x_status mimir::Model::finalize(int64_t max_tokens) {
+    Model* m = this;
     if (!m->embed.set() || !m->norm.set()) return capi_fail(MI355X_ERR_SHAPE, "mi355x: llama: token_embd.weight or output_norm.weight missing");
     m->tied = !m->output.set();  // llm/model.go:283-288
     for (int i = 0; i < c.layers; i++) {
@@ -722,16 +688,14 @@ mi355x_status mi355x_llama_finalize(void* model, int64_t max_tokens) {
         LLM_HIP(hipMemset(m->values[i].p, 0, cache_bytes), "hipMemset(KV cache)");
     }
     m->cache_len = 0;
-    const int64_t rows = (int64_t)c.batch * max_tokens;
+    const int64_t rows = (int64_t)c.batch * max_tokens;  // of a call, here and below (not the member)
     const int64_t qd = (int64_t)c.heads * c.head_dim, kvd = (int64_t)c.kv_heads * c.head_dim;
-    m->max_rows = rows;
+    if (mi355x_status st = alloc_common(rows, rows)) return st;
     LLM_HIP(m->x.alloc(rows * c.embed * 4), "hipMalloc"); LLM_HIP(m->h.alloc(rows * c.embed * 4), "hipMalloc");
     LLM_HIP(m->q.alloc(rows * qd * 4), "hipMalloc"); LLM_HIP(m->k.alloc(rows * kvd * 4), "hipMalloc"); LLM_HIP(m->v.alloc(rows * kvd * 4), "hipMalloc");
     LLM_HIP(m->a.alloc(rows * qd * 4), "hipMalloc"); LLM_HIP(m->o.alloc(rows * c.embed * 4), "hipMalloc");
     LLM_HIP(m->gate.alloc(rows * c.hidden * 4), "hipMalloc"); LLM_HIP(m->up.alloc(rows * c.hidden * 4), "hipMalloc"); LLM_HIP(m->s.alloc(rows * c.hidden * 4), "hipMalloc");
     LLM_HIP(m->hlast.alloc(rows * c.embed * 4), "hipMalloc");
-    LLM_HIP(m->logits.alloc((size_t)rows * c.vocab * 4), "hipMalloc(logits)");
-    LLM_HIP(m->tokens_dev.alloc(rows * 4), "hipMalloc"); LLM_HIP(m->next_tok.alloc(c.batch * 4), "hipMalloc");
     const int64_t kmax = c.hidden > qd ? (c.hidden > c.embed ? c.hidden : c.embed) : (qd > c.embed ? qd : c.embed);
     for (int cls = 1; cls < kActClasses; cls++) {
         int64_t kk = cls == kActKQ ? (kmax + 255) / 256 * 256 : cls == kActFx || cls == kActFxPairs ? (kmax + 127) / 128 * 128 : (kmax + 63) / 64 * 64;
@@ -770,17 +734,6 @@ mi355x_status mi355x_llama_finalize(void* model, int64_t max_tokens) {
         LLM_HIP(m->attn_flags.alloc(fb + 64), "hipMalloc(attention hand-over)");
         LLM_HIP(hipMemset(m->attn_flags.p, 0, fb + 64), "hipMemset(attention hand-over)");
     }
-    if (!m->stream) LLM_HIP(hipStreamCreate(&m->stream), "hipStreamCreate");
-    if (m->step_graph) {
-        (void)hipGraphExecDestroy(m->step_graph);
-        m->step_graph = nullptr;
-    }
-    LLM_HIP(m->state.alloc(256), "hipMalloc");
-    if (c.batch <= (int)(kArgmaxTicketBytes / 4)) {
-        LLM_HIP(m->argmax_ws.alloc(argmax_workspace_bytes(c.batch)), "hipMalloc");
-        LLM_HIP(hipMemset(m->argmax_ws.p, 0, kArgmaxTicketBytes), "hipMemset");
-    }
-    LLM_HIP(m->record.alloc(((size_t)c.context + 1) * c.batch * 4), "hipMalloc");  // a graph keeps its address
     LLM_HIP(m->qkv.alloc((size_t)c.batch * (qd + 2 * kvd) * 4), "hipMalloc");
     m->fast = rmsnorm_q4act_ok(c.embed) && c.head_dim % 2 == 0;
     bool biased = false;  // q, k, v with biases: the generic step, whose rotation launch adds them first
@@ -858,12 +811,7 @@ mi355x_status mi355x_llama_finalize(void* model, int64_t max_tokens) {
     return MI355X_OK;
 }
 
-mi355x_status mi355x_llama_reset(void* model) {
-    Model* m = (Model*)model;
-    if (!m) return mimir::capi_fail(MI355X_ERR_INTERNAL, "mi355x: llama_reset: null pointer");
-    m->cache_len = 0;  // KVCache.Reset (nn/transformer.go:377)
-    return MI355X_OK;
-}
+extern "C" {
 
 // Loads positions [0, n) of one block's caches from the host (keys and values
 // [batch, kv_heads, n, head_dim] in the cache's dtype) and makes n the length
@@ -871,7 +819,7 @@ mi355x_status mi355x_llama_reset(void* model) {
 // (nn/transformer.go:348-423), for callers that keep caches of their own.
 mi355x_status mi355x_llama_set_cache(void* model, int32_t layer, const void* keys, const void* values, int64_t n) {
     using namespace mimir;
-    Model* m = (Model*)model;
+    Model* m = (Model*)(mimir::Decoder*)model;
     if (!m || !keys || !values) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: llama_set_cache: null pointer");
     const auto& c = m->c;
     if (!m->ready) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: llama: model is not finalized");
@@ -888,149 +836,19 @@ mi355x_status mi355x_llama_set_cache(void* model, int32_t layer, const void* key
     return MI355X_OK;
 }
 
-int64_t mi355x_llama_cache_len(void* model) { return model ? ((Model*)model)->cache_len : -1; }
-
-static mi355x_status check_tokens(Model* m, const int32_t* tokens, int64_t n) {
-    using namespace mimir;
-    const auto& c = m->c;
-    if (!m->ready) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: llama: model is not finalized");
-    // llm/model.go:393-400
-    if (n <= 0 || (int64_t)c.batch * n > m->max_rows) return capi_fail(MI355X_ERR_SHAPE, "mi355x: llama: %lld tokens a sequence, at most %lld a call", (long long)n, (long long)(m->max_rows / c.batch));
-    if (m->cache_len + n > c.context)
-        return capi_fail(MI355X_ERR_SHAPE, "mi355x: llama: append %lld positions to a cache holding %lld of %d", (long long)n, (long long)m->cache_len, c.context);
-    for (int64_t i = 0; i < (int64_t)c.batch * n; i++)
-        if (tokens[i] < 0 || tokens[i] >= c.vocab) return capi_fail(MI355X_ERR_INDEX, "mi355x: llama: token %d of a vocabulary of %d", tokens[i], c.vocab);
-    return MI355X_OK;
+// The rest of a llama handle's calls are any decoder's (decoder.hip).
+mi355x_status mi355x_llama_destroy(void* model) { return mi355x_model_destroy(model); }
+mi355x_status mi355x_llama_set_tensor(void* model, const char* name, int dtype, const void* host, int64_t n_elems) {
+    return mi355x_model_set_tensor(model, name, dtype, host, n_elems);
 }
-
-// Model.Logits (llm/model.go:391-437): runs tokens [batch, n], which follow the
-// positions the caches hold, and copies to the host the logits of the last
-// token, [batch, vocab], or of every token, [batch, n, vocab], if all is set.
+mi355x_status mi355x_llama_finalize(void* model, int64_t max_tokens) { return mi355x_model_finalize(model, max_tokens); }
+mi355x_status mi355x_llama_reset(void* model) { return mi355x_model_reset(model); }  // KVCache.Reset (nn/transformer.go:377)
+int64_t mi355x_llama_cache_len(void* model) { return mi355x_model_cache_len(model); }
 mi355x_status mi355x_llama_logits(void* model, const int32_t* tokens, int64_t n, int all, float* logits_host) {
-    using namespace mimir;
-    Model* m = (Model*)model;
-    if (!m || !tokens || !logits_host) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: llama_logits: null pointer");
-    if (mi355x_status st = check_tokens(m, tokens, n)) return st;
-    const auto& c = m->c;
-    const int64_t rows = (int64_t)c.batch * n;
-    LLM_HIP(hipMemcpyAsync(m->tokens_dev.p, tokens, rows * 4, hipMemcpyHostToDevice, m->stream), "upload tokens");
-    if (mi355x_status st = forward(*m, n)) return st;
-    int64_t out_rows = all ? rows : c.batch;
-    if (mi355x_status st = all ? head(*m, m->x.as<float>(), rows, c.embed) : head(*m, m->x.as<float>() + (n - 1) * c.embed, c.batch, n * c.embed)) return st;
-    LLM_HIP(hipMemcpyAsync(logits_host, m->logits.p, (size_t)out_rows * c.vocab * 4, hipMemcpyDeviceToHost, m->stream), "download logits");
-    return mi355x_sync(m->stream);
+    return mi355x_model_logits(model, tokens, n, all, logits_host);
 }
-
-// Greedy generation (examples/llama/generate.go:162-202 with Sample at :44-53):
-// the prompt [batch, n_prompt], then n_new steps. Each step's token is chosen on
-// the device and read by the next step's embedding lookup from device memory;
-// out_tokens [batch, n_new] comes back once at the end. seconds, if not NULL,
-// gets the wall time of the prompt pass and of the n_new - 1 decoding steps.
 mi355x_status mi355x_llama_generate(void* model, const int32_t* prompt, int64_t n_prompt, int64_t n_new, int32_t* out_tokens, double* seconds) {
-    using namespace mimir;
-    Model* m = (Model*)model;
-    if (!m || !prompt || !out_tokens || n_new <= 0) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: llama_generate: bad arguments");
-    if (mi355x_status st = check_tokens(m, prompt, n_prompt)) return st;
-    const auto& c = m->c;
-    if (m->cache_len + n_prompt + n_new - 1 > c.context)
-        return capi_fail(MI355X_ERR_SHAPE, "mi355x: llama: %lld positions for a context of %d", (long long)(m->cache_len + n_prompt + n_new - 1), c.context);
-    const int64_t B = c.batch;
-    const bool use_graph = g_llama_step_mode == 0, use_fast = g_llama_step_mode != 2;  // 2: forward() with the position from the host
-    DevBuf picked;  // [n_new, batch]
-    LLM_HIP(picked.alloc((size_t)n_new * B * 4), "hipMalloc(tokens)");
-    hipEvent_t e0, e1, e2;
-    LLM_HIP(hipEventCreate(&e0), "hipEventCreate"); LLM_HIP(hipEventCreate(&e1), "hipEventCreate"); LLM_HIP(hipEventCreate(&e2), "hipEventCreate");
-    LLM_HIP(hipMemcpyAsync(m->tokens_dev.p, prompt, B * n_prompt * 4, hipMemcpyHostToDevice, m->stream), "upload tokens");
-    LLM_HIP(hipEventRecord(e0, m->stream), "hipEventRecord");
-    mi355x_status st = forward(*m, n_prompt);
-    if (!st) st = head(*m, m->x.as<float>() + (n_prompt - 1) * c.embed, B, n_prompt * c.embed);
-    if (!st) {
-        hipError_t e = argmax(m->logits.as<float>(), B, c.vocab, picked.as<int32_t>(), m->argmax_ws.p, m->stream);
-        if (e != hipSuccess) st = capi_fail((mi355x_status)e, "mi355x: llama: argmax: %s", hipGetErrorName(e));
-    }
-    if (!st) (void)hipEventRecord(e1, m->stream);
-    if (!st && use_fast) {
-        // record[0] is the prompt's choice; each step then reads next_tok and the
-        // position from the device, and leaves its own choice in both places
-        hipError_t e = hipSuccess;  // n_new <= context: the record holds it
-        if (!st) e = hipMemcpyAsync(m->next_tok.p, picked.p, B * 4, hipMemcpyDeviceToDevice, m->stream);
-        if (!st && e == hipSuccess) e = set_state(m->state.as<int32_t>(), (int)m->cache_len, 0, m->stream);
-        if (!st && e == hipSuccess) e = advance(m->state.as<int32_t>(), m->next_tok.as<int32_t>(), m->record.as<int32_t>(), (int)B, 0, m->stream);
-        if (!st && e != hipSuccess) st = capi_fail((mi355x_status)e, "mi355x: llama: step state: %s", hipGetErrorName(e));
-        auto one_step = [&]() -> mi355x_status {
-            if (mi355x_status s2 = m->rows && !g_llama_rows_off ? step_rows(*m) : m->fast ? step_fast(*m) : step_any(*m)) return s2;
-            if (mi355x_status s2 = head(*m, m->x.as<float>(), B, c.embed)) return s2;
-            LLM_HIP(argmax(m->logits.as<float>(), B, c.vocab, m->next_tok.as<int32_t>(), m->argmax_ws.p, m->stream), "argmax");
-            LLM_HIP(advance(m->state.as<int32_t>(), m->next_tok.as<int32_t>(), m->record.as<int32_t>(), (int)B, 1, m->stream), "advance");
-            return MI355X_OK;
-        };
-        const int rows_now = m->rows && !g_llama_rows_off ? 1 + g_llama_rows_plain : 0;
-        if (m->step_graph && m->graph_rows != rows_now) {  // the measurement aid changed which step runs
-            (void)hipGraphExecDestroy(m->step_graph);
-            m->step_graph = nullptr;
-        }
-        if (!st && n_new > 1 && !m->step_graph && use_graph) {
-            m->graph_rows = rows_now;
-            hipGraph_t g = nullptr;
-            e = hipStreamBeginCapture(m->stream, hipStreamCaptureModeThreadLocal);
-            if (e != hipSuccess) st = capi_fail((mi355x_status)e, "mi355x: llama: begin capture: %s", hipGetErrorName(e));
-            if (!st) {
-                mi355x_status cst = one_step();
-                e = hipStreamEndCapture(m->stream, &g);
-                if (cst) st = cst;
-                else if (e != hipSuccess) st = capi_fail((mi355x_status)e, "mi355x: llama: end capture: %s", hipGetErrorName(e));
-            }
-            if (!st) {
-                e = hipGraphInstantiate(&m->step_graph, g, nullptr, nullptr, 0);
-                if (e != hipSuccess) st = capi_fail((mi355x_status)e, "mi355x: llama: instantiate graph: %s", hipGetErrorName(e));
-            }
-            if (g) (void)hipGraphDestroy(g);
-        }
-        for (int64_t t = 1; t < n_new && !st; t++) {
-            if (m->step_graph && use_graph) {
-                e = hipGraphLaunch(m->step_graph, m->stream);
-                if (e != hipSuccess) st = capi_fail((mi355x_status)e, "mi355x: llama: graph launch: %s", hipGetErrorName(e));
-            } else {
-                st = one_step();
-            }
-            if (!st) m->cache_len += 1;
-        }
-        if (!st) {
-            e = hipMemcpyAsync(picked.p, m->record.p, (size_t)n_new * B * 4, hipMemcpyDeviceToDevice, m->stream);
-            if (e != hipSuccess) st = capi_fail((mi355x_status)e, "mi355x: llama: copy record: %s", hipGetErrorName(e));
-        }
-    } else
-    for (int64_t t = 1; t < n_new && !st; t++) {
-        // the step reads its tokens where the last step's argmax wrote them
-        hipError_t e = hipMemcpyAsync(m->tokens_dev.p, picked.as<int32_t>() + (t - 1) * B, B * 4, hipMemcpyDeviceToDevice, m->stream);
-        if (e != hipSuccess) { st = capi_fail((mi355x_status)e, "mi355x: llama: token copy: %s", hipGetErrorName(e)); break; }
-        st = forward(*m, 1);
-        if (!st) st = head(*m, m->x.as<float>(), B, c.embed);
-        if (!st) {
-            e = argmax(m->logits.as<float>(), B, c.vocab, picked.as<int32_t>() + t * B, m->argmax_ws.p, m->stream);
-            if (e != hipSuccess) st = capi_fail((mi355x_status)e, "mi355x: llama: argmax: %s", hipGetErrorName(e));
-        }
-    }
-    if (!st) (void)hipEventRecord(e2, m->stream);
-    std::vector<int32_t> host((size_t)n_new * B);
-    if (!st) {
-        hipError_t e = hipMemcpyAsync(host.data(), picked.p, host.size() * 4, hipMemcpyDeviceToHost, m->stream);
-        if (e != hipSuccess) st = capi_fail((mi355x_status)e, "mi355x: llama: download tokens: %s", hipGetErrorName(e));
-    }
-    if (!st) st = mi355x_sync(m->stream);
-    if (!st) {
-        for (int64_t t = 0; t < n_new; t++)
-            for (int64_t b = 0; b < B; b++) out_tokens[b * n_new + t] = host[t * B + b];
-        if (seconds) {
-            float ms01 = 0, ms12 = 0;
-            (void)hipEventElapsedTime(&ms01, e0, e1);
-            (void)hipEventElapsedTime(&ms12, e1, e2);
-            seconds[0] = ms01 * 1e-3;
-            seconds[1] = ms12 * 1e-3;
-        }
-    }
-    (void)hipEventDestroy(e0); (void)hipEventDestroy(e1); (void)hipEventDestroy(e2);
-    return st;
+    return mi355x_model_generate(model, prompt, n_prompt, n_new, out_tokens, seconds);
 }
 
 }  // extern "C"

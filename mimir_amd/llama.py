@@ -11,6 +11,7 @@ import ctypes as C
 import numpy as np
 
 from . import capi
+from .decoder import Decoder
 from .mimfile import MimFile
 
 # container dtype codes (mimfile) -> C-ABI dtype codes
@@ -18,8 +19,8 @@ from .mimfile import MimFile
 _MIM_TO_ABI = {"f32": capi.F32, "f16": capi.F16, "bf16": capi.BF16, "q8_0": capi.Q8_0, "q4_K": capi.Q4_K, "q6_K": capi.Q6_K, "q4_0": capi.Q4_0}
 
 
-class Llama:
-    """A handle on mi355x_llama_*."""
+class Llama(Decoder):
+    """A handle on a mi355x_llama_* decoder."""
 
     def __init__(self, config: capi.LlamaConfig):
         self.lib = capi.load()
@@ -27,58 +28,15 @@ class Llama:
         self._h = C.c_void_p()
         capi.check(self.lib.mi355x_llama_create(C.byref(config), C.byref(self._h)))
 
-    def close(self):
-        if self._h:
-            self.lib.mi355x_llama_destroy(self._h)
-            self._h = C.c_void_p()
-
-    def __del__(self):
-        try:
-            self.close()
-        except Exception:
-            pass
-
-    def set_tensor(self, name: str, dtype: int, data: np.ndarray, n_elems: int):
-        data = np.ascontiguousarray(data)
-        capi.check(self.lib.mi355x_llama_set_tensor(self._h, name.encode(), dtype, data.ctypes.data, n_elems))
-
     def set_rope_factors(self, factors):
         f = np.ascontiguousarray(factors, np.float32)
         capi.check(self.lib.mi355x_llama_set_rope_factors(self._h, f.ctypes.data, f.size))
-
-    def finalize(self, max_tokens: int):
-        capi.check(self.lib.mi355x_llama_finalize(self._h, max_tokens))
-
-    def reset(self):
-        capi.check(self.lib.mi355x_llama_reset(self._h))
 
     def set_cache(self, layer: int, keys, values):
         """keys, values [batch, kv_heads, n, head_dim] in the cache's dtype
         (float32, or binary16 bits as uint16)."""
         k = np.ascontiguousarray(keys); v = np.ascontiguousarray(values)
         capi.check(self.lib.mi355x_llama_set_cache(self._h, layer, k.ctypes.data, v.ctypes.data, k.shape[2]))
-
-    @property
-    def cache_len(self) -> int:
-        return self.lib.mi355x_llama_cache_len(self._h)
-
-    def logits(self, tokens, all: bool = False) -> np.ndarray:
-        """tokens [batch, n] (or [n] for batch 1) -> [batch, vocab] or [batch, n, vocab]."""
-        c = self.config
-        t = np.ascontiguousarray(tokens, np.int32).reshape(c.batch, -1)
-        n = t.shape[1]
-        out = np.empty((c.batch, n, c.vocab) if all else (c.batch, c.vocab), np.float32)
-        capi.check(self.lib.mi355x_llama_logits(self._h, t.ctypes.data, n, int(all), out.ctypes.data))
-        return out
-
-    def generate(self, prompt, n_new: int):
-        """Greedy tokens [batch, n_new] and (prompt seconds, decode seconds)."""
-        c = self.config
-        t = np.ascontiguousarray(prompt, np.int32).reshape(c.batch, -1)
-        out = np.empty((c.batch, n_new), np.int32)
-        secs = (C.c_double * 2)()
-        capi.check(self.lib.mi355x_llama_generate(self._h, t.ctypes.data, t.shape[1], n_new, out.ctypes.data, secs))
-        return out, (secs[0], secs[1])
 
 
 def config_from_metadata(md: dict, vocab: int, context: int | None = None, batch: int = 1, cache_dtype: int = capi.F32) -> capi.LlamaConfig:
