@@ -1,0 +1,72 @@
+// y = act(x . W^T) for many rows of float32 x and bfloat16 weights on the float32 matrix cores
+// (v_mfma_f32_32x32x2_f32): nothing is rounded below float32 on the way. The prompt product of a model that runs in
+// float32, and in any model that of the few columns that must not be rounded (a recurrence's gates).
+// A workgroup of four wavefronts owns 64 x 64 of y, a wavefront 32 x 32; steps of 32 along K go through LDS.
+#include "device_util.h"
+#include "stack_ops.h"
+
+namespace mimir {
+
+namespace {
+
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+
+constexpr int kTile = 64, kStep = 32, kPad = kStep + 1;
+
+__global__ __launch_bounds__(256) void gemm_f32_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx, int64_t M,
+                                                       int64_t N, int64_t K, ProductOut out) {
+    __shared__ float xs[2][kTile * kPad], ws[2][kTile * kPad];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r32 = lane & 31, hi = lane >> 5;
+    const int64_t m0 = (int64_t)blockIdx.y * kTile, n0 = (int64_t)blockIdx.x * kTile;
+    const int wm = (wave >> 1) * 32, wn = (wave & 1) * 32;
+    // a thread brings eight neighbouring elements of one row of each operand
+    const int lr = tid >> 2, lk = (tid & 3) * 8;
+    const float* xp = x + (m0 + lr < M ? m0 + lr : M - 1) * ldx + lk;
+    const uint16_t* wp = W + (n0 + lr < N ? n0 + lr : N - 1) * ldw + lk;
+    f32x16 acc;
+#pragma unroll
+    for (int i = 0; i < 16; i++) acc[i] = 0.f;
+    float xv[8];
+    uint16_t wv[8];
+    auto fetch = [&](int64_t k0) {
+#pragma unroll
+        for (int i = 0; i < 8; i++) xv[i] = k0 + lk + i < K ? xp[k0 + i] : 0.f;
+#pragma unroll
+        for (int i = 0; i < 8; i++) wv[i] = k0 + lk + i < K ? wp[k0 + i] : (uint16_t)0;
+    };
+    fetch(0);
+    int p = 0;
+    for (int64_t k0 = 0; k0 < K; k0 += kStep, p ^= 1) {
+#pragma unroll
+        for (int i = 0; i < 8; i++) {
+            xs[p][lr * kPad + lk + i] = xv[i];
+            ws[p][lr * kPad + lk + i] = bf16_bits_to_f32(wv[i]);
+        }
+        __syncthreads();  // the other stage is written next only after everyone has passed the next barrier
+        if (k0 + kStep < K) fetch(k0 + kStep);
+#pragma unroll
+        for (int k = 0; k < kStep; k += 2)
+            acc = __builtin_amdgcn_mfma_f32_32x32x2f32(xs[p][(wm + r32) * kPad + k + hi], ws[p][(wn + r32) * kPad + k + hi], acc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < 16; i++) {
+        const int64_t m = m0 + wm + (i & 3) + 8 * (i >> 2) + 4 * hi, n = n0 + wn + r32;
+        if (m >= M || n >= N) continue;
+        float v = acc[i];
+        if (out.relu2) v = v > 0.f ? v * v : 0.f;
+        else if (n < out.silu_n) v = v / (1.f + expf(-v));
+        if (out.f32) out.f32[m * out.ld + n] = v;
+        else out.bf16[m * out.ld + n] = f32_to_bf16_bits(v);
+    }
+}
+
+}  // namespace
+
+hipError_t gemm_f32(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st) {
+    if (M == 0 || N == 0) return hipSuccess;
+    hipLaunchKernelGGL(gemm_f32_kernel, dim3((unsigned)((N + kTile - 1) / kTile), (unsigned)((M + kTile - 1) / kTile)), dim3(256), 0, st, W, ldw, x, ldx, M,
+                       N, K, out);
+    return hipGetLastError();
+}
+
+}  // namespace mimir

@@ -4,8 +4,12 @@
 // are widened to float32 and multiplied there). Tiny Llama fixtures keep some
 // projections in these types; the decode path of a quantized model does not
 // come here. One wavefront per row of W.
+//
+// gemv_bf16 is the product of a decoding step whose weights are bfloat16 (the mixer stack's): a wavefront takes a few
+// rows of W for up to eight rows of x, sixteen bytes of W a lane at a time, and applies the activation behind it.
 #include "device_util.h"
 #include "kernels.h"
+#include "stack_ops.h"
 
 namespace mimir {
 
@@ -43,6 +47,90 @@ hipError_t gemv_float(int dt, const void* W, const float* x, float* y, int64_t M
         hipLaunchKernelGGL(gemv_float_kernel<half_bits>, grid, dim3(256), 0, st, (const half_bits*)W, x, y, (int)N, (int)K, x_row_stride);
     else
         hipLaunchKernelGGL(gemv_float_kernel<bf16_bits>, grid, dim3(256), 0, st, (const bf16_bits*)W, x, y, (int)N, (int)K, x_row_stride);
+    return hipGetLastError();
+}
+
+// M rows of x against R rows of W a wavefront, eight elements of K a lane and step (the rows are padded with zeros to
+// a multiple of 64). The x of a step serves all R rows from registers.
+template <int M, int R>
+__global__ __launch_bounds__(256) void gemv_bf16_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx, int N, int K,
+                                                        ProductOut out) {
+    const int lane = threadIdx.x & 63, n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * R;
+    if (n0 >= N) return;
+    const int64_t m0 = (int64_t)blockIdx.y * M;
+    const uint16_t* w[R];
+#pragma unroll
+    for (int r = 0; r < R; r++) w[r] = W + (int64_t)(n0 + r < N ? n0 + r : N - 1) * ldw;
+    float acc[M][R];
+#pragma unroll
+    for (int m = 0; m < M; m++)
+#pragma unroll
+        for (int r = 0; r < R; r++) acc[m][r] = 0.f;
+#pragma unroll 4
+    for (int k = lane * 8; k < K; k += 512) {
+        u32x4 wv[R];
+#pragma unroll
+        for (int r = 0; r < R; r++) wv[r] = *(const u32x4*)(w[r] + k);
+#pragma unroll
+        for (int m = 0; m < M; m++) {
+            const f32x4* xp = (const f32x4*)(x + (m0 + m) * ldx + k);
+            const f32x4 a = xp[0], b = xp[1];
+#pragma unroll
+            for (int r = 0; r < R; r++) {
+                float t = acc[m][r];
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const float x0 = i < 2 ? a[2 * i] : b[2 * i - 4], x1 = i < 2 ? a[2 * i + 1] : b[2 * i - 3];
+                    t = fmaf(x0, __uint_as_float(wv[r][i] << 16), t);
+                    t = fmaf(x1, __uint_as_float(wv[r][i] & 0xffff0000u), t);
+                }
+                acc[m][r] = t;
+            }
+        }
+    }
+#pragma unroll
+    for (int m = 0; m < M; m++)
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            float v = wave_sum(acc[m][r]);
+            if (lane != 0 || n0 + r >= N) continue;
+            if (out.relu2) v = v > 0.f ? v * v : 0.f;
+            else if (n0 + r < out.silu_n) v = v / (1.f + expf(-v));
+            const int64_t at = (m0 + m) * out.ld + n0 + r;
+            if (out.f32) out.f32[at] = v;
+            else out.bf16[at] = f32_to_bf16_bits(v);
+        }
+}
+
+namespace {
+
+template <int M>
+void launch_gemv_bf16(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t groups, int64_t N, int64_t K, const ProductOut& out, hipStream_t st) {
+    const int k = (int)((K + 63) / 64 * 64);
+    // more rows a wavefront read x less often; fewer give a small matrix enough wavefronts
+    if (N >= 8192 && M <= 4) hipLaunchKernelGGL((gemv_bf16_kernel<M, 4>), dim3((unsigned)((N + 15) / 16), (unsigned)groups), dim3(256), 0, st, W, ldw, x, ldx, (int)N, k, out);
+    else if (N >= 2048) hipLaunchKernelGGL((gemv_bf16_kernel<M, 2>), dim3((unsigned)((N + 7) / 8), (unsigned)groups), dim3(256), 0, st, W, ldw, x, ldx, (int)N, k, out);
+    else hipLaunchKernelGGL((gemv_bf16_kernel<M, 1>), dim3((unsigned)((N + 3) / 4), (unsigned)groups), dim3(256), 0, st, W, ldw, x, ldx, (int)N, k, out);
+}
+
+}  // namespace
+
+hipError_t gemv_bf16(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st) {
+    int64_t m = 0;
+    auto rest = [&](int64_t rows, int64_t each) {  // whole groups of `each` rows from row m on
+        ProductOut o = out;
+        if (o.f32) o.f32 += m * o.ld;
+        else o.bf16 += m * o.ld;
+        const float* xr = x + m * ldx;
+        const int64_t groups = rows / each;
+        if (each == 8) launch_gemv_bf16<8>(W, ldw, xr, ldx, groups, N, K, o, st);
+        else if (each == 4) launch_gemv_bf16<4>(W, ldw, xr, ldx, groups, N, K, o, st);
+        else if (each == 2) launch_gemv_bf16<2>(W, ldw, xr, ldx, groups, N, K, o, st);
+        else launch_gemv_bf16<1>(W, ldw, xr, ldx, groups, N, K, o, st);
+        m += groups * each;
+    };
+    for (int64_t each = 8; each >= 1; each >>= 1)
+        if (M - m >= each) rest(M - m, each);
     return hipGetLastError();
 }
 

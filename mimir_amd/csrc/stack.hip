@@ -1,0 +1,468 @@
+// A decoder whose layers are a list of mixers, each with its own sizes (mi355x_stack_create): the Fuvolix design's. A layer
+// is x += norm1b(mixer(conv(norm1(x)))), x += norm2b(mlp(norm2(x))) where it has an mlp, then the depth average over
+// the embedding output and all layers' results so far; norms are RMS norms in groups, conv adds a short causal
+// convolution over time. Mixers: latent attention (attention_latent.hip), gated and decaying linear recurrences
+// (linear_recurrence.hip). What a sequence holds between calls: the last inputs of each layer's convolution, the latents
+// and rotated keys of latent attention, the recurrences' states.
+//
+// Weights are bfloat16 on the device; matrices that read the same input lie in one buffer and are multiplied in one
+// product. Activations: a pass of up to kGemvRows rows, and every pass of a model that runs in float32, multiplies
+// float32 activations; longer passes of a bfloat16 model round the products' inputs to bfloat16. The residual, norms,
+// recurrent states, gates, scores and softmax weights are float32 either way.
+#include <cmath>
+#include <cstring>
+#include <map>
+#include <memory>
+#include <string>
+#include <vector>
+
+#include "decoder.h"
+#include "stack_ops.h"
+
+namespace mimir {
+
+namespace {
+
+#define STACK_HIP(expr, what) DECODER_HIP(expr, "stack", what)
+
+int64_t pad64(int64_t n) { return (n + 63) / 64 * 64; }
+
+struct Mat {  // [n, k] bfloat16, rows ld apart, zeros from k on
+    int64_t n = 0, k = 0, ld = 0;
+    DevBuf buf;
+    const uint16_t* row(int64_t i) const { return buf.as<uint16_t>() + i * ld; }
+};
+struct Vec {  // float32
+    int64_t n = 0;
+    DevBuf buf;
+    const float* p() const { return buf.as<float>(); }
+};
+
+// Where a tensor of the file goes.
+struct Slot {
+    Mat* mat = nullptr;
+    Vec* vec = nullptr;
+    int64_t row0 = 0, rows = 0, cols = 0;
+    bool set = false;
+};
+
+struct StackLayer {
+    mi355x_stack_layer c{};
+    std::vector<double> decay;
+    Vec norm1, norm1b, norm2, norm2b, canon, dwa, mix_norm, dkv_norm, bias_i, bias_f;
+    Mat in, o, ukv, up, down;          // in: every projection of the mixer's input, one after the other
+    int64_t g_at = 0, gates_at = 0;    // rows of `in` where W_g and the two gates' begin
+    DevBuf cos_t, sin_t, cache, S, n, m, conv_state, decay_f, decay_pow;
+    int64_t ldc = 0;
+    int64_t mixed() const { return (int64_t)c.heads * c.vdim; }
+    bool recurrent() const { return c.mixer != MI355X_MIXER_LATENT; }
+};
+
+struct Stack : Decoder {
+    mi355x_stack_config c{};
+    std::vector<StackLayer> layers;
+    Mat embed;
+    Vec embed_norm, final_norm;
+    std::map<std::string, Slot> slots;
+
+    // activations of up to max_rows rows; *_f float32, *_b bfloat16
+    DevBuf streams, x, h, y, in_f, in_b, proj_f, proj_b, gates, scanned, mix_f, mix_b, up_f, up_b, last_f, last_b, rows_dev, ws;
+
+    mi355x_status set_tensor(const char* tensor, int dtype, const void* host, int64_t n_elems) override;
+    mi355x_status finalize(int64_t max_tokens) override;
+    mi355x_status forward(int64_t s) override;
+    mi355x_status head(const int64_t* rows, int64_t n) override;
+    mi355x_status step() override;
+    mi355x_status reset() override;
+    bool runs_in_portions() const override { return true; }
+
+    bool half() const { return c.dtype == MI355X_BF16; }
+    int64_t width() const { return c.width; }
+    void name_tensors();
+    Latent latent(const StackLayer& l, int64_t s, const int32_t* pos) const;
+    Recurrence recurrence(const StackLayer& l, int64_t s) const;
+    mi355x_status pass(const int32_t* tokens, int64_t s, const int32_t* pos);
+    mi355x_status mix(StackLayer& l, int64_t s, bool tiles, const int32_t* pos);
+    // out = act(x . W[row0, row0 + n)^T) by the kernel for this many rows and x's form (bfloat16 if b, else float32)
+    mi355x_status product(const Mat& w, int64_t row0, int64_t n, const DevBuf& f, const DevBuf& b, bool tiles, int64_t rows, const ProductOut& out);
+};
+
+mi355x_status Stack::product(const Mat& w, int64_t row0, int64_t n, const DevBuf& f, const DevBuf& b, bool tiles, int64_t rows, const ProductOut& out) {
+    if (tiles) STACK_HIP(gemm_bf16(w.row(row0), w.ld, b.as<uint16_t>(), w.ld, rows, n, w.k, out, stream), "product");
+    else if (rows <= kGemvRows) STACK_HIP(gemv_bf16(w.row(row0), w.ld, f.as<float>(), w.ld, rows, n, w.k, out, stream), "product");
+    else STACK_HIP(gemm_f32(w.row(row0), w.ld, f.as<float>(), w.ld, rows, n, w.k, out, stream), "product");
+    return MI355X_OK;
+}
+
+Latent Stack::latent(const StackLayer& l, int64_t s, const int32_t* pos) const {
+    Latent a;
+    a.heads = l.c.heads; a.dim = l.c.dim; a.rot_dim = l.c.rot_dim; a.vdim = l.c.vdim; a.rank = l.c.kv_rank;
+    a.scale = (float)l.c.scale; a.eps = (float)c.eps;
+    a.cos_t = l.cos_t.as<float>(); a.sin_t = l.sin_t.as<float>();
+    a.norm_w = l.dkv_norm.p();
+    a.w_uk = l.ukv.row(0); a.w_uv = l.ukv.row((int64_t)l.c.heads * l.c.dim); a.ldw = l.ukv.ld;
+    a.cache = l.cache.p; a.cache_bf16 = half(); a.ldc = l.ldc; a.context = context;
+    a.batch = batch; a.s = s;
+    a.past = pos ? 0 : cache_len; a.past_dev = pos;
+    return a;
+}
+
+Recurrence Stack::recurrence(const StackLayer& l, int64_t s) const {
+    Recurrence r;
+    const int64_t qk = (int64_t)l.c.heads * l.c.dim;
+    r.ld = l.in.n;
+    r.q = proj_f.as<float>(); r.k = proj_f.as<float>() + qk; r.v = proj_f.as<float>() + 2 * qk;
+    if (l.c.mixer == MI355X_MIXER_MLSTM) {
+        r.gates = proj_f.as<float>() + l.gates_at; r.ldg = l.in.n;
+        r.bias_i = l.bias_i.p(); r.bias_f = l.bias_f.p();
+        r.cap = (float)l.c.gate_cap;
+        r.q_scale = (float)(1.0 / std::sqrt((double)l.c.dim));
+        r.n = l.n.as<float>(); r.m = l.m.as<float>();
+    } else {
+        r.decay = l.decay_f.as<float>(); r.decay_pow = l.decay_pow.as<float>();
+    }
+    r.S = l.S.as<float>();
+    r.out = scanned.as<float>(); r.ldo = l.mixed();
+    r.batch = batch; r.heads = l.c.heads; r.dim = l.c.dim; r.vdim = l.c.vdim; r.s = s;
+    r.ws = ws.as<float>();
+    return r;
+}
+
+// y = mixer(in), for s positions a sequence.
+mi355x_status Stack::mix(StackLayer& l, int64_t s, bool tiles, const int32_t* pos) {
+    const int64_t rows = (int64_t)batch * s, mixed = l.mixed();
+    if (!l.recurrent()) {
+        ProductOut p;
+        p.f32 = proj_f.as<float>(); p.ld = l.in.n;
+        if (mi355x_status st = product(l.in, 0, l.in.n, in_f, in_b, tiles, rows, p)) return st;
+        const Latent a = latent(l, s, pos);
+        STACK_HIP(latent_prepare(a, proj_f.as<float>(), l.in.n, nullptr, 0, stream), "latents and rotation");
+        STACK_HIP(latent_absorbed(a, proj_f.as<float>(), l.in.n, ws.as<float>(), tiles ? nullptr : mix_f.as<float>(), tiles ? mix_b.as<uint16_t>() : nullptr,
+                                  l.o.ld, stream), "latent attention");
+    } else {
+        ProductOut p;
+        p.f32 = proj_f.as<float>(); p.ld = l.in.n;
+        p.silu_n = l.c.mixer == MI355X_MIXER_LIGHTNING ? l.g_at : 0;
+        if (mi355x_status st = product(l.in, 0, l.in.n, in_f, in_b, tiles, rows, p)) return st;
+        const Recurrence r = recurrence(l, s);
+        STACK_HIP(recurrence_scan(r, stream), "recurrence");
+        STACK_HIP(gated_norm(scanned.as<float>(), proj_f.as<float>() + l.g_at, false, l.in.n, l.mix_norm.p(), rows, (int)mixed,
+                             l.c.mixer == MI355X_MIXER_MLSTM ? l.c.heads : 1, (float)c.eps, tiles ? nullptr : mix_f.as<float>(),
+                             tiles ? mix_b.as<uint16_t>() : nullptr, l.o.ld, stream), "gated norm");
+    }
+    ProductOut p;
+    p.f32 = y.as<float>(); p.ld = width();
+    return product(l.o, 0, l.o.n, mix_f, mix_b, tiles, rows, p);
+}
+
+// s positions a sequence through all layers. pos: a decoding step, whose position is read from the device (s is 1) and
+// which leaves the final norm of its rows in last_f; otherwise the residual is left in x.
+mi355x_status Stack::pass(const int32_t* tokens, int64_t s, const int32_t* pos) {
+    const int64_t rows = (int64_t)batch * s, W = width(), ldw = pad64(W);
+    const bool tiles = false;
+    NormChain base;
+    base.width = c.width; base.groups = c.norm_groups; base.eps = (float)c.eps; base.taps = c.taps;
+    auto into_layer = [&](NormChain& a, size_t i) {  // the end of a chain: layer i's norm, or the final one
+        if (i == layers.size()) {
+            if (!pos) return;
+            a.w_next = final_norm.p(); a.h_f32 = last_f.as<float>(); a.ldh = ldw;
+            return;
+        }
+        a.w_next = layers[i].norm1.p();
+        if (pos) {
+            a.conv_w = layers[i].canon.p(); a.conv_state = layers[i].conv_state.as<float>();
+            a.h_f32 = in_f.as<float>(); a.ldh = ldw;
+        } else {
+            a.h_f32 = h.as<float>(); a.ldh = W;
+        }
+    };
+    {
+        NormChain a = base;
+        a.tokens = tokens; a.table = embed.row(0); a.table_ld = embed.ld; a.w_post = embed_norm.p();
+        a.stream_out = streams.as<float>(); a.x_out = x.as<float>();
+        into_layer(a, 0);
+        STACK_HIP(norm_chain(a, rows, stream), "embedding");
+    }
+    for (size_t i = 0; i < layers.size(); i++) {
+        StackLayer& l = layers[i];
+        if (!pos) {
+            const bool both = tiles && l.c.mixer == MI355X_MIXER_MLSTM;  // the gates read float32
+            STACK_HIP(causal_conv(h.as<float>(), l.canon.p(), l.conv_state.as<float>(), c.taps, batch, s, c.width, tiles && !both ? nullptr : in_f.as<float>(),
+                                  tiles ? in_b.as<uint16_t>() : nullptr, ldw, stream), "convolution");
+        }
+        if (mi355x_status st = mix(l, s, tiles, pos)) return st;
+        NormChain a = base;
+        a.x = x.as<float>(); a.y = y.as<float>(); a.ldy = W; a.w_post = l.norm1b.p(); a.x_out = x.as<float>();
+        if (l.c.ff > 0) {
+            a.w_next = l.norm2.p(); a.ldh = ldw;
+            if (tiles) a.h_bf16 = in_b.as<uint16_t>();
+            else a.h_f32 = in_f.as<float>();
+            STACK_HIP(norm_chain(a, rows, stream), "norms");
+            ProductOut p;
+            p.relu2 = true; p.ld = l.down.ld;
+            if (tiles) p.bf16 = up_b.as<uint16_t>();
+            else p.f32 = up_f.as<float>();
+            if (mi355x_status st = product(l.up, 0, l.up.n, in_f, in_b, tiles, rows, p)) return st;
+            ProductOut d;
+            d.f32 = y.as<float>(); d.ld = W;
+            if (mi355x_status st = product(l.down, 0, l.down.n, up_f, up_b, tiles, rows, d)) return st;
+            a = base;
+            a.x = x.as<float>(); a.y = y.as<float>(); a.ldy = W; a.w_post = l.norm2b.p(); a.x_out = x.as<float>();
+        }
+        a.stream_out = i + 1 < layers.size() ? streams.as<float>() + (i + 1) * max_rows * W : nullptr;
+        a.streams = streams.as<float>(); a.stream_stride = max_rows * W; a.n_streams = (int)i + 1; a.dwa = l.dwa.p();
+        into_layer(a, i + 1);
+        STACK_HIP(norm_chain(a, rows, stream), "norms and depth average");
+    }
+    return MI355X_OK;
+}
+
+mi355x_status Stack::forward(int64_t s) {
+    if (mi355x_status st = pass(tokens_dev.as<int32_t>(), s, nullptr)) return st;
+    cache_len += s;
+    return MI355X_OK;
+}
+
+mi355x_status Stack::head(const int64_t* rows, int64_t n) {
+    if (n <= 0) return MI355X_OK;
+    const bool tiles = false;
+    STACK_HIP(hipMemcpyAsync(rows_dev.p, rows, (size_t)n * 8, hipMemcpyHostToDevice, stream), "upload rows");
+    STACK_HIP(norm_rows(x.as<float>(), rows_dev.as<int64_t>(), n, final_norm.p(), c.width, c.norm_groups, (float)c.eps, tiles ? nullptr : last_f.as<float>(),
+                        tiles ? last_b.as<uint16_t>() : nullptr, embed.ld, stream), "final norm");
+    ProductOut p;
+    p.f32 = logits.as<float>(); p.ld = vocab;
+    return product(embed, 0, vocab, last_f, last_b, tiles, n, p);
+}
+
+mi355x_status Stack::step() {
+    if (mi355x_status st = pass(next_tok.as<int32_t>(), 1, state.as<int32_t>())) return st;
+    ProductOut p;
+    p.f32 = logits.as<float>(); p.ld = vocab;
+    return product(embed, 0, vocab, last_f, last_b, false, batch, p);
+}
+
+mi355x_status Stack::reset() {
+    cache_len = 0;
+    if (!ready) return MI355X_OK;
+    for (StackLayer& l : layers)  // a cache's rows are written before they are read; the rest is read as it is
+        for (DevBuf* b : {&l.conv_state, &l.S, &l.n, &l.m})
+            if (b->p) STACK_HIP(hipMemsetAsync(b->p, 0, b->bytes, stream), "clear states");
+    return MI355X_OK;
+}
+
+// The tensors' names and where each goes. Sizes are known from the configuration.
+void Stack::name_tensors() {
+    const int64_t W = width();
+    auto mat = [&](const std::string& s, Mat& m, int64_t row0, int64_t rows, int64_t cols) {
+        Slot v;
+        v.mat = &m; v.row0 = row0; v.rows = rows; v.cols = cols;
+        slots[s] = v;
+        if (row0 + rows > m.n) m.n = row0 + rows;
+        m.k = cols;
+        m.ld = pad64(cols);
+    };
+    auto vec = [&](const std::string& s, Vec& d, int64_t n) {
+        Slot v;
+        v.vec = &d; v.rows = 1; v.cols = n;
+        slots[s] = v;
+        d.n = n;
+    };
+    mat("embed", embed, 0, vocab, W);
+    vec("embed.norm", embed_norm, W);
+    vec("final.norm", final_norm, W);
+    for (size_t i = 0; i < layers.size(); i++) {
+        StackLayer& l = layers[i];
+        const std::string p = "l" + std::to_string(i) + ".", mp = p + "mix.";
+        const int64_t H = l.c.heads, qk = H * l.c.dim, mixed = l.mixed();
+        vec(p + "norm1", l.norm1, W);
+        vec(p + "norm1b", l.norm1b, W);
+        vec(p + "canon1", l.canon, W * c.taps);
+        vec(p + "dwa", l.dwa, (int64_t)i + 2);
+        if (l.c.ff > 0) {
+            vec(p + "norm2", l.norm2, W);
+            vec(p + "norm2b", l.norm2b, W);
+            mat(p + "mlp.up", l.up, 0, l.c.ff, W);
+            mat(p + "mlp.down", l.down, 0, W, l.c.ff);
+        }
+        mat(mp + "o", l.o, 0, W, mixed);
+        if (!l.recurrent()) {
+            const int64_t qn = H * (l.c.dim + l.c.rot_dim);
+            mat(mp + "q", l.in, 0, qn, W);
+            mat(mp + "dkv", l.in, qn, l.c.kv_rank + l.c.rot_dim, W);
+            vec(mp + "dkv.norm", l.dkv_norm, l.c.kv_rank);
+            mat(mp + "uk", l.ukv, 0, qk, l.c.kv_rank);
+            mat(mp + "uv", l.ukv, qk, mixed, l.c.kv_rank);
+            continue;
+        }
+        mat(mp + "q", l.in, 0, qk, W);
+        mat(mp + "k", l.in, qk, qk, W);
+        mat(mp + "v", l.in, 2 * qk, mixed, W);
+        l.g_at = 2 * qk + mixed;
+        mat(mp + "g", l.in, l.g_at, mixed, W);
+        l.gates_at = l.g_at + mixed;
+        vec(mp + "norm", l.mix_norm, mixed);
+        if (l.c.mixer == MI355X_MIXER_MLSTM) {
+            mat(mp + "i", l.in, l.gates_at, H, W);
+            mat(mp + "f", l.in, l.gates_at + H, H, W);
+            vec(mp + "i.b", l.bias_i, H);
+            vec(mp + "f.b", l.bias_f, H);
+        }
+    }
+}
+
+mi355x_status Stack::set_tensor(const char* tensor, int dtype, const void* host, int64_t n_elems) {
+    auto it = slots.find(tensor);
+    if (it == slots.end()) return capi_fail(MI355X_ERR_SHAPE, "mi355x: stack: unknown tensor %s", tensor);
+    Slot& v = it->second;
+    if (v.rows * v.cols != n_elems)
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: stack: %s of %lld elements, want [%lld, %lld]", tensor, (long long)n_elems, (long long)v.rows, (long long)v.cols);
+    if (dtype != kBF16 && !(v.vec && dtype == kF32)) return capi_fail(MI355X_ERR_DTYPE, "mi355x: stack: %s of dtype %d, want bfloat16", tensor, dtype);
+    if (v.vec) {
+        std::vector<float> f((size_t)n_elems);
+        if (dtype == kF32) {
+            memcpy(f.data(), host, f.size() * 4);
+        } else {
+            for (int64_t i = 0; i < n_elems; i++) {
+                const uint32_t bits = (uint32_t)((const uint16_t*)host)[i] << 16;
+                memcpy(&f[(size_t)i], &bits, 4);
+            }
+        }
+        if (!v.vec->buf.p) STACK_HIP(v.vec->buf.alloc(f.size() * 4), "hipMalloc(weight)");
+        STACK_HIP(hipMemcpy(v.vec->buf.p, f.data(), f.size() * 4, hipMemcpyHostToDevice), "hipMemcpy(weight)");
+    } else {
+        Mat& m = *v.mat;
+        if (!m.buf.p) {
+            STACK_HIP(m.buf.alloc((size_t)m.n * m.ld * 2), "hipMalloc(weight)");
+            STACK_HIP(hipMemset(m.buf.p, 0, (size_t)m.n * m.ld * 2), "hipMemset(weight)");
+        }
+        STACK_HIP(hipMemcpy2D(m.buf.as<uint16_t>() + v.row0 * m.ld, (size_t)m.ld * 2, host, (size_t)v.cols * 2, (size_t)v.cols * 2, (size_t)v.rows,
+                              hipMemcpyHostToDevice), "hipMemcpy(weight)");
+    }
+    v.set = true;
+    ready = false;
+    return MI355X_OK;
+}
+
+mi355x_status Stack::finalize(int64_t max_tokens) {
+    for (const auto& kv : slots)
+        if (!kv.second.set) return capi_fail(MI355X_ERR_SHAPE, "mi355x: stack: tensor %s missing", kv.first.c_str());
+    const int64_t W = width();
+    int64_t per = 8192 / batch;  // rows of a pass: longer calls go in portions
+    per = per < 1 ? 1 : per;
+    if (max_tokens > context) max_tokens = context;
+    const int64_t R = batch * (max_tokens < per ? max_tokens : per);
+    const int64_t logit_n = R < 256 ? R : 256 > batch ? 256 : batch;
+    if (mi355x_status st = alloc_common(R, logit_n < batch ? batch : logit_n)) return st;
+    auto zeroed = [&](DevBuf& b, size_t bytes) -> mi355x_status {
+        STACK_HIP(b.alloc(bytes), "hipMalloc");
+        STACK_HIP(hipMemset(b.p, 0, b.bytes), "hipMemset");
+        return MI355X_OK;
+    };
+#define STACK_BUF(buf, n)                                              \
+    do {                                                               \
+        if (mi355x_status st_ = zeroed(buf, (size_t)(n))) return st_;  \
+    } while (0)
+    int64_t in_n = 0, mixed = 0, ff = 0, gate_n = 0;
+    size_t ws_floats = 0;
+    for (StackLayer& l : layers) {
+        in_n = l.in.n > in_n ? l.in.n : in_n;
+        mixed = l.mixed() > mixed ? l.mixed() : mixed;
+        ff = l.c.ff > ff ? l.c.ff : ff;
+        const int64_t H = l.c.heads;
+        if (c.taps > 1) STACK_BUF(l.conv_state, (size_t)batch * (c.taps - 1) * W * 4);
+        if (!l.recurrent()) {
+            l.ldc = (l.c.kv_rank + l.c.rot_dim + 7) / 8 * 8;
+            // rows are read to a multiple of 64 elements of the latent: one row more than the context
+            STACK_BUF(l.cache, ((size_t)batch * context * l.ldc + pad64(l.ldc) + 64) * (half() ? 2 : 4));
+            const int half_n = l.c.rot_dim / 2;
+            std::vector<float> cs((size_t)context * half_n), sn((size_t)context * half_n);
+            for (int i = 0; i < half_n; i++) {
+                const double f = std::pow(l.c.rot_base, -2.0 * i / (double)l.c.rot_dim);
+                for (int64_t p = 0; p < context; p++) {
+                    cs[p * half_n + i] = (float)std::cos((double)p * f);
+                    sn[p * half_n + i] = (float)std::sin((double)p * f);
+                }
+            }
+            STACK_BUF(l.cos_t, cs.size() * 4);
+            STACK_BUF(l.sin_t, sn.size() * 4);
+            STACK_HIP(hipMemcpy(l.cos_t.p, cs.data(), cs.size() * 4, hipMemcpyHostToDevice), "hipMemcpy(angles)");
+            STACK_HIP(hipMemcpy(l.sin_t.p, sn.data(), sn.size() * 4, hipMemcpyHostToDevice), "hipMemcpy(angles)");
+            const size_t need = latent_absorbed_ws_floats(latent(l, 1, nullptr), R);
+            ws_floats = need > ws_floats ? need : ws_floats;
+            continue;
+        }
+        STACK_BUF(l.S, (size_t)batch * H * l.c.dim * l.c.vdim * 4);
+        if (l.c.mixer == MI355X_MIXER_MLSTM) {
+            gate_n = 2 * H > gate_n ? 2 * H : gate_n;
+            STACK_BUF(l.n, (size_t)batch * H * recurrence_slices(l.c.vdim) * l.c.dim * 4);
+            STACK_BUF(l.m, (size_t)batch * H * recurrence_slices(l.c.vdim) * 4);
+        } else {
+            std::vector<float> d(H), pw((size_t)H * (kRecurrenceChunk + 1));
+            for (int64_t i = 0; i < H; i++) {
+                d[i] = (float)l.decay[i];
+                for (int j = 0; j <= kRecurrenceChunk; j++) pw[i * (kRecurrenceChunk + 1) + j] = (float)std::pow((double)d[i], j);
+            }
+            STACK_BUF(l.decay_f, d.size() * 4);
+            STACK_BUF(l.decay_pow, pw.size() * 4);
+            STACK_HIP(hipMemcpy(l.decay_f.p, d.data(), d.size() * 4, hipMemcpyHostToDevice), "hipMemcpy(decays)");
+            STACK_HIP(hipMemcpy(l.decay_pow.p, pw.data(), pw.size() * 4, hipMemcpyHostToDevice), "hipMemcpy(decays)");
+        }
+    }
+    // rows are padded to a multiple of 64 elements that a product may read; the layers' sizes share the buffers
+    STACK_BUF(streams, (size_t)layers.size() * R * W * 4);
+    STACK_BUF(x, (size_t)R * W * 4);
+    STACK_BUF(h, (size_t)R * W * 4);
+    STACK_BUF(y, (size_t)R * W * 4);
+    STACK_BUF(in_f, (size_t)R * pad64(W) * 4);
+    STACK_BUF(proj_f, (size_t)R * in_n * 4);
+    STACK_BUF(scanned, (size_t)R * mixed * 4);
+    STACK_BUF(mix_f, (size_t)R * pad64(mixed) * 4);
+    STACK_BUF(up_f, (size_t)R * pad64(ff) * 4);
+    STACK_BUF(last_f, (size_t)logit_rows * pad64(W) * 4);
+    STACK_BUF(rows_dev, (size_t)logit_rows * 8);
+    STACK_BUF(ws, ws_floats * 4);
+#undef STACK_BUF
+    cache_len = 0;
+    ready = true;
+    return MI355X_OK;
+}
+
+}  // namespace
+
+}  // namespace mimir
+
+extern "C" {
+
+mi355x_status mi355x_stack_create(const mi355x_stack_config* cfg, const mi355x_stack_layer* layers, void** out) {
+    using namespace mimir;
+    if (!cfg || !layers || !out) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: stack_create: null pointer");
+    const auto& c = *cfg;
+    if (c.width <= 0 || c.width > 15360 || c.vocab <= 0 || c.layers <= 0 || c.layers > 1024 || c.context <= 0 || c.batch <= 0 || c.batch > 8192 || c.taps <= 0 ||
+        c.norm_groups <= 0 || c.norm_groups > 512 || c.width % c.norm_groups != 0 || !(c.eps > 0))
+        return capi_fail(MI355X_ERR_SHAPE, "mi355x: stack: hyperparameters: width %d in %d groups, %d layers, %d taps, vocabulary %d, context %d, batch %d",
+                         c.width, c.norm_groups, c.layers, c.taps, c.vocab, c.context, c.batch);
+    if (c.dtype != MI355X_F32 && c.dtype != MI355X_BF16) return capi_fail(MI355X_ERR_DTYPE, "mi355x: stack: compute dtype %d", c.dtype);
+    auto m = std::make_unique<Stack>();
+    m->c = c;
+    m->name = "stack"; m->vocab = c.vocab; m->context = c.context; m->batch = c.batch;
+    m->layers.resize(c.layers);
+    for (int i = 0; i < c.layers; i++) {
+        const auto& l = layers[i];
+        bool ok = l.heads > 0 && l.heads <= 4096 && l.dim > 0 && l.vdim > 0 && l.ff >= 0 && (int64_t)l.heads * l.vdim <= 15360;
+        if (l.mixer == MI355X_MIXER_LATENT) ok = ok && l.rot_dim > 0 && l.rot_dim % 2 == 0 && l.kv_rank > 0 && l.kv_rank <= 1024 && l.rot_dim <= 1024 && l.rot_base > 0;
+        else if (l.mixer == MI355X_MIXER_MLSTM) ok = ok && l.dim <= kRecurrenceMaxDim && l.gate_cap > 0;
+        else if (l.mixer == MI355X_MIXER_LIGHTNING) ok = ok && l.dim <= kRecurrenceMaxDim && l.decay;
+        else ok = false;
+        if (!ok)
+            return capi_fail(MI355X_ERR_SHAPE, "mi355x: stack: layer %d: mixer %d with %d heads of %d and %d features, %d rotated, latent of %d", i, l.mixer, l.heads,
+                             l.dim, l.vdim, l.rot_dim, l.kv_rank);
+        m->layers[i].c = l;
+        if (l.mixer == MI355X_MIXER_LIGHTNING) m->layers[i].decay.assign(l.decay, l.decay + l.heads);
+        m->layers[i].c.decay = nullptr;
+    }
+    m->name_tensors();
+    *out = (Decoder*)m.release();
+    return MI355X_OK;
+}
+
+}  // extern "C"
