@@ -305,6 +305,190 @@ hipError_t launch_attend(const Latent& a, const float* proj, int64_t ldp, const 
     return hipGetLastError();
 }
 
+// ---- many query rows ------------------------------------------------------------------------
+// A wavefront owns 32 query rows of one head and walks the keys in tiles of 64 with a running maximum and sum per row.
+// Both products are computed transposed (scores^T = K Q^T, result^T = V^T P^T), so that a row's scores and results lie in
+// one lane and its partner 32 lanes on, and the weights go from the exponential straight into the second product's
+// operand: the order in which the scores' registers hold the keys is the order in which V^T's fragment is read. Four
+// wavefronts with consecutive rows share a tile of keys and values in LDS; the next tile is requested while one is used.
+
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+
+__device__ __forceinline__ f32x16 mfma_bf16(u32x4 a, u32x4 b, f32x16 c) {
+    return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+}
+__device__ __forceinline__ uint32_t pack2(float lo, float hi) { return (uint32_t)f32_to_bf16_bits(lo) | (uint32_t)f32_to_bf16_bits(hi) << 16; }
+__device__ __forceinline__ float low_part(float v) { return v - bf16_bits_to_f32(f32_to_bf16_bits(v)); }
+
+struct PromptArgs {
+    const uint16_t *q, *keys, *vt, *cache;  // cache: the sequence's rows
+    uint16_t* out;
+    int64_t ldq, ldk, ldv, ldc, ldo;
+    int heads, dim, rot_dim, vdim, rank;
+    int past, s;
+    float scale;  // times log2(e)
+};
+
+constexpr int kPromptRows = 128;
+
+// DT: sixteenths of dim + rot_dim, rounded up; VT: 32nds of vdim, rounded up. WHOLE: rows and their parts are multiples of
+// 16 bytes (else keys and queries are brought element by element).
+template <int DT, int VT, bool WHOLE>
+__global__ __launch_bounds__(256, DT > 12 ? 1 : 2) void latent_prompt_kernel(PromptArgs p) {
+    constexpr int kKey = DT * 16 + 8, kVal = kKeys + 8;  // elements between rows in LDS
+    constexpr int kKeyLoads = (kKeys * DT * 2 + 255) / 256;
+    __shared__ __align__(16) uint16_t ks[kKeys * kKey];
+    __shared__ __align__(16) uint16_t vs[VT * 32 * kVal];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r32 = lane & 31, hi = lane >> 5;
+    const int h = blockIdx.x, first = (int)(gridDim.y - 1 - blockIdx.y) * kPromptRows;  // the last rows first: they see the most keys
+    const int D = p.dim + p.rot_dim, n_keys = p.past + p.s;
+    const int row = first + wave * 32 + r32, pos = p.past + row;  // sees keys 0 .. pos
+    const int last_wg = first + kPromptRows < p.s ? first + kPromptRows : p.s;
+    const int seen_wg = p.past + last_wg;
+    const int seen_wave = first + wave * 32 < p.s ? (p.past + (first + wave * 32 + 32 < p.s ? first + wave * 32 + 32 : p.s)) : 0;
+
+    u32x4 q[DT];
+    {
+        const uint16_t* qr = p.q + (int64_t)(row < p.s ? row : p.s - 1) * p.ldq + (int64_t)h * D;
+#pragma unroll
+        for (int k = 0; k < DT; k++) {
+            const int d = k * 16 + hi * 8;
+            if (WHOLE) {
+                q[k] = d < D ? *(const u32x4*)(qr + d) : u32x4{0, 0, 0, 0};
+                continue;
+            }
+            uint16_t e[8];
+#pragma unroll
+            for (int i = 0; i < 8; i++) e[i] = d + i < D ? qr[d + i] : (uint16_t)0;
+            __builtin_memcpy(&q[k], e, 16);
+        }
+    }
+    u32x4 kreg[kKeyLoads], vreg[VT];
+    auto fetch = [&](int j0) {
+#pragma unroll
+        for (int n = 0; n < kKeyLoads; n++) {
+            const int item = tid + 256 * n, r = item / (DT * 2), d = item % (DT * 2) * 8;
+            if (kKeys * DT * 2 % 256 != 0 && item >= kKeys * DT * 2) break;
+            const int64_t j = j0 + r < n_keys ? j0 + r : n_keys - 1;  // past the last key: never seen
+            const uint16_t* k = p.keys + j * p.ldk + (int64_t)h * p.dim;
+            const uint16_t* c = p.cache + j * p.ldc + p.rank - p.dim;
+            if (WHOLE) {  // pieces past the last feature meet zeros of q: any finite value does
+                kreg[n] = *(const u32x4*)(d < p.dim ? k + d : d < D ? c + d : k);
+            } else {
+                uint16_t e[8];
+#pragma unroll
+                for (int i = 0; i < 8; i++) e[i] = d + i < p.dim ? k[d + i] : d + i < D ? c[d + i] : (uint16_t)0;
+                __builtin_memcpy(&kreg[n], e, 16);
+            }
+        }
+#pragma unroll
+        for (int n = 0; n < VT; n++) {
+            const int item = tid + 256 * n, r = item >> 3;
+            vreg[n] = *(const u32x4*)(p.vt + ((int64_t)h * p.vdim + (r < p.vdim ? r : p.vdim - 1)) * p.ldv + j0 + (item & 7) * 8);
+        }
+    };
+    auto stage = [&]() {
+#pragma unroll
+        for (int n = 0; n < kKeyLoads; n++) {
+            const int item = tid + 256 * n;
+            if (kKeys * DT * 2 % 256 != 0 && item >= kKeys * DT * 2) break;
+            *(u32x4*)(ks + item / (DT * 2) * kKey + item % (DT * 2) * 8) = kreg[n];
+        }
+#pragma unroll
+        for (int n = 0; n < VT; n++) {
+            const int item = tid + 256 * n;
+            *(u32x4*)(vs + (item >> 3) * kVal + (item & 7) * 8) = vreg[n];
+        }
+    };
+    f32x16 o[VT];
+#pragma unroll
+    for (int t = 0; t < VT; t++)
+#pragma unroll
+        for (int i = 0; i < 16; i++) o[t][i] = 0.f;
+    float m = -__builtin_inff(), l = 0.f;  // the row's maximum (in units of log2); the sum over the keys this half of the lanes holds
+    fetch(0);
+    for (int j0 = 0; j0 < seen_wg; j0 += kKeys) {
+        __syncthreads();  // the tile before has been read
+        stage();
+        __syncthreads();
+        if (j0 + kKeys < seen_wg) fetch(j0 + kKeys);
+        if (j0 >= seen_wave) continue;
+        f32x16 sc[2];
+#pragma unroll
+        for (int b = 0; b < 2; b++) {
+#pragma unroll
+            for (int i = 0; i < 16; i++) sc[b][i] = 0.f;
+#pragma unroll
+            for (int k = 0; k < DT; k++) sc[b] = mfma_bf16(*(const u32x4*)(ks + (b * 32 + r32) * kKey + k * 16 + hi * 8), q[k], sc[b]);
+        }
+        const bool whole = j0 + kKeys - 1 <= p.past + first + wave * 32;  // every row of the wavefront sees the whole tile
+        float top = -__builtin_inff();
+#pragma unroll
+        for (int b = 0; b < 2; b++)
+#pragma unroll
+            for (int i = 0; i < 16; i++) {
+                float v = sc[b][i] * p.scale;
+                if (!whole && j0 + b * 32 + (i & 3) + 8 * (i >> 2) + 4 * hi > pos) v = -__builtin_inff();
+                sc[b][i] = v;
+                top = fmaxf(top, v);
+            }
+        top = fmaxf(top, __shfl_xor(top, 32));
+        const float next = fmaxf(m, top);  // a row past the end sees keys too: finite from the first tile on
+        if (__any(next > m)) {
+            const float back = __builtin_amdgcn_exp2f(m - next);
+            l *= back;
+#pragma unroll
+            for (int t = 0; t < VT; t++)
+#pragma unroll
+                for (int i = 0; i < 16; i++) o[t][i] *= back;
+            m = next;
+        }
+#pragma unroll
+        for (int b = 0; b < 2; b++)
+#pragma unroll
+            for (int half = 0; half < 2; half++) {
+                u32x4 high, low;
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const float x = __builtin_amdgcn_exp2f(sc[b][half * 8 + 2 * i] - m), y = __builtin_amdgcn_exp2f(sc[b][half * 8 + 2 * i + 1] - m);
+                    l += x + y;
+                    high[i] = pack2(x, y);
+                    low[i] = pack2(low_part(x), low_part(y));
+                }
+#pragma unroll
+                for (int t = 0; t < VT; t++) {
+                    const uint16_t* v = vs + (t * 32 + r32) * kVal + b * 32 + half * 16 + hi * 4;
+                    const u32x2 v0 = *(const u32x2*)v, v1 = *(const u32x2*)(v + 8);
+                    const u32x4 a = {v0[0], v0[1], v1[0], v1[1]};
+                    o[t] = mfma_bf16(a, high, o[t]);
+                    o[t] = mfma_bf16(a, low, o[t]);
+                }
+            }
+    }
+    const float inv = 1.f / (l + __shfl_xor(l, 32));
+    if (row >= p.s) return;
+    uint16_t* out = p.out + (int64_t)row * p.ldo + (int64_t)h * p.vdim;
+#pragma unroll
+    for (int t = 0; t < VT; t++)
+#pragma unroll
+        for (int g = 0; g < 4; g++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int e = t * 32 + 8 * g + 4 * hi + i;
+                if (e < p.vdim) out[e] = f32_to_bf16_bits(o[t][4 * g + i] * inv);
+            }
+}
+
+template <int DT, int VT>
+void launch_prompt(const PromptArgs& p, hipStream_t st) {
+    const dim3 grid((unsigned)p.heads, (unsigned)((p.s + kPromptRows - 1) / kPromptRows));
+    const bool whole = p.dim % 8 == 0 && p.rot_dim % 8 == 0 && p.rank % 8 == 0 && p.ldq % 8 == 0 && p.ldk % 8 == 0 && p.ldc % 8 == 0 &&
+                       (((uintptr_t)p.q | (uintptr_t)p.keys | (uintptr_t)p.cache) & 15) == 0;
+    if (whole) hipLaunchKernelGGL((latent_prompt_kernel<DT, VT, true>), grid, dim3(256), 0, st, p);
+    else hipLaunchKernelGGL((latent_prompt_kernel<DT, VT, false>), grid, dim3(256), 0, st, p);
+}
+
 }  // namespace
 
 hipError_t latent_prepare(const Latent& a, float* proj, int64_t ldp, uint16_t* q_bf16, int64_t ldq, hipStream_t st) {
@@ -346,6 +530,28 @@ hipError_t latent_absorbed(const Latent& a, const float* proj, int64_t ldp, floa
     if (e != hipSuccess) return e;
     hipLaunchKernelGGL(latent_combine_kernel, dim3((unsigned)rows, (unsigned)a.heads, (unsigned)((a.vdim + kValues - 1) / kValues)), dim3(256),
                        (size_t)((a.rank + 63) / 64 * 64) * 4, st, a, splits, po, ml, out_f32, out_bf16, ldo);
+    return hipGetLastError();
+}
+
+bool latent_prompt_ok(const Latent& a) {
+    return a.cache_bf16 && a.dim + a.rot_dim <= 256 && a.vdim <= 256 && a.past + a.s < 1 << 30 && !a.past_dev;
+}
+
+hipError_t latent_prompt(const Latent& a, int sequence, const uint16_t* q, int64_t ldq, const uint16_t* keys, int64_t ldk, const uint16_t* values_t,
+                         int64_t ldv, uint16_t* out, int64_t ldo, hipStream_t st) {
+    if (a.s == 0) return hipSuccess;
+    if (!latent_prompt_ok(a) || ldv % 64 || ((uintptr_t)values_t & 15)) return hipErrorInvalidValue;
+    PromptArgs p;
+    p.q = q; p.keys = keys; p.vt = values_t; p.cache = (const uint16_t*)a.cache + sequence * a.context * a.ldc; p.out = out;
+    p.ldq = ldq; p.ldk = ldk; p.ldv = ldv; p.ldc = a.ldc; p.ldo = ldo;
+    p.heads = a.heads; p.dim = a.dim; p.rot_dim = a.rot_dim; p.vdim = a.vdim; p.rank = a.rank;
+    p.past = (int)a.past; p.s = (int)a.s;
+    p.scale = a.scale * 1.4426950408889634f;
+    const int d = a.dim + a.rot_dim, v = a.vdim;
+    if (d <= 64 && v <= 64) launch_prompt<4, 2>(p, st);
+    else if (d <= 128 && v <= 128) launch_prompt<8, 4>(p, st);
+    else if (d <= 192 && v <= 128) launch_prompt<12, 4>(p, st);
+    else launch_prompt<16, 8>(p, st);
     return hipGetLastError();
 }
 

@@ -1,5 +1,112 @@
-#include "device_util.h"
+// y = act(x . W^T) for many rows of bfloat16 x and bfloat16 weights on the bfloat16 matrix cores, float32 sums: the
+// prompt product of a model whose weights are bfloat16. The tiles are those of gemm_nt_tile.h, cut as tile_plan.h
+// chooses; products with too few tiles of 128 x 256 for the device take tiles of 64 x 128. The activation and the
+// rounding to the output's dtype happen as the tile is stored.
+#include "gemm_nt_tile.h"
+#include "kernels.h"
 #include "stack_ops.h"
+#include "tile_plan.h"
+
 namespace mimir {
-hipError_t gemm_bf16(const uint16_t* W, int64_t ldw, const uint16_t* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st) { return hipErrorNotSupported; }
+
+namespace {
+
+constexpr size_t kLdsBytes = 2 * (size_t)Wide::kStageBytes;
+
+// Costs in Wide tiles' time (qgemm_f16_panel.hip), a Tiny tile's share of the MFMAs with as many more reads from LDS.
+constexpr double kNarrowCost = 0.78, kLowCost = 0.56, kTinyCost = 0.19;
+
+struct ActStore {
+    ProductOut out;
+    bool wide_ok;
+    __device__ __forceinline__ float row(int, int) const { return 0.f; }
+    __device__ __forceinline__ void operator()(int m, int n, int N, float, float v[4]) const {
+        if (out.relu2) {
+#pragma unroll
+            for (int k = 0; k < 4; k++) v[k] = v[k] > 0.f ? v[k] * v[k] : 0.f;
+        } else if (n < out.silu_n) {
+#pragma unroll
+            for (int k = 0; k < 4; k++)
+                if (n + k < out.silu_n) v[k] = v[k] / (1.f + __expf(-v[k]));
+        }
+        const int64_t at = m * out.ld + n;
+        if (wide_ok && n + 3 < N) {
+            if (out.f32) {
+                const f32x4 o = {v[0], v[1], v[2], v[3]};
+                *(f32x4*)(out.f32 + at) = o;
+            } else {
+                const u32x2 o = {(uint32_t)f32_to_bf16_bits(v[0]) | (uint32_t)f32_to_bf16_bits(v[1]) << 16,
+                                 (uint32_t)f32_to_bf16_bits(v[2]) | (uint32_t)f32_to_bf16_bits(v[3]) << 16};
+                *(u32x2*)(out.bf16 + at) = o;
+            }
+            return;
+        }
+#pragma unroll
+        for (int k = 0; k < 4; k++) {
+            if (n + k >= N) continue;
+            if (out.f32) out.f32[at + k] = v[k];
+            else out.bf16[at + k] = f32_to_bf16_bits(v[k]);
+        }
+    }
+};
+
+template <class T>
+__device__ __forceinline__ void one_tile(const uint16_t* X, int64_t ldx, const uint16_t* W, int64_t ldw, const ActStore& store, int M, int N, int K, int b,
+                                         int tiles_m, int tiles_n, int col0, char* lds) {
+    const int t = tile_of(b, tiles_m * tiles_n);
+    if (t >= tiles_m * tiles_n) return;  // the whole workgroup
+    tile_body<T, Bf16Element>(X, ldx, W, ldw, store, M, N, K, (t % tiles_m) * T::BM, col0 + (t / tiles_m) * T::BN, lds);
 }
+
+__global__ __launch_bounds__(512, 2) void gemm_bf16_kernel(const uint16_t* __restrict__ X, int64_t ldx, const uint16_t* __restrict__ W, int64_t ldw, ActStore store,
+                                                           int M, int N, int K, PanelPlan plan) {
+    extern __shared__ __align__(1024) char lds_gemm[];
+    int b = (int)blockIdx.x;
+    if (plan.low) {
+        one_tile<Low>(X, ldx, W, ldw, store, M, N, K, b, plan.tiles_m, plan.wide_cols, 0, lds_gemm);
+        return;
+    }
+    const int wide_wgs = ((plan.tiles_m * plan.wide_cols + 7) >> 3) << 3;
+    if (b < wide_wgs) one_tile<Wide>(X, ldx, W, ldw, store, M, N, K, b, plan.tiles_m, plan.wide_cols, 0, lds_gemm);
+    else one_tile<Narrow>(X, ldx, W, ldw, store, M, N, K, b - wide_wgs, plan.tiles_m, plan.narrow_cols, plan.wide_cols * Wide::BN, lds_gemm);
+}
+
+// Two workgroups a compute unit: 48 KB of LDS and few registers each.
+__global__ __launch_bounds__(512, 4) void gemm_bf16_tiny_kernel(const uint16_t* __restrict__ X, int64_t ldx, const uint16_t* __restrict__ W, int64_t ldw,
+                                                                ActStore store, int M, int N, int K, int tiles_m, int tiles_n) {
+    extern __shared__ __align__(1024) char lds_gemm[];
+    one_tile<Tiny>(X, ldx, W, ldw, store, M, N, K, (int)blockIdx.x, tiles_m, tiles_n, 0, lds_gemm);
+}
+
+unsigned die_grid(int tiles) { return (unsigned)((tiles + 7) / 8 * 8); }
+
+}  // namespace
+
+hipError_t gemm_bf16(const uint16_t* W, int64_t ldw, const uint16_t* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st) {
+    if (M == 0 || N == 0) return hipSuccess;
+    if (M >= 1 << 24 || N >= 1 << 24 || K >= 1 << 24 || ldx % 8 || ldw % 8) return hipErrorInvalidValue;
+    {
+        static std::atomic<bool> raised{false};  // threads may race here: both then set the same attribute
+        if (!raised) {
+            hipError_t e = hipFuncSetAttribute((const void*)gemm_bf16_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)kLdsBytes);
+            if (e != hipSuccess) return e;
+            raised = true;
+        }
+    }
+    const int k = (int)((K + 63) / 64 * 64);
+    const void* y = out.f32 ? (const void*)out.f32 : (const void*)out.bf16;
+    const ActStore store{out, out.ld % 4 == 0 && ((uintptr_t)y & 15) == 0};
+    PanelPlan plan;
+    const double end = plan_panel(M, N, kNarrowCost, kLowCost, &plan);
+    const int tm = (int)((M + Tiny::BM - 1) / Tiny::BM), tn = (int)((N + Tiny::BN - 1) / Tiny::BN);
+    if (makespan(tm * tn, kTinyCost, 0, 0.0) < end - 1e-9) {
+        hipLaunchKernelGGL(gemm_bf16_tiny_kernel, dim3(die_grid(tm * tn)), dim3(512), 2 * (size_t)Tiny::kStageBytes, st, x, ldx, W, ldw, store, (int)M, (int)N, k,
+                           tm, tn);
+        return hipGetLastError();
+    }
+    const int first = plan.tiles_m * plan.wide_cols, then = plan.tiles_m * plan.narrow_cols;
+    hipLaunchKernelGGL(gemm_bf16_kernel, dim3(die_grid(first) + die_grid(then)), dim3(512), kLdsBytes, st, x, ldx, W, ldw, store, (int)M, (int)N, k, plan);
+    return hipGetLastError();
+}
+
+}  // namespace mimir

@@ -25,6 +25,10 @@ namespace {
 
 #define STACK_HIP(expr, what) DECODER_HIP(expr, "stack", what)
 
+// From how many positions of a sequence in one pass a prompt's forms are taken (bfloat16, more than kGemvRows rows):
+// keys and values formed for latent attention, recurrences in chunks.
+constexpr int64_t kFormKeys = 32, kChunked = 16;
+
 int64_t pad64(int64_t n) { return (n + 63) / 64 * 64; }
 
 struct Mat {  // [n, k] bfloat16, rows ld apart, zeros from k on
@@ -67,6 +71,7 @@ struct Stack : Decoder {
 
     // activations of up to max_rows rows; *_f float32, *_b bfloat16
     DevBuf streams, x, h, y, in_f, in_b, proj_f, proj_b, gates, scanned, mix_f, mix_b, up_f, up_b, last_f, last_b, rows_dev, ws;
+    DevBuf q_b, keys_b, values_b;  // latent attention of a prompt: turned queries; one sequence's keys, and its values transposed
 
     mi355x_status set_tensor(const char* tensor, int dtype, const void* host, int64_t n_elems) override;
     mi355x_status finalize(int64_t max_tokens) override;
@@ -80,9 +85,10 @@ struct Stack : Decoder {
     int64_t width() const { return c.width; }
     void name_tensors();
     Latent latent(const StackLayer& l, int64_t s, const int32_t* pos) const;
-    Recurrence recurrence(const StackLayer& l, int64_t s) const;
+    Recurrence recurrence(const StackLayer& l, int64_t s, bool tiles) const;
     mi355x_status pass(const int32_t* tokens, int64_t s, const int32_t* pos);
     mi355x_status mix(StackLayer& l, int64_t s, bool tiles, const int32_t* pos);
+    mi355x_status prompt_attention(const StackLayer& l, const Latent& a);
     // out = act(x . W[row0, row0 + n)^T) by the kernel for this many rows and x's form (bfloat16 if b, else float32)
     mi355x_status product(const Mat& w, int64_t row0, int64_t n, const DevBuf& f, const DevBuf& b, bool tiles, int64_t rows, const ProductOut& out);
 };
@@ -107,13 +113,19 @@ Latent Stack::latent(const StackLayer& l, int64_t s, const int32_t* pos) const {
     return a;
 }
 
-Recurrence Stack::recurrence(const StackLayer& l, int64_t s) const {
+Recurrence Stack::recurrence(const StackLayer& l, int64_t s, bool tiles) const {
     Recurrence r;
     const int64_t qk = (int64_t)l.c.heads * l.c.dim;
-    r.ld = l.in.n;
-    r.q = proj_f.as<float>(); r.k = proj_f.as<float>() + qk; r.v = proj_f.as<float>() + 2 * qk;
+    r.bf16 = tiles;
+    if (tiles) {
+        r.ld = pad64(l.gates_at);
+        r.q = proj_b.as<uint16_t>(); r.k = proj_b.as<uint16_t>() + qk; r.v = proj_b.as<uint16_t>() + 2 * qk;
+    } else {
+        r.ld = l.in.n;
+        r.q = proj_f.as<float>(); r.k = proj_f.as<float>() + qk; r.v = proj_f.as<float>() + 2 * qk;
+    }
     if (l.c.mixer == MI355X_MIXER_MLSTM) {
-        r.gates = proj_f.as<float>() + l.gates_at; r.ldg = l.in.n;
+        r.gates = tiles ? gates.as<float>() : proj_f.as<float>() + l.gates_at; r.ldg = tiles ? 2 * l.c.heads : l.in.n;
         r.bias_i = l.bias_i.p(); r.bias_f = l.bias_f.p();
         r.cap = (float)l.c.gate_cap;
         r.q_scale = (float)(1.0 / std::sqrt((double)l.c.dim));
@@ -128,25 +140,61 @@ Recurrence Stack::recurrence(const StackLayer& l, int64_t s) const {
     return r;
 }
 
+// A prompt's latent attention, sequence by sequence: keys and transposed values of all positions from the cached
+// latents, then the attention on them.
+mi355x_status Stack::prompt_attention(const StackLayer& l, const Latent& a) {
+    const int64_t n = a.past + a.s, kn = (int64_t)a.heads * a.dim, vn = l.mixed(), ldv = pad64(context), qn = (int64_t)a.heads * (a.dim + a.rot_dim);
+    for (int b = 0; b < batch; b++) {
+        const uint16_t* latents = l.cache.as<uint16_t>() + (int64_t)b * context * a.ldc;
+        ProductOut k;
+        k.bf16 = keys_b.as<uint16_t>(); k.ld = kn;
+        STACK_HIP(gemm_bf16(a.w_uk, a.ldw, latents, a.ldc, n, kn, a.rank, k, stream), "keys");
+        ProductOut v;
+        v.bf16 = values_b.as<uint16_t>(); v.ld = ldv;
+        STACK_HIP(gemm_bf16(latents, a.ldc, a.w_uv, a.ldw, vn, n, a.rank, v, stream), "values");
+        STACK_HIP(latent_prompt(a, b, q_b.as<uint16_t>() + b * a.s * qn, qn, keys_b.as<uint16_t>(), kn, values_b.as<uint16_t>(), ldv,
+                                mix_b.as<uint16_t>() + b * a.s * l.o.ld, l.o.ld, stream), "latent attention");
+    }
+    return MI355X_OK;
+}
+
 // y = mixer(in), for s positions a sequence.
 mi355x_status Stack::mix(StackLayer& l, int64_t s, bool tiles, const int32_t* pos) {
     const int64_t rows = (int64_t)batch * s, mixed = l.mixed();
     if (!l.recurrent()) {
-        ProductOut p;
+        ProductOut p;  // float32: the latent's norm and the rotation see what the product summed
         p.f32 = proj_f.as<float>(); p.ld = l.in.n;
         if (mi355x_status st = product(l.in, 0, l.in.n, in_f, in_b, tiles, rows, p)) return st;
         const Latent a = latent(l, s, pos);
-        STACK_HIP(latent_prepare(a, proj_f.as<float>(), l.in.n, nullptr, 0, stream), "latents and rotation");
-        STACK_HIP(latent_absorbed(a, proj_f.as<float>(), l.in.n, ws.as<float>(), tiles ? nullptr : mix_f.as<float>(), tiles ? mix_b.as<uint16_t>() : nullptr,
-                                  l.o.ld, stream), "latent attention");
+        const bool formed = tiles && s >= kFormKeys && latent_prompt_ok(a);
+        STACK_HIP(latent_prepare(a, proj_f.as<float>(), l.in.n, formed ? q_b.as<uint16_t>() : nullptr, (int64_t)l.c.heads * (l.c.dim + l.c.rot_dim), stream),
+                  "latents and rotation");
+        if (formed) {
+            if (mi355x_status st = prompt_attention(l, a)) return st;
+        } else {
+            STACK_HIP(latent_absorbed(a, proj_f.as<float>(), l.in.n, ws.as<float>(), tiles ? nullptr : mix_f.as<float>(),
+                                      tiles ? mix_b.as<uint16_t>() : nullptr, l.o.ld, stream), "latent attention");
+        }
     } else {
         ProductOut p;
-        p.f32 = proj_f.as<float>(); p.ld = l.in.n;
         p.silu_n = l.c.mixer == MI355X_MIXER_LIGHTNING ? l.g_at : 0;
-        if (mi355x_status st = product(l.in, 0, l.in.n, in_f, in_b, tiles, rows, p)) return st;
-        const Recurrence r = recurrence(l, s);
-        STACK_HIP(recurrence_scan(r, stream), "recurrence");
-        STACK_HIP(gated_norm(scanned.as<float>(), proj_f.as<float>() + l.g_at, false, l.in.n, l.mix_norm.p(), rows, (int)mixed,
+        if (tiles) {
+            p.bf16 = proj_b.as<uint16_t>(); p.ld = pad64(l.gates_at);
+            if (mi355x_status st = product(l.in, 0, l.gates_at, in_f, in_b, true, rows, p)) return st;
+            if (l.in.n > l.gates_at) {  // the recurrence's gates are not rounded
+                ProductOut g;
+                g.f32 = gates.as<float>(); g.ld = l.in.n - l.gates_at;
+                if (mi355x_status st = product(l.in, l.gates_at, g.ld, in_f, in_b, false, rows, g)) return st;
+            }
+        } else {
+            p.f32 = proj_f.as<float>(); p.ld = l.in.n;
+            if (mi355x_status st = product(l.in, 0, l.in.n, in_f, in_b, false, rows, p)) return st;
+        }
+        const Recurrence r = recurrence(l, s, tiles);
+        if (tiles && s >= kChunked && recurrence_chunks_ok(r)) STACK_HIP(recurrence_chunks(r, stream), "recurrence in chunks");
+        else STACK_HIP(recurrence_scan(r, stream), "recurrence");
+        const void* g = tiles ? (const void*)(proj_b.as<uint16_t>() + l.g_at) : (const void*)(proj_f.as<float>() + l.g_at);
+        STACK_HIP(gated_norm(scanned.as<float>(), g, tiles, tiles ? p.ld : l.in.n, l.mix_norm.p(), rows, (int)mixed,
                              l.c.mixer == MI355X_MIXER_MLSTM ? l.c.heads : 1, (float)c.eps, tiles ? nullptr : mix_f.as<float>(),
                              tiles ? mix_b.as<uint16_t>() : nullptr, l.o.ld, stream), "gated norm");
     }
@@ -159,7 +207,7 @@ mi355x_status Stack::mix(StackLayer& l, int64_t s, bool tiles, const int32_t* po
 // which leaves the final norm of its rows in last_f; otherwise the residual is left in x.
 mi355x_status Stack::pass(const int32_t* tokens, int64_t s, const int32_t* pos) {
     const int64_t rows = (int64_t)batch * s, W = width(), ldw = pad64(W);
-    const bool tiles = false;
+    const bool tiles = half() && rows > kGemvRows;
     NormChain base;
     base.width = c.width; base.groups = c.norm_groups; base.eps = (float)c.eps; base.taps = c.taps;
     auto into_layer = [&](NormChain& a, size_t i) {  // the end of a chain: layer i's norm, or the final one
@@ -225,7 +273,7 @@ mi355x_status Stack::forward(int64_t s) {
 
 mi355x_status Stack::head(const int64_t* rows, int64_t n) {
     if (n <= 0) return MI355X_OK;
-    const bool tiles = false;
+    const bool tiles = half() && n > kGemvRows;
     STACK_HIP(hipMemcpyAsync(rows_dev.p, rows, (size_t)n * 8, hipMemcpyHostToDevice, stream), "upload rows");
     STACK_HIP(norm_rows(x.as<float>(), rows_dev.as<int64_t>(), n, final_norm.p(), c.width, c.norm_groups, (float)c.eps, tiles ? nullptr : last_f.as<float>(),
                         tiles ? last_b.as<uint16_t>() : nullptr, embed.ld, stream), "final norm");
@@ -238,7 +286,7 @@ mi355x_status Stack::step() {
     if (mi355x_status st = pass(next_tok.as<int32_t>(), 1, state.as<int32_t>())) return st;
     ProductOut p;
     p.f32 = logits.as<float>(); p.ld = vocab;
-    return product(embed, 0, vocab, last_f, last_b, false, batch, p);
+    return product(embed, 0, vocab, last_f, last_b, false, batch, p);  // float32 rows, however many
 }
 
 mi355x_status Stack::reset() {
@@ -362,7 +410,7 @@ mi355x_status Stack::finalize(int64_t max_tokens) {
     do {                                                               \
         if (mi355x_status st_ = zeroed(buf, (size_t)(n))) return st_;  \
     } while (0)
-    int64_t in_n = 0, mixed = 0, ff = 0, gate_n = 0;
+    int64_t in_n = 0, mixed = 0, ff = 0, gate_n = 0, q_n = 0, keys_n = 0, values_n = 0;
     size_t ws_floats = 0;
     for (StackLayer& l : layers) {
         in_n = l.in.n > in_n ? l.in.n : in_n;
@@ -389,9 +437,16 @@ mi355x_status Stack::finalize(int64_t max_tokens) {
             STACK_HIP(hipMemcpy(l.sin_t.p, sn.data(), sn.size() * 4, hipMemcpyHostToDevice), "hipMemcpy(angles)");
             const size_t need = latent_absorbed_ws_floats(latent(l, 1, nullptr), R);
             ws_floats = need > ws_floats ? need : ws_floats;
+            q_n = H * (l.c.dim + l.c.rot_dim) > q_n ? H * (l.c.dim + l.c.rot_dim) : q_n;
+            keys_n = H * l.c.dim > keys_n ? H * l.c.dim : keys_n;
+            values_n = l.mixed() > values_n ? l.mixed() : values_n;
             continue;
         }
         STACK_BUF(l.S, (size_t)batch * H * l.c.dim * l.c.vdim * 4);
+        if (half()) {
+            const size_t need = recurrence_chunk_ws_floats(batch, l.c.heads, l.c.dim, l.c.vdim, R / batch);
+            ws_floats = need > ws_floats ? need : ws_floats;
+        }
         if (l.c.mixer == MI355X_MIXER_MLSTM) {
             gate_n = 2 * H > gate_n ? 2 * H : gate_n;
             STACK_BUF(l.n, (size_t)batch * H * recurrence_slices(l.c.vdim) * l.c.dim * 4);
@@ -421,6 +476,20 @@ mi355x_status Stack::finalize(int64_t max_tokens) {
     STACK_BUF(last_f, (size_t)logit_rows * pad64(W) * 4);
     STACK_BUF(rows_dev, (size_t)logit_rows * 8);
     STACK_BUF(ws, ws_floats * 4);
+    if (half() && R > kGemvRows) {
+        STACK_BUF(in_b, (size_t)R * pad64(W) * 2);
+        STACK_BUF(mix_b, (size_t)R * pad64(mixed) * 2);
+        STACK_BUF(up_b, (size_t)R * pad64(ff) * 2);
+        STACK_BUF(proj_b, (size_t)R * pad64(in_n) * 2);
+        STACK_BUF(gates, (size_t)R * gate_n * 4);
+        STACK_BUF(last_b, (size_t)logit_rows * pad64(W) * 2);
+        if (keys_n > 0) {
+            // a product reads rows of latents to a multiple of 64; whole tiles of 64 keys are read of the transposed values
+            STACK_BUF(q_b, (size_t)R * q_n * 2);
+            STACK_BUF(keys_b, (size_t)context * keys_n * 2);
+            STACK_BUF(values_b, (size_t)values_n * pad64(context) * 2);
+        }
+    }
 #undef STACK_BUF
     cache_len = 0;
     ready = true;
