@@ -44,9 +44,16 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const uint16_t* __restric
         }
         __syncthreads();  // the other stage is written next only after everyone has passed the next barrier
         if (k0 + kStep < K) fetch(k0 + kStep);
+        // a step's sum on its own and then added: the matrix cores add one product after the other, and the error of a
+        // long chain grows with its length
+        f32x16 part;
+#pragma unroll
+        for (int i = 0; i < 16; i++) part[i] = 0.f;
 #pragma unroll
         for (int k = 0; k < kStep; k += 2)
-            acc = __builtin_amdgcn_mfma_f32_32x32x2f32(xs[p][(wm + r32) * kPad + k + hi], ws[p][(wn + r32) * kPad + k + hi], acc, 0, 0, 0);
+            part = __builtin_amdgcn_mfma_f32_32x32x2f32(xs[p][(wm + r32) * kPad + k + hi], ws[p][(wn + r32) * kPad + k + hi], part, 0, 0, 0);
+#pragma unroll
+        for (int i = 0; i < 16; i++) acc[i] += part[i];
     }
 #pragma unroll
     for (int i = 0; i < 16; i++) {

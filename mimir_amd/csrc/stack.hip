@@ -210,6 +210,8 @@ mi355x_status Stack::pass(const int32_t* tokens, int64_t s, const int32_t* pos) 
     const bool tiles = half() && rows > kGemvRows;
     NormChain base;
     base.width = c.width; base.groups = c.norm_groups; base.eps = (float)c.eps; base.taps = c.taps;
+    // whether a layer's products read float32 rows; the gates of a recurrence always do
+    auto in_float = [&](const StackLayer& l) { return !tiles || l.c.mixer == MI355X_MIXER_MLSTM; };
     auto into_layer = [&](NormChain& a, size_t i) {  // the end of a chain: layer i's norm, or the final one
         if (i == layers.size()) {
             if (!pos) return;
@@ -219,7 +221,9 @@ mi355x_status Stack::pass(const int32_t* tokens, int64_t s, const int32_t* pos) 
         a.w_next = layers[i].norm1.p();
         if (pos) {
             a.conv_w = layers[i].canon.p(); a.conv_state = layers[i].conv_state.as<float>();
-            a.h_f32 = in_f.as<float>(); a.ldh = ldw;
+            a.ldh = ldw;
+            if (tiles) a.h_bf16 = in_b.as<uint16_t>();
+            if (in_float(layers[i])) a.h_f32 = in_f.as<float>();
         } else {
             a.h_f32 = h.as<float>(); a.ldh = W;
         }
@@ -234,8 +238,7 @@ mi355x_status Stack::pass(const int32_t* tokens, int64_t s, const int32_t* pos) 
     for (size_t i = 0; i < layers.size(); i++) {
         StackLayer& l = layers[i];
         if (!pos) {
-            const bool both = tiles && l.c.mixer == MI355X_MIXER_MLSTM;  // the gates read float32
-            STACK_HIP(causal_conv(h.as<float>(), l.canon.p(), l.conv_state.as<float>(), c.taps, batch, s, c.width, tiles && !both ? nullptr : in_f.as<float>(),
+            STACK_HIP(causal_conv(h.as<float>(), l.canon.p(), l.conv_state.as<float>(), c.taps, batch, s, c.width, in_float(l) ? in_f.as<float>() : nullptr,
                                   tiles ? in_b.as<uint16_t>() : nullptr, ldw, stream), "convolution");
         }
         if (mi355x_status st = mix(l, s, tiles, pos)) return st;

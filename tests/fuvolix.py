@@ -66,7 +66,7 @@ def weights(c, seed=0):
         elif name.endswith("f.b"):
             w = 3 + w
         elif leaf not in ("embed", "b"):
-            w = w * 1.5 / np.sqrt(shape[-1])
+            w = w / np.sqrt(shape[-1])
         out[name] = to_bf16(w)
     return out
 
@@ -92,9 +92,10 @@ def tokens(c, n, seed=0, batch=None):
     return rng.integers(0, c["vocab"], n if batch is None else (batch, n)).astype(np.int32)
 
 
-def error(got, want):
-    """The largest row error: root mean square over the vocabulary with the mean taken off, over that of all the wanted logits."""
+def error(got, want, quantile=1.0):
+    """A row's error: root mean square over the vocabulary with the mean taken off, over that of all the wanted logits. The
+    largest, or another quantile of the rows'."""
     d = np.asarray(got, np.float64) - want
     d = d - d.mean(axis=-1, keepdims=True)
     spread = want - want.mean(axis=-1, keepdims=True)
-    return float(np.sqrt((d * d).mean(axis=-1)).max() / np.sqrt((spread * spread).mean()))
+    return float(np.quantile(np.sqrt((d * d).mean(axis=-1)), quantile) / np.sqrt((spread * spread).mean()))

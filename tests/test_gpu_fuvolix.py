@@ -158,27 +158,29 @@ def test_one_far_key_stands_out(tmp_path, place, dtype):
     """One token that no other position has, whose key a sharp query finds among hundreds: the rows that see it differ
     from those of a sequence without it by far more than the tolerance, and agree with the plain forward."""
     c = X.config([X.latent(heads=2, dim=32, rot_dim=4, vdim=32, kv_rank=64, scale=1.0, base=1e6)], width=64, vocab=80, groups=1, taps=1)
-    w = changed(X.weights(c, 3), canon1=off, dkv__norm=lambda t: t * 0 + 1)
+    w = changed(X.weights(c, 3), canon1=off, dkv__norm=lambda t: t * 0 + 1, dwa=lambda t: np.array([0.0, 1.0]), norm1b=lambda t: 3 * t)
     rng = np.random.default_rng(4)
-    # tokens 0..77 are ordinary, 78 is the key and 79 the query: opposite to one another in the features both heads look at
+    # tokens 0..77 are ordinary; 78 is the key (features 0..15, which keys are made of) and 79 asks (48..63, which queries
+    # are made of)
     e = w["embed"].copy()
     e[:78, :16] = 0.1 * rng.normal(size=(78, 16))
+    e[:78, 48:] = 0.1 * rng.normal(size=(78, 16))
     e[78], e[79] = 0, 0
-    e[78, :16] = 3
-    e[79, :16], e[79, 16:32] = 3, 1
+    e[78, :16], e[78, 16:48] = 3, rng.normal(size=32)
+    e[79, 48:], e[79, 16:48] = 3, rng.normal(size=32)
     w["embed"] = X.to_bf16(e)
     toks = rng.integers(0, 78, 333).astype(np.int32)
     toks[-1] = toks[place + 1] = 79
     without = toks.copy()
     toks[place] = 78
-    # queries and keys agree on the first features
+    # both heads' queries and keys meet in the latent's first features
     q, dkv, uk = w["l0.mix.q"] * 0.1, w["l0.mix.dkv"].copy(), w["l0.mix.uk"] * 0.05
     dkv[:16, :] = 0
     dkv[np.arange(16), np.arange(16)] = 2
     for h in range(2):
         uk[h * 32:h * 32 + 16, :] = 0
         uk[h * 32 + np.arange(16), np.arange(16)] = 1
-        q[h * 36 + np.arange(16), np.arange(16)] = 1
+        q[h * 36 + np.arange(16), 48 + np.arange(16)] = 1
     w |= {"l0.mix.q": X.to_bf16(q), "l0.mix.dkv": X.to_bf16(dkv), "l0.mix.uk": X.to_bf16(uk)}
     want = F.forward(c, w, toks)
     apart = X.error(F.forward(c, w, without)[-1:], want[-1:])
@@ -196,18 +198,17 @@ def test_one_far_position_in_a_state(tmp_path, layer, dtype):
     """A position whose key and value are far larger than the others', in a state that hardly forgets: every later row
     carries it, over chunk edges and into decoding."""
     c = X.config([layer], width=64, vocab=50, groups=1, taps=1)
-    edits = dict(canon1=off)
-    if layer["type"] == "mlstm":
-        edits |= {"f__b": lambda t: t * 0 + 8, "f": off, "i": lambda t: t * 3}
-    w = changed(X.weights(c, 6), **edits)
-    toks = X.tokens(c, 200, 3)
+    # only token 45 has the first feature; keys, values and the input gate grow with it
+    w = changed(X.weights(c, 6), canon1=off, dwa=lambda t: np.array([0.0, 1.0]), embed=lambda t: t * (np.arange(64) > 0) + 6 * np.eye(50, 64, -45))
+    loud = lambda t: t + 4 * (np.arange(64) == 0)
+    w = changed(w, k=loud, v=loud, **({"f__b": lambda t: t * 0 + 8, "f": off, "i__b": lambda t: t * 0 - 2, "i": lambda t: loud(t * 0)} if layer["type"] == "mlstm" else {}))
+    toks = X.tokens(c, 200, 3) % 40
     for place in (0, 62, 63, 64, 130):
-        one = toks % 40
+        one = toks.copy()
         one[place] = 45
-        other = one.copy()
-        other[place] = 46
         want = F.forward(c, w, one)
-        assert X.error(F.forward(c, w, other)[-1:], want[-1:]) > 3 * TOL["float32"]  # it is still there at the end
+        apart = X.error(F.forward(c, w, toks)[-1:], want[-1:])
+        assert apart > 0.25, apart  # it is still what the last row is about
         gpu.say(f"fuvolix far position {layer['type']} {place} {dtype}")
         m = load(tmp_path, c, w, context=200, dtype=dtype)
         for sizes in ([200], [64, 1], [190, 1, 2]):
@@ -219,7 +220,7 @@ SIZES = {
                     vocab=101, groups=5, taps=2, eps=1e-3),
     "one_of_each": X.config([X.latent(heads=1, dim=1, rot_dim=2, vdim=1, kv_rank=1, ff=1), X.mlstm(heads=1, dim=1, vdim=1), X.lightning(heads=1, dim=1, vdim=1, decay=[0.9])],
                             width=32, vocab=40, groups=1, taps=1),
-    "many_heads": X.config([X.latent(heads=33, dim=8, rot_dim=8, vdim=8, kv_rank=72), X.mlstm(heads=19, dim=8, vdim=8), X.lightning(heads=17, dim=8, vdim=8)], width=160),
+    "many_heads": X.config([X.latent(heads=33, dim=8, rot_dim=8, vdim=8, kv_rank=72), X.mlstm(heads=19, dim=8, vdim=8), X.lightning(heads=17, dim=8, vdim=8)], width=160, groups=4),
     "wide_heads": X.config([X.latent(heads=2, dim=128, rot_dim=64, vdim=128, kv_rank=512, ff=512), X.mlstm(heads=2, dim=128, vdim=192), X.lightning(heads=2, dim=256, vdim=136)],
                            width=256, groups=4),
     "wider_heads": X.config([X.latent(heads=2, dim=192, rot_dim=32, vdim=160, kv_rank=600), X.mlstm(heads=1, dim=256, vdim=64), X.lightning(heads=2, dim=64, vdim=256)], width=192),
@@ -244,7 +245,8 @@ def test_other_sizes(tmp_path, name, dtype):
 
 
 def test_gates_and_states_far_from_one(tmp_path):
-    """Gates driven to their cap in both directions, and a state that decays to nothing and starts anew."""
+    """Gates driven to their cap in both directions, and a state that decays to nothing and starts anew. A state of one
+    key only gives o = v sign(k . q): the few rows where k . q is within its rounding of zero are not looked at."""
     c = X.config([X.mlstm(gate_cap=15.0)])
     w = changed(X.weights(c, 8), i=lambda t: t * 12, f=lambda t: t * 12)
     toks = X.tokens(c, 150, 8)
@@ -253,9 +255,9 @@ def test_gates_and_states_far_from_one(tmp_path):
     for dtype in DTYPES:
         m = load(tmp_path, c, w, dtype=dtype)
         for sizes in ([150], [1], [65, 20]):
-            e = X.error(in_portions(m, toks, sizes), want)
+            e = X.error(in_portions(m, toks, sizes), want, quantile=0.95)
             print(dtype, sizes, e)
-            assert e < 3 * TOL[dtype]
+            assert e < TOL[dtype]
 
 
 def test_greedy_generation(mixed):
