@@ -416,6 +416,87 @@ def layer_step_bench(capi, cached=2048, new=33):
     return out
 
 
+FUVOLIX_SIZES = {
+    # width, feed-forward, heads; a head has 128 features of queries, keys and values (latent attention 64 rotated ones besides,
+    # over a latent of 512)
+    "4096": (4096, 14336, 32),
+    "2048": (2048, 8192, 16),
+}
+
+
+def fuvolix_layer(kind, ff, heads):
+    """config.json's entry of a layer that resembles a real model's."""
+    mx = {"latent_attention": dict(heads=heads, dim=128, rot_dim=64, vdim=128, kv_rank=512, scale=192 ** -0.5, rot=dict(base=10000.0, dims=64)),
+          "mlstm": dict(heads=heads, dim=128, vdim=128, gate_cap=15.0),
+          "lightning": dict(heads=heads, dim=128, vdim=128, decay=[float(np.exp(-2.0 ** (-8 * (h + 1) / heads))) for h in range(heads)])}[kind]
+    return dict(type=kind, mixer=mx, mlp=None if ff is None else dict(kind="dense", ff=ff))
+
+
+def build_fuvolix(capi, kinds, size, batch, context, max_tokens, vocab=32768):
+    """A random-init Fuvolix decoder with layers of these kinds, bfloat16."""
+    from mimir_amd import stack
+    width, ff, heads = FUVOLIX_SIZES[size]
+    cfg = dict(width=width, vocab=vocab, canon=dict(taps=4), norm=dict(groups=2, eps=1e-6), layers=[fuvolix_layer(k, ff, heads) for k in kinds])
+    m = stack.Stack(*stack.fuvolix_config(cfg, context, batch))
+    rng = np.random.default_rng(0)
+    pool = rng.standard_normal(1 << 24, np.float32)  # tensors are cut from it, each from another place, and scaled
+    for name, n, k in m.tensors():
+        leaf = name.rsplit(".", 1)[-1]
+        scale, at = (1.0, 1.0) if "norm" in leaf else (k ** -0.5 if n > 1 else 0.5, 0.0)
+        if "norm" in leaf:
+            scale = 0.02
+        start = int(rng.integers(0, pool.size))
+        w = np.take(pool, np.arange(start, start + n * k), mode="wrap") * np.float32(scale) + np.float32(at)
+        m.set_tensor(name, capi.BF16, (w.view(np.uint32) >> 16).astype(np.uint16), n * k)
+    m.finalize(max_tokens)
+    return m
+
+
+def fuvolix_bench(capi, sizes=("4096", "2048"), kinds=("latent_attention", "mlstm", "lightning"), prompts=((1, 2048), (8, 512)), new=65, layers=(2, 6)):
+    """Prompt passes and decoding of the Fuvolix design's three kinds of layer, beside the Llama decoder's (Q4_0) at equal
+    width, feed-forward and heads: microseconds a layer (models of two and of six layers; the difference over four, so
+    that embedding and head drop out), the best of three runs."""
+    out = {}
+    for size in sizes:
+        width, ff, heads = FUVOLIX_SIZES[size]
+        kv_heads = max(1, heads // 4)
+        for kind in kinds + ("llama_q4_0",):
+            for batch, prompt in prompts:
+                secs = {}
+                for n in layers:
+                    if kind == "llama_q4_0":
+                        m = build_llama(capi, layers=n, batch=batch, context=prompt + new, max_tokens=prompt, embed=width, hidden=ff, heads=heads, kv_heads=kv_heads,
+                                        vocab=32768)
+                    else:
+                        m = build_fuvolix(capi, [kind] * n, size, batch, prompt + new, prompt)
+                    toks = np.random.default_rng(0).integers(0, 32768, (batch, prompt))
+                    runs = []
+                    for _ in range(4):
+                        m.reset()
+                        runs.append(m.generate(toks, new)[1])
+                    secs[n] = [min(r[i] for r in runs[1:]) for i in range(2)]
+                    del m
+                span = layers[1] - layers[0]
+                p_us = (secs[layers[1]][0] - secs[layers[0]][0]) / span * 1e6
+                d_us = (secs[layers[1]][1] - secs[layers[0]][1]) / span / (new - 1) * 1e6
+                if kind == "llama_q4_0":
+                    weights = width * (2 * heads + 2 * kv_heads) * 128 + 3 * width * ff
+                    weight_bytes, state = weights * 18 // 32, batch * (prompt + new // 2) * kv_heads * 128 * 4
+                elif kind == "latent_attention":
+                    weights = width * (heads * 192 + 576 + heads * 128) + heads * 256 * 512 + 2 * width * ff
+                    weight_bytes, state = weights * 2, batch * (prompt + new // 2) * 576 * 2
+                else:
+                    weights = width * heads * 128 * 5 + 2 * width * ff
+                    weight_bytes, state = weights * 2, batch * heads * 128 * 128 * 8
+                row = out.setdefault(size, {}).setdefault(kind, {})
+                row[f"prompt_{batch}x{prompt}"] = {"us_per_layer": round(p_us, 1), "TFLOPs_of_products": round(2 * weights * batch * prompt / p_us * 1e-6, 1),
+                                                   "tok_per_s_per_layer": round(batch * prompt / p_us * 1e6)}
+                row[f"decode_{batch}"] = {"us_per_layer": round(d_us, 2), "bytes_per_layer": weight_bytes + state,
+                                          "frac_of_hbm": round((weight_bytes + state) / (d_us * 1e-6) / 1e9 / HBM_PEAK_GBS, 4)}
+                print(f"bench.py: {size} {kind} batch {batch}: {row}", file=sys.stderr, flush=True)
+    return out
+
+
 def bench_blocks_kquant(rng, dtype_bytes, n_elems):
     """Random Q4_K (144-byte) or Q6_K (210-byte) super-blocks: every field uniform, the binary16 scales |N(0, 0.02)|."""
     raw = rng.integers(0, 256, size=(n_elems // 256, dtype_bytes), dtype=np.uint8)
@@ -669,6 +750,8 @@ def main():
     ap.add_argument("--decode-batch", type=int, default=1)
     ap.add_argument("--decode-linear", choices=("q4_0", "q4_K", "q6_K"), default="q4_0",
                     help="block dtype of the decoder's linear weights (the oracle check is for q4_0)")
+    ap.add_argument("--fuvolix", action="store_true", help="only: prompt passes and decoding of the Fuvolix design's layers at sizes like a real model's, beside the Llama decoder's")
+    ap.add_argument("--fuvolix-only", default=None, metavar="SIZE[:KIND[:BATCHxPROMPT]]", help="with --fuvolix: one size, kind of layer, call (for profiles)")
     ap.add_argument("--tune", action="append", default=[], metavar="KEY=VALUE",
                     help="a launch-plan override for mi355x_tune before anything runs (may be repeated), e.g. q4_0.stream=1")
     args = ap.parse_args()
@@ -685,6 +768,17 @@ def main():
         key, _, val = kv.partition("=")
         capi.check(lib.mi355x_tune(key.encode(), int(val)))
 
+    if args.fuvolix:
+        kw = {}
+        if args.fuvolix_only:
+            parts = args.fuvolix_only.split(":")
+            kw["sizes"] = (parts[0],)
+            if len(parts) > 1:
+                kw["kinds"] = tuple(k for k in parts[1].split(",") if k)
+            if len(parts) > 2:
+                kw["prompts"] = (tuple(int(v) for v in parts[2].split("x")),)
+        print(json.dumps({"fuvolix": fuvolix_bench(capi, **kw)}))
+        return
     if args.rows_counters:
         rows_bench(lib, capi, torch, shapes=((14336, 4096),), only=args.rows_counters)
         per_weight = {"q4_K": 144 / 256, "q6_K": 210 / 256}.get(args.rows_counters[:4], 18 / 32)

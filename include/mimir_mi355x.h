@@ -365,6 +365,10 @@ typedef struct mi355x_stack_config {
 } mi355x_stack_config;
 
 MI355X_API mi355x_status mi355x_stack_create(const mi355x_stack_config* cfg, const mi355x_stack_layer* layers, void** model);
+/* Tensor i that the model takes, in the order of their names: the name (cut to
+ * size - 1 characters), rows and columns (a vector: one row). MI355X_ERR_INDEX
+ * behind the last one. */
+MI355X_API mi355x_status mi355x_stack_tensor(void* model, int64_t i, char* name, size_t size, int64_t* rows, int64_t* cols);
 
 /* ---- the reference's operator interface for this path ---------------------------
  * backend.Backend and backend.Batcher (backend/backend.go:141-171,

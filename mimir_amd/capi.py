@@ -58,6 +58,7 @@ SYMBOLS = {
     "mi355x_model_logits_at": (C.c_uint32, [_vp, _vp, _i64, _vp, _i64, _vp]),
     "mi355x_model_generate": (C.c_uint32, [_vp, _vp, _i64, _i64, _vp, _vp]),
     "mi355x_stack_create": (C.c_uint32, [_vp, _vp, C.POINTER(_vp)]),
+    "mi355x_stack_tensor": (C.c_uint32, [_vp, _i64, _vp, _sz, _vp, _vp]),
     "mi355x_llama_create": (C.c_uint32, [_vp, C.POINTER(_vp)]),
     "mi355x_llama_destroy": (C.c_uint32, [_vp]),
     "mi355x_llama_set_tensor": (C.c_uint32, [_vp, C.c_char_p, _int, _vp, _i64]),

@@ -10,7 +10,9 @@
 // float32 activations; longer passes of a bfloat16 model round the products' inputs to bfloat16. The residual, norms,
 // recurrent states, gates, scores and softmax weights are float32 either way.
 #include <cmath>
+#include <cstdio>
 #include <cstring>
+#include <iterator>
 #include <map>
 #include <memory>
 #include <string>
@@ -534,6 +536,19 @@ mi355x_status mi355x_stack_create(const mi355x_stack_config* cfg, const mi355x_s
     }
     m->name_tensors();
     *out = (Decoder*)m.release();
+    return MI355X_OK;
+}
+
+mi355x_status mi355x_stack_tensor(void* model, int64_t i, char* name, size_t size, int64_t* rows, int64_t* cols) {
+    using namespace mimir;
+    if (!model || !name || size == 0 || !rows || !cols) return capi_fail(MI355X_ERR_INTERNAL, "mi355x: stack_tensor: null pointer");
+    const auto& slots = ((Stack*)(Decoder*)model)->slots;
+    if (i < 0 || i >= (int64_t)slots.size()) return capi_fail(MI355X_ERR_INDEX, "mi355x: stack_tensor: tensor %lld of %zu", (long long)i, slots.size());
+    auto it = slots.begin();
+    std::advance(it, i);
+    snprintf(name, size, "%s", it->first.c_str());
+    *rows = it->second.rows;
+    *cols = it->second.cols;
     return MI355X_OK;
 }
 

@@ -27,6 +27,15 @@ class Stack(Decoder):
         self._h = C.c_void_p()
         capi.check(self.lib.mi355x_stack_create(C.byref(config), self._layers, C.byref(self._h)))
 
+    def tensors(self):
+        """(name, rows, columns) of every tensor that the model takes (vectors: one row)."""
+        out, i = [], 0
+        name, n, k = C.create_string_buffer(64), C.c_int64(), C.c_int64()
+        while self.lib.mi355x_stack_tensor(self._h, i, name, 64, C.byref(n), C.byref(k)) == capi.OK:
+            out.append((name.value.decode(), n.value, k.value))
+            i += 1
+        return out
+
 
 def _latent_layer(mx: dict) -> dict:
     rot = mx["rot"]
