@@ -3,8 +3,10 @@
 //
 // latent_absorbed serves few query rows (a decoding step, a short portion) and everything in float32 without forming
 // keys or values: q_h . (W_uk,h c_j) = (W_uk,h^T q_h) . c_j, so a head's query goes to the latents' space once
-// (latent_absorb_kernel) and all heads read the same cache rows; the weighted sum of the latents comes back through W_uv,h
-// (latent_combine_kernel). The keys of a row are cut into shares that workgroups take side by side.
+// (latent_queries_kernel, which also turns the rotated parts and writes the new cache rows) and all heads read the same
+// cache rows; the weighted sum of the latents comes back through W_uv,h (latent_combine_kernel). The keys of a row are cut
+// into shares that workgroups take side by side, on the vector units (latent_attend_kernel, any sizes, float32 or
+// bfloat16 cache) or, for a bfloat16 cache, on the matrix cores (latent_attend_mfma_kernel).
 #include "device_util.h"
 #include "stack_ops.h"
 
@@ -21,14 +23,9 @@ __device__ __forceinline__ float block_sum_256(float v, float* part) {
 
 __device__ __forceinline__ int64_t past_of(const Latent& a) { return a.past + (a.past_dev ? *a.past_dev : 0); }
 
-// One workgroup a row: the latent's norm and the rotations.
-__global__ __launch_bounds__(256) void latent_prepare_kernel(Latent a, float* __restrict__ proj, int64_t ldp, uint16_t* __restrict__ q16, int64_t ldq) {
+// A row's cache entry: the latent over its root mean square times the norm's weight, and the turned key part. 256 threads.
+__device__ __forceinline__ void write_cache_row(const Latent& a, const float* low, int64_t b, int64_t pos, const float* cs, const float* sn) {
     __shared__ float part[4];
-    const int64_t r = blockIdx.x, b = r / a.s, pos = past_of(a) + r % a.s;
-    const int D = a.dim + a.rot_dim, half = a.rot_dim / 2;
-    float* p = proj + r * ldp;
-    const float* low = p + (int64_t)a.heads * D;
-    const float *cs = a.cos_t + pos * half, *sn = a.sin_t + pos * half;
     float ss = 0.f;
     for (int i = threadIdx.x; i < a.rank; i += 256) ss = fmaf(low[i], low[i], ss);
     ss = block_sum_256(ss, part);
@@ -38,44 +35,57 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(Latent a, float* __
     uint16_t* c16 = a.cache_bf16 ? (uint16_t*)a.cache + at : nullptr;
     auto keep = [&](int i, float v) {
         if (c32) c32[i] = v;
-        else c16[i] = f32_to_bf16_bits(v);
+        else c16[i] = round_bf16(v);
     };
     for (int i = threadIdx.x; i < a.rank; i += 256) keep(i, low[i] * scale * a.norm_w[i]);
-    for (int i = threadIdx.x; i < half; i += 256) {
+    for (int i = threadIdx.x; i < a.rot_dim / 2; i += 256) {
         const float u = low[a.rank + 2 * i], v = low[a.rank + 2 * i + 1];
         keep(a.rank + 2 * i, u * cs[i] - v * sn[i]);
         keep(a.rank + 2 * i + 1, v * cs[i] + u * sn[i]);
     }
+}
+
+// For formed keys, one workgroup a row: the cache row, and the queries turned and rounded.
+__global__ __launch_bounds__(256) void latent_prepare_kernel(Latent a, const float* __restrict__ proj, int64_t ldp, uint16_t* __restrict__ q16, int64_t ldq) {
+    const int64_t r = blockIdx.x, b = r / a.s, pos = past_of(a) + r % a.s;
+    const int D = a.dim + a.rot_dim, half = a.rot_dim / 2;
+    const float* p = proj + r * ldp;
+    const float *cs = a.cos_t + pos * half, *sn = a.sin_t + pos * half;
+    write_cache_row(a, p + (int64_t)a.heads * D, b, pos, cs, sn);
     for (int i = threadIdx.x; i < a.heads * half; i += 256) {
         const int h = i / half, j = i % half;
         const int64_t o = (int64_t)h * D + a.dim + 2 * j;
         const float u = p[o], v = p[o + 1];
-        const float x = u * cs[j] - v * sn[j], y = v * cs[j] + u * sn[j];
-        if (q16) {
-            q16[r * ldq + o] = f32_to_bf16_bits(x);
-            q16[r * ldq + o + 1] = f32_to_bf16_bits(y);
-        } else {
-            p[o] = x;
-            p[o + 1] = y;
-        }
+        q16[r * ldq + o] = round_bf16(u * cs[j] - v * sn[j]);
+        q16[r * ldq + o + 1] = round_bf16(v * cs[j] + u * sn[j]);
     }
-    if (q16)
-        for (int i = threadIdx.x; i < a.heads * a.dim; i += 256) {
-            const int64_t o = (int64_t)(i / a.dim) * D + i % a.dim;
-            q16[r * ldq + o] = f32_to_bf16_bits(p[o]);
-        }
+    for (int i = threadIdx.x; i < a.heads * a.dim; i += 256) {
+        const int64_t o = (int64_t)(i / a.dim) * D + i % a.dim;
+        q16[r * ldq + o] = round_bf16(p[o]);
+    }
 }
 
-// q'[row, h, :] = W_uk,h^T q_h: 256 columns a workgroup, eight a thread, the head's rows of W_uk shared by eight groups.
-__global__ __launch_bounds__(256) void latent_absorb_kernel(Latent a, const float* __restrict__ proj, int64_t ldp, float* __restrict__ qa) {
-    __shared__ float red[8][256 + 8];
-    const int64_t r = blockIdx.x;
-    const int h = blockIdx.y, c0 = blockIdx.z * 256 + (threadIdx.x & 31) * 8, g = threadIdx.x >> 5;
-    const float* q = proj + r * ldp + (int64_t)h * (a.dim + a.rot_dim);
+constexpr int kAbsorbCols = 128;  // latent features a workgroup
+
+__device__ __forceinline__ int query_ld(const Latent& a) { return (a.rank + a.rot_dim + 31) / 32 * 32; }
+
+// Without formed keys: qa[row, h, :] = (W_uk,h^T q_h | the turned part) * scale, zeros up to query_ld. Workgroups (row, h, z):
+// 128 latent features each, eight a thread, the head's rows of W_uk shared by sixteen groups; those of head 0's first
+// piece also write the row's cache entry.
+__global__ __launch_bounds__(256) void latent_queries_kernel(Latent a, const float* __restrict__ proj, int64_t ldp, float* __restrict__ qa) {
+    __shared__ float red[16][kAbsorbCols + 4];
+    const int64_t r = blockIdx.x, pos = past_of(a) + r % a.s;
+    const int h = blockIdx.y, half = a.rot_dim / 2, D = a.dim + a.rot_dim, lq = query_ld(a);
+    const int c0 = blockIdx.z * kAbsorbCols + (threadIdx.x & 15) * 8, g = threadIdx.x >> 4;
+    const float *cs = a.cos_t + pos * half, *sn = a.sin_t + pos * half;
+    const float* q = proj + r * ldp + (int64_t)h * D;
+    float* to = qa + (r * a.heads + h) * lq;
     float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    if (c0 < a.rank)
-        for (int d = g; d < a.dim; d += 8) {
-            const u32x4 w = *(const u32x4*)(a.w_uk + ((int64_t)h * a.dim + d) * a.ldw + c0);  // rows are padded with zeros
+    if (c0 < a.rank) {
+        const uint16_t* w0 = a.w_uk + (int64_t)h * a.dim * a.ldw + c0;  // rows are padded with zeros
+#pragma unroll 4
+        for (int d = g; d < a.dim; d += 16) {
+            const u32x4 w = *(const u32x4*)(w0 + (int64_t)d * a.ldw);
             const float x = q[d];
 #pragma unroll
             for (int i = 0; i < 4; i++) {
@@ -83,15 +93,26 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(Latent a, const floa
                 acc[2 * i + 1] = fmaf(x, __uint_as_float(w[i] & 0xffff0000u), acc[2 * i + 1]);
             }
         }
+    }
 #pragma unroll
-    for (int i = 0; i < 8; i++) red[g][(threadIdx.x & 31) * 8 + i] = acc[i];
+    for (int i = 0; i < 8; i++) red[g][(threadIdx.x & 15) * 8 + i] = acc[i];
     __syncthreads();
-    const int c = blockIdx.z * 256 + threadIdx.x;
-    if (c >= a.rank) return;
-    float v = 0.f;
+    const int c = blockIdx.z * kAbsorbCols + threadIdx.x;
+    if (threadIdx.x < kAbsorbCols && c < a.rank) {
+        float v = 0.f;
 #pragma unroll
-    for (int i = 0; i < 8; i++) v += red[i][threadIdx.x];
-    qa[(r * a.heads + h) * a.rank + c] = v;
+        for (int i = 0; i < 16; i++) v += red[i][threadIdx.x];
+        to[c] = v * a.scale;
+    }
+    if (blockIdx.z == 0) {
+        for (int i = threadIdx.x; i < half; i += 256) {
+            const float u = q[a.dim + 2 * i], v = q[a.dim + 2 * i + 1];
+            to[a.rank + 2 * i] = (u * cs[i] - v * sn[i]) * a.scale;
+            to[a.rank + 2 * i + 1] = (v * cs[i] + u * sn[i]) * a.scale;
+        }
+        for (int i = a.rank + a.rot_dim + threadIdx.x; i < lq; i += 256) to[i] = 0.f;
+        if (h == 0) write_cache_row(a, proj + r * ldp + (int64_t)a.heads * D, r / a.s, pos, cs, sn);  // the whole workgroup
+    }
 }
 
 constexpr int kHeads = 16;  // heads a workgroup
@@ -115,12 +136,18 @@ __device__ __forceinline__ void load8<uint16_t>(const uint16_t* p, float v[8]) {
 __device__ __forceinline__ float widen1(float v) { return v; }
 __device__ __forceinline__ float widen1(uint16_t v) { return bf16_bits_to_f32(v); }
 
+// How many of a row's keys a share has: whole tiles.
+__device__ __forceinline__ int64_t share_of(int64_t seen, int splits) {
+    const int64_t share = (seen + splits - 1) / splits;
+    return (share + kKeys - 1) / kKeys * kKeys;
+}
+
 // The share `split` of the keys of one row, for kHeads heads: scores with a lane's key against four heads a
 // wavefront, a running softmax, and the weighted sum of the latents with a thread's columns tid + 256 u.
 // parts: [rows, splits, heads, rank] sums, then [rows, splits, heads, 2] (maximum, sum of weights).
 template <typename T, int U>
-__global__ __launch_bounds__(256) void latent_attend_kernel(Latent a, const float* __restrict__ proj, int64_t ldp, const float* __restrict__ qa, int splits,
-                                                            float* __restrict__ part_o, float* __restrict__ part_ml) {
+__global__ __launch_bounds__(256) void latent_attend_kernel(Latent a, const float* __restrict__ qa, int splits, float* __restrict__ part_o,
+                                                            float* __restrict__ part_ml) {
     extern __shared__ __align__(16) float lds_latent[];
     const int L8 = (a.rank + a.rot_dim + 7) / 8 * 8;
     float* qs = lds_latent;                    // [L8][kHeads]
@@ -130,25 +157,13 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(Latent a, const floa
     const int split = blockIdx.x, h0 = blockIdx.y * kHeads;
     const int64_t r = blockIdx.z, b = r / a.s;
     const int64_t seen = past_of(a) + r % a.s + 1;
-    int64_t share = (seen + splits - 1) / splits;
-    share = (share + kKeys - 1) / kKeys * kKeys;
+    const int64_t share = share_of(seen, splits);
     const int64_t lo = split * share, hi = lo + share < seen ? lo + share : seen;
     const int64_t pr = (r * splits + split) * a.heads;
-    if (lo >= hi) {  // the whole workgroup: nothing to add
-        if (tid < kHeads && h0 + tid < a.heads) {
-            part_ml[(pr + h0 + tid) * 2] = -__builtin_inff();
-            part_ml[(pr + h0 + tid) * 2 + 1] = 0.f;
-        }
-        return;
-    }
+    if (lo >= hi) return;  // the whole workgroup: latent_combine_kernel does not look at this share
     for (int i = tid; i < L8 * kHeads; i += 256) {
         const int d = i / kHeads, h = h0 + i % kHeads;
-        float v = 0.f;
-        if (h < a.heads) {
-            if (d < a.rank) v = qa[(r * a.heads + h) * a.rank + d];
-            else if (d < a.rank + a.rot_dim) v = proj[r * ldp + (int64_t)h * (a.dim + a.rot_dim) + a.dim + d - a.rank];
-        }
-        qs[i] = v * a.scale;
+        qs[i] = h < a.heads ? qa[(r * a.heads + h) * query_ld(a) + d] : 0.f;
     }
     const T* cache = (const T*)a.cache + b * a.context * a.ldc;
     float acc[kHeads][U];
@@ -243,66 +258,273 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(Latent a, const floa
     }
 }
 
-constexpr int kValues = 32;  // values a workgroup of latent_combine_kernel
+// The same on the matrix cores, a bfloat16 cache: tiles of 64 keys in LDS, 32 heads a workgroup. Scores: the wavefronts cut the
+// features into four (KS steps of 32 each at most), queries as the sum of two bfloat16 in registers, and the four partial
+// sums meet in LDS, where eight threads a head do the softmax. Sum of latents: the wavefronts cut the latent's features
+// (RT tiles of sixteen each at most), weights as the sum of two bfloat16.
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+
+__device__ __forceinline__ f32x4 mfma16_bf16(u32x4 a, u32x4 b, f32x4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+}
+
+constexpr int kMHeads = 32;
+constexpr int kScoreLd = kMHeads + 1, kWeightLd = kKeys + 8;
+
+size_t attend_mfma_lds(const Latent& a) {
+    const int lq = (a.rank + a.rot_dim + 31) / 32 * 32;
+    return (size_t)kKeys * (lq + 8) * 2 + (size_t)4 * kKeys * kScoreLd * 4 + (size_t)2 * kMHeads * kWeightLd * 2 + kMHeads * 4;
+}
+
+template <int KS, int RT>
+__global__ __launch_bounds__(256) void latent_attend_mfma_kernel(Latent a, const float* __restrict__ qa, int splits, float* __restrict__ part_o,
+                                                                 float* __restrict__ part_ml) {
+    extern __shared__ __align__(16) float lds_latent[];
+    const int lq = query_ld(a), ldt = lq + 8, steps = lq / 32, L = a.rank + a.rot_dim;
+    float* ps = lds_latent;                                    // [4][kKeys][kScoreLd]
+    float* back = ps + 4 * kKeys * kScoreLd;                   // [kMHeads]
+    uint16_t* tile = (uint16_t*)(back + kMHeads);              // [kKeys][ldt]
+    uint16_t* wH = tile + (size_t)kKeys * ldt;                 // [kMHeads][kWeightLd], high parts
+    uint16_t* wL = wH + kMHeads * kWeightLd;                   // low parts
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
+    const int split = blockIdx.x, h0 = blockIdx.y * kMHeads;
+    const int64_t r = blockIdx.z, b = r / a.s;
+    const int64_t seen = past_of(a) + r % a.s + 1, share = share_of(seen, splits);
+    const int64_t lo = split * share, hi = lo + share < seen ? lo + share : seen;
+    const int64_t pr = (r * splits + split) * a.heads;
+    if (lo >= hi) return;  // the whole workgroup: latent_combine_kernel does not look at this share
+    const uint16_t* cache = (const uint16_t*)a.cache + b * a.context * a.ldc;
+    // this wavefront's steps of the features: wave, wave + 4, ...
+    u32x4 qh[KS][2], ql[KS][2];
+#pragma unroll
+    for (int i = 0; i < KS; i++)
+#pragma unroll
+        for (int t = 0; t < 2; t++) {
+            const int h = h0 + t * 16 + r16, step = wave + 4 * i;
+            f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = x;
+            if (h < a.heads && step < steps) {
+                const f32x4* q = (const f32x4*)(qa + (r * a.heads + h) * lq + step * 32 + g * 8);
+                x = q[0];
+                y = q[1];
+            }
+            qh[i][t] = u32x4{pack_bf16(x[0], x[1]), pack_bf16(x[2], x[3]), pack_bf16(y[0], y[1]), pack_bf16(y[2], y[3])};
+            ql[i][t] = u32x4{pack_bf16(low_part(x[0]), low_part(x[1])), pack_bf16(low_part(x[2]), low_part(x[3])), pack_bf16(low_part(y[0]), low_part(y[1])),
+                             pack_bf16(low_part(y[2]), low_part(y[3]))};
+        }
+    f32x4 acc[RT][2];
+#pragma unroll
+    for (int t = 0; t < RT; t++)
+#pragma unroll
+        for (int i = 0; i < 2; i++) acc[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int sh = tid >> 3, sk = tid & 7;  // the softmax's head and first key of this thread
+    float m = -__builtin_inff(), l = 0.f;
+    const int pieces = lq / 8;
+    for (int64_t j0 = lo; j0 < hi; j0 += kKeys) {
+        for (int i = tid; i < kKeys * pieces; i += 256) {
+            const int j = i / pieces, d = i % pieces * 8;
+            const int64_t row = j0 + j < hi ? j0 + j : hi - 1;
+            u32x4 v = {0, 0, 0, 0};
+            if (d < L) v = *(const u32x4*)(cache + row * a.ldc + d);  // a row is padded with zeros to a multiple of 8
+            *(u32x4*)(tile + j * ldt + d) = v;
+        }
+        __syncthreads();
+        f32x4 sc[4][2];
+#pragma unroll
+        for (int k = 0; k < 4; k++)
+#pragma unroll
+            for (int t = 0; t < 2; t++) sc[k][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i = 0; i < KS; i++) {
+            const int step = wave + 4 * i;
+            if (step >= steps) break;
+#pragma unroll
+            for (int k = 0; k < 4; k++) {
+                const u32x4 c = *(const u32x4*)(tile + (k * 16 + r16) * ldt + step * 32 + g * 8);
+#pragma unroll
+                for (int t = 0; t < 2; t++) {
+                    sc[k][t] = mfma16_bf16(c, qh[i][t], sc[k][t]);
+                    sc[k][t] = mfma16_bf16(c, ql[i][t], sc[k][t]);
+                }
+            }
+        }
+#pragma unroll
+        for (int k = 0; k < 4; k++)
+#pragma unroll
+            for (int t = 0; t < 2; t++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) ps[(wave * kKeys + k * 16 + 4 * g + i) * kScoreLd + t * 16 + r16] = sc[k][t][i];
+        __syncthreads();
+        {
+            float s[8], top = -__builtin_inff();
+#pragma unroll
+            for (int i = 0; i < 8; i++) {
+                const int j = sk * 8 + i;
+                float v = 0.f;
+#pragma unroll
+                for (int w = 0; w < 4; w++) v += ps[(w * kKeys + j) * kScoreLd + sh];
+                s[i] = j0 + j < hi ? v : -__builtin_inff();
+                top = fmaxf(top, s[i]);
+            }
+            top = group8_max(top);
+            const float next = fmaxf(m, top), scale = expf(m - next);  // the first tile's m: exp(-inf) = 0
+            float sum = 0.f;
+#pragma unroll
+            for (int i = 0; i < 8; i++) {
+                s[i] = expf(s[i] - next);
+                sum += s[i];
+            }
+            *(u32x4*)(wH + sh * kWeightLd + sk * 8) = u32x4{pack_bf16(s[0], s[1]), pack_bf16(s[2], s[3]), pack_bf16(s[4], s[5]), pack_bf16(s[6], s[7])};
+            *(u32x4*)(wL + sh * kWeightLd + sk * 8) = u32x4{pack_bf16(low_part(s[0]), low_part(s[1])), pack_bf16(low_part(s[2]), low_part(s[3])),
+                                                            pack_bf16(low_part(s[4]), low_part(s[5])), pack_bf16(low_part(s[6]), low_part(s[7]))};
+            l = l * scale + group8_sum(sum);
+            m = next;
+            if (sk == 0) back[sh] = scale;
+        }
+        __syncthreads();
+        if (j0 > lo)
+#pragma unroll
+            for (int t = 0; t < 2; t++) {
+                const f32x4 f = *(const f32x4*)(back + t * 16 + 4 * g);
+#pragma unroll
+                for (int k = 0; k < RT; k++) acc[k][t] = acc[k][t] * f;
+            }
+#pragma unroll
+        for (int half = 0; half < 2; half++) {
+            u32x4 pw[2][2];
+#pragma unroll
+            for (int t = 0; t < 2; t++) {
+                pw[t][0] = *(const u32x4*)(wH + (t * 16 + r16) * kWeightLd + half * 32 + g * 8);
+                pw[t][1] = *(const u32x4*)(wL + (t * 16 + r16) * kWeightLd + half * 32 + g * 8);
+            }
+#pragma unroll
+            for (int k = 0; k < RT; k++) {
+                const int c0 = (wave + 4 * k) * 16;
+                if (c0 >= a.rank) break;
+                // eight keys of one feature: a column of the tile (features past the rank are the rotated part or zeros: not stored)
+                const uint16_t* col = tile + (half * 32 + g * 8) * ldt + c0 + r16;
+                u32x4 v;
+#pragma unroll
+                for (int i = 0; i < 4; i++) v[i] = (uint32_t)col[2 * i * ldt] | (uint32_t)col[(2 * i + 1) * ldt] << 16;
+#pragma unroll
+                for (int t = 0; t < 2; t++) {
+                    acc[k][t] = mfma16_bf16(pw[t][0], v, acc[k][t]);
+                    acc[k][t] = mfma16_bf16(pw[t][1], v, acc[k][t]);
+                }
+            }
+        }
+        __syncthreads();
+    }
+#pragma unroll
+    for (int k = 0; k < RT; k++) {
+        const int c = (wave + 4 * k) * 16 + r16;
+#pragma unroll
+        for (int t = 0; t < 2; t++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const int h = h0 + t * 16 + 4 * g + i;
+                if (c < a.rank && h < a.heads) part_o[(pr + h) * a.rank + c] = acc[k][t][i];
+            }
+    }
+    if (sk == 0 && h0 + sh < a.heads) {
+        part_ml[(pr + h0 + sh) * 2] = m;
+        part_ml[(pr + h0 + sh) * 2 + 1] = l;
+    }
+}
+
+constexpr int kValues = 64;      // values a workgroup of latent_combine_kernel
+constexpr int kMaxSplits = 512;
 
 // The shares of a head brought together, then its values: out[row, h, e] = W_uv[h, e, :] . (sum of latents).
 __global__ __launch_bounds__(256) void latent_combine_kernel(Latent a, int splits, const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                                              float* __restrict__ out_f32, uint16_t* __restrict__ out_bf16, int64_t ldo) {
     extern __shared__ __align__(16) float lds_latent[];
+    __shared__ float weight[kMaxSplits];
     float* oc = lds_latent;  // [rank to a multiple of 64]
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.y;
     const int64_t r = blockIdx.x;
     const int R64 = (a.rank + 63) / 64 * 64;
+    const int64_t seen = past_of(a) + r % a.s + 1, share = share_of(seen, splits);
+    const int live = (int)((seen + share - 1) / share);  // shares that have keys
     const float* mlp = part_ml + (r * splits * a.heads + h) * 2;
     const int64_t step = (int64_t)a.heads * 2;
-    float top = -__builtin_inff();
-    for (int s = lane; s < splits; s += 64) top = fmaxf(top, mlp[s * step]);
-    top = wave_max(top);
-    float sum = 0.f;
-    for (int s = lane; s < splits; s += 64) sum = fmaf(mlp[s * step + 1], expf(mlp[s * step] - top), sum);
-    const float inv = 1.f / wave_sum(sum);
-    for (int c = tid; c < R64; c += 256) {
-        float v = 0.f;
-        if (c < a.rank)
-            for (int s = 0; s < splits; s++) {
-                const float m = mlp[s * step];
-                if (m == -__builtin_inff()) continue;  // a share without keys wrote no sums
-                v = fmaf(part_o[((r * splits + s) * a.heads + h) * a.rank + c], expf(m - top), v);
-            }
-        oc[c] = v * inv;
+    if (wave == 0) {
+        float top = -__builtin_inff();
+        for (int s = lane; s < live; s += 64) top = fmaxf(top, mlp[s * step]);
+        top = wave_max(top);
+        float sum = 0.f;
+        for (int s = lane; s < live; s += 64) {
+            const float w = expf(mlp[s * step] - top);
+            weight[s] = w;
+            sum = fmaf(mlp[s * step + 1], w, sum);
+        }
+        const float inv = 1.f / wave_sum(sum);
+        for (int s = lane; s < live; s += 64) weight[s] *= inv;
     }
     __syncthreads();
-    const int e1 = (int)(blockIdx.z + 1) * kValues < a.vdim ? (int)(blockIdx.z + 1) * kValues : a.vdim;
-    for (int e = blockIdx.z * kValues + wave; e < e1; e += 4) {
-        const uint16_t* w = a.w_uv + ((int64_t)h * a.vdim + e) * a.ldw;
+    const float* po = part_o + (r * splits * a.heads + h) * a.rank;
+    const int64_t ostep = (int64_t)a.heads * a.rank;
+    for (int c = tid; c < R64; c += 256) {
         float v = 0.f;
-        for (int c = lane * 8; c < R64; c += 512) {
-            const u32x4 x = *(const u32x4*)(w + c);
-#pragma unroll
-            for (int i = 0; i < 4; i++) {
-                v = fmaf(oc[c + 2 * i], __uint_as_float(x[i] << 16), v);
-                v = fmaf(oc[c + 2 * i + 1], __uint_as_float(x[i] & 0xffff0000u), v);
-            }
+        if (c < a.rank) {
+#pragma unroll 8
+            for (int s = 0; s < live; s++) v = fmaf(po[s * ostep + c], weight[s], v);
         }
-        v = wave_sum(v);
-        if (lane == 0) {
-            const int64_t at = r * ldo + (int64_t)h * a.vdim + e;
-            if (out_f32) out_f32[at] = v;
-            else out_bf16[at] = f32_to_bf16_bits(v);
+        oc[c] = v;
+    }
+    __syncthreads();
+    const int e0 = blockIdx.z * kValues, e1 = e0 + kValues < a.vdim ? e0 + kValues : a.vdim;
+    const uint16_t* w0 = a.w_uv + (int64_t)h * a.vdim * a.ldw;
+    for (int e = e0 + wave * 4; e < e1; e += 16) {  // four values a wavefront at a time
+        float v[4] = {0.f, 0.f, 0.f, 0.f};
+        for (int c = lane * 8; c < R64; c += 512) {
+            u32x4 x[4];
+#pragma unroll
+            for (int u = 0; u < 4; u++) x[u] = *(const u32x4*)(w0 + (int64_t)(e + u < e1 ? e + u : e1 - 1) * a.ldw + c);
+#pragma unroll
+            for (int u = 0; u < 4; u++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    v[u] = fmaf(oc[c + 2 * i], __uint_as_float(x[u][i] << 16), v[u]);
+                    v[u] = fmaf(oc[c + 2 * i + 1], __uint_as_float(x[u][i] & 0xffff0000u), v[u]);
+                }
+        }
+#pragma unroll
+        for (int u = 0; u < 4; u++) {
+            const float sum = wave_sum(v[u]);
+            if (lane == 0 && e + u < e1) {
+                const int64_t at = r * ldo + (int64_t)h * a.vdim + e + u;
+                if (out_f32) out_f32[at] = sum;
+                else out_bf16[at] = round_bf16(sum);
+            }
         }
     }
 }
 
 template <typename T, int U>
-hipError_t launch_attend(const Latent& a, const float* proj, int64_t ldp, const float* qa, int splits, float* po, float* ml, hipStream_t st) {
+hipError_t launch_attend(const Latent& a, const float* qa, int splits, float* po, float* ml, hipStream_t st) {
     const size_t lds = ((size_t)(a.rank + a.rot_dim + 7) / 8 * 8 * kHeads + kKeys * kHeads + kHeads) * 4;
     if (lds > 64 * 1024) {
         hipError_t e = hipFuncSetAttribute((const void*)latent_attend_kernel<T, U>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
     }
     const dim3 grid((unsigned)splits, (unsigned)((a.heads + kHeads - 1) / kHeads), (unsigned)(a.batch * a.s));
-    hipLaunchKernelGGL((latent_attend_kernel<T, U>), grid, dim3(256), lds, st, a, proj, ldp, qa, splits, po, ml);
+    hipLaunchKernelGGL((latent_attend_kernel<T, U>), grid, dim3(256), lds, st, a, qa, splits, po, ml);
     return hipGetLastError();
+}
+
+template <int KS, int RT>
+hipError_t launch_attend_mfma(const Latent& a, const float* qa, int splits, float* po, float* ml, hipStream_t st) {
+    const size_t lds = attend_mfma_lds(a);
+    hipError_t e = hipFuncSetAttribute((const void*)latent_attend_mfma_kernel<KS, RT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return e;
+    const dim3 grid((unsigned)splits, (unsigned)((a.heads + kMHeads - 1) / kMHeads), (unsigned)(a.batch * a.s));
+    hipLaunchKernelGGL((latent_attend_mfma_kernel<KS, RT>), grid, dim3(256), lds, st, a, qa, splits, po, ml);
+    return hipGetLastError();
+}
+
+bool attend_mfma_ok(const Latent& a) {
+    return a.cache_bf16 && a.rank <= 512 && a.rank + a.rot_dim <= 640 && a.ldc % 8 == 0 && attend_mfma_lds(a) <= 160 * 1024;
 }
 
 // ---- many query rows ------------------------------------------------------------------------
@@ -312,14 +534,9 @@ hipError_t launch_attend(const Latent& a, const float* proj, int64_t ldp, const 
 // operand: the order in which the scores' registers hold the keys is the order in which V^T's fragment is read. Four
 // wavefronts with consecutive rows share a tile of keys and values in LDS; the next tile is requested while one is used.
 
-typedef float f32x16 __attribute__((ext_vector_type(16)));
-typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
-
 __device__ __forceinline__ f32x16 mfma_bf16(u32x4 a, u32x4 b, f32x16 c) {
     return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
 }
-__device__ __forceinline__ uint32_t pack2(float lo, float hi) { return (uint32_t)f32_to_bf16_bits(lo) | (uint32_t)f32_to_bf16_bits(hi) << 16; }
-__device__ __forceinline__ float low_part(float v) { return v - bf16_bits_to_f32(f32_to_bf16_bits(v)); }
 
 struct PromptArgs {
     const uint16_t *q, *keys, *vt, *cache;  // cache: the sequence's rows
@@ -453,8 +670,8 @@ __global__ __launch_bounds__(256, DT > 12 ? 1 : 2) void latent_prompt_kernel(Pro
                 for (int i = 0; i < 4; i++) {
                     const float x = __builtin_amdgcn_exp2f(sc[b][half * 8 + 2 * i] - m), y = __builtin_amdgcn_exp2f(sc[b][half * 8 + 2 * i + 1] - m);
                     l += x + y;
-                    high[i] = pack2(x, y);
-                    low[i] = pack2(low_part(x), low_part(y));
+                    high[i] = pack_bf16(x, y);
+                    low[i] = pack_bf16(low_part(x), low_part(y));
                 }
 #pragma unroll
                 for (int t = 0; t < VT; t++) {
@@ -476,7 +693,7 @@ __global__ __launch_bounds__(256, DT > 12 ? 1 : 2) void latent_prompt_kernel(Pro
 #pragma unroll
             for (int i = 0; i < 4; i++) {
                 const int e = t * 32 + 8 * g + 4 * hi + i;
-                if (e < p.vdim) out[e] = f32_to_bf16_bits(o[t][4 * g + i] * inv);
+                if (e < p.vdim) out[e] = round_bf16(o[t][4 * g + i] * inv);
             }
 }
 
@@ -491,7 +708,7 @@ void launch_prompt(const PromptArgs& p, hipStream_t st) {
 
 }  // namespace
 
-hipError_t latent_prepare(const Latent& a, float* proj, int64_t ldp, uint16_t* q_bf16, int64_t ldq, hipStream_t st) {
+hipError_t latent_prepare(const Latent& a, const float* proj, int64_t ldp, uint16_t* q_bf16, int64_t ldq, hipStream_t st) {
     if (a.batch * a.s == 0) return hipSuccess;
     hipLaunchKernelGGL(latent_prepare_kernel, dim3((unsigned)(a.batch * a.s)), dim3(256), 0, st, a, proj, ldp, q_bf16, ldq);
     return hipGetLastError();
@@ -499,14 +716,15 @@ hipError_t latent_prepare(const Latent& a, float* proj, int64_t ldp, uint16_t* q
 
 // By the capacity, not by how many positions are held: a recorded step keeps its grid.
 int latent_splits(const Latent& a) {
-    const int64_t wgs = (int64_t)a.batch * a.s * ((a.heads + kHeads - 1) / kHeads), most = (a.context + kKeys - 1) / kKeys;
-    const int64_t want = (512 + wgs - 1) / wgs;
+    const int heads = attend_mfma_ok(a) ? kMHeads : kHeads;
+    const int64_t wgs = (int64_t)a.batch * a.s * ((a.heads + heads - 1) / heads), most = (a.context + kKeys - 1) / kKeys;
+    const int64_t want = (kMaxSplits + wgs - 1) / wgs;
     return (int)(want < most ? want : most);
 }
 
-// rows * splits <= rows * (512 / rows + 1)
+// rows * splits <= rows * (kMaxSplits / rows + 1)
 size_t latent_absorbed_ws_floats(const Latent& a, int64_t rows) {
-    return (size_t)rows * a.heads * a.rank + (size_t)(512 + rows) * a.heads * (a.rank + 2);
+    return (size_t)rows * a.heads * ((a.rank + a.rot_dim + 31) / 32 * 32) + (size_t)(kMaxSplits + rows) * a.heads * (a.rank + 2);
 }
 
 hipError_t latent_absorbed(const Latent& a, const float* proj, int64_t ldp, float* ws, float* out_f32, uint16_t* out_bf16, int64_t ldo, hipStream_t st) {
@@ -515,18 +733,21 @@ hipError_t latent_absorbed(const Latent& a, const float* proj, int64_t ldp, floa
     if (a.rank > 1024 || rows > 65535) return hipErrorInvalidValue;
     const int splits = latent_splits(a);
     float* qa = ws;
-    float* po = qa + (size_t)rows * a.heads * a.rank;
+    float* po = qa + (size_t)rows * a.heads * ((a.rank + a.rot_dim + 31) / 32 * 32);
     float* ml = po + (size_t)rows * splits * a.heads * a.rank;
-    hipLaunchKernelGGL(latent_absorb_kernel, dim3((unsigned)rows, (unsigned)a.heads, (unsigned)((a.rank + 255) / 256)), dim3(256), 0, st, a, proj, ldp, qa);
+    hipLaunchKernelGGL(latent_queries_kernel, dim3((unsigned)rows, (unsigned)a.heads, (unsigned)((a.rank + kAbsorbCols - 1) / kAbsorbCols)), dim3(256), 0, st, a,
+                       proj, ldp, qa);
     hipError_t e;
-    if (a.cache_bf16)
-        e = a.rank <= 256   ? launch_attend<uint16_t, 1>(a, proj, ldp, qa, splits, po, ml, st)
-            : a.rank <= 512 ? launch_attend<uint16_t, 2>(a, proj, ldp, qa, splits, po, ml, st)
-                            : launch_attend<uint16_t, 4>(a, proj, ldp, qa, splits, po, ml, st);
+    if (attend_mfma_ok(a))
+        e = a.rank + a.rot_dim <= 256 ? launch_attend_mfma<2, 4>(a, qa, splits, po, ml, st) : launch_attend_mfma<5, 8>(a, qa, splits, po, ml, st);
+    else if (a.cache_bf16)
+        e = a.rank <= 256   ? launch_attend<uint16_t, 1>(a, qa, splits, po, ml, st)
+            : a.rank <= 512 ? launch_attend<uint16_t, 2>(a, qa, splits, po, ml, st)
+                            : launch_attend<uint16_t, 4>(a, qa, splits, po, ml, st);
     else
-        e = a.rank <= 256   ? launch_attend<float, 1>(a, proj, ldp, qa, splits, po, ml, st)
-            : a.rank <= 512 ? launch_attend<float, 2>(a, proj, ldp, qa, splits, po, ml, st)
-                            : launch_attend<float, 4>(a, proj, ldp, qa, splits, po, ml, st);
+        e = a.rank <= 256   ? launch_attend<float, 1>(a, qa, splits, po, ml, st)
+            : a.rank <= 512 ? launch_attend<float, 2>(a, qa, splits, po, ml, st)
+                            : launch_attend<float, 4>(a, qa, splits, po, ml, st);
     if (e != hipSuccess) return e;
     hipLaunchKernelGGL(latent_combine_kernel, dim3((unsigned)rows, (unsigned)a.heads, (unsigned)((a.vdim + kValues - 1) / kValues)), dim3(256),
                        (size_t)((a.rank + 63) / 64 * 64) * 4, st, a, splits, po, ml, out_f32, out_bf16, ldo);

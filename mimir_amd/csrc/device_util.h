@@ -125,6 +125,17 @@ __device__ __forceinline__ uint16_t f32_to_bf16_bits(float f) {  // half.go:42-5
     return (uint16_t)(b >> 16);
 }
 
+// Two values rounded to bfloat16 (to nearest, ties to even) in one v_cvt_pk_bf16_f32, `lo` in the low half. A NaN stays one,
+// its payload the instruction's: for kernels whose bits no CPU backend defines.
+typedef __bf16 bf16x2_t __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ uint32_t pack_bf16(float lo, float hi) {
+    const bf16x2_t v = {(__bf16)lo, (__bf16)hi};
+    return __builtin_bit_cast(uint32_t, v);
+}
+__device__ __forceinline__ uint16_t round_bf16(float v) { return __builtin_bit_cast(uint16_t, (__bf16)v); }
+// What rounding v to bfloat16 leaves: v = (rounded v) + low_part(v) exactly.
+__device__ __forceinline__ float low_part(float v) { return v - (float)(__bf16)v; }
+
 // ---- loads ----------------------------------------------------------------
 // ggml blocks are 2-byte aligned. gfx950 serves unaligned dword..dwordx4
 // global loads in hardware, so these compile to single wide loads.

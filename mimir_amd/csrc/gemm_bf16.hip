@@ -35,8 +35,8 @@ struct ActStore {
                 const f32x4 o = {v[0], v[1], v[2], v[3]};
                 *(f32x4*)(out.f32 + at) = o;
             } else {
-                const u32x2 o = {(uint32_t)f32_to_bf16_bits(v[0]) | (uint32_t)f32_to_bf16_bits(v[1]) << 16,
-                                 (uint32_t)f32_to_bf16_bits(v[2]) | (uint32_t)f32_to_bf16_bits(v[3]) << 16};
+                const u32x2 o = {pack_bf16(v[0], v[1]),
+                                 pack_bf16(v[2], v[3])};
                 *(u32x2*)(out.bf16 + at) = o;
             }
             return;
@@ -45,7 +45,7 @@ struct ActStore {
         for (int k = 0; k < 4; k++) {
             if (n + k >= N) continue;
             if (out.f32) out.f32[at + k] = v[k];
-            else out.bf16[at + k] = f32_to_bf16_bits(v[k]);
+            else out.bf16[at + k] = round_bf16(v[k]);
         }
     }
 };

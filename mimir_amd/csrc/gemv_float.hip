@@ -98,7 +98,7 @@ __global__ __launch_bounds__(256) void gemv_bf16_kernel(const uint16_t* __restri
             else if (n0 + r < out.silu_n) v = v / (1.f + expf(-v));
             const int64_t at = (m0 + m) * out.ld + n0 + r;
             if (out.f32) out.f32[at] = v;
-            else out.bf16[at] = f32_to_bf16_bits(v);
+            else out.bf16[at] = round_bf16(v);
         }
 }
 

@@ -128,9 +128,6 @@ constexpr int kValueTile = 128;  // rows of S (values) a workgroup
 __device__ __forceinline__ f32x16 mfma_bf16(u32x4 a, u32x4 b, f32x16 c) {
     return __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
 }
-__device__ __forceinline__ uint32_t pack2(float lo, float hi) { return (uint32_t)f32_to_bf16_bits(lo) | (uint32_t)f32_to_bf16_bits(hi) << 16; }
-// v = high + low + at most 2^-17 |v|
-__device__ __forceinline__ float low_part(float v) { return v - bf16_bits_to_f32(f32_to_bf16_bits(v)); }
 
 struct ChunkWs {
     float* states;   // [chunks, batch * heads, vdim, dp]; chunk_carry leaves 8 high and 8 low bfloat16 parts in the place of 8 floats
@@ -191,8 +188,8 @@ __device__ __forceinline__ void stage_transposed(const uint16_t* __restrict__ sr
                 float f[4];
 #pragma unroll
                 for (int i = 0; i < 4; i++) f[i] = __uint_as_float(bits[i] << 16) * w[s0 + i];
-                *(u32x2*)at = u32x2{pack2(f[0], f[1]), pack2(f[2], f[3])};
-                *(u32x2*)(low + (p * 8 + e) * kRow + s0) = u32x2{pack2(low_part(f[0]), low_part(f[1])), pack2(low_part(f[2]), low_part(f[3]))};
+                *(u32x2*)at = u32x2{pack_bf16(f[0], f[1]), pack_bf16(f[2], f[3])};
+                *(u32x2*)(low + (p * 8 + e) * kRow + s0) = u32x2{pack_bf16(low_part(f[0]), low_part(f[1])), pack_bf16(low_part(f[2]), low_part(f[3]))};
             }
         }
     }
@@ -304,8 +301,8 @@ __global__ __launch_bounds__(256) void chunk_carry_kernel(Recurrence r, ChunkWs 
             u32x4 high, low;
 #pragma unroll
             for (int i = 0; i < 4; i++) {
-                high[i] = pack2(s[2 * i], s[2 * i + 1]);
-                low[i] = pack2(low_part(s[2 * i]), low_part(s[2 * i + 1]));
+                high[i] = pack_bf16(s[2 * i], s[2 * i + 1]);
+                low[i] = pack_bf16(low_part(s[2 * i]), low_part(s[2 * i + 1]));
             }
             ((u32x4*)at)[0] = high;
             ((u32x4*)at)[1] = low;
@@ -423,8 +420,8 @@ __global__ __launch_bounds__(256) void chunk_outputs_kernel(Recurrence r, ChunkW
 #pragma unroll
             for (int i = 0; i < 4; i++) {
                 const float x = p[half * 8 + 2 * i], y = p[half * 8 + 2 * i + 1];
-                high[i] = pack2(x, y);
-                low[i] = pack2(low_part(x), low_part(y));
+                high[i] = pack_bf16(x, y);
+                low[i] = pack_bf16(low_part(x), low_part(y));
             }
 #pragma unroll
             for (int et = 0; et < ET; et++) {

@@ -97,6 +97,7 @@ struct Stack : Decoder {
 
 mi355x_status Stack::product(const Mat& w, int64_t row0, int64_t n, const DevBuf& f, const DevBuf& b, bool tiles, int64_t rows, const ProductOut& out) {
     if (tiles) STACK_HIP(gemm_bf16(w.row(row0), w.ld, b.as<uint16_t>(), w.ld, rows, n, w.k, out, stream), "product");
+    else if (half() && rows > 1 && rows <= kGemvRows) STACK_HIP(gemv_bf16_rows(w.row(row0), w.ld, f.as<float>(), w.ld, rows, n, w.k, out, stream), "product");
     else if (rows <= kGemvRows) STACK_HIP(gemv_bf16(w.row(row0), w.ld, f.as<float>(), w.ld, rows, n, w.k, out, stream), "product");
     else STACK_HIP(gemm_f32(w.row(row0), w.ld, f.as<float>(), w.ld, rows, n, w.k, out, stream), "product");
     return MI355X_OK;
@@ -169,9 +170,9 @@ mi355x_status Stack::mix(StackLayer& l, int64_t s, bool tiles, const int32_t* po
         if (mi355x_status st = product(l.in, 0, l.in.n, in_f, in_b, tiles, rows, p)) return st;
         const Latent a = latent(l, s, pos);
         const bool formed = tiles && s >= kFormKeys && latent_prompt_ok(a);
-        STACK_HIP(latent_prepare(a, proj_f.as<float>(), l.in.n, formed ? q_b.as<uint16_t>() : nullptr, (int64_t)l.c.heads * (l.c.dim + l.c.rot_dim), stream),
-                  "latents and rotation");
         if (formed) {
+            STACK_HIP(latent_prepare(a, proj_f.as<float>(), l.in.n, q_b.as<uint16_t>(), (int64_t)l.c.heads * (l.c.dim + l.c.rot_dim), stream),
+                      "latents and rotation");
             if (mi355x_status st = prompt_attention(l, a)) return st;
         } else {
             STACK_HIP(latent_absorbed(a, proj_f.as<float>(), l.in.n, ws.as<float>(), tiles ? nullptr : mix_f.as<float>(),

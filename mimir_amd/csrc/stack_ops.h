@@ -67,6 +67,8 @@ struct ProductOut {
 constexpr int64_t kGemvRows = 8;  // rows of x that gemv_bf16 takes at once (more are several passes over W)
 // float32 x, few rows: W read once for up to kGemvRows of them (gemv_float.hip)
 hipError_t gemv_bf16(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st);
+// the same on the bfloat16 matrix cores, x as the sum of two bfloat16: at most kGemvRows rows (gemv_bf16_rows.hip)
+hipError_t gemv_bf16_rows(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st);
 // float32 x, many rows, on the float32 matrix cores: nothing is rounded to 16 bits (gemm_float.hip)
 hipError_t gemm_f32(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st);
 // bfloat16 x, many rows, on the bfloat16 matrix cores with float32 sums (gemm_bf16.hip): ldx and ldw multiples of 8
@@ -130,15 +132,15 @@ struct Latent {
     int64_t past = 0;    // positions before them: past + *past_dev
     const int32_t* past_dev = nullptr;
 };
-// From projections [rows, heads * (dim + rot_dim) | rank + rot_dim] (float32, rows ldp apart): the cache rows of the new
-// positions, and the queries with their rotated parts turned, in place or (q_bf16) as bfloat16 rows ldq apart.
-hipError_t latent_prepare(const Latent& a, float* proj, int64_t ldp, uint16_t* q_bf16, int64_t ldq, hipStream_t st);
-// Few query rows: keys and values are never formed. q' = W_uk^T q per head against the latents, and W_uv on what they sum
-// to. ws: latent_absorbed_ws_floats floats. out [rows, heads * vdim] float32 or bfloat16, rows ldo apart.
+// From projections [rows, heads * (dim + rot_dim) | rank + rot_dim] (float32, rows ldp apart), for latent_prompt: the cache
+// rows of the new positions, and the queries with their rotated parts turned, as bfloat16 rows ldq apart.
+hipError_t latent_prepare(const Latent& a, const float* proj, int64_t ldp, uint16_t* q_bf16, int64_t ldq, hipStream_t st);
+// Few query rows, from the same projections: cache rows, then attention without ever forming keys or values: q' = W_uk^T q
+// per head against the latents, and W_uv on what they sum to. ws: latent_absorbed_ws_floats floats. out
+// [rows, heads * vdim] float32 or bfloat16, rows ldo apart.
 int latent_splits(const Latent& a);
 size_t latent_absorbed_ws_floats(const Latent& a, int64_t rows);
 hipError_t latent_absorbed(const Latent& a, const float* proj, int64_t ldp, float* ws, float* out_f32, uint16_t* out_bf16, int64_t ldo, hipStream_t st);
-
 // Many query rows of one sequence (bfloat16 cache and queries), on keys and values formed beforehand for all its past + s
 // positions: keys [positions, heads * dim], values transposed [heads * vdim, positions], rows ldk and ldv (a multiple of
 // 64) elements apart. q, out: the sequence's rows. Products on the bfloat16 matrix cores; a weight goes to them as the
