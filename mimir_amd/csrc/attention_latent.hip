@@ -321,12 +321,20 @@ __global__ __launch_bounds__(256) void latent_attend_mfma_kernel(Latent a, const
     float m = -__builtin_inff(), l = 0.f;
     const int pieces = lq / 8;
     for (int64_t j0 = lo; j0 < hi; j0 += kKeys) {
-        for (int i = tid; i < kKeys * pieces; i += 256) {
-            const int j = i / pieces, d = i % pieces * 8;
-            const int64_t row = j0 + j < hi ? j0 + j : hi - 1;
-            u32x4 v = {0, 0, 0, 0};
-            if (d < L) v = *(const u32x4*)(cache + row * a.ldc + d);  // a row is padded with zeros to a multiple of 8
-            *(u32x4*)(tile + j * ldt + d) = v;
+        for (int i0 = tid; i0 < kKeys * pieces; i0 += 6 * 256) {  // six pieces requested at a time
+            u32x4 v[6];
+#pragma unroll
+            for (int u = 0; u < 6; u++) {
+                const int i = i0 + 256 * u, j = i / pieces, d = i % pieces * 8;
+                const int64_t row = j0 + j < hi ? j0 + j : hi - 1;
+                v[u] = u32x4{0, 0, 0, 0};
+                if (i < kKeys * pieces && d < L) v[u] = *(const u32x4*)(cache + row * a.ldc + d);  // a row is padded with zeros to a multiple of 8
+            }
+#pragma unroll
+            for (int u = 0; u < 6; u++) {
+                const int i = i0 + 256 * u, j = i / pieces, d = i % pieces * 8;
+                if (i < kKeys * pieces) *(u32x4*)(tile + j * ldt + d) = v[u];
+            }
         }
         __syncthreads();
         f32x4 sc[4][2];
@@ -539,11 +547,12 @@ __device__ __forceinline__ f32x16 mfma_bf16(u32x4 a, u32x4 b, f32x16 c) {
 }
 
 struct PromptArgs {
-    const uint16_t *q, *keys, *vt, *cache;  // cache: the sequence's rows
+    const uint16_t *q, *keys, *vt, *cache;
     uint16_t* out;
-    int64_t ldq, ldk, ldv, ldc, ldo;
+    int64_t ldq, ldk, ldv, ldc, ldo, context;
     int heads, dim, rot_dim, vdim, rank;
-    int past, s;
+    int past, s, batch;
+    int fold;
     float scale;  // times log2(e)
 };
 
@@ -558,7 +567,16 @@ __global__ __launch_bounds__(256, DT > 12 ? 1 : 2) void latent_prompt_kernel(Pro
     __shared__ __align__(16) uint16_t ks[kKeys * kKey];
     __shared__ __align__(16) uint16_t vs[VT * 32 * kVal];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r32 = lane & 31, hi = lane >> 5;
-    const int h = blockIdx.x, first = (int)(gridDim.y - 1 - blockIdx.y) * kPromptRows;  // the last rows first: they see the most keys
+    // the last rows first: they see the most keys. Where all workgroups fit the device at once, two a compute unit, the
+    // second half goes the other way, so that long ones and short ones share a unit.
+    const int h = blockIdx.x, nb = gridDim.y, by = blockIdx.y;
+    const int first = (p.fold && by >= (nb + 1) / 2 ? by - (nb + 1) / 2 : nb - 1 - by) * kPromptRows;
+    const int64_t seq = blockIdx.z;
+    p.q += seq * p.s * p.ldq;
+    p.keys += seq * p.context * p.ldk;
+    p.vt += seq * p.context;
+    p.cache += seq * p.context * p.ldc;
+    p.out += seq * p.s * p.ldo;
     const int D = p.dim + p.rot_dim, n_keys = p.past + p.s;
     const int row = first + wave * 32 + r32, pos = p.past + row;  // sees keys 0 .. pos
     const int last_wg = first + kPromptRows < p.s ? first + kPromptRows : p.s;
@@ -698,8 +716,9 @@ __global__ __launch_bounds__(256, DT > 12 ? 1 : 2) void latent_prompt_kernel(Pro
 }
 
 template <int DT, int VT>
-void launch_prompt(const PromptArgs& p, hipStream_t st) {
-    const dim3 grid((unsigned)p.heads, (unsigned)((p.s + kPromptRows - 1) / kPromptRows));
+void launch_prompt(PromptArgs p, hipStream_t st) {
+    const dim3 grid((unsigned)p.heads, (unsigned)((p.s + kPromptRows - 1) / kPromptRows), (unsigned)p.batch);
+    p.fold = (int64_t)grid.x * grid.y * grid.z <= 512;
     const bool whole = p.dim % 8 == 0 && p.rot_dim % 8 == 0 && p.rank % 8 == 0 && p.ldq % 8 == 0 && p.ldk % 8 == 0 && p.ldc % 8 == 0 &&
                        (((uintptr_t)p.q | (uintptr_t)p.keys | (uintptr_t)p.cache) & 15) == 0;
     if (whole) hipLaunchKernelGGL((latent_prompt_kernel<DT, VT, true>), grid, dim3(256), 0, st, p);
@@ -758,15 +777,15 @@ bool latent_prompt_ok(const Latent& a) {
     return a.cache_bf16 && a.dim + a.rot_dim <= 256 && a.vdim <= 256 && a.past + a.s < 1 << 30 && !a.past_dev;
 }
 
-hipError_t latent_prompt(const Latent& a, int sequence, const uint16_t* q, int64_t ldq, const uint16_t* keys, int64_t ldk, const uint16_t* values_t,
-                         int64_t ldv, uint16_t* out, int64_t ldo, hipStream_t st) {
-    if (a.s == 0) return hipSuccess;
-    if (!latent_prompt_ok(a) || ldv % 64 || ((uintptr_t)values_t & 15)) return hipErrorInvalidValue;
+hipError_t latent_prompt(const Latent& a, const uint16_t* q, int64_t ldq, const uint16_t* keys, int64_t ldk, const uint16_t* values_t, int64_t ldv,
+                         uint16_t* out, int64_t ldo, hipStream_t st) {
+    if (a.batch * a.s == 0) return hipSuccess;
+    if (!latent_prompt_ok(a) || ldv % 8 || a.context % 64 || ((uintptr_t)values_t & 15)) return hipErrorInvalidValue;
     PromptArgs p;
-    p.q = q; p.keys = keys; p.vt = values_t; p.cache = (const uint16_t*)a.cache + sequence * a.context * a.ldc; p.out = out;
-    p.ldq = ldq; p.ldk = ldk; p.ldv = ldv; p.ldc = a.ldc; p.ldo = ldo;
+    p.q = q; p.keys = keys; p.vt = values_t; p.cache = (const uint16_t*)a.cache; p.out = out;
+    p.ldq = ldq; p.ldk = ldk; p.ldv = ldv; p.ldc = a.ldc; p.ldo = ldo; p.context = a.context;
     p.heads = a.heads; p.dim = a.dim; p.rot_dim = a.rot_dim; p.vdim = a.vdim; p.rank = a.rank;
-    p.past = (int)a.past; p.s = (int)a.s;
+    p.past = (int)a.past; p.s = (int)a.s; p.batch = a.batch; p.fold = 0;
     p.scale = a.scale * 1.4426950408889634f;
     const int d = a.dim + a.rot_dim, v = a.vdim;
     if (d <= 64 && v <= 64) launch_prompt<4, 2>(p, st);

@@ -2,7 +2,7 @@
 // (v_mfma_f32_32x32x2_f32): nothing is rounded below float32 on the way. The prompt product of a model that runs in
 // float32, and in any model that of the few columns that must not be rounded (a recurrence's gates).
 // A workgroup of four wavefronts owns 64 x 64 of y, a wavefront 32 x 32; steps of 32 along K go through LDS. Where W has
-// few rows, a workgroup owns 16 rows of x and up to 64 of W instead, and its wavefronts cut K into four
+// few rows, a workgroup owns 16 rows of x and up to 64 of W instead, and its eight wavefronts cut K
 // (gemm_f32_narrow_kernel): the tiles above would leave most of the device without work.
 #include "device_util.h"
 #include "stack_ops.h"
@@ -73,12 +73,12 @@ constexpr int kNarrow = 64;  // rows of W a workgroup
 
 // v_mfma_f32_16x16x4: lane (row, k). A lane brings four neighbouring elements of K of its row, so the four products of a step
 // of sixteen take K in the order 4 k + j, in both operands alike.
-__global__ __launch_bounds__(256) void gemm_f32_narrow_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx, int64_t M,
+__global__ __launch_bounds__(512) void gemm_f32_narrow_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx, int64_t M,
                                                               int64_t N, int64_t K, ProductOut out) {
-    __shared__ float red[4][16][kNarrow + 1];
+    __shared__ float red[8][16][kNarrow + 1];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
     const int64_t m0 = (int64_t)blockIdx.y * 16, n0 = (int64_t)blockIdx.x * kNarrow;
-    const int64_t steps = (K + 15) / 16, per = (steps + 3) / 4, k0 = wave * per * 16, k1 = k0 + per * 16 < steps * 16 ? k0 + per * 16 : steps * 16;
+    const int64_t steps = (K + 15) / 16, per = (steps + 7) / 8, k0 = wave * per * 16, k1 = k0 + per * 16 < steps * 16 ? k0 + per * 16 : steps * 16;
     const float* xp = x + (m0 + r16 < M ? m0 + r16 : M - 1) * ldx + g * 4;
     const uint16_t* wp[kNarrow / 16];
 #pragma unroll
@@ -103,11 +103,13 @@ __global__ __launch_bounds__(256) void gemm_f32_narrow_kernel(const uint16_t* __
 #pragma unroll
         for (int i = 0; i < 4; i++) red[wave][4 * g + i][t * 16 + r16] = acc[t][i];
     __syncthreads();
-    for (int o = tid; o < 16 * kNarrow; o += 256) {
+    for (int o = tid; o < 16 * kNarrow; o += 512) {
         const int row = o / kNarrow, col = o % kNarrow;
         const int64_t m = m0 + row, n = n0 + col;
         if (m >= M || n >= N) continue;
-        float v = (red[0][row][col] + red[1][row][col]) + (red[2][row][col] + red[3][row][col]);
+        float v = 0.f;
+#pragma unroll
+        for (int i = 0; i < 8; i++) v += red[i][row][col];
         if (out.relu2) v = v > 0.f ? v * v : 0.f;
         else if (n < out.silu_n) v = v / (1.f + expf(-v));
         if (out.f32) out.f32[m * out.ld + n] = v;
@@ -120,7 +122,7 @@ __global__ __launch_bounds__(256) void gemm_f32_narrow_kernel(const uint16_t* __
 hipError_t gemm_f32(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st) {
     if (M == 0 || N == 0) return hipSuccess;
     if (N <= 2 * kNarrow && ldx % 4 == 0 && ldw % 4 == 0) {
-        hipLaunchKernelGGL(gemm_f32_narrow_kernel, dim3((unsigned)((N + kNarrow - 1) / kNarrow), (unsigned)((M + 15) / 16)), dim3(256), 0, st, W, ldw, x, ldx, M, N,
+        hipLaunchKernelGGL(gemm_f32_narrow_kernel, dim3((unsigned)((N + kNarrow - 1) / kNarrow), (unsigned)((M + 15) / 16)), dim3(512), 0, st, W, ldw, x, ldx, M, N,
                            K, out);
         return hipGetLastError();
     }

@@ -2,7 +2,7 @@
 // product of a decoding step of several sequences. v_mfma_f32_16x16x32_bf16 multiplies sixteen rows of W by sixteen
 // columns; the columns are the rows of x twice, once their bfloat16 value and once what rounding left of them (a float32's
 // first sixteen bits of significand), whose results are added at the end: near float32's accuracy for the price of one
-// product. The eight wavefronts of a workgroup share its rows of W and cut K into pieces; W goes from memory straight into
+// product. The wavefronts of a workgroup (eight, or sixteen for long rows) share its rows of W and cut K into pieces; W goes from memory straight into
 // the operand registers (a lane's sixteen bytes of one row), x is converted on the way.
 #include "device_util.h"
 #include "stack_ops.h"
@@ -13,10 +13,8 @@ namespace {
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
-constexpr int kWaves = 8;
-
 // T: groups of sixteen rows of W a workgroup.
-template <int T>
+template <int T, int kWaves>
 __global__ __launch_bounds__(64 * kWaves) void gemv_bf16_rows_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx,
                                                                      int M, int N, int K, ProductOut out) {
     __shared__ float red[kWaves][T * 16][17];
@@ -85,10 +83,12 @@ hipError_t gemv_bf16_rows(const uint16_t* W, int64_t ldw, const float* x, int64_
     if (M == 0 || N == 0) return hipSuccess;
     if (M > kGemvRows || ldw % 8 || ldx % 4) return hipErrorInvalidValue;
     const int k = (int)((K + 63) / 64 * 64);
-    if (N >= 8192)
-        hipLaunchKernelGGL(gemv_bf16_rows_kernel<2>, dim3((unsigned)((N + 31) / 32)), dim3(64 * kWaves), 0, st, W, ldw, x, ldx, (int)M, (int)N, k, out);
-    else
-        hipLaunchKernelGGL(gemv_bf16_rows_kernel<1>, dim3((unsigned)((N + 15) / 16)), dim3(64 * kWaves), 0, st, W, ldw, x, ldx, (int)M, (int)N, k, out);
+    auto launch = [&](auto kernel, int rows, int waves) {
+        hipLaunchKernelGGL(kernel, dim3((unsigned)((N + rows - 1) / rows)), dim3(64 * waves), 0, st, W, ldw, x, ldx, (int)M, (int)N, k, out);
+    };
+    if (N >= 8192) launch(gemv_bf16_rows_kernel<2, 8>, 32, 8);
+    else if (k >= 8192) launch(gemv_bf16_rows_kernel<1, 16>, 16, 16);
+    else launch(gemv_bf16_rows_kernel<1, 8>, 16, 8);
     return hipGetLastError();
 }
 

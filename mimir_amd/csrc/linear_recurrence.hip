@@ -115,8 +115,10 @@ void launch_scan(const Recurrence& r, hipStream_t st) {
 //   chunk_states   each chunk's own sum of weighted v k^T (and of k), relative to its largest a_s
 //   chunk_carry    S at every chunk's start, chunk after chunk, and the state behind the last
 //   chunk_outputs  o of the chunk's positions from S and from the chunk itself
-// States are kept transposed, [vdim, dim], so that a lane's part of an operand is contiguous. Operands that are not q, k, v
-// (weighted keys, weights, S) go to the matrix cores as the sum of two bfloat16.
+// Operands that are not q, k, v (weighted keys, weights, S) go to the matrix cores as the sum of two bfloat16. The states
+// between the launches lie as their operand does: blocks of 32 values by 16 features, 512 floats each; value e, features
+// 8 p .. 8 p + 7 belong to lane e + 32 p (p 0 or 1), whose first four floats are at 4 lane and whose others 256 behind. In
+// their place chunk_carry leaves the eight high and the eight low bfloat16 parts.
 
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -130,11 +132,11 @@ __device__ __forceinline__ f32x16 mfma_bf16(u32x4 a, u32x4 b, f32x16 c) {
 }
 
 struct ChunkWs {
-    float* states;   // [chunks, batch * heads, vdim, dp]; chunk_carry leaves 8 high and 8 low bfloat16 parts in the place of 8 floats
+    float* states;   // [chunks, batch * heads, ep / 32, dp / 16, 512]
     float* norms;    // [chunks, batch * heads, dp]: the sums of k, then n at the chunk's start
     float* gates;    // [chunks, batch * heads, 2]: the chunk's log decay, its largest a_s
     float* m_start;  // [chunks, batch * heads]
-    int dp;          // dim to a multiple of 16
+    int dp, ep;      // dim to a multiple of 16, vdim to one of 32
     int chunks;
 };
 
@@ -227,26 +229,27 @@ __global__ __launch_bounds__(256) void chunk_states_kernel(Recurrence r, ChunkWs
     __syncthreads();
     stage_transposed((const uint16_t*)r.k + row0 * r.ld + (int64_t)h * r.dim, r.ld, n, r.dim, dp32, kH, kL, weight);
     __syncthreads();
-    float* out = ws.states + (head * r.vdim + e0) * ws.dp;
     const int e = wave * 32;
     if (e < cols) {
-        u32x4 a[kC / 16];
+        float* out = ws.states + (head * (ws.ep / 32) + (e0 + e) / 32) * (ws.dp / 16) * 512;
+        u32x4 v[kC / 16];
 #pragma unroll
-        for (int k = 0; k < kC / 16; k++) a[k] = *(const u32x4*)(vT + (e + r32) * kRow + k * 16 + hi * 8);
+        for (int k = 0; k < kC / 16; k++) v[k] = *(const u32x4*)(vT + (e + r32) * kRow + k * 16 + hi * 8);
         for (int d = 0; d < dp32; d += 32) {
             f32x16 acc;
 #pragma unroll
             for (int i = 0; i < 16; i++) acc[i] = 0.f;
 #pragma unroll
             for (int k = 0; k < kC / 16; k++) {
-                acc = mfma_bf16(a[k], *(const u32x4*)(kH + (d + r32) * kRow + k * 16 + hi * 8), acc);
-                acc = mfma_bf16(a[k], *(const u32x4*)(kL + (d + r32) * kRow + k * 16 + hi * 8), acc);
+                acc = mfma_bf16(*(const u32x4*)(kH + (d + r32) * kRow + k * 16 + hi * 8), v[k], acc);
+                acc = mfma_bf16(*(const u32x4*)(kL + (d + r32) * kRow + k * 16 + hi * 8), v[k], acc);
             }
+            // a lane holds value r32 and features d + 8 g + 4 hi .. + 3 for g = 0 .. 3
 #pragma unroll
-            for (int i = 0; i < 16; i++) {
-                const int row = e + (i & 3) + 8 * (i >> 2) + 4 * hi;
-                if (row < cols && d + r32 < ws.dp) out[(int64_t)row * ws.dp + d + r32] = acc[i];
-            }
+            for (int g = 0; g < 4; g++)
+                if (d + 8 * g < ws.dp)
+                    *(f32x4*)(out + (d / 16 + g / 2) * 512 + hi * 256 + (r32 + 32 * (g & 1)) * 4) =
+                        f32x4{acc[4 * g], acc[4 * g + 1], acc[4 * g + 2], acc[4 * g + 3]};
         }
     }
     if (GATED && e0 == 0)
@@ -260,28 +263,29 @@ __global__ __launch_bounds__(256) void chunk_states_kernel(Recurrence r, ChunkWs
 // A thread carries eight features of one value's row of S (or of n, behind them) through the chunks.
 template <bool GATED>
 __global__ __launch_bounds__(256) void chunk_carry_kernel(Recurrence r, ChunkWs ws) {
-    const int h = blockIdx.y, b = blockIdx.z, per = ws.dp / 8, total = r.vdim * per;
+    const int h = blockIdx.y, b = blockIdx.z, per = ws.dp / 8, total = ws.ep * per;
     const int item = blockIdx.x * 256 + threadIdx.x;
     const bool is_n = GATED && item >= total && item < total + per;
     if (item >= total && !is_n) return;
-    const int e = is_n ? 0 : item / per, d0 = (is_n ? item - total : item % per) * 8;
+    const int block = item / 64, lane = item % 64;
+    const int e = is_n ? 0 : block / (ws.dp / 16) * 32 + lane % 32, d0 = is_n ? (item - total) * 8 : block % (ws.dp / 16) * 16 + lane / 32 * 8;
     const int64_t head = (int64_t)b * r.heads + h, heads = (int64_t)r.batch * r.heads;
     const int slices = (r.vdim + kCols - 1) / kCols;
     float s[8];
 #pragma unroll
     for (int i = 0; i < 8; i++)
-        s[i] = d0 + i >= r.dim ? 0.f : is_n ? r.n[head * slices * r.dim + d0 + i] : r.S[(head * r.dim + d0 + i) * r.vdim + e];
+        s[i] = d0 + i >= r.dim || e >= r.vdim ? 0.f : is_n ? r.n[head * slices * r.dim + d0 + i] : r.S[(head * r.dim + d0 + i) * r.vdim + e];
     float m = GATED ? r.m[head * slices] : 0.f;
-    float* at = is_n ? ws.norms + head * ws.dp + d0 : ws.states + (head * r.vdim + e) * ws.dp + d0;
-    const int64_t step = is_n ? heads * ws.dp : heads * r.vdim * ws.dp;
+    float* at = is_n ? ws.norms + head * ws.dp + d0 : ws.states + head * ws.ep * ws.dp + block * 512 + lane * 4;
+    const int64_t step = is_n ? heads * ws.dp : heads * ws.ep * ws.dp, second = is_n ? 4 : 256;  // floats to the other four
     const int last = (int)(r.s - (int64_t)(ws.chunks - 1) * kC);
     f32x4 x[2], y[2];  // the next chunk's sums are requested before this chunk's are used
-    x[0] = ((const f32x4*)at)[0];
-    x[1] = ((const f32x4*)at)[1];
+    x[0] = *(const f32x4*)at;
+    x[1] = *(const f32x4*)(at + second);
     for (int c = 0; c < ws.chunks; c++, at += step) {
         if (c + 1 < ws.chunks) {
-            y[0] = ((const f32x4*)(at + step))[0];
-            y[1] = ((const f32x4*)(at + step))[1];
+            y[0] = *(const f32x4*)(at + step);
+            y[1] = *(const f32x4*)(at + step + second);
         }
         float keep, take = 1.f;
         if (GATED) {
@@ -304,8 +308,8 @@ __global__ __launch_bounds__(256) void chunk_carry_kernel(Recurrence r, ChunkWs 
                 high[i] = pack_bf16(s[2 * i], s[2 * i + 1]);
                 low[i] = pack_bf16(low_part(s[2 * i]), low_part(s[2 * i + 1]));
             }
-            ((u32x4*)at)[0] = high;
-            ((u32x4*)at)[1] = low;
+            *(u32x4*)at = high;
+            *(u32x4*)(at + second) = low;
         }
 #pragma unroll
         for (int i = 0; i < 8; i++) s[i] = fmaf(take, x[i >> 2][i & 3], keep * s[i]);
@@ -314,7 +318,7 @@ __global__ __launch_bounds__(256) void chunk_carry_kernel(Recurrence r, ChunkWs 
     }
 #pragma unroll
     for (int i = 0; i < 8; i++) {
-        if (d0 + i >= r.dim) continue;
+        if (d0 + i >= r.dim || e >= r.vdim) continue;
         if (is_n)
             for (int k = 0; k < slices; k++) r.n[(head * slices + k) * r.dim + d0 + i] = s[i];
         else
@@ -329,6 +333,7 @@ template <bool GATED, int DT, int ET>
 __global__ __launch_bounds__(256) void chunk_outputs_kernel(Recurrence r, ChunkWs ws) {
     constexpr int kKey = DT * 16 + 8;
     __shared__ __align__(16) uint16_t ks[kC * kKey];
+    __shared__ __align__(16) uint16_t qs[DT <= 8 ? kC * kKey : 1];  // up to 128 features; more would not leave room for two workgroups
     __shared__ __align__(16) uint16_t vT[2 * ET * 32 * kRow];
     __shared__ float as[kC], bs[kC], tops[kC], n0[DT * 16], pw[kC + 1];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r32 = lane & 31, hi = lane >> 5;
@@ -362,12 +367,17 @@ __global__ __launch_bounds__(256) void chunk_outputs_kernel(Recurrence r, ChunkW
             u32x4 v = {0, 0, 0, 0};
             if (s < n && p * 8 < r.dim) v = *(const u32x4*)(k + (int64_t)s * r.ld + p * 8);
             *(u32x4*)(ks + s * kKey + p * 8) = v;
+            if constexpr (DT <= 8) {
+                v = u32x4{0, 0, 0, 0};
+                if (s < n && p * 8 < r.dim) v = *(const u32x4*)((const uint16_t*)r.q + (row0 + s) * r.ld + (int64_t)h * r.dim + p * 8);
+                *(u32x4*)(qs + s * kKey + p * 8) = v;
+            }
         }
     }
     stage_transposed((const uint16_t*)r.v + row0 * r.ld + (int64_t)h * r.vdim + e0, r.ld, n, cols, kTile, vT, nullptr, nullptr);
     const int t = (wave >> 1) * 32 + r32, e1 = (wave & 1) * ET * 32;  // this lane's position; the wavefront's first value
     u32x4 q[DT];
-    {
+    if constexpr (DT > 8) {
         const uint16_t* qr = (const uint16_t*)r.q + (row0 + (t < n ? t : n - 1)) * r.ld + (int64_t)h * r.dim + hi * 8;
 #pragma unroll
         for (int k = 0; k < DT; k++) {
@@ -376,21 +386,27 @@ __global__ __launch_bounds__(256) void chunk_outputs_kernel(Recurrence r, ChunkW
         }
     }
     __syncthreads();
+    if constexpr (DT <= 8) {
+#pragma unroll
+        for (int k = 0; k < DT; k++) q[k] = *(const u32x4*)(qs + t * kKey + k * 16 + hi * 8);
+    }
     const float inter = (GATED ? expf(m0 - tops[t]) : pw[t + 1]) * r.q_scale;
     f32x16 acc[ET];
+#pragma unroll
+    for (int et = 0; et < ET; et++)
+#pragma unroll
+        for (int i = 0; i < 16; i++) acc[et][i] = 0.f;
     // from the state at the chunk's start
 #pragma unroll
     for (int et = 0; et < ET; et++) {
-#pragma unroll
-        for (int i = 0; i < 16; i++) acc[et][i] = 0.f;
-        const int e = e1 + et * 32 + r32;
-        const float* S = ws.states + (head * r.vdim + e0 + (e < cols ? e : cols - 1)) * ws.dp;
+        const int block = (e0 + e1 + et * 32) / 32;
+        if (block >= ws.ep / 32) break;
+        const float* S = ws.states + (head * (ws.ep / 32) + block) * (ws.dp / 16) * 512 + lane * 4;
 #pragma unroll
         for (int k = 0; k < DT; k++) {
             if (k * 16 < ws.dp) {  // dp is a multiple of 16
-                const u32x4* pair = (const u32x4*)(S + k * 16 + hi * 8);
-                acc[et] = mfma_bf16(pair[0], q[k], acc[et]);
-                acc[et] = mfma_bf16(pair[1], q[k], acc[et]);
+                acc[et] = mfma_bf16(*(const u32x4*)(S + k * 512), q[k], acc[et]);
+                acc[et] = mfma_bf16(*(const u32x4*)(S + k * 512 + 256), q[k], acc[et]);
             }
         }
 #pragma unroll
@@ -477,7 +493,7 @@ hipError_t launch_chunks(const Recurrence& r, const ChunkWs& ws, hipStream_t st)
     }
     const unsigned vt = (unsigned)((r.vdim + kValueTile - 1) / kValueTile);
     hipLaunchKernelGGL(chunk_states_kernel<GATED>, dim3((unsigned)ws.chunks, (unsigned)r.heads, (unsigned)r.batch * vt), dim3(256), lds, st, r, ws);
-    const int items = (r.vdim + (GATED ? 1 : 0)) * ws.dp / 8;
+    const int items = (ws.ep + (GATED ? 1 : 0)) * ws.dp / 8;
     hipLaunchKernelGGL(chunk_carry_kernel<GATED>, dim3((unsigned)((items + 255) / 256), (unsigned)r.heads, (unsigned)r.batch), dim3(256), 0, st, r, ws);
     if (ws.dp <= 32) launch_outputs<GATED, 2>(r, ws, st);
     else if (ws.dp <= 64) launch_outputs<GATED, 4>(r, ws, st);
@@ -508,7 +524,7 @@ bool recurrence_chunks_ok(const Recurrence& r) {
 
 size_t recurrence_chunk_ws_floats(int batch, int heads, int dim, int vdim, int64_t s) {
     const int64_t dp = chunk_dp(dim);
-    return (size_t)((s + kC - 1) / kC) * batch * heads * (vdim * dp + dp + 4) + 64;
+    return (size_t)((s + kC - 1) / kC) * batch * heads * ((vdim + 31) / 32 * 32 * dp + dp + 4) + 64;
 }
 
 hipError_t recurrence_chunks(const Recurrence& r, hipStream_t st) {
@@ -519,7 +535,8 @@ hipError_t recurrence_chunks(const Recurrence& r, hipStream_t st) {
     ws.chunks = (int)((r.s + kC - 1) / kC);
     const size_t heads = (size_t)ws.chunks * r.batch * r.heads;
     ws.states = r.ws;
-    ws.norms = ws.states + heads * r.vdim * ws.dp;
+    ws.ep = (r.vdim + 31) / 32 * 32;
+    ws.norms = ws.states + heads * ws.ep * ws.dp;
     ws.gates = ws.norms + heads * ws.dp;
     ws.m_start = ws.gates + heads * 2;
     return r.gates ? launch_chunks<true>(r, ws, st) : launch_chunks<false>(r, ws, st);

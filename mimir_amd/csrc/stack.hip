@@ -73,7 +73,7 @@ struct Stack : Decoder {
 
     // activations of up to max_rows rows; *_f float32, *_b bfloat16
     DevBuf streams, x, h, y, in_f, in_b, proj_f, proj_b, gates, scanned, mix_f, mix_b, up_f, up_b, last_f, last_b, rows_dev, ws;
-    DevBuf q_b, keys_b, values_b;  // latent attention of a prompt: turned queries; one sequence's keys, and its values transposed
+    DevBuf q_b, keys_b, values_b;  // latent attention of a prompt: turned queries; all positions' keys, and their values transposed
 
     mi355x_status set_tensor(const char* tensor, int dtype, const void* host, int64_t n_elems) override;
     mi355x_status finalize(int64_t max_tokens) override;
@@ -90,7 +90,7 @@ struct Stack : Decoder {
     Recurrence recurrence(const StackLayer& l, int64_t s, bool tiles) const;
     mi355x_status pass(const int32_t* tokens, int64_t s, const int32_t* pos);
     mi355x_status mix(StackLayer& l, int64_t s, bool tiles, const int32_t* pos);
-    mi355x_status prompt_attention(const StackLayer& l, const Latent& a);
+    mi355x_status prompt_attention(const Latent& a, const Mat& o);
     // out = act(x . W[row0, row0 + n)^T) by the kernel for this many rows and x's form (bfloat16 if b, else float32)
     mi355x_status product(const Mat& w, int64_t row0, int64_t n, const DevBuf& f, const DevBuf& b, bool tiles, int64_t rows, const ProductOut& out);
 };
@@ -110,7 +110,7 @@ Latent Stack::latent(const StackLayer& l, int64_t s, const int32_t* pos) const {
     a.cos_t = l.cos_t.as<float>(); a.sin_t = l.sin_t.as<float>();
     a.norm_w = l.dkv_norm.p();
     a.w_uk = l.ukv.row(0); a.w_uv = l.ukv.row((int64_t)l.c.heads * l.c.dim); a.ldw = l.ukv.ld;
-    a.cache = l.cache.p; a.cache_bf16 = half(); a.ldc = l.ldc; a.context = context;
+    a.cache = l.cache.p; a.cache_bf16 = half(); a.ldc = l.ldc; a.context = pad64(context);
     a.batch = batch; a.s = s;
     a.past = pos ? 0 : cache_len; a.past_dev = pos;
     return a;
@@ -143,21 +143,24 @@ Recurrence Stack::recurrence(const StackLayer& l, int64_t s, bool tiles) const {
     return r;
 }
 
-// A prompt's latent attention, sequence by sequence: keys and transposed values of all positions from the cached
-// latents, then the attention on them.
-mi355x_status Stack::prompt_attention(const StackLayer& l, const Latent& a) {
-    const int64_t n = a.past + a.s, kn = (int64_t)a.heads * a.dim, vn = l.mixed(), ldv = pad64(context), qn = (int64_t)a.heads * (a.dim + a.rot_dim);
-    for (int b = 0; b < batch; b++) {
-        const uint16_t* latents = l.cache.as<uint16_t>() + (int64_t)b * context * a.ldc;
+// A prompt's latent attention: keys and transposed values of all positions from the cached latents, then the attention on
+// them. The sequences' caches lie one behind the other: one product for all of them where most of the capacity is held
+// (what lies behind a sequence's positions is finite and is not looked at), else one a sequence.
+mi355x_status Stack::prompt_attention(const Latent& a, const Mat& o) {
+    const int64_t n = a.past + a.s, kn = (int64_t)a.heads * a.dim, vn = (int64_t)a.heads * a.vdim, ldv = batch * a.context, qn = (int64_t)a.heads * (a.dim + a.rot_dim);
+    const bool at_once = batch > 1 && 2 * n > a.context;
+    for (int b = 0; b < (at_once ? 1 : batch); b++) {
+        const uint16_t* latents = (const uint16_t*)a.cache + b * a.context * a.ldc;
+        const int64_t rows = at_once ? batch * a.context : n;
         ProductOut k;
-        k.bf16 = keys_b.as<uint16_t>(); k.ld = kn;
-        STACK_HIP(gemm_bf16(a.w_uk, a.ldw, latents, a.ldc, n, kn, a.rank, k, stream), "keys");
+        k.bf16 = keys_b.as<uint16_t>() + b * a.context * kn; k.ld = kn;
+        STACK_HIP(gemm_bf16(a.w_uk, a.ldw, latents, a.ldc, rows, kn, a.rank, k, stream), "keys");
         ProductOut v;
-        v.bf16 = values_b.as<uint16_t>(); v.ld = ldv;
-        STACK_HIP(gemm_bf16(latents, a.ldc, a.w_uv, a.ldw, vn, n, a.rank, v, stream), "values");
-        STACK_HIP(latent_prompt(a, b, q_b.as<uint16_t>() + b * a.s * qn, qn, keys_b.as<uint16_t>(), kn, values_b.as<uint16_t>(), ldv,
-                                mix_b.as<uint16_t>() + b * a.s * l.o.ld, l.o.ld, stream), "latent attention");
+        v.bf16 = values_b.as<uint16_t>() + b * a.context; v.ld = ldv;
+        STACK_HIP(gemm_bf16(latents, a.ldc, a.w_uv, a.ldw, vn, rows, a.rank, v, stream), "values");
     }
+    STACK_HIP(latent_prompt(a, q_b.as<uint16_t>(), qn, keys_b.as<uint16_t>(), kn, values_b.as<uint16_t>(), ldv, mix_b.as<uint16_t>(), o.ld, stream),
+              "latent attention");
     return MI355X_OK;
 }
 
@@ -173,7 +176,7 @@ mi355x_status Stack::mix(StackLayer& l, int64_t s, bool tiles, const int32_t* po
         if (formed) {
             STACK_HIP(latent_prepare(a, proj_f.as<float>(), l.in.n, q_b.as<uint16_t>(), (int64_t)l.c.heads * (l.c.dim + l.c.rot_dim), stream),
                       "latents and rotation");
-            if (mi355x_status st = prompt_attention(l, a)) return st;
+            if (mi355x_status st = prompt_attention(a, l.o)) return st;
         } else {
             STACK_HIP(latent_absorbed(a, proj_f.as<float>(), l.in.n, ws.as<float>(), tiles ? nullptr : mix_f.as<float>(),
                                       tiles ? mix_b.as<uint16_t>() : nullptr, l.o.ld, stream), "latent attention");
@@ -426,8 +429,8 @@ mi355x_status Stack::finalize(int64_t max_tokens) {
         if (c.taps > 1) STACK_BUF(l.conv_state, (size_t)batch * (c.taps - 1) * W * 4);
         if (!l.recurrent()) {
             l.ldc = (l.c.kv_rank + l.c.rot_dim + 7) / 8 * 8;
-            // rows are read to a multiple of 64 elements of the latent: one row more than the context
-            STACK_BUF(l.cache, ((size_t)batch * context * l.ldc + pad64(l.ldc) + 64) * (half() ? 2 : 4));
+            // rows are read to a multiple of 64 elements of the latent: more than the last row has
+            STACK_BUF(l.cache, ((size_t)batch * pad64(context) * l.ldc + pad64(l.ldc) + 64) * (half() ? 2 : 4));
             const int half_n = l.c.rot_dim / 2;
             std::vector<float> cs((size_t)context * half_n), sn((size_t)context * half_n);
             for (int i = 0; i < half_n; i++) {
@@ -490,10 +493,9 @@ mi355x_status Stack::finalize(int64_t max_tokens) {
         STACK_BUF(gates, (size_t)R * gate_n * 4);
         STACK_BUF(last_b, (size_t)logit_rows * pad64(W) * 2);
         if (keys_n > 0) {
-            // a product reads rows of latents to a multiple of 64; whole tiles of 64 keys are read of the transposed values
             STACK_BUF(q_b, (size_t)R * q_n * 2);
-            STACK_BUF(keys_b, (size_t)context * keys_n * 2);
-            STACK_BUF(values_b, (size_t)values_n * pad64(context) * 2);
+            STACK_BUF(keys_b, (size_t)batch * pad64(context) * keys_n * 2);
+            STACK_BUF(values_b, (size_t)values_n * batch * pad64(context) * 2);  // read in whole tiles of 64 keys
         }
     }
 #undef STACK_BUF

@@ -123,7 +123,7 @@ struct Latent {
     const uint16_t* w_uk = nullptr;                  // [heads * dim, rank], rows ldw apart
     const uint16_t* w_uv = nullptr;                  // [heads * vdim, rank]
     int64_t ldw = 0;
-    void* cache = nullptr;  // [batch, context, ldc]
+    void* cache = nullptr;  // [batch, context, ldc]: context is the capacity
     bool cache_bf16 = false;
     int64_t ldc = 0;
     int64_t context = 0;
@@ -141,12 +141,11 @@ hipError_t latent_prepare(const Latent& a, const float* proj, int64_t ldp, uint1
 int latent_splits(const Latent& a);
 size_t latent_absorbed_ws_floats(const Latent& a, int64_t rows);
 hipError_t latent_absorbed(const Latent& a, const float* proj, int64_t ldp, float* ws, float* out_f32, uint16_t* out_bf16, int64_t ldo, hipStream_t st);
-// Many query rows of one sequence (bfloat16 cache and queries), on keys and values formed beforehand for all its past + s
-// positions: keys [positions, heads * dim], values transposed [heads * vdim, positions], rows ldk and ldv (a multiple of
-// 64) elements apart. q, out: the sequence's rows. Products on the bfloat16 matrix cores; a weight goes to them as the
-// sum of two bfloat16.
+// Many query rows (bfloat16 cache and queries), on keys and values formed beforehand for all past + s positions of every
+// sequence: keys [batch * context, heads * dim], values transposed [heads * vdim, batch * context], rows ldk and ldv elements
+// apart; context a multiple of 64. Products on the bfloat16 matrix cores; a weight goes to them as the sum of two bfloat16.
 bool latent_prompt_ok(const Latent& a);
-hipError_t latent_prompt(const Latent& a, int sequence, const uint16_t* q, int64_t ldq, const uint16_t* keys, int64_t ldk, const uint16_t* values_t,
-                         int64_t ldv, uint16_t* out, int64_t ldo, hipStream_t st);
+hipError_t latent_prompt(const Latent& a, const uint16_t* q, int64_t ldq, const uint16_t* keys, int64_t ldk, const uint16_t* values_t, int64_t ldv,
+                         uint16_t* out, int64_t ldo, hipStream_t st);
 
 }  // namespace mimir
