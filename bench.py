@@ -452,7 +452,7 @@ def build_fuvolix(capi, kinds, size, batch, context, max_tokens, vocab=32768):
     return m
 
 
-def fuvolix_bench(capi, sizes=("4096", "2048"), kinds=("latent_attention", "mlstm", "lightning"), prompts=((1, 2048), (8, 512)), new=65, layers=(2, 6)):
+def fuvolix_bench(capi, sizes=("4096", "2048"), kinds=("latent_attention", "mlstm", "lightning"), prompts=((1, 2048), (8, 512)), new=65, layers=(2, 6), llama=True):
     """Prompt passes and decoding of the Fuvolix design's three kinds of layer, beside the Llama decoder's (Q4_0) at equal
     width, feed-forward and heads: microseconds a layer (models of two and of six layers; the difference over four, so
     that embedding and head drop out), the best of three runs."""
@@ -460,7 +460,7 @@ def fuvolix_bench(capi, sizes=("4096", "2048"), kinds=("latent_attention", "mlst
     for size in sizes:
         width, ff, heads = FUVOLIX_SIZES[size]
         kv_heads = max(1, heads // 4)
-        for kind in kinds + ("llama_q4_0",):
+        for kind in kinds + (("llama_q4_0",) if llama else ()):
             for batch, prompt in prompts:
                 secs = {}
                 for n in layers:
@@ -752,6 +752,7 @@ def main():
                     help="block dtype of the decoder's linear weights (the oracle check is for q4_0)")
     ap.add_argument("--fuvolix", action="store_true", help="only: prompt passes and decoding of the Fuvolix design's layers at sizes like a real model's, beside the Llama decoder's")
     ap.add_argument("--fuvolix-only", default=None, metavar="SIZE[:KIND[:BATCHxPROMPT]]", help="with --fuvolix: one size, kind of layer, call (for profiles)")
+    ap.add_argument("--fuvolix-no-llama", action="store_true", help="with --fuvolix: without the Llama decoder's figures")
     ap.add_argument("--tune", action="append", default=[], metavar="KEY=VALUE",
                     help="a launch-plan override for mi355x_tune before anything runs (may be repeated), e.g. q4_0.stream=1")
     args = ap.parse_args()
@@ -769,7 +770,7 @@ def main():
         capi.check(lib.mi355x_tune(key.encode(), int(val)))
 
     if args.fuvolix:
-        kw = {}
+        kw = {"llama": not args.fuvolix_no_llama}
         if args.fuvolix_only:
             parts = args.fuvolix_only.split(":")
             kw["sizes"] = (parts[0],)
