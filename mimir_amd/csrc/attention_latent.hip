@@ -258,10 +258,10 @@ __global__ __launch_bounds__(256) void latent_attend_kernel(Latent a, const floa
     }
 }
 
-// The same on the matrix cores, a bfloat16 cache: tiles of 64 keys in LDS, 32 heads a workgroup. Scores: the wavefronts cut the
-// features into four (KS steps of 32 each at most), queries as the sum of two bfloat16 in registers, and the four partial
-// sums meet in LDS, where eight threads a head do the softmax. Sum of latents: the wavefronts cut the latent's features
-// (RT tiles of sixteen each at most), weights as the sum of two bfloat16.
+// The same on the matrix cores, a bfloat16 cache: tiles of 64 keys in LDS, 32 heads a workgroup. Scores: the eight
+// wavefronts cut the features (KS steps of 32 each), queries as the sum of two bfloat16 in registers, and the partial
+// sums meet in LDS, where sixteen threads a head do the softmax. Sum of latents: the wavefronts cut the latent's features
+// (RT tiles of sixteen each), weights as the sum of two bfloat16.
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
@@ -269,21 +269,27 @@ __device__ __forceinline__ f32x4 mfma16_bf16(u32x4 a, u32x4 b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
 }
 
-constexpr int kMHeads = 32;
+constexpr int kMHeads = 32, kMWaves = 8;
 constexpr int kScoreLd = kMHeads + 1, kWeightLd = kKeys + 8;
 
-size_t attend_mfma_lds(const Latent& a) {
-    const int lq = (a.rank + a.rot_dim + 31) / 32 * 32;
-    return (size_t)kKeys * (lq + 8) * 2 + (size_t)4 * kKeys * kScoreLd * 4 + (size_t)2 * kMHeads * kWeightLd * 2 + kMHeads * 4;
+// Features of a tile's row in LDS: a constant, so that the addresses of a column are one register and immediate offsets.
+int attend_mfma_row(const Latent& a) {
+    const int n = a.rank + a.rot_dim;
+    return n <= 128 ? 128 : n <= 256 ? 256 : n <= 576 ? 576 : 640;
 }
+constexpr size_t attend_mfma_lds(int lq) {
+    return (size_t)kKeys * (lq + 8) * 2 + (size_t)kMWaves * kKeys * kScoreLd * 4 + (size_t)2 * kMHeads * kWeightLd * 2 + kMHeads * 4;
+}
+static_assert(attend_mfma_lds(640) <= 160 * 1024, "a compute unit's LDS");
 
-template <int KS, int RT>
-__global__ __launch_bounds__(256) void latent_attend_mfma_kernel(Latent a, const float* __restrict__ qa, int splits, float* __restrict__ part_o,
-                                                                 float* __restrict__ part_ml) {
+template <int LQ>
+__global__ __launch_bounds__(64 * kMWaves) void latent_attend_mfma_kernel(Latent a, const float* __restrict__ qa, int splits, float* __restrict__ part_o,
+                                                                              float* __restrict__ part_ml) {
     extern __shared__ __align__(16) float lds_latent[];
-    const int lq = query_ld(a), ldt = lq + 8, steps = lq / 32, L = a.rank + a.rot_dim;
-    float* ps = lds_latent;                                    // [4][kKeys][kScoreLd]
-    float* back = ps + 4 * kKeys * kScoreLd;                   // [kMHeads]
+    constexpr int ldt = LQ + 8, steps = LQ / 32, KS = (steps + kMWaves - 1) / kMWaves, RT = LQ <= 128 ? 1 : LQ <= 256 ? 2 : 4;
+    const int lq = query_ld(a), L = a.rank + a.rot_dim;
+    float* ps = lds_latent;                                    // [kMWaves][kKeys][kScoreLd]
+    float* back = ps + kMWaves * kKeys * kScoreLd;             // [kMHeads]
     uint16_t* tile = (uint16_t*)(back + kMHeads);              // [kKeys][ldt]
     uint16_t* wH = tile + (size_t)kKeys * ldt;                 // [kMHeads][kWeightLd], high parts
     uint16_t* wL = wH + kMHeads * kWeightLd;                   // low parts
@@ -295,15 +301,33 @@ __global__ __launch_bounds__(256) void latent_attend_mfma_kernel(Latent a, const
     const int64_t pr = (r * splits + split) * a.heads;
     if (lo >= hi) return;  // the whole workgroup: latent_combine_kernel does not look at this share
     const uint16_t* cache = (const uint16_t*)a.cache + b * a.context * a.ldc;
-    // this wavefront's steps of the features: wave, wave + 4, ...
+    // a tile's pieces of 16 bytes, this thread's: all requested at once, the first tile's before the queries
+    constexpr int pieces = LQ / 8, kPieces = kKeys * pieces / (64 * kMWaves);
+    auto each_piece = [&](auto body) {
+#pragma unroll
+        for (int u = 0; u < kPieces; u++) {
+            const int i = tid + 64 * kMWaves * u;
+            body(u, i / pieces, i % pieces * 8);
+        }
+    };
+    u32x4 piece[kPieces];
+    auto fetch = [&](int64_t j0) {
+        each_piece([&](int u, int j, int d) {
+            const int64_t row = j0 + j < hi ? j0 + j : hi - 1;
+            piece[u] = u32x4{0, 0, 0, 0};
+            if (d < L) piece[u] = *(const u32x4*)(cache + row * a.ldc + d);  // a row is padded with zeros to a multiple of 8
+        });
+    };
+    fetch(lo);
+    // this wavefront's steps of the features: wave, wave + kMWaves, ...
     u32x4 qh[KS][2], ql[KS][2];
 #pragma unroll
     for (int i = 0; i < KS; i++)
 #pragma unroll
         for (int t = 0; t < 2; t++) {
-            const int h = h0 + t * 16 + r16, step = wave + 4 * i;
+            const int h = h0 + t * 16 + r16, step = wave + kMWaves * i;
             f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = x;
-            if (h < a.heads && step < steps) {
+            if (h < a.heads && step * 32 < lq) {
                 const f32x4* q = (const f32x4*)(qa + (r * a.heads + h) * lq + step * 32 + g * 8);
                 x = q[0];
                 y = q[1];
@@ -317,26 +341,14 @@ __global__ __launch_bounds__(256) void latent_attend_mfma_kernel(Latent a, const
     for (int t = 0; t < RT; t++)
 #pragma unroll
         for (int i = 0; i < 2; i++) acc[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const int sh = tid >> 3, sk = tid & 7;  // the softmax's head and first key of this thread
+    const int sh = tid >> 4, sk = tid & 15;  // the softmax's head and first key of this thread
     float m = -__builtin_inff(), l = 0.f;
-    const int pieces = lq / 8;
     for (int64_t j0 = lo; j0 < hi; j0 += kKeys) {
-        for (int i0 = tid; i0 < kKeys * pieces; i0 += 6 * 256) {  // six pieces requested at a time
-            u32x4 v[6];
-#pragma unroll
-            for (int u = 0; u < 6; u++) {
-                const int i = i0 + 256 * u, j = i / pieces, d = i % pieces * 8;
-                const int64_t row = j0 + j < hi ? j0 + j : hi - 1;
-                v[u] = u32x4{0, 0, 0, 0};
-                if (i < kKeys * pieces && d < L) v[u] = *(const u32x4*)(cache + row * a.ldc + d);  // a row is padded with zeros to a multiple of 8
-            }
-#pragma unroll
-            for (int u = 0; u < 6; u++) {
-                const int i = i0 + 256 * u, j = i / pieces, d = i % pieces * 8;
-                if (i < kKeys * pieces) *(u32x4*)(tile + j * ldt + d) = v[u];
-            }
-        }
+        each_piece([&](int u, int j, int d) {
+            *(u32x4*)(tile + j * ldt + d) = piece[u];
+        });
         __syncthreads();
+        if (j0 + kKeys < hi) fetch(j0 + kKeys);
         f32x4 sc[4][2];
 #pragma unroll
         for (int k = 0; k < 4; k++)
@@ -344,7 +356,7 @@ __global__ __launch_bounds__(256) void latent_attend_mfma_kernel(Latent a, const
             for (int t = 0; t < 2; t++) sc[k][t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int i = 0; i < KS; i++) {
-            const int step = wave + 4 * i;
+            const int step = wave + kMWaves * i;
             if (step >= steps) break;
 #pragma unroll
             for (int k = 0; k < 4; k++) {
@@ -364,28 +376,29 @@ __global__ __launch_bounds__(256) void latent_attend_mfma_kernel(Latent a, const
                 for (int i = 0; i < 4; i++) ps[(wave * kKeys + k * 16 + 4 * g + i) * kScoreLd + t * 16 + r16] = sc[k][t][i];
         __syncthreads();
         {
-            float s[8], top = -__builtin_inff();
+            float s[4], top = -__builtin_inff();
 #pragma unroll
-            for (int i = 0; i < 8; i++) {
-                const int j = sk * 8 + i;
+            for (int i = 0; i < 4; i++) {
+                const int j = sk * 4 + i;
                 float v = 0.f;
 #pragma unroll
-                for (int w = 0; w < 4; w++) v += ps[(w * kKeys + j) * kScoreLd + sh];
+                for (int w = 0; w < kMWaves; w++) v += ps[(w * kKeys + j) * kScoreLd + sh];
                 s[i] = j0 + j < hi ? v : -__builtin_inff();
                 top = fmaxf(top, s[i]);
             }
             top = group8_max(top);
+            top = fmaxf(top, __shfl_xor(top, 8));
             const float next = fmaxf(m, top), scale = expf(m - next);  // the first tile's m: exp(-inf) = 0
             float sum = 0.f;
 #pragma unroll
-            for (int i = 0; i < 8; i++) {
+            for (int i = 0; i < 4; i++) {
                 s[i] = expf(s[i] - next);
                 sum += s[i];
             }
-            *(u32x4*)(wH + sh * kWeightLd + sk * 8) = u32x4{pack_bf16(s[0], s[1]), pack_bf16(s[2], s[3]), pack_bf16(s[4], s[5]), pack_bf16(s[6], s[7])};
-            *(u32x4*)(wL + sh * kWeightLd + sk * 8) = u32x4{pack_bf16(low_part(s[0]), low_part(s[1])), pack_bf16(low_part(s[2]), low_part(s[3])),
-                                                            pack_bf16(low_part(s[4]), low_part(s[5])), pack_bf16(low_part(s[6]), low_part(s[7]))};
-            l = l * scale + group8_sum(sum);
+            *(u32x2*)(wH + sh * kWeightLd + sk * 4) = u32x2{pack_bf16(s[0], s[1]), pack_bf16(s[2], s[3])};
+            *(u32x2*)(wL + sh * kWeightLd + sk * 4) = u32x2{pack_bf16(low_part(s[0]), low_part(s[1])), pack_bf16(low_part(s[2]), low_part(s[3]))};
+            sum = group8_sum(sum);
+            l = l * scale + (sum + __shfl_xor(sum, 8));
             m = next;
             if (sk == 0) back[sh] = scale;
         }
@@ -407,7 +420,7 @@ __global__ __launch_bounds__(256) void latent_attend_mfma_kernel(Latent a, const
             }
 #pragma unroll
             for (int k = 0; k < RT; k++) {
-                const int c0 = (wave + 4 * k) * 16;
+                const int c0 = (wave + kMWaves * k) * 16;
                 if (c0 >= a.rank) break;
                 // eight keys of one feature: a column of the tile (features past the rank are the rotated part or zeros: not stored)
                 const uint16_t* col = tile + (half * 32 + g * 8) * ldt + c0 + r16;
@@ -425,7 +438,7 @@ __global__ __launch_bounds__(256) void latent_attend_mfma_kernel(Latent a, const
     }
 #pragma unroll
     for (int k = 0; k < RT; k++) {
-        const int c = (wave + 4 * k) * 16 + r16;
+        const int c = (wave + kMWaves * k) * 16 + r16;
 #pragma unroll
         for (int t = 0; t < 2; t++)
 #pragma unroll
@@ -521,19 +534,17 @@ hipError_t launch_attend(const Latent& a, const float* qa, int splits, float* po
     return hipGetLastError();
 }
 
-template <int KS, int RT>
+template <int LQ>
 hipError_t launch_attend_mfma(const Latent& a, const float* qa, int splits, float* po, float* ml, hipStream_t st) {
-    const size_t lds = attend_mfma_lds(a);
-    hipError_t e = hipFuncSetAttribute((const void*)latent_attend_mfma_kernel<KS, RT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    constexpr size_t lds = attend_mfma_lds(LQ);
+    hipError_t e = hipFuncSetAttribute((const void*)latent_attend_mfma_kernel<LQ>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return e;
     const dim3 grid((unsigned)splits, (unsigned)((a.heads + kMHeads - 1) / kMHeads), (unsigned)(a.batch * a.s));
-    hipLaunchKernelGGL((latent_attend_mfma_kernel<KS, RT>), grid, dim3(256), lds, st, a, qa, splits, po, ml);
+    hipLaunchKernelGGL(latent_attend_mfma_kernel<LQ>, grid, dim3(64 * kMWaves), lds, st, a, qa, splits, po, ml);
     return hipGetLastError();
 }
 
-bool attend_mfma_ok(const Latent& a) {
-    return a.cache_bf16 && a.rank <= 512 && a.rank + a.rot_dim <= 640 && a.ldc % 8 == 0 && attend_mfma_lds(a) <= 160 * 1024;
-}
+bool attend_mfma_ok(const Latent& a) { return a.cache_bf16 && a.rank <= 512 && a.rank + a.rot_dim <= 640 && a.ldc % 8 == 0; }
 
 // ---- many query rows ------------------------------------------------------------------------
 // A wavefront owns 32 query rows of one head and walks the keys in tiles of 64 with a running maximum and sum per row.
@@ -757,8 +768,12 @@ hipError_t latent_absorbed(const Latent& a, const float* proj, int64_t ldp, floa
     hipLaunchKernelGGL(latent_queries_kernel, dim3((unsigned)rows, (unsigned)a.heads, (unsigned)((a.rank + kAbsorbCols - 1) / kAbsorbCols)), dim3(256), 0, st, a,
                        proj, ldp, qa);
     hipError_t e;
+    const int row = attend_mfma_row(a);
     if (attend_mfma_ok(a))
-        e = a.rank + a.rot_dim <= 256 ? launch_attend_mfma<2, 4>(a, qa, splits, po, ml, st) : launch_attend_mfma<5, 8>(a, qa, splits, po, ml, st);
+        e = row == 128   ? launch_attend_mfma<128>(a, qa, splits, po, ml, st)
+            : row == 256 ? launch_attend_mfma<256>(a, qa, splits, po, ml, st)
+            : row == 576 ? launch_attend_mfma<576>(a, qa, splits, po, ml, st)
+                         : launch_attend_mfma<640>(a, qa, splits, po, ml, st);
     else if (a.cache_bf16)
         e = a.rank <= 256   ? launch_attend<uint16_t, 1>(a, qa, splits, po, ml, st)
             : a.rank <= 512 ? launch_attend<uint16_t, 2>(a, qa, splits, po, ml, st)

@@ -225,6 +225,8 @@ SIZES = {
                            width=256, groups=4),
     "wider_heads": X.config([X.latent(heads=2, dim=192, rot_dim=32, vdim=160, kv_rank=600), X.mlstm(heads=1, dim=256, vdim=64), X.lightning(heads=2, dim=64, vdim=256)], width=192),
     "past_the_prompt_kernel": X.config([X.latent(heads=2, dim=300, rot_dim=10, vdim=288, kv_rank=96)], width=96),
+    "latents": X.config([X.latent(heads=35, dim=16, rot_dim=104, vdim=16, kv_rank=504), X.latent(heads=4, dim=8, rot_dim=40, vdim=40, kv_rank=200),
+                         X.latent(heads=4, dim=8, rot_dim=6, vdim=24, kv_rank=124)], width=96),
     "eight_rows_wide": X.config([X.latent(heads=2, dim=96, rot_dim=24, vdim=72, kv_rank=88), X.mlstm(heads=3, dim=24, vdim=104)], width=2080, groups=13),
 }
 
