@@ -331,37 +331,58 @@ MI355X_API mi355x_status mi355x_llama_generate(void* model, const int32_t* promp
 
 /* ---- the mixer stack ------------------------------------------------------------
  * A decoder whose layers are a list of mixers with sizes of their own, beside the
- * reference's architectures (which have no counterpart of it): norms in groups
- * before and after every sublayer, a short causal convolution in front of every
- * mixer, an average over all earlier layers' results behind every layer, and the
- * embedding table as output matrix. A handle takes the mi355x_model_* calls;
- * tensors have the names of the model's file (embed, l0.norm1, l0.mix.q, ...) and
- * are bfloat16. */
-enum { MI355X_MIXER_LATENT = 1, MI355X_MIXER_MLSTM = 2, MI355X_MIXER_LIGHTNING = 3 };
+ * reference's architectures (which have no counterpart of it). What surrounds the
+ * mixers is chosen by flags. A handle takes the mi355x_model_* calls; tensors have
+ * the names of the model's file (embed, l0.norm1, l0.mix.q, ...) and are bfloat16. */
+enum { MI355X_MIXER_LATENT = 1, MI355X_MIXER_MLSTM = 2, MI355X_MIXER_LIGHTNING = 3, MI355X_MIXER_ATTENTION = 4 };
+enum { MI355X_MLP_RELU2 = 0, /* down (max(0, up h)^2) */
+       MI355X_MLP_SWIGLU = 1 /* down (silu(gate h) * (up h)) */ };
 
 typedef struct mi355x_stack_layer {
     int32_t mixer;    /* MI355X_MIXER_* */
     int32_t heads;
+    int32_t kv_heads; /* attention: key and value heads, a divisor of heads (neighbouring heads share one) */
     int32_t dim;      /* features of a query and key (latent attention: of their part without positions) */
     int32_t vdim;     /* features of a value */
-    int32_t rot_dim;  /* latent attention: rotated features of a query and key, interleaved pairs */
+    int32_t rot_dim;  /* latent attention: rotated features of a query and key, interleaved pairs; attention: of its
+                       * first features, i with i + rot_dim / 2 (0: no rotation) */
     int32_t kv_rank;  /* latent attention: size of the latent */
-    int32_t ff;       /* rows of the feed-forward's up matrix (squared ReLU), 0: no feed-forward */
-    int32_t reserved;
-    double scale;     /* latent attention: of the scores */
+    int32_t ff;       /* inner size of the feed-forward, 0: no feed-forward */
+    int32_t mlp;      /* MI355X_MLP_* */
+    int32_t unit_qk;  /* attention: queries and keys over their root mean square */
+    int32_t value_mix; /* attention: values mixed with those of the first layer that has this */
+    int32_t head_gate; /* attention: a head's result times the sigmoid of a gate */
+    double scale;     /* attention and latent attention: of the scores */
+    double softcap;   /* attention: score <- softcap tanh(score / softcap); 0: not */
     double rot_base;
+    double rot_factor, rot_low, rot_high, rot_original; /* attention: Llama 3.1's scaling of the frequencies; factor 0: none */
     double gate_cap;  /* mLSTM: soft cap of its two gates */
     const double* decay; /* lightning attention: [heads] */
 } mi355x_stack_layer;
+
+enum {
+    MI355X_STACK_EMBED_NORM = 1,     /* a norm of the embedding's row */
+    MI355X_STACK_POST_NORMS = 2,     /* a norm of every sublayer's result */
+    MI355X_STACK_DEPTH_AVERAGE = 4,  /* behind a layer, an average over the embedding output and all layers' results */
+    MI355X_STACK_PARALLEL = 8,       /* mixer and feed-forward read the same norm and are added together (attention only;
+                                      * without convolution, norms of results and average) */
+    MI355X_STACK_LAYER_SCALE = 16,   /* a factor for every feature of a sublayer's result */
+    MI355X_STACK_OUTPUT_MATRIX = 32  /* an output matrix of its own; else the embedding table */
+};
 
 typedef struct mi355x_stack_config {
     int32_t width, vocab, layers;
     int32_t context;      /* capacity of the caches, in positions */
     int32_t batch;
-    int32_t taps;         /* of the causal convolutions */
+    int32_t taps;         /* of the causal convolution in front of every mixer, 0: none */
     int32_t norm_groups;
     int32_t dtype;        /* MI355X_BF16: prompts on the bfloat16 matrix cores; MI355X_F32: float32 throughout */
+    int32_t flags;        /* MI355X_STACK_* */
+    int32_t reserved;
+    int64_t pair_buckets; /* rows of a second table, added to the embedding: (previous token * mul_prev + token * mul_cur) */
+    int64_t pair_mul_prev, pair_mul_cur; /* mod pair_buckets, for a first token row pair_buckets; 0 buckets: none */
     double eps;
+    double logit_scale;
 } mi355x_stack_config;
 
 MI355X_API mi355x_status mi355x_stack_create(const mi355x_stack_config* cfg, const mi355x_stack_layer* layers, void** model);

@@ -29,7 +29,7 @@ FLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-fvisibility=h
 
 # Sources that make a library of their own: what the decoders of one kind need.
 PARTS = {
-    "stack": ("runtime", "decoder", "stack", "residual_ops", "linear_recurrence", "attention_latent", "gemv_float", "gemv_bf16_rows",
+    "stack": ("runtime", "decoder", "stack", "residual_ops", "linear_recurrence", "attention_latent", "attention_heads", "gemv_float", "gemv_bf16_rows",
               "gemm_float", "gemm_bf16", "decode_ops"),
 }
 

@@ -100,18 +100,22 @@ class LlamaConfig(C.Structure):
                                           "interleaved", "cache_dtype", "batch")] + [(n, C.c_double) for n in ("rope_base", "rope_scale", "eps")]
 
 
-MIXER_LATENT, MIXER_MLSTM, MIXER_LIGHTNING = 1, 2, 3
+MIXER_LATENT, MIXER_MLSTM, MIXER_LIGHTNING, MIXER_ATTENTION = 1, 2, 3, 4
+MLP_RELU2, MLP_SWIGLU = 0, 1
+STACK_EMBED_NORM, STACK_POST_NORMS, STACK_DEPTH_AVERAGE, STACK_PARALLEL, STACK_LAYER_SCALE, STACK_OUTPUT_MATRIX = 1, 2, 4, 8, 16, 32
 
 
 class StackConfig(C.Structure):
     """mi355x_stack_config."""
-    _fields_ = [(n, C.c_int32) for n in ("width", "vocab", "layers", "context", "batch", "taps", "norm_groups", "dtype")] + [("eps", C.c_double)]
+    _fields_ = [(n, C.c_int32) for n in ("width", "vocab", "layers", "context", "batch", "taps", "norm_groups", "dtype", "flags", "reserved")] + \
+               [(n, C.c_int64) for n in ("pair_buckets", "pair_mul_prev", "pair_mul_cur")] + [("eps", C.c_double), ("logit_scale", C.c_double)]
 
 
 class StackLayer(C.Structure):
     """mi355x_stack_layer."""
-    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "dim", "vdim", "rot_dim", "kv_rank", "ff", "reserved")] + \
-               [(n, C.c_double) for n in ("scale", "rot_base", "gate_cap")] + [("decay", C.POINTER(C.c_double))]
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "vdim", "rot_dim", "kv_rank", "ff", "mlp", "unit_qk", "value_mix", "head_gate")] + \
+               [(n, C.c_double) for n in ("scale", "softcap", "rot_base", "rot_factor", "rot_low", "rot_high", "rot_original", "gate_cap")] + \
+               [("decay", C.POINTER(C.c_double))]
 
 
 class AttentionDesc(C.Structure):

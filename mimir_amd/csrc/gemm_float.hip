@@ -5,6 +5,7 @@
 // few rows, a workgroup owns 16 rows of x and up to 64 of W instead, and its eight wavefronts cut K
 // (gemm_f32_narrow_kernel): the tiles above would leave most of the device without work.
 #include "device_util.h"
+#include "product_store.h"
 #include "stack_ops.h"
 
 namespace mimir {
@@ -56,16 +57,19 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const uint16_t* __restric
             part = __builtin_amdgcn_mfma_f32_32x32x2f32(xs[p][(wm + r32) * kPad + k + hi], ws[p][(wn + r32) * kPad + k + hi], part, 0, 0, 0);
 #pragma unroll
         for (int i = 0; i < 16; i++) acc[i] += part[i];
+        if (out.mid && k0 + kStep == out.split) {
+            const float f = out.mid[n0 + wn + r32 < N ? n0 + wn + r32 : N - 1];
+#pragma unroll
+            for (int i = 0; i < 16; i++) acc[i] *= f;
+        }
     }
 #pragma unroll
     for (int i = 0; i < 16; i++) {
         const int64_t m = m0 + wm + (i & 3) + 8 * (i >> 2) + 4 * hi, n = n0 + wn + r32;
+        const float beside = __shfl_xor(acc[i], 1);  // the column beside this one
         if (m >= M || n >= N) continue;
-        float v = acc[i];
-        if (out.relu2) v = v > 0.f ? v * v : 0.f;
-        else if (n < out.silu_n) v = v / (1.f + expf(-v));
-        if (out.f32) out.f32[m * out.ld + n] = v;
-        else out.bf16[m * out.ld + n] = round_bf16(v);
+        if (n < out.pair_from) store_column(out, m, n, acc[i]);
+        else if ((n & 1) == 0) store_pair(out, m, n, acc[i], beside);
     }
 }
 
@@ -73,6 +77,8 @@ constexpr int kNarrow = 64;  // rows of W a workgroup
 
 // v_mfma_f32_16x16x4: lane (row, k). A lane brings four neighbouring elements of K of its row, so the four products of a step
 // of sixteen take K in the order 4 k + j, in both operands alike.
+// TWO: the sums below and from out.split on have factors of their own.
+template <bool TWO>
 __global__ __launch_bounds__(512) void gemm_f32_narrow_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx, int64_t M,
                                                               int64_t N, int64_t K, ProductOut out) {
     __shared__ float red[8][16][kNarrow + 1];
@@ -86,18 +92,29 @@ __global__ __launch_bounds__(512) void gemm_f32_narrow_kernel(const uint16_t* __
     f32x4 acc[kNarrow / 16];
 #pragma unroll
     for (int t = 0; t < kNarrow / 16; t++) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    auto sum_of = [&](int64_t from, int64_t to) {
 #pragma unroll 4
-    for (int64_t k = k0; k < k1; k += 16) {  // both operands' rows are padded to a multiple of 64
-        const f32x4 a = *(const f32x4*)(xp + k);
-        u32x2 w[kNarrow / 16];
+        for (int64_t k = from; k < to; k += 16) {  // both operands' rows are padded to a multiple of 64
+            const f32x4 a = *(const f32x4*)(xp + k);
+            u32x2 w[kNarrow / 16];
 #pragma unroll
-        for (int t = 0; t < kNarrow / 16; t++) w[t] = *(const u32x2*)(wp[t] + k);
+            for (int t = 0; t < kNarrow / 16; t++) w[t] = *(const u32x2*)(wp[t] + k);
 #pragma unroll
-        for (int t = 0; t < kNarrow / 16; t++)
+            for (int t = 0; t < kNarrow / 16; t++)
 #pragma unroll
-            for (int j = 0; j < 4; j++)
-                acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], __uint_as_float(j & 1 ? w[t][j >> 1] & 0xffff0000u : w[t][j >> 1] << 16), acc[t], 0, 0, 0);
+                for (int j = 0; j < 4; j++)
+                    acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], __uint_as_float(j & 1 ? w[t][j >> 1] & 0xffff0000u : w[t][j >> 1] << 16), acc[t], 0, 0, 0);
+        }
+    };
+    int64_t from = k0;
+    if constexpr (TWO) {  // what of this wavefront's piece lies below split
+        const int64_t to = out.split < k1 ? out.split : k1;
+        sum_of(k0, to);
+#pragma unroll
+        for (int t = 0; t < kNarrow / 16; t++) acc[t] = acc[t] * out.mid[n0 + t * 16 + r16 < N ? n0 + t * 16 + r16 : N - 1];
+        if (to > from) from = to;
     }
+    sum_of(from, k1);
 #pragma unroll
     for (int t = 0; t < kNarrow / 16; t++)
 #pragma unroll
@@ -107,13 +124,14 @@ __global__ __launch_bounds__(512) void gemm_f32_narrow_kernel(const uint16_t* __
         const int row = o / kNarrow, col = o % kNarrow;
         const int64_t m = m0 + row, n = n0 + col;
         if (m >= M || n >= N) continue;
-        float v = 0.f;
+        auto sum = [&](int c) {
+            float v = 0.f;
 #pragma unroll
-        for (int i = 0; i < 8; i++) v += red[i][row][col];
-        if (out.relu2) v = v > 0.f ? v * v : 0.f;
-        else if (n < out.silu_n) v = v / (1.f + expf(-v));
-        if (out.f32) out.f32[m * out.ld + n] = v;
-        else out.bf16[m * out.ld + n] = round_bf16(v);
+            for (int i = 0; i < 8; i++) v += red[i][row][c];
+            return v;
+        };
+        if (n < out.pair_from) store_column(out, m, n, sum(col));
+        else if ((col & 1) == 0) store_pair(out, m, n, sum(col), sum(col + 1));
     }
 }
 
@@ -122,8 +140,9 @@ __global__ __launch_bounds__(512) void gemm_f32_narrow_kernel(const uint16_t* __
 hipError_t gemm_f32(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st) {
     if (M == 0 || N == 0) return hipSuccess;
     if (N <= 2 * kNarrow && ldx % 4 == 0 && ldw % 4 == 0) {
-        hipLaunchKernelGGL(gemm_f32_narrow_kernel, dim3((unsigned)((N + kNarrow - 1) / kNarrow), (unsigned)((M + 15) / 16)), dim3(512), 0, st, W, ldw, x, ldx, M, N,
-                           K, out);
+        const dim3 grid((unsigned)((N + kNarrow - 1) / kNarrow), (unsigned)((M + 15) / 16));
+        if (out.mid) hipLaunchKernelGGL(gemm_f32_narrow_kernel<true>, grid, dim3(512), 0, st, W, ldw, x, ldx, M, N, K, out);
+        else hipLaunchKernelGGL(gemm_f32_narrow_kernel<false>, grid, dim3(512), 0, st, W, ldw, x, ldx, M, N, K, out);
         return hipGetLastError();
     }
     hipLaunchKernelGGL(gemm_f32_kernel, dim3((unsigned)((N + kTile - 1) / kTile), (unsigned)((M + kTile - 1) / kTile)), dim3(256), 0, st, W, ldw, x, ldx, M,

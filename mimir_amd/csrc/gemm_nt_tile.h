@@ -62,6 +62,8 @@ __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(
 // Y [m0 .. m0 + BM) x [n0 .. n0 + BN) of X [M, K] (rows ldx apart) by P [N, K] (rows ldp apart), float32 sums; K a
 // multiple of 64, rows 16-byte aligned. store.row(m, M) is called once a row (also for rows past M), then
 // store(m, n, N, its value, v) with the results of columns n .. n + 3 (n < N; those past N are not to be stored).
+// After the first store.first_steps(steps) of the steps of K the sums so far are multiplied by store.mid(n, N) (called for
+// columns past N too); a store object without such a factor returns `steps`.
 template <class T, class E, class S>
 __device__ __forceinline__ void tile_body(const uint16_t* __restrict__ X16, int64_t ldx, const uint16_t* __restrict__ P, int64_t ldp, const S& store, int M,
                                           int N, int K, int m0, int n0, char* lds) {
@@ -114,7 +116,18 @@ __device__ __forceinline__ void tile_body(const uint16_t* __restrict__ X16, int6
         load_to_lds(from[j], __builtin_amdgcn_readfirstlane(lds0 + into[j]));
         from[j] += kRowBytes;
     }
+    const int first = store.first_steps(nk);
     for (int i = 0; i < nk; i++) {
+        if (i == first) {  // the sums over the first steps have a factor of their own (a lane has one column)
+#pragma unroll
+            for (int nt = 0; nt < NT; nt++) {
+                const float f = store.mid(n0 + wn * 32 * NT + nt * 32 + r32, N);
+#pragma unroll
+                for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+                    for (int e = 0; e < 16; e++) acc[mt][nt][e] *= f;
+            }
+        }
         wait_loads();   // this wavefront's part of step i has landed
         lds_barrier();  // everyone's has, and everyone has read the other stage for the last time
         const bool more = i + 1 < nk;

@@ -5,6 +5,7 @@
 // product. The wavefronts of a workgroup (eight, or sixteen for long rows) share its rows of W and cut K into pieces; W goes from memory straight into
 // the operand registers (a lane's sixteen bytes of one row), x is converted on the way.
 #include "device_util.h"
+#include "product_store.h"
 #include "stack_ops.h"
 
 namespace mimir {
@@ -13,8 +14,8 @@ namespace {
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
-// T: groups of sixteen rows of W a workgroup.
-template <int T, int kWaves>
+// T: groups of sixteen rows of W a workgroup. TWO: the sums below and from out.split on have factors of their own.
+template <int T, int kWaves, bool TWO>
 __global__ __launch_bounds__(64 * kWaves) void gemv_bf16_rows_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx,
                                                                      int M, int N, int K, ProductOut out) {
     __shared__ float red[kWaves][T * 16][17];
@@ -32,31 +33,47 @@ __global__ __launch_bounds__(64 * kWaves) void gemv_bf16_rows_kernel(const uint1
     f32x4 acc[T];
 #pragma unroll
     for (int t = 0; t < T; t++) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    auto sum_of = [&](int from, int to) {
 #pragma unroll 2
-    for (int k = k0; k < k1; k += 64) {
-        u32x4 w[2][T];
+        for (int k = from; k < to; k += 64) {
+            u32x4 w[2][T];
+#pragma unroll
+            for (int t = 0; t < T; t++)
+#pragma unroll
+                for (int s = 0; s < 2; s++) w[s][t] = *(const u32x4*)(wp[t] + k + 32 * s);
+#pragma unroll
+            for (int s = 0; s < 2; s++) {
+                const f32x4 a = *(const f32x4*)(xp + k + 32 * s), b = *(const f32x4*)(xp + k + 32 * s + 4);
+                float v[8] = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+                u32x4 q;
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    if (low) {
+                        v[2 * i] = low_part(v[2 * i]);
+                        v[2 * i + 1] = low_part(v[2 * i + 1]);
+                    }
+                    q[i] = pack_bf16(v[2 * i], v[2 * i + 1]);
+                }
+#pragma unroll
+                for (int t = 0; t < T; t++)
+                    acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, w[s][t]), __builtin_bit_cast(bf16x8, q), acc[t], 0, 0, 0);
+            }
+        }
+    };
+    int from = k0;
+    if constexpr (TWO) {  // what of this wavefront's piece lies below split
+        const int to = out.split < k1 ? (int)out.split : k1;
+        sum_of(k0, to);
 #pragma unroll
         for (int t = 0; t < T; t++)
 #pragma unroll
-            for (int s = 0; s < 2; s++) w[s][t] = *(const u32x4*)(wp[t] + k + 32 * s);
-#pragma unroll
-        for (int s = 0; s < 2; s++) {
-            const f32x4 a = *(const f32x4*)(xp + k + 32 * s), b = *(const f32x4*)(xp + k + 32 * s + 4);
-            float v[8] = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
-            u32x4 q;
-#pragma unroll
             for (int i = 0; i < 4; i++) {
-                if (low) {
-                    v[2 * i] = low_part(v[2 * i]);
-                    v[2 * i + 1] = low_part(v[2 * i + 1]);
-                }
-                q[i] = pack_bf16(v[2 * i], v[2 * i + 1]);
+                const int n = n0 + t * 16 + 4 * g + i;
+                acc[t][i] *= out.mid[n < N ? n : N - 1];
             }
-#pragma unroll
-            for (int t = 0; t < T; t++)
-                acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, w[s][t]), __builtin_bit_cast(bf16x8, q), acc[t], 0, 0, 0);
-        }
+        if (to > from) from = to;
     }
+    sum_of(from, k1);
     // a lane holds column r16 of rows 4 g .. 4 g + 3
 #pragma unroll
     for (int t = 0; t < T; t++)
@@ -66,14 +83,14 @@ __global__ __launch_bounds__(64 * kWaves) void gemv_bf16_rows_kernel(const uint1
     for (int o = tid; o < T * 128; o += 64 * kWaves) {
         const int row = o >> 3, col = o & 7, n = n0 + row;
         if (col >= M || n >= N) continue;
-        float v = 0.f;
+        auto sum = [&](int r) {
+            float v = 0.f;
 #pragma unroll
-        for (int i = 0; i < kWaves; i++) v += red[i][row][col] + red[i][row][col + 8];
-        if (out.relu2) v = v > 0.f ? v * v : 0.f;
-        else if (n < out.silu_n) v = v / (1.f + expf(-v));
-        const int64_t at = (int64_t)col * out.ld + n;
-        if (out.f32) out.f32[at] = v;
-        else out.bf16[at] = round_bf16(v);
+            for (int i = 0; i < kWaves; i++) v += red[i][r][col] + red[i][r][col + 8];
+            return v;
+        };
+        if (n < out.pair_from) store_column(out, col, n, sum(row));
+        else if ((row & 1) == 0) store_pair(out, col, n, sum(row), sum(row + 1));
     }
 }
 
@@ -86,9 +103,16 @@ hipError_t gemv_bf16_rows(const uint16_t* W, int64_t ldw, const float* x, int64_
     auto launch = [&](auto kernel, int rows, int waves) {
         hipLaunchKernelGGL(kernel, dim3((unsigned)((N + rows - 1) / rows)), dim3(64 * waves), 0, st, W, ldw, x, ldx, (int)M, (int)N, k, out);
     };
-    if (N >= 8192) launch(gemv_bf16_rows_kernel<2, 8>, 32, 8);
-    else if (k >= 8192) launch(gemv_bf16_rows_kernel<1, 16>, 16, 16);
-    else launch(gemv_bf16_rows_kernel<1, 8>, 16, 8);
+    if (N >= 8192) {
+        if (out.mid) launch(gemv_bf16_rows_kernel<2, 8, true>, 32, 8);
+        else launch(gemv_bf16_rows_kernel<2, 8, false>, 32, 8);
+    } else if (k >= 8192) {
+        if (out.mid) launch(gemv_bf16_rows_kernel<1, 16, true>, 16, 16);
+        else launch(gemv_bf16_rows_kernel<1, 16, false>, 16, 16);
+    } else {
+        if (out.mid) launch(gemv_bf16_rows_kernel<1, 8, true>, 16, 8);
+        else launch(gemv_bf16_rows_kernel<1, 8, false>, 16, 8);
+    }
     return hipGetLastError();
 }
 

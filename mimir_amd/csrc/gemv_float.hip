@@ -9,6 +9,7 @@
 // rows of W for up to eight rows of x, sixteen bytes of W a lane at a time, and applies the activation behind it.
 #include "device_util.h"
 #include "kernels.h"
+#include "product_store.h"
 #include "stack_ops.h"
 
 namespace mimir {
@@ -52,7 +53,8 @@ hipError_t gemv_float(int dt, const void* W, const float* x, float* y, int64_t M
 
 // M rows of x against R rows of W a wavefront, eight elements of K a lane and step (the rows are padded with zeros to
 // a multiple of 64). The x of a step serves all R rows from registers.
-template <int M, int R>
+// TWO: the sums below and from out.split on have factors of their own.
+template <int M, int R, bool TWO>
 __global__ __launch_bounds__(256) void gemv_bf16_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx, int N, int K,
                                                         ProductOut out) {
     const int lane = threadIdx.x & 63, n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * R;
@@ -66,40 +68,54 @@ __global__ __launch_bounds__(256) void gemv_bf16_kernel(const uint16_t* __restri
     for (int m = 0; m < M; m++)
 #pragma unroll
         for (int r = 0; r < R; r++) acc[m][r] = 0.f;
+    auto sum = [&](int from, int to) {
 #pragma unroll 4
-    for (int k = lane * 8; k < K; k += 512) {
-        u32x4 wv[R];
+        for (int k = from + lane * 8; k < to; k += 512) {
+            u32x4 wv[R];
 #pragma unroll
-        for (int r = 0; r < R; r++) wv[r] = *(const u32x4*)(w[r] + k);
+            for (int r = 0; r < R; r++) wv[r] = *(const u32x4*)(w[r] + k);
 #pragma unroll
-        for (int m = 0; m < M; m++) {
-            const f32x4* xp = (const f32x4*)(x + (m0 + m) * ldx + k);
-            const f32x4 a = xp[0], b = xp[1];
+            for (int m = 0; m < M; m++) {
+                const f32x4* xp = (const f32x4*)(x + (m0 + m) * ldx + k);
+                const f32x4 a = xp[0], b = xp[1];
 #pragma unroll
-            for (int r = 0; r < R; r++) {
-                float t = acc[m][r];
+                for (int r = 0; r < R; r++) {
+                    float t = acc[m][r];
 #pragma unroll
-                for (int i = 0; i < 4; i++) {
-                    const float x0 = i < 2 ? a[2 * i] : b[2 * i - 4], x1 = i < 2 ? a[2 * i + 1] : b[2 * i - 3];
-                    t = fmaf(x0, __uint_as_float(wv[r][i] << 16), t);
-                    t = fmaf(x1, __uint_as_float(wv[r][i] & 0xffff0000u), t);
+                    for (int i = 0; i < 4; i++) {
+                        const float x0 = i < 2 ? a[2 * i] : b[2 * i - 4], x1 = i < 2 ? a[2 * i + 1] : b[2 * i - 3];
+                        t = fmaf(x0, __uint_as_float(wv[r][i] << 16), t);
+                        t = fmaf(x1, __uint_as_float(wv[r][i] & 0xffff0000u), t);
+                    }
+                    acc[m][r] = t;
                 }
-                acc[m][r] = t;
             }
         }
-    }
-#pragma unroll
-    for (int m = 0; m < M; m++)
+    };
+    if constexpr (TWO) {
+        sum(0, (int)out.split);
 #pragma unroll
         for (int r = 0; r < R; r++) {
-            float v = wave_sum(acc[m][r]);
-            if (lane != 0 || n0 + r >= N) continue;
-            if (out.relu2) v = v > 0.f ? v * v : 0.f;
-            else if (n0 + r < out.silu_n) v = v / (1.f + expf(-v));
-            const int64_t at = (m0 + m) * out.ld + n0 + r;
-            if (out.f32) out.f32[at] = v;
-            else out.bf16[at] = round_bf16(v);
+            const float f = out.mid[n0 + r < N ? n0 + r : N - 1];
+#pragma unroll
+            for (int m = 0; m < M; m++) acc[m][r] *= f;
         }
+    }
+    sum(TWO ? (int)out.split : 0, K);
+#pragma unroll
+    for (int m = 0; m < M; m++) {
+        float v[R];
+#pragma unroll
+        for (int r = 0; r < R; r++) v[r] = wave_sum(acc[m][r]);
+        if (lane != 0) continue;
+#pragma unroll
+        for (int r = 0; r < R; r++) {
+            const int n = n0 + r;
+            if (n >= N) break;
+            if (n < out.pair_from) store_column(out, m0 + m, n, v[r]);
+            else if (r + 1 < R && (r & 1) == 0) store_pair(out, m0 + m, n, v[r], v[r + 1 < R ? r + 1 : r]);
+        }
+    }
 }
 
 namespace {
@@ -107,10 +123,18 @@ namespace {
 template <int M>
 void launch_gemv_bf16(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t groups, int64_t N, int64_t K, const ProductOut& out, hipStream_t st) {
     const int k = (int)((K + 63) / 64 * 64);
+    auto launch = [&](auto kernel, int rows) {
+        hipLaunchKernelGGL(kernel, dim3((unsigned)((N + 4 * rows - 1) / (4 * rows)), (unsigned)groups), dim3(256), 0, st, W, ldw, x, ldx, (int)N, k, out);
+    };
     // more rows a wavefront read x less often; fewer give a small matrix enough wavefronts
-    if (N >= 8192 && M <= 4) hipLaunchKernelGGL((gemv_bf16_kernel<M, 4>), dim3((unsigned)((N + 15) / 16), (unsigned)groups), dim3(256), 0, st, W, ldw, x, ldx, (int)N, k, out);
-    else if (N >= 2048) hipLaunchKernelGGL((gemv_bf16_kernel<M, 2>), dim3((unsigned)((N + 7) / 8), (unsigned)groups), dim3(256), 0, st, W, ldw, x, ldx, (int)N, k, out);
-    else hipLaunchKernelGGL((gemv_bf16_kernel<M, 1>), dim3((unsigned)((N + 3) / 4), (unsigned)groups), dim3(256), 0, st, W, ldw, x, ldx, (int)N, k, out);
+    const int rows = N >= 8192 && M <= 4 ? 4 : N >= 2048 || N > out.pair_from ? 2 : 1;
+    if (out.mid) {
+        if (rows == 4) launch(gemv_bf16_kernel<M, (M <= 4 ? 4 : 2), true>, 4);
+        else if (rows == 2) launch(gemv_bf16_kernel<M, 2, true>, 2);
+        else launch(gemv_bf16_kernel<M, 1, true>, 1);
+    } else if (rows == 4) launch(gemv_bf16_kernel<M, (M <= 4 ? 4 : 2), false>, 4);
+    else if (rows == 2) launch(gemv_bf16_kernel<M, 2, false>, 2);
+    else launch(gemv_bf16_kernel<M, 1, false>, 1);
 }
 
 }  // namespace
@@ -120,7 +144,9 @@ hipError_t gemv_bf16(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx
     auto rest = [&](int64_t rows, int64_t each) {  // whole groups of `each` rows from row m on
         ProductOut o = out;
         if (o.f32) o.f32 += m * o.ld;
-        else o.bf16 += m * o.ld;
+        else if (o.bf16) o.bf16 += m * o.ld;
+        if (o.pair_f32) o.pair_f32 += m * o.pair_ld;
+        else if (o.pair_bf16) o.pair_bf16 += m * o.pair_ld;
         const float* xr = x + m * ldx;
         const int64_t groups = rows / each;
         if (each == 8) launch_gemv_bf16<8>(W, ldw, xr, ldx, groups, N, K, o, st);

@@ -78,6 +78,8 @@ struct ScaledStore {
     void* Yv;
     const float* row_scale;
     bool wide_ok;
+    __device__ __forceinline__ int first_steps(int steps) const { return steps; }
+    __device__ __forceinline__ float mid(int, int) const { return 1.f; }
     __device__ __forceinline__ float row(int m, int M) const { return m < M ? row_scale[m] : 0.f; }
     __device__ __forceinline__ void operator()(int m, int n, int N, float back, float v[4]) const {
 #pragma unroll

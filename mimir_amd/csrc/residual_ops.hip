@@ -40,6 +40,17 @@ __device__ __forceinline__ void put(float* f, uint16_t* b, int64_t at, float v) 
     if (b) b[at] = round_bf16(v);
 }
 
+// The pair table's row for one row of the call, whose token is kept for the next: the thread with `keeps` does that.
+__device__ __forceinline__ const uint16_t* pair_row(const PairTable& p, const int32_t* tokens, int64_t r, bool keeps) {
+    const int64_t b = r / p.s, t = r % p.s, pos = p.past + (p.past_dev ? *p.past_dev : 0) + t;
+    int32_t* held = p.held + b * p.held_ld;
+    const int64_t token = tokens[r];
+    int64_t row = p.buckets;
+    if (pos > 0) row = ((int64_t)(t > 0 ? tokens[r - 1] : held[pos - 1]) * p.mul_prev + token * p.mul_cur) % p.buckets;
+    if (keeps) held[pos] = (int32_t)token;
+    return p.table + row * p.ld;
+}
+
 // floats of LDS: the row, the groups' parts and scales
 size_t chain_lds(int width, int groups, int threads) {
     const int nw = threads / 64;
@@ -57,14 +68,18 @@ __global__ __launch_bounds__(1024) void norm_chain_kernel(NormChain a) {
     if (a.tokens) {
         const uint16_t* e = a.table + (int64_t)a.tokens[r] * a.table_ld;
         for (int i = threadIdx.x; i < W; i += blockDim.x) row[i] = bf16_bits_to_f32(e[i]);
+        if (a.pairs.table) {
+            const uint16_t* pr = pair_row(a.pairs, a.tokens, r, threadIdx.x == 0);
+            for (int i = threadIdx.x; i < W; i += blockDim.x) row[i] += bf16_bits_to_f32(pr[i]);
+        }
     } else {
-        for (int i = threadIdx.x; i < W; i += blockDim.x) row[i] = a.y[r * a.ldy + i];
+        for (int i = threadIdx.x; i < W; i += blockDim.x) row[i] = a.y ? a.y[r * a.ldy + i] : 0.f;
     }
     __syncthreads();
-    group_scales(row, W, a.groups, a.eps, part, scale);
+    if (a.w_post) group_scales(row, W, a.groups, a.eps, part, scale);
     const float own = a.dwa ? a.dwa[a.n_streams] : 1.f;
     for (int i = threadIdx.x; i < W; i += blockDim.x) {
-        float z = row[i] * scale[i / gs] * a.w_post[i];
+        float z = a.w_post ? row[i] * scale[i / gs] * a.w_post[i] : row[i];
         if (!a.tokens) z += a.x[r * W + i];
         if (a.stream_out) a.stream_out[r * W + i] = z;
         if (a.dwa) {
@@ -141,18 +156,23 @@ __global__ __launch_bounds__(1024) void norm_chain_wide_kernel(NormChain a) {
     };
     f32x4 y[E], x[E], wp[E], wn[E], z[E], avg[E];
     const uint16_t* row = a.tokens ? a.table + (int64_t)a.tokens[r] * a.table_ld : nullptr;
+    const uint16_t* pair = a.tokens && a.pairs.table ? pair_row(a.pairs, a.tokens, r, threadIdx.x == 0) : nullptr;
 #pragma unroll
     for (int e = 0; e < E; e++) {
         if (row) {
             u32x2 v = {0, 0};
             if (in[e]) v = *(const u32x2*)(row + at[e]);
             y[e] = f32x4{__uint_as_float(v[0] << 16), __uint_as_float(v[0] & 0xffff0000u), __uint_as_float(v[1] << 16), __uint_as_float(v[1] & 0xffff0000u)};
+            if (pair && in[e]) {
+                v = *(const u32x2*)(pair + at[e]);
+                y[e] = y[e] + f32x4{__uint_as_float(v[0] << 16), __uint_as_float(v[0] & 0xffff0000u), __uint_as_float(v[1] << 16), __uint_as_float(v[1] & 0xffff0000u)};
+            }
             x[e] = zero;
         } else {
-            y[e] = read(a.y + r * a.ldy, e);
+            y[e] = a.y ? read(a.y + r * a.ldy, e) : zero;
             x[e] = read(a.x + r * W, e);
         }
-        wp[e] = read(a.w_post, e);
+        wp[e] = a.w_post ? read(a.w_post, e) : zero;
         wn[e] = a.w_next ? read(a.w_next, e) : zero;
         avg[e] = zero;
     }
@@ -166,12 +186,12 @@ __global__ __launch_bounds__(1024) void norm_chain_wide_kernel(NormChain a) {
                 for (int i = 0; i < 4; i++) avg[e][i] = fmaf(w, v[i], avg[e][i]);
             }
         }
-    norm(y, part[0], z);
+    if (a.w_post) norm(y, part[0], z);
     const float own = a.dwa ? a.dwa[a.n_streams] : 1.f;
 #pragma unroll
     for (int e = 0; e < E; e++) {
         if (!in[e]) continue;
-        z[e] = x[e] + z[e] * wp[e];
+        z[e] = a.w_post ? x[e] + z[e] * wp[e] : x[e] + y[e];
         if (a.stream_out) *(f32x4*)(a.stream_out + r * W + at[e]) = z[e];
         if (a.dwa) {
 #pragma unroll
@@ -350,7 +370,7 @@ __global__ __launch_bounds__(256) void conv_state_kernel(const float* __restrict
 hipError_t norm_chain(const NormChain& a, int64_t rows, hipStream_t st) {
     if (rows == 0) return hipSuccess;
     auto whole = [](const void* p, int64_t ld) { return !p || (((uintptr_t)p & 15) == 0 && ld % 4 == 0); };
-    if (a.width / a.groups % 256 == 0 && a.width <= 16384 && whole(a.table, a.table_ld) && whole(a.y, a.ldy) && whole(a.x, 4) && whole(a.h_f32, a.ldh) &&
+    if (a.width / a.groups % 256 == 0 && a.width <= 16384 && whole(a.table, a.table_ld) && whole(a.pairs.table, a.pairs.ld) && whole(a.y, a.ldy) && whole(a.x, 4) && whole(a.h_f32, a.ldh) &&
         whole(a.h_bf16, a.ldh) && whole(a.streams, a.stream_stride) && whole(a.stream_out, 4) && whole(a.x_out, 4) && whole(a.conv_state, 4)) {
         const int threads = a.width < 4096 ? a.width / 4 : 1024;  // a multiple of 64
         if (a.width <= 4096) hipLaunchKernelGGL(norm_chain_wide_kernel<1>, dim3((unsigned)rows), dim3(threads), 0, st, a);

@@ -1,5 +1,5 @@
 // Kernels of the mixer stack (stack.hip): group norms with what surrounds them, short causal convolutions, the products
-// of bfloat16 weights, latent attention and the linear recurrences. Each launches on the given stream and returns the
+// of bfloat16 weights, latent attention, attention by key heads and the linear recurrences. Each launches on the given stream and returns the
 // launch status. Sizes and constants are parameters; rows are sequences' positions one after the other (b * s + t).
 #pragma once
 
@@ -10,18 +10,28 @@ namespace mimir {
 
 // ---- residual_ops.hip -------------------------------------------------------------------
 // The steps between two products on one row of `width`, in this order, those with a null pointer left out:
-//   z = group_norm(table[tokens[row]]) * w_post            (tokens set), or
-//   z = x + group_norm(y) * w_post
+//   z = group_norm(table[tokens[row]] + pair_table[pair]) * w_post            (tokens set), or
+//   z = x + group_norm(y) * w_post                 (w_post null: no norm of y, or of the table's row)
 //   stream_out = z;  z = sum_j dwa[j] streams[j] + dwa[n_streams] z   (the depth average: n_streams earlier results)
 //   x_out = z
 //   h = group_norm(z) * w_next, and with conv_w (one position a sequence): h += the causal convolution of h with the
 //   taps - 1 rows of conv_state [batch, taps - 1, width], which then moves on by one
 //   h_f32, h_bf16: h, rows ldh elements apart.
 // group_norm: `groups` equal parts, each over sqrt(mean(part^2) + eps); all of it in float32.
+// pair: (previous token * mul_prev + token * mul_cur) mod buckets, or row `buckets` for a sequence's first token. The tokens
+// of every position are kept in held [batch, held_ld], where the first of a call finds the one before.
+struct PairTable {
+    const uint16_t* table = nullptr;  // [buckets + 1, width]; null: none
+    int64_t ld = 0, buckets = 0, mul_prev = 0, mul_cur = 0;
+    int32_t* held = nullptr;
+    int64_t held_ld = 0, s = 1, past = 0;  // s positions a sequence in this call, after past + *past_dev
+    const int32_t* past_dev = nullptr;
+};
 struct NormChain {
     const int32_t* tokens = nullptr;
     const uint16_t* table = nullptr;
     int64_t table_ld = 0;
+    PairTable pairs;
     const float* x = nullptr;
     const float* y = nullptr;
     int64_t ldy = 0;
@@ -63,6 +73,18 @@ struct ProductOut {
     int64_t ld = 0;
     int64_t silu_n = 0;
     bool relu2 = false;
+    // Columns from pair_from (a multiple of 4) on come in pairs (z, u), side by side, and leave one value silu(z) u a pair, in
+    // one of these, rows pair_ld apart. N is even then.
+    int64_t pair_from = INT64_MAX;
+    float* pair_f32 = nullptr;
+    uint16_t* pair_bf16 = nullptr;
+    int64_t pair_ld = 0;
+    // y_n = scale[n] (mid[n] (the sum over k < split) + the rest of it), with null pointers for ones: two products of the same
+    // row, each with factors of its own (s in front of the first: mid = s / scale), in one. split: a multiple of 64 below K.
+    const float* scale = nullptr;
+    const float* mid = nullptr;
+    int64_t split = 0;
+    bool add = false;  // to what f32 holds
 };
 constexpr int64_t kGemvRows = 8;  // rows of x that gemv_bf16 takes at once (more are several passes over W)
 // float32 x, few rows: W read once for up to kGemvRows of them (gemv_float.hip)
@@ -147,5 +169,40 @@ hipError_t latent_absorbed(const Latent& a, const float* proj, int64_t ldp, floa
 bool latent_prompt_ok(const Latent& a);
 hipError_t latent_prompt(const Latent& a, const uint16_t* q, int64_t ldq, const uint16_t* keys, int64_t ldk, const uint16_t* values_t, int64_t ldv,
                          uint16_t* out, int64_t ldo, hipStream_t st);
+
+// ---- attention with a key and value for every key head (attention_heads.hip) -------------------
+// Query heads share key heads in neighbouring groups; causal. score = softcap tanh(scale q.k / softcap) (softcap 0: scale q.k).
+struct HeadAttention {
+    int heads = 1, kv_heads = 1, dim = 0, vdim = 0;
+    float scale = 1.f, softcap = 0.f;
+    bool unit = false;  // queries and keys over their root mean square, sqrt(mean(x^2) + eps)
+    float eps = 0.f;
+    int rot_dim = 0;  // the first features of queries and keys turn, feature i with feature i + rot_dim / 2
+    const float *cos_t = nullptr, *sin_t = nullptr;  // [context, rot_dim / 2]
+    const float* proj = nullptr;  // [rows, heads * dim of q | kv_heads * dim of k | kv_heads * vdim of v | gated: heads], rows ldp apart
+    int64_t ldp = 0;
+    bool gated = false;  // a head's result times the sigmoid of its gate
+    // values: (1 - mix) v + mix first, where `first` is set ([rows, kv_heads * vdim]); first_out, where set, gets v
+    const float* mix = nullptr;
+    const float* first = nullptr;
+    float* first_out = nullptr;
+    void* keys = nullptr;    // [batch, kv_heads, context, ldk]
+    void* values = nullptr;  // [batch, kv_heads, vdim, context], positions in the kernels' own order
+    bool cache_bf16 = false;
+    int64_t ldk = 0;      // a multiple of 8, zeros behind dim
+    int64_t context = 0;  // the capacity, a multiple of 64
+    int batch = 1;
+    int64_t s = 1;     // new positions a sequence
+    int64_t past = 0;  // positions before them: past + *past_dev
+    const int32_t* past_dev = nullptr;
+};
+constexpr int kHeadAttentionMax = 1024;  // features of a head
+// Cache entries of the new positions, then attention of few query rows. ws: heads_attend_ws_floats floats. out
+// [rows, heads * vdim] float32 or bfloat16, rows ldo apart.
+size_t heads_attend_ws_floats(const HeadAttention& a, int64_t rows);
+hipError_t heads_attend(const HeadAttention& a, float* ws, float* out_f32, uint16_t* out_bf16, int64_t ldo, hipStream_t st);
+// The same for many query rows on a bfloat16 cache. q: [rows, heads, ldk] of workspace.
+bool heads_prompt_ok(const HeadAttention& a);
+hipError_t heads_prompt(const HeadAttention& a, uint16_t* q, uint16_t* out, int64_t ldo, hipStream_t st);
 
 }  // namespace mimir

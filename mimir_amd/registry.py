@@ -18,13 +18,13 @@ def _llama(path: str, dtype: str | None = None, **kw) -> Decoder:
     return load_mim(path, **kw)
 
 
-def _fuvolix(path: str, **kw) -> Decoder:
-    from .stack import load_fuvolix
-    return load_fuvolix(path, **kw)
+def _stack(path: str, **kw) -> Decoder:
+    from .stack import load_stack
+    return load_stack(path, **kw)
 
 
 # architecture -> (loader, the part of the library that it needs: a name of build.PARTS, None: the whole library)
-ARCHITECTURES = {"llama": (_llama, None), "qwen2": (_llama, None), "Fuvolix": (_fuvolix, "stack")}
+ARCHITECTURES = {"llama": (_llama, None), "qwen2": (_llama, None), "Fuvolix": (_stack, "stack"), "Genetar": (_stack, "stack")}
 
 
 def architecture(path: str) -> str:

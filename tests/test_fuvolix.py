@@ -174,7 +174,7 @@ def test_configuration_errors_come_before_a_device_is_touched():
 
     ok = X.config([X.latent(ff=8), X.mlstm(), X.lightning()])
     assert create(ok) == capi.OK
-    for edit in (dict(norm_groups=7), dict(taps=0), dict(width=0), dict(context=0), dict(eps=0.0), dict(rot_dim=7), dict(kv_rank=0), dict(heads=0), dict(mixer=9)):
+    for edit in (dict(norm_groups=7), dict(taps=-1), dict(width=0), dict(context=0), dict(eps=0.0), dict(rot_dim=7), dict(kv_rank=0), dict(heads=0), dict(mixer=9)):
         assert create(ok, **edit) == capi.ERR_SHAPE, edit
     assert create(ok, dtype=capi.F16) == capi.ERR_DTYPE
     assert create(X.config([X.mlstm(dim=257)])) == capi.ERR_SHAPE
