@@ -23,7 +23,7 @@ def unit_rms(x, eps):
 
 
 def soft_cap(s, cap):
-    return cap * np.tanh(s / cap)
+    return cap * np.tanh(s / cap) if cap else s
 
 
 def embed_pairs(tokens, table, pairs, mul_prev, mul_cur):
