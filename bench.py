@@ -416,35 +416,41 @@ def layer_step_bench(capi, cached=2048, new=33):
     return out
 
 
-FUVOLIX_SIZES = {
+STACK_SIZES = {
     # width, feed-forward, heads; a head has 128 features of queries, keys and values (latent attention 64 rotated ones besides,
-    # over a latent of 512)
+    # over a latent of 512; attention has a quarter as many key heads)
     "4096": (4096, 14336, 32),
     "2048": (2048, 8192, 16),
 }
+# the kinds of layer of the designs that are a mixer stack (mimir_amd.stack)
+STACK_KINDS = {"Fuvolix": ("latent_attention", "mlstm", "lightning"), "Genetar": ("attention", "attention_2")}
 
 
-def fuvolix_layer(kind, ff, heads):
+def stack_layer(kind, ff, heads):
     """config.json's entry of a layer that resembles a real model's."""
+    by_heads = dict(heads=heads, kv_heads=max(1, heads // 4), dim=128, vdim=128, scale=128 ** -0.5, softcap=30.0, v_mix=True)
     mx = {"latent_attention": dict(heads=heads, dim=128, rot_dim=64, vdim=128, kv_rank=512, scale=192 ** -0.5, rot=dict(base=10000.0, dims=64)),
           "mlstm": dict(heads=heads, dim=128, vdim=128, gate_cap=15.0),
-          "lightning": dict(heads=heads, dim=128, vdim=128, decay=[float(np.exp(-2.0 ** (-8 * (h + 1) / heads))) for h in range(heads)])}[kind]
+          "lightning": dict(heads=heads, dim=128, vdim=128, decay=[float(np.exp(-2.0 ** (-8 * (h + 1) / heads))) for h in range(heads)]),
+          "attention": by_heads,
+          "attention_2": dict(by_heads, rot=dict(base=500000.0, dims=128, scaling=dict(factor=8.0, low=1.0, high=4.0, original=8192)))}[kind]
     return dict(type=kind, mixer=mx, mlp=None if ff is None else dict(kind="dense", ff=ff))
 
 
-def build_fuvolix(capi, kinds, size, batch, context, max_tokens, vocab=32768):
-    """A random-init Fuvolix decoder with layers of these kinds, bfloat16."""
+def build_stack(capi, design, kinds, size, batch, context, max_tokens, vocab=32768):
+    """A random-init decoder of a design with layers of these kinds, bfloat16."""
     from mimir_amd import stack
-    width, ff, heads = FUVOLIX_SIZES[size]
-    cfg = dict(width=width, vocab=vocab, canon=dict(taps=4), norm=dict(groups=2, eps=1e-6), layers=[fuvolix_layer(k, ff, heads) for k in kinds])
-    m = stack.Stack(*stack.fuvolix_config(cfg, context, batch))
+    width, ff, heads = STACK_SIZES[size]
+    cfg = dict(width=width, vocab=vocab, canon=dict(taps=4), norm=dict(groups=2, eps=1e-6), layers=[stack_layer(k, ff, heads) for k in kinds],
+               embedding=dict(bigram=dict(buckets=vocab, mul_prev=31, mul_cur=7)), logit_scale=1.0)
+    m = stack.Stack(*stack.CONFIGS[design](cfg, context, batch))
     rng = np.random.default_rng(0)
     pool = rng.standard_normal(1 << 24, np.float32)  # tensors are cut from it, each from another place, and scaled
     for name, n, k in m.tensors():
         leaf = name.rsplit(".", 1)[-1]
-        scale, at = (1.0, 1.0) if "norm" in leaf else (k ** -0.5 if n > 1 else 0.5, 0.0)
-        if "norm" in leaf:
-            scale = 0.02
+        scale, at = (k ** -0.5 if n > 1 else 0.5, 0.0)
+        if "norm" in leaf or leaf in ("ls1", "ls2"):
+            scale, at = 0.02, 1.0
         start = int(rng.integers(0, pool.size))
         w = np.take(pool, np.arange(start, start + n * k), mode="wrap") * np.float32(scale) + np.float32(at)
         m.set_tensor(name, capi.BF16, (w.view(np.uint32) >> 16).astype(np.uint16), n * k)
@@ -452,15 +458,15 @@ def build_fuvolix(capi, kinds, size, batch, context, max_tokens, vocab=32768):
     return m
 
 
-def fuvolix_bench(capi, sizes=("4096", "2048"), kinds=("latent_attention", "mlstm", "lightning"), prompts=((1, 2048), (8, 512)), new=65, layers=(2, 6), llama=True):
-    """Prompt passes and decoding of the Fuvolix design's three kinds of layer, beside the Llama decoder's (Q4_0) at equal
-    width, feed-forward and heads: microseconds a layer (models of two and of six layers; the difference over four, so
+def stack_bench(capi, kinds, sizes=("4096", "2048"), prompts=((1, 2048), (8, 512)), new=65, layers=(2, 6)):
+    """Prompt passes and decoding of layers of these kinds at equal width, feed-forward and heads: those of a mixer stack, and
+    llama_q4_0, the Llama decoder's. Microseconds a layer (models of two and of six layers; the difference over four, so
     that embedding and head drop out), the best of three runs."""
     out = {}
     for size in sizes:
-        width, ff, heads = FUVOLIX_SIZES[size]
+        width, ff, heads = STACK_SIZES[size]
         kv_heads = max(1, heads // 4)
-        for kind in kinds + (("llama_q4_0",) if llama else ()):
+        for kind in kinds:
             for batch, prompt in prompts:
                 secs = {}
                 for n in layers:
@@ -468,7 +474,7 @@ def fuvolix_bench(capi, sizes=("4096", "2048"), kinds=("latent_attention", "mlst
                         m = build_llama(capi, layers=n, batch=batch, context=prompt + new, max_tokens=prompt, embed=width, hidden=ff, heads=heads, kv_heads=kv_heads,
                                         vocab=32768)
                     else:
-                        m = build_fuvolix(capi, [kind] * n, size, batch, prompt + new, prompt)
+                        m = build_stack(capi, next(d for d, k in STACK_KINDS.items() if kind in k), [kind] * n, size, batch, prompt + new, prompt)
                     toks = np.random.default_rng(0).integers(0, 32768, (batch, prompt))
                     runs = []
                     for _ in range(4):
@@ -479,9 +485,9 @@ def fuvolix_bench(capi, sizes=("4096", "2048"), kinds=("latent_attention", "mlst
                 span = layers[1] - layers[0]
                 p_us = (secs[layers[1]][0] - secs[layers[0]][0]) / span * 1e6
                 d_us = (secs[layers[1]][1] - secs[layers[0]][1]) / span / (new - 1) * 1e6
-                if kind == "llama_q4_0":
+                if kind in ("llama_q4_0", *STACK_KINDS["Genetar"]):
                     weights = width * (2 * heads + 2 * kv_heads) * 128 + 3 * width * ff
-                    weight_bytes, state = weights * 18 // 32, batch * (prompt + new // 2) * kv_heads * 128 * 4
+                    weight_bytes, state = weights * 18 // 32 if kind == "llama_q4_0" else weights * 2, batch * (prompt + new // 2) * kv_heads * 128 * 4
                 elif kind == "latent_attention":
                     weights = width * (heads * 192 + 576 + heads * 128) + heads * 256 * 512 + 2 * width * ff
                     weight_bytes, state = weights * 2, batch * (prompt + new // 2) * 576 * 2
@@ -751,8 +757,10 @@ def main():
     ap.add_argument("--decode-linear", choices=("q4_0", "q4_K", "q6_K"), default="q4_0",
                     help="block dtype of the decoder's linear weights (the oracle check is for q4_0)")
     ap.add_argument("--fuvolix", action="store_true", help="only: prompt passes and decoding of the Fuvolix design's layers at sizes like a real model's, beside the Llama decoder's")
-    ap.add_argument("--fuvolix-only", default=None, metavar="SIZE[:KIND[:BATCHxPROMPT]]", help="with --fuvolix: one size, kind of layer, call (for profiles)")
-    ap.add_argument("--fuvolix-no-llama", action="store_true", help="with --fuvolix: without the Llama decoder's figures")
+    ap.add_argument("--genetar", action="store_true", help="only: the same of the Genetar design's layers, beside the Llama decoder's and Fuvolix's latent attention")
+    ap.add_argument("--fuvolix-only", "--stack-only", dest="stack_only", default=None, metavar="SIZE[:KIND[:BATCHxPROMPT]]",
+                    help="with --fuvolix or --genetar: one size, kind of layer, call (for profiles)")
+    ap.add_argument("--fuvolix-no-llama", "--stack-alone", dest="stack_alone", action="store_true", help="with --fuvolix or --genetar: without the other decoders' figures")
     ap.add_argument("--tune", action="append", default=[], metavar="KEY=VALUE",
                     help="a launch-plan override for mi355x_tune before anything runs (may be repeated), e.g. q4_0.stream=1")
     args = ap.parse_args()
@@ -769,16 +777,18 @@ def main():
         key, _, val = kv.partition("=")
         capi.check(lib.mi355x_tune(key.encode(), int(val)))
 
-    if args.fuvolix:
-        kw = {"llama": not args.fuvolix_no_llama}
-        if args.fuvolix_only:
-            parts = args.fuvolix_only.split(":")
+    if args.fuvolix or args.genetar:
+        design = "Fuvolix" if args.fuvolix else "Genetar"
+        beside = () if args.stack_alone else ("llama_q4_0",) if args.fuvolix else ("latent_attention", "llama_q4_0")
+        kw = {"kinds": STACK_KINDS[design] + beside}
+        if args.stack_only:
+            parts = args.stack_only.split(":")
             kw["sizes"] = (parts[0],)
             if len(parts) > 1:
-                kw["kinds"] = tuple(k for k in parts[1].split(",") if k)
+                kw["kinds"] = tuple(k for k in parts[1].split(",") if k) + (() if args.stack_alone else ("llama_q4_0",))
             if len(parts) > 2:
                 kw["prompts"] = (tuple(int(v) for v in parts[2].split("x")),)
-        print(json.dumps({"fuvolix": fuvolix_bench(capi, **kw)}))
+        print(json.dumps({design.lower(): stack_bench(capi, **kw)}))
         return
     if args.rows_counters:
         rows_bench(lib, capi, torch, shapes=((14336, 4096),), only=args.rows_counters)
