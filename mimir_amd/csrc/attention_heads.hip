@@ -49,15 +49,14 @@ __device__ __forceinline__ void head_features(const HeadAttention& a, const floa
     }
 }
 
+__device__ __forceinline__ float mixed_with(float own, float first, float mix) { return fmaf(mix, first, (1.f - mix) * own); }
+
 // The value that a position keeps, of feature c of all value features; what later layers mix in is kept beside.
 __device__ __forceinline__ float mixed_value(const HeadAttention& a, int64_t row, int c) {
     const int64_t vn = (int64_t)a.kv_heads * a.vdim;
     float v = a.proj[row * a.ldp + (int64_t)(a.heads + a.kv_heads) * a.dim + c];
     if (a.first_out) a.first_out[row * vn + c] = v;
-    if (a.first) {
-        const float w = *a.mix;
-        v = fmaf(w, a.first[row * vn + c], (1.f - w) * v);
-    }
+    if (a.first) v = mixed_with(v, a.first[row * vn + c], *a.mix);
     return v;
 }
 __device__ __forceinline__ void keep(void* cache, bool bf16, int64_t at, float v) {
@@ -70,45 +69,106 @@ __device__ __forceinline__ float gate_of(const HeadAttention& a, int64_t row, in
     return a.gated ? sigmoid_f32(a.proj[row * a.ldp + (int64_t)(a.heads + a.kv_heads) * a.dim + (int64_t)a.kv_heads * a.vdim + h]) : 1.f;
 }
 
-// The cache entries of all new positions, and the queries: as bfloat16 rows of heads * ldk for heads_prompt_kernel (zeros
-// behind a head's features), or as float32 times the scale, [rows, heads, dim]. The first `rows` workgroups take a row's queries and keys, a
-// head a wavefront; the others 64 positions of 64 value features, which change places through LDS.
-__global__ __launch_bounds__(256) void heads_prepare_kernel(HeadAttention a, uint16_t* __restrict__ q16, float* __restrict__ q32) {
+// The same of a head on LANES lanes, four neighbouring features a lane (head_fours_ok): put(i, features i .. i + 3).
+template <int LANES, class F>
+__device__ __forceinline__ void head_fours(const HeadAttention& a, const float* x, int64_t pos, F put) {
+    const int i = (threadIdx.x & (LANES - 1)) * 4, half = a.rot_dim >> 1;
+    const bool in = i < a.dim, turns = i < a.rot_dim;
+    f32x4 v = {0.f, 0.f, 0.f, 0.f}, other = v, cs = v, sn = v;
+    if (in) v = *(const f32x4*)(x + i);
+    if (turns) {
+        const int j = i < half ? i : i - half;
+        other = *(const f32x4*)(x + (i < half ? i + half : i - half));
+        cs = *(const f32x4*)(a.cos_t + pos * half + j);
+        sn = *(const f32x4*)(a.sin_t + pos * half + j);
+    }
+    float scale = 1.f;
+    if (a.unit) {
+        float ss = fmaf(v[0], v[0], fmaf(v[1], v[1], fmaf(v[2], v[2], v[3] * v[3])));
+#pragma unroll
+        for (int d = LANES / 2; d > 0; d >>= 1) ss += __shfl_xor(ss, d);
+        scale = 1.f / __builtin_sqrtf(ss / (float)a.dim + a.eps);
+    }
+    v = v * scale;
+    if (turns) {
+        other = other * (i < half ? -scale : scale);
+#pragma unroll
+        for (int e = 0; e < 4; e++) v[e] = v[e] * cs[e] + other[e] * sn[e];
+    }
+    if (i < a.ldk) put(i, v);  // zeros behind the last feature
+}
+bool head_fours_ok(const HeadAttention& a) {
+    return a.dim % 4 == 0 && a.dim <= 256 && a.rot_dim % 8 == 0 && a.ldp % 4 == 0 && ((uintptr_t)a.proj & 15) == 0;
+}
+
+__device__ __forceinline__ u32x2 pack_four(f32x4 v) { return u32x2{pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3])}; }
+
+// The cache entries of all new positions, and the queries times q_scale: as bfloat16 rows of heads * ldk for
+// heads_prompt_kernel (zeros behind a head's features), or as float32, [rows, heads, dim]. The first workgroups take queries and keys,
+// 256 / LANES heads of a row each (LANES 0: a head a wavefront, any size); the others 64 positions of 64 value features,
+// which change places through LDS.
+template <int LANES>
+__global__ __launch_bounds__(256) void heads_prepare_kernel(HeadAttention a, uint16_t* __restrict__ q16, float* __restrict__ q32, float q_scale) {
     __shared__ float tile[64][65];
+    constexpr int kAtOnce = LANES ? 256 / LANES : 4;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int units = a.heads + a.kv_heads, chunks = (units + kAtOnce - 1) / kAtOnce;
     const int64_t rows = a.batch * a.s;
-    if ((int64_t)blockIdx.x < rows) {
-        const int64_t r = blockIdx.x, b = r / a.s, pos = past_of(a) + r % a.s;
-        const float* p = a.proj + r * a.ldp;
-        for (int u = wave; u < a.heads + a.kv_heads; u += 4) {
-            const float* x = p + (int64_t)u * a.dim;
-            if (u >= a.heads) {
-                const int64_t at = key_row(a, b, u - a.heads, pos);
-                head_features(a, x, pos, [&](int i, float v) { keep(a.keys, a.cache_bf16, at + i, v); });
-            } else if (q16) {
-                uint16_t* to = q16 + (r * a.heads + u) * a.ldk;
-                head_features(a, x, pos, [&](int i, float v) { to[i] = round_bf16(v); });
-                for (int i = a.dim + lane; i < a.ldk; i += 64) to[i] = 0;
-            } else {
-                float* to = q32 + (r * a.heads + u) * a.dim;
-                head_features(a, x, pos, [&](int i, float v) { to[i] = v * a.scale; });
-            }
+    if ((int64_t)blockIdx.x < rows * chunks) {
+        const int64_t r = blockIdx.x / chunks, b = r / a.s, pos = past_of(a) + r % a.s;
+        const int u = (int)(blockIdx.x % chunks) * kAtOnce + (int)threadIdx.x / (LANES ? LANES : 64);
+        if (u >= units) return;  // whole groups of lanes
+        const float* x = a.proj + r * a.ldp + (int64_t)u * a.dim;
+        const int64_t key = u < a.heads ? 0 : key_row(a, b, u - a.heads, pos), query = r * a.heads + u;
+        if constexpr (LANES > 0) {
+            head_fours<LANES>(a, x, pos, [&](int i, f32x4 v) {
+                if (u >= a.heads) {
+                    if (a.cache_bf16) *(u32x2*)((uint16_t*)a.keys + key + i) = pack_four(v);
+                    else *(f32x4*)((float*)a.keys + key + i) = v;
+                } else if (q16) {
+                    *(u32x2*)(q16 + query * a.ldk + i) = pack_four(v * q_scale);
+                } else if (i < a.dim) {
+                    *(f32x4*)(q32 + query * a.dim + i) = v * q_scale;
+                }
+            });
+        } else {
+            head_features(a, x, pos, [&](int i, float v) {
+                if (u >= a.heads) keep(a.keys, a.cache_bf16, key + i, v);
+                else if (q16) q16[query * a.ldk + i] = round_bf16(v * q_scale);
+                else q32[query * a.dim + i] = v * q_scale;
+            });
+            if (u < a.heads && q16)
+                for (int i = a.dim + lane; i < a.ldk; i += 64) q16[query * a.ldk + i] = 0;
         }
         return;
     }
     const int vn = a.kv_heads * a.vdim, cols = (vn + 63) / 64;
-    const int64_t w = blockIdx.x - rows, runs = (a.s + 63) / 64;
-    const int c0 = (int)(w % cols) * 64;
-    const int64_t b = w / cols / runs, t0 = w / cols % runs * 64, past = past_of(a);
-    for (int i = wave; i < 64; i += 4)
-        if (t0 + i < a.s && c0 + lane < vn) tile[i][lane] = mixed_value(a, b * a.s + t0 + i, c0 + lane);
+    const int64_t w = blockIdx.x - rows * chunks, runs = (a.s + 63) / 64;
+    const int c = (int)(w % cols) * 64 + lane;
+    const int64_t b = w / cols / runs, t0 = w / cols % runs * 64, r0 = b * a.s + t0;
+    const float* from = a.proj + (int64_t)(a.heads + a.kv_heads) * a.dim;
+    float own[16], first[16];
+    auto in = [&](int u) { return t0 + wave + 4 * u < a.s && c < vn; };
+#pragma unroll
+    for (int u = 0; u < 16; u++) own[u] = in(u) ? from[(r0 + wave + 4 * u) * a.ldp + c] : 0.f;
+    if (a.first) {
+#pragma unroll
+        for (int u = 0; u < 16; u++) first[u] = in(u) ? a.first[(r0 + wave + 4 * u) * vn + c] : 0.f;
+        const float mix = *a.mix;
+#pragma unroll
+        for (int u = 0; u < 16; u++) own[u] = mixed_with(own[u], first[u], mix);
+    }
+#pragma unroll
+    for (int u = 0; u < 16; u++) {
+        tile[wave + 4 * u][lane] = own[u];
+        if (a.first_out && in(u)) a.first_out[(r0 + wave + 4 * u) * vn + c] = own[u];
+    }
     __syncthreads();
     if (t0 + lane >= a.s) return;
-    const int64_t slot = value_slot((int)(past + t0) + lane);
-    for (int i = wave; i < 64 && c0 + i < vn; i += 4) {
-        const int c = c0 + i;
-        keep(a.values, a.cache_bf16, value_row(a, b, c / a.vdim, c % a.vdim) + slot, tile[lane][i]);
-    }
+    const int64_t slot = value_slot((int)(past_of(a) + t0) + lane);
+    const int c0 = c - lane;
+    for (int i = wave; i < 64 && c0 + i < vn; i += 4)
+        keep(a.values, a.cache_bf16, value_row(a, b, (c0 + i) / a.vdim, (c0 + i) % a.vdim) + slot, tile[lane][i]);
 }
 
 // ---- few query rows -------------------------------------------------------------------------
@@ -486,11 +546,17 @@ __global__ __launch_bounds__(256) void heads_combine_kernel(HeadAttention a, Par
 // and the weights go from the exponential straight into the second product's operand, as the sum of two bfloat16. Four
 // wavefronts with consecutive rows share a tile of keys and values in LDS, which goes there straight from the cache while the
 // tile before is used; a row's pieces of sixteen bytes are exchanged so that the reads of 32 rows spread over the banks.
+// Products are issued between the exponentials of the other half of the tile: a wavefront's MFMAs run beside its own
+// vector instructions, which take longer.
 //
-// A capped score is cap (1 - 2 / (exp(2 s / cap) + 1)), at most cap: where exp(-2 cap) is far from float32's smallest
-// number the weights are taken relative to exp(cap), and no running maximum is needed (CAP 1; CAP 2 keeps one, CAP 0 has
-// no cap).
+// The queries come times scale log2(e) (a capped score's: 2 scale / cap log2(e)). A capped score is
+// cap (1 - 2 / (exp(2 s / cap) + 1)), at most cap: where exp(-2 cap) is far from float32's smallest number the weights are
+// taken relative to exp(cap), and no running maximum is needed (CAP 1; CAP 2 keeps one, CAP 0 has no cap).
 
+// 16 bytes a lane from a wavefront's address and a lane's offset into LDS (load_to_lds, gemm_nt_tile.h).
+__device__ __forceinline__ void load_to_lds(const void* g, uint32_t offset, uint32_t lds_base) {
+    asm volatile("s_mov_b32 m0, %0\n\tglobal_load_lds_dwordx4 %1, %2" ::"s"(lds_base), "v"(offset), "s"(g) : "memory");
+}
 __device__ __forceinline__ f32x16 mfma_bf16(u32x4 a, u32x4 b, f32x16 c) { return Bf16Element::mfma(a, b, c); }
 
 struct PromptArgs {
@@ -499,8 +565,7 @@ struct PromptArgs {
     uint16_t* out;
     int64_t ldo;
     int past, s, fold;
-    float to_arg;  // a score's product becomes the exponential's argument: of 2 s / cap, or of s itself; times log2(e)
-    float cap2;    // cap log2(e)
+    float cap2, inv_cap2;  // 2 cap log2(e), and -1 over it
 };
 
 constexpr int kPromptRows = 128;
@@ -527,35 +592,28 @@ __global__ __launch_bounds__(256, DT > 8 ? 1 : 2) void heads_prompt_kernel(Promp
     const int seen_wg = p.past + last_wg;
     const int seen_wave = first + wave * 32 < p.s ? (p.past + (first + wave * 32 + 32 < p.s ? first + wave * 32 + 32 : p.s)) : 0;
 
-    // where this lane's pieces of a tile come from: the same for every tile but for the tile's place
-    const char* kfrom[NK];
-    const char* vfrom[NV];
-    const uint32_t lds0 = (uint32_t)(uintptr_t)lds_prompt;
-    {
-        const uint16_t* keys = (const uint16_t*)a.keys + key_row(a, b, hk, 0);
-        const uint16_t* values = (const uint16_t*)a.values + value_row(a, b, hk, 0);
+    // where this lane's pieces of a tile come from: offsets that are the same for every tile
+    uint32_t kfrom[NK], vfrom[NV];
+    const char* keys = (const char*)((const uint16_t*)a.keys + key_row(a, b, hk, 0));
+    const char* values = (const char*)((const uint16_t*)a.values + value_row(a, b, hk, 0));
+    const uint32_t lds0 = (uint32_t)(uintptr_t)lds_prompt + wave * 1024;
 #pragma unroll
-        for (int n = 0; n < NK; n++) {
-            const int item = (wave * NK + n) * 64 + lane, r = item / P, piece = item % P ^ (P % 16 == 0 ? r & 15 : r >> 1 & 7);
-            kfrom[n] = (const char*)(keys + r * a.ldk + (piece * 8 < a.ldk ? piece * 8 : 0));  // pieces past the last feature meet zeros of q
-        }
+    for (int n = 0; n < NK; n++) {
+        const int item = (wave + 4 * n) * 64 + lane, r = item / P, piece = item % P ^ (P % 16 == 0 ? r & 15 : r >> 1 & 7);
+        kfrom[n] = (uint32_t)(r * a.ldk + (piece * 8 < a.ldk ? piece * 8 : 0)) * 2;  // pieces past the last feature meet zeros of q
+    }
 #pragma unroll
-        for (int n = 0; n < NV; n++) {
-            const int item = (wave * NV + n) * 64 + lane, r = item >> 3, piece = (item & 7) ^ (r >> 1 & 7);
-            vfrom[n] = (const char*)(values + (int64_t)(r < a.vdim ? r : a.vdim - 1) * a.context + piece * 8);
-        }
+    for (int n = 0; n < NV; n++) {
+        const int item = (wave + 4 * n) * 64 + lane, r = item >> 3, piece = (item & 7) ^ (r >> 1 & 7);
+        vfrom[n] = (uint32_t)((r < a.vdim ? r : a.vdim - 1) * a.context + piece * 8) * 2;
     }
     auto fetch = [&](uint32_t stage) {
 #pragma unroll
-        for (int n = 0; n < NK; n++) {
-            load_to_lds(kfrom[n], __builtin_amdgcn_readfirstlane(stage + (wave * NK + n) * 1024));
-            kfrom[n] += kKeys * a.ldk * 2;
-        }
+        for (int n = 0; n < NK; n++) load_to_lds(keys, kfrom[n], __builtin_amdgcn_readfirstlane(stage + n * 4096));
 #pragma unroll
-        for (int n = 0; n < NV; n++) {
-            load_to_lds(vfrom[n], __builtin_amdgcn_readfirstlane(stage + kKeyBytes + (wave * NV + n) * 1024));
-            vfrom[n] += kKeys * 2;
-        }
+        for (int n = 0; n < NV; n++) load_to_lds(values, vfrom[n], __builtin_amdgcn_readfirstlane(stage + kKeyBytes + n * 4096));
+        keys += kKeys * a.ldk * 2;
+        values += kKeys * 2;
     };
     u32x4 q[DT];
     {
@@ -572,8 +630,9 @@ __global__ __launch_bounds__(256, DT > 8 ? 1 : 2) void heads_prompt_kernel(Promp
     for (int t = 0; t < VT; t++)
 #pragma unroll
         for (int i = 0; i < 16; i++) o[t][i] = 0.f;
-    float m = CAP == 1 ? p.cap2 : -__builtin_inff(), l = 0.f;  // the reference of the weights (in units of log2); the sum over the keys this half of the lanes holds
+    float m = -__builtin_inff(), l = 0.f;  // the running maximum (in units of log2; not with CAP 1); the sum over the keys this half of the lanes holds
     const int kswz = P % 16 == 0 ? r32 & 15 : r32 >> 1 & 7, vswz = r32 >> 1 & 7;
+
     fetch(lds0);
     int stage = 0;
     for (int j0 = 0; j0 < seen_wg; j0 += kKeys, stage ^= 1) {
@@ -585,27 +644,57 @@ __global__ __launch_bounds__(256, DT > 8 ? 1 : 2) void heads_prompt_kernel(Promp
         const char* vs = ks + kKeyBytes;
         const bool whole = j0 + kKeys - 1 <= p.past + first + wave * 32;  // every row of the wavefront sees the whole tile
         f32x16 sc[2];
+        u32x4 high[2], low[2];
+        auto multiply_keys = [&](int c, int k) { sc[c] = mfma_bf16(*(const u32x4*)(ks + ((c * 32 + r32) * P + ((2 * k + hi) ^ kswz)) * 16), q[k], sc[c]); };
+        auto hide = [&](int c, float v) {  // what stands for keys that a row does not see
+            if (whole) return;
 #pragma unroll
-        for (int c = 0; c < 2; c++) {
+            for (int i = 0; i < 16; i++) sc[c][i] = j0 + c * 32 + (i & 3) + 8 * (i >> 2) + 4 * hi > pos ? v : sc[c][i];
+        };
+        auto weight = [&](int c, int i) {  // of a score, in its place
+            if constexpr (CAP == 1) sc[c][i] = __builtin_amdgcn_exp2f(__builtin_amdgcn_rcpf(fmaf(__builtin_amdgcn_exp2f(sc[c][i]), p.inv_cap2, p.inv_cap2)));
+            else sc[c][i] = __builtin_amdgcn_exp2f(sc[c][i] - m);
+        };
+        auto split = [&](int c, int half) {  // eight weights as the sum of two bfloat16
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const float x = sc[c][half * 8 + 2 * i], y = sc[c][half * 8 + 2 * i + 1];
+                l += x + y;
+                high[half][i] = pack_bf16(x, y);
+                low[half][i] = pack_bf16(x - __uint_as_float(high[half][i] << 16), y - __uint_as_float(high[half][i] & 0xffff0000u));
+            }
+        };
+        auto value = [&](int c, int half, int t) { return *(const u32x4*)(vs + (t * 32 + r32) * 128 + ((c * 4 + half * 2 + hi) ^ vswz) * 16); };
+#pragma unroll
+        for (int c = 0; c < 2; c++)
 #pragma unroll
             for (int i = 0; i < 16; i++) sc[c][i] = 0.f;
 #pragma unroll
-            for (int k = 0; k < DT; k++)
-                sc[c] = mfma_bf16(*(const u32x4*)(ks + ((c * 32 + r32) * P + ((2 * k + hi) ^ kswz)) * 16), q[k], sc[c]);
-        }
-        auto masked = [&](int c, int i) { return !whole && j0 + c * 32 + (i & 3) + 8 * (i >> 2) + 4 * hi > pos; };
-        if constexpr (CAP != 1) {
+        for (int k = 0; k < DT; k++) multiply_keys(0, k);
+        if constexpr (CAP == 1) {
+#pragma unroll
+            for (int k = 0; k < DT; k++) {
+                multiply_keys(1, k);
+#pragma unroll
+                for (int i = 16 * k / DT; i < 16 * (k + 1) / DT; i++) weight(0, i);
+            }
+            hide(0, 0.f);
+        } else {
+#pragma unroll
+            for (int k = 0; k < DT; k++) multiply_keys(1, k);
+            if constexpr (CAP == 2) {  // capped scores less their cap
+#pragma unroll
+                for (int c = 0; c < 2; c++)
+#pragma unroll
+                    for (int i = 0; i < 16; i++) sc[c][i] = __builtin_amdgcn_rcpf(fmaf(__builtin_amdgcn_exp2f(sc[c][i]), p.inv_cap2, p.inv_cap2));
+            }
+            hide(0, -__builtin_inff());
+            hide(1, -__builtin_inff());
             float top = -__builtin_inff();
 #pragma unroll
             for (int c = 0; c < 2; c++)
 #pragma unroll
-                for (int i = 0; i < 16; i++) {
-                    float v = sc[c][i] * p.to_arg;
-                    if constexpr (CAP == 2) v = fmaf(-2.f * p.cap2, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(v) + 1.f), p.cap2);
-                    if (masked(c, i)) v = -__builtin_inff();
-                    sc[c][i] = v;
-                    top = fmaxf(top, v);
-                }
+                for (int i = 0; i < 16; i++) top = fmaxf(top, sc[c][i]);
             top = fmaxf(top, __shfl_xor(top, 32));
             const float next = fmaxf(m, top);  // a row past the end sees keys too: finite from the first tile on
             if (__any(next > m)) {
@@ -617,34 +706,32 @@ __global__ __launch_bounds__(256, DT > 8 ? 1 : 2) void heads_prompt_kernel(Promp
                     for (int i = 0; i < 16; i++) o[t][i] *= back;
                 m = next;
             }
-        }
-        auto weight = [&](int c, int i) -> float {
-            if constexpr (CAP == 1) {
-                const float w = __builtin_amdgcn_exp2f(-2.f * p.cap2 * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(sc[c][i] * p.to_arg) + 1.f));
-                return masked(c, i) ? 0.f : w;
-            } else {
-                return __builtin_amdgcn_exp2f(sc[c][i] - m);
-            }
-        };
 #pragma unroll
-        for (int c = 0; c < 2; c++)
+            for (int i = 0; i < 16; i++) weight(0, i);
+        }
+#pragma unroll
+        for (int c = 0; c < 2; c++) {
+            split(c, 0);
+            split(c, 1);
 #pragma unroll
             for (int half = 0; half < 2; half++) {
-                u32x4 high, low;
+                u32x4 v[VT];
 #pragma unroll
-                for (int i = 0; i < 4; i++) {
-                    const float x = weight(c, half * 8 + 2 * i), y = weight(c, half * 8 + 2 * i + 1);
-                    l += x + y;
-                    high[i] = pack_bf16(x, y);
-                    low[i] = pack_bf16(low_part(x), low_part(y));
-                }
+                for (int t = 0; t < VT; t++) v[t] = value(c, half, t);
 #pragma unroll
-                for (int t = 0; t < VT; t++) {
-                    const u32x4 v = *(const u32x4*)(vs + (t * 32 + r32) * 128 + ((c * 4 + half * 2 + hi) ^ vswz) * 16);
-                    o[t] = mfma_bf16(v, high, o[t]);
-                    o[t] = mfma_bf16(v, low, o[t]);
-                }
+                for (int part = 0; part < 2; part++)
+#pragma unroll
+                    for (int t = 0; t < VT; t++) {
+                        o[t] = mfma_bf16(v[t], part ? low[half] : high[half], o[t]);
+                        if (c == 0) {  // the other half's weights between these
+                            const int at = (half * 2 + part) * VT + t;
+#pragma unroll
+                            for (int i = 16 * at / (4 * VT); i < 16 * (at + 1) / (4 * VT); i++) weight(1, i);
+                        }
+                    }
             }
+            if (CAP == 1 && c == 0) hide(1, 0.f);
+        }
     }
     const float sum = l + __shfl_xor(l, 32);
     if (row >= p.s) return;
@@ -680,7 +767,7 @@ hipError_t launch_prompt(PromptArgs p, hipStream_t st) {
 template <int DT, int VT>
 hipError_t launch_prompt(const PromptArgs& p, hipStream_t st) {
     if (p.a.softcap <= 0.f) return launch_prompt<DT, VT, 0>(p, st);
-    return p.cap2 <= 45.f ? launch_prompt<DT, VT, 1>(p, st) : launch_prompt<DT, VT, 2>(p, st);  // weights of 2^-90 and more
+    return p.cap2 <= 90.f ? launch_prompt<DT, VT, 1>(p, st) : launch_prompt<DT, VT, 2>(p, st);  // weights of 2^-90 and more
 }
 
 bool attend_mfma_ok(const HeadAttention& a) { return a.cache_bf16 && a.dim <= 256 && a.vdim <= 256; }
@@ -697,9 +784,14 @@ void launch_attend_any(const HeadAttention& a, const float* q32, const Parts& pa
     else hipLaunchKernelGGL((heads_attend_any_kernel<T, 4>), grid, dim3(256), lds, st, a, q32, parts);
 }
 
-hipError_t prepare(const HeadAttention& a, uint16_t* q16, float* q32, hipStream_t st) {
-    const int64_t rows = a.batch * a.s, blocks = rows + a.batch * ((a.s + 63) / 64) * (((int64_t)a.kv_heads * a.vdim + 63) / 64);
-    hipLaunchKernelGGL(heads_prepare_kernel, dim3((unsigned)blocks), dim3(256), 0, st, a, q16, q32);
+hipError_t prepare(const HeadAttention& a, uint16_t* q16, float* q32, float q_scale, hipStream_t st) {
+    const int lanes = !head_fours_ok(a) ? 0 : a.dim <= 64 ? 16 : a.dim <= 128 ? 32 : 64, at_once = lanes ? 256 / lanes : 4;
+    const int64_t heads = a.batch * a.s * ((a.heads + a.kv_heads + at_once - 1) / at_once);
+    const dim3 grid((unsigned)(heads + a.batch * ((a.s + 63) / 64) * (((int64_t)a.kv_heads * a.vdim + 63) / 64)));
+    if (lanes == 16) hipLaunchKernelGGL(heads_prepare_kernel<16>, grid, dim3(256), 0, st, a, q16, q32, q_scale);
+    else if (lanes == 32) hipLaunchKernelGGL(heads_prepare_kernel<32>, grid, dim3(256), 0, st, a, q16, q32, q_scale);
+    else if (lanes == 64) hipLaunchKernelGGL(heads_prepare_kernel<64>, grid, dim3(256), 0, st, a, q16, q32, q_scale);
+    else hipLaunchKernelGGL(heads_prepare_kernel<0>, grid, dim3(256), 0, st, a, q16, q32, q_scale);
     return hipGetLastError();
 }
 
@@ -731,7 +823,7 @@ hipError_t heads_attend(const HeadAttention& a, float* ws, float* out_f32, uint1
     const dim3 grid((unsigned)parts.splits, (unsigned)(a.kv_heads * ((per + kHeads - 1) / kHeads)), (unsigned)rows);
     const bool mfma = attend_mfma_ok(a), step = mfma && a.s == 1;
     if (!step)
-        if (hipError_t e = prepare(a, nullptr, ws, st)) return e;
+        if (hipError_t e = prepare(a, nullptr, ws, a.scale, st)) return e;
     if (mfma) {
         if (a.dim <= 64 && a.vdim <= 64) launch_attend<2, 1>(a, ws, parts, grid, step, st);
         else if (a.dim <= 128 && a.vdim <= 128) launch_attend<4, 2>(a, ws, parts, grid, step, st);
@@ -747,20 +839,20 @@ hipError_t heads_attend(const HeadAttention& a, float* ws, float* out_f32, uint1
 }
 
 bool heads_prompt_ok(const HeadAttention& a) {
-    return attend_mfma_ok(a) && a.past + a.s < 1 << 30 && !a.past_dev && a.batch <= 65535 && a.s <= (int64_t)65535 * kPromptRows;
+    return attend_mfma_ok(a) && a.vdim * a.context < 1ll << 30 && a.past + a.s < 1 << 30 && !a.past_dev && a.batch <= 65535 && a.s <= (int64_t)65535 * kPromptRows;
 }
 
 hipError_t heads_prompt(const HeadAttention& a, uint16_t* q, uint16_t* out, int64_t ldo, hipStream_t st) {
     if (a.batch * a.s == 0) return hipSuccess;
     if (!heads_prompt_ok(a) || a.ldk % 8 || a.context % kKeys || a.past + a.s > a.context || a.heads % a.kv_heads) return hipErrorInvalidValue;
-    if (hipError_t e = prepare(a, q, nullptr, st)) return e;
     constexpr float kLog2e = 1.4426950408889634f;
+    if (hipError_t e = prepare(a, q, nullptr, a.softcap > 0.f ? 2.f * a.scale / a.softcap * kLog2e : a.scale * kLog2e, st)) return e;
     PromptArgs p;
     p.a = a;
     p.q = q; p.out = out; p.ldo = ldo;
     p.past = (int)a.past; p.s = (int)a.s; p.fold = 0;
-    p.cap2 = a.softcap * kLog2e;
-    p.to_arg = a.softcap > 0.f ? 2.f * a.scale / a.softcap * kLog2e : a.scale * kLog2e;
+    p.cap2 = 2.f * a.softcap * kLog2e;
+    p.inv_cap2 = -1.f / p.cap2;
     if (a.dim <= 64 && a.vdim <= 64) return launch_prompt<4, 2>(p, st);
     if (a.dim <= 128 && a.vdim <= 128) return launch_prompt<8, 4>(p, st);
     return launch_prompt<16, 8>(p, st);
