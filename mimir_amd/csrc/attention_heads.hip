@@ -645,7 +645,17 @@ __global__ __launch_bounds__(256, DT > 8 ? 1 : 2) void heads_prompt_kernel(Promp
         const bool whole = j0 + kKeys - 1 <= p.past + first + wave * 32;  // every row of the wavefront sees the whole tile
         f32x16 sc[2];
         u32x4 high[2], low[2];
-        auto multiply_keys = [&](int c, int k) { sc[c] = mfma_bf16(*(const u32x4*)(ks + ((c * 32 + r32) * P + ((2 * k + hi) ^ kswz)) * 16), q[k], sc[c]); };
+        auto key = [&](int c, int k) { return *(const u32x4*)(ks + ((c * 32 + r32) * P + ((2 * k + hi) ^ kswz)) * 16); };
+        // all fragments of the keys are requested first, those of the values (a half of the tile's) before its weights are split
+        u32x4 kf[2][DT], vf[2][VT];
+        if constexpr (DT <= 8) {
+#pragma unroll
+            for (int c = 0; c < 2; c++)
+#pragma unroll
+                for (int k = 0; k < DT; k++) kf[c][k] = key(c, k);
+            __builtin_amdgcn_sched_barrier(0);
+        }
+        auto multiply_keys = [&](int c, int k) { sc[c] = mfma_bf16(DT <= 8 ? kf[c][k] : key(c, k), q[k], sc[c]); };
         auto hide = [&](int c, float v) {  // what stands for keys that a row does not see
             if (whole) return;
 #pragma unroll
@@ -664,7 +674,13 @@ __global__ __launch_bounds__(256, DT > 8 ? 1 : 2) void heads_prompt_kernel(Promp
                 low[half][i] = pack_bf16(x - __uint_as_float(high[half][i] << 16), y - __uint_as_float(high[half][i] & 0xffff0000u));
             }
         };
-        auto value = [&](int c, int half, int t) { return *(const u32x4*)(vs + (t * 32 + r32) * 128 + ((c * 4 + half * 2 + hi) ^ vswz) * 16); };
+        auto fetch_values = [&](int c) {
+#pragma unroll
+            for (int half = 0; half < 2; half++)
+#pragma unroll
+                for (int t = 0; t < VT; t++) vf[half][t] = *(const u32x4*)(vs + (t * 32 + r32) * 128 + ((c * 4 + half * 2 + hi) ^ vswz) * 16);
+            __builtin_amdgcn_sched_barrier(0);
+        };
 #pragma unroll
         for (int c = 0; c < 2; c++)
 #pragma unroll
@@ -711,18 +727,16 @@ __global__ __launch_bounds__(256, DT > 8 ? 1 : 2) void heads_prompt_kernel(Promp
         }
 #pragma unroll
         for (int c = 0; c < 2; c++) {
+            fetch_values(c);
             split(c, 0);
             split(c, 1);
 #pragma unroll
             for (int half = 0; half < 2; half++) {
-                u32x4 v[VT];
-#pragma unroll
-                for (int t = 0; t < VT; t++) v[t] = value(c, half, t);
 #pragma unroll
                 for (int part = 0; part < 2; part++)
 #pragma unroll
                     for (int t = 0; t < VT; t++) {
-                        o[t] = mfma_bf16(v[t], part ? low[half] : high[half], o[t]);
+                        o[t] = mfma_bf16(vf[half][t], part ? low[half] : high[half], o[t]);
                         if (c == 0) {  // the other half's weights between these
                             const int at = (half * 2 + part) * VT + t;
 #pragma unroll
