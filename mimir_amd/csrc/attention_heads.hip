@@ -18,7 +18,7 @@ namespace mimir {
 
 namespace {
 
-constexpr int kKeys = 64;   // keys a tile; a prompt's stage has up to two
+constexpr int kKeys = 64;   // keys a tile
 constexpr int kHeads = 8;   // heads of a group that a workgroup of few rows takes
 constexpr int kMaxSplits = 512;
 
@@ -547,8 +547,7 @@ __global__ __launch_bounds__(256) void heads_combine_kernel(HeadAttention a, Par
 // wavefronts with consecutive rows share a tile of keys and values in LDS, which goes there straight from the cache while the
 // tile before is used; a row's pieces of sixteen bytes are exchanged so that the reads of 32 rows spread over the banks.
 // Products are issued between the exponentials of the other half of the tile: a wavefront's MFMAs run beside its own
-// vector instructions, which take longer. Four more wavefronts take the same rows and every other tile (GROUPS 2), so that
-// a SIMD has work while one of them waits, however few workgroups there are; their sums meet at the end.
+// vector instructions, which take longer.
 //
 // The queries come times scale log2(e) (a capped score's: 2 scale / cap log2(e)). A capped score is
 // cap (1 - 2 / (exp(2 s / cap) + 1)), at most cap: where exp(-2 cap) is far from float32's smallest number the weights are
@@ -565,258 +564,218 @@ struct PromptArgs {
     const uint16_t* q;
     uint16_t* out;
     int64_t ldo;
-    int past, s;
-    int pair;              // a workgroup takes a block of rows from the end and then one from the start
+    int past, s, fold;
     float cap2, inv_cap2;  // 2 cap log2(e), and -1 over it
 };
 
 constexpr int kPromptRows = 128;
-constexpr int prompt_groups(int DT) { return DT > 8 ? 1 : 2; }  // one where results fill a SIMD's registers
-// Bytes of a stage in LDS: the tiles of all groups.
-constexpr size_t prompt_stage(int DT, int VT) { return prompt_groups(DT) * ((size_t)kKeys * DT * 32 + VT * 32 * kKeys * 2); }
 
 // DT: sixteenths of dim, rounded up to a multiple of four; VT: 32nds of vdim, rounded up.
 template <int DT, int VT, int CAP>
-__global__ __launch_bounds__(256 * prompt_groups(DT), DT > 8 ? 1 : DT > 4 ? 2 : 4) void heads_prompt_kernel(PromptArgs p) {
-    constexpr int GROUPS = prompt_groups(DT), kStep = GROUPS * kKeys, kWaves = 4 * GROUPS;
-    constexpr int P = DT * 2, VP = GROUPS * 8;  // pieces of a row of keys and of values in LDS
-    constexpr int kKeyBytes = kStep * P * 16, kStage = (int)prompt_stage(DT, VT);
-    constexpr int NK = DT / 2, NV = VT;  // loads of 1 KB a wavefront issues a stage
+__global__ __launch_bounds__(256, DT > 8 ? 1 : 2) void heads_prompt_kernel(PromptArgs p) {
+    constexpr int P = DT * 2;  // pieces of a key's row in LDS
+    constexpr int kKeyBytes = kKeys * P * 16, kValBytes = VT * 32 * 128, kStage = kKeyBytes + kValBytes;
+    constexpr int NK = DT / 2, NV = VT;  // loads of 1 KB a wavefront issues a tile
     extern __shared__ __align__(1024) char lds_prompt[];
     const HeadAttention& a = p.a;
     const int tid = threadIdx.x, lane = tid & 63, r32 = lane & 31, hi = lane >> 5;
-    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), group = wave >> 2, w4 = wave & 3;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     // heads of different groups beside each other: with as many groups as dies, a group's workgroups share a die's cache
     const int per = a.heads / a.kv_heads, hk = blockIdx.x % a.kv_heads, h = hk * per + blockIdx.x / a.kv_heads;
+    // the last rows first: they see the most keys. Where all workgroups fit the device at once, two a compute unit, the
+    // second half goes the other way, so that long ones and short ones share a unit.
+    const int nb = gridDim.y, by = blockIdx.y;
+    const int first = (p.fold && by >= (nb + 1) / 2 ? by - (nb + 1) / 2 : nb - 1 - by) * kPromptRows;
     const int64_t b = blockIdx.z;
+    const int row = first + wave * 32 + r32, pos = p.past + row;  // sees keys 0 .. pos
+    const int last_wg = first + kPromptRows < p.s ? first + kPromptRows : p.s;
+    const int seen_wg = p.past + last_wg;
+    const int seen_wave = first + wave * 32 < p.s ? (p.past + (first + wave * 32 + 32 < p.s ? first + wave * 32 + 32 : p.s)) : 0;
 
-    // where this lane's pieces of a stage come from: offsets that are the same for every stage
+    // where this lane's pieces of a tile come from: offsets that are the same for every tile
     uint32_t kfrom[NK], vfrom[NV];
+    const char* keys = (const char*)((const uint16_t*)a.keys + key_row(a, b, hk, 0));
+    const char* values = (const char*)((const uint16_t*)a.values + value_row(a, b, hk, 0));
     const uint32_t lds0 = (uint32_t)(uintptr_t)lds_prompt + wave * 1024;
 #pragma unroll
     for (int n = 0; n < NK; n++) {
-        const int item = (wave + kWaves * n) * 64 + lane, r = item / P, piece = item % P ^ (P % 16 == 0 ? r & 15 : r >> 1 & 7);
+        const int item = (wave + 4 * n) * 64 + lane, r = item / P, piece = item % P ^ (P % 16 == 0 ? r & 15 : r >> 1 & 7);
         kfrom[n] = (uint32_t)(r * a.ldk + (piece * 8 < a.ldk ? piece * 8 : 0)) * 2;  // pieces past the last feature meet zeros of q
     }
 #pragma unroll
     for (int n = 0; n < NV; n++) {
-        const int item = (wave + kWaves * n) * 64 + lane, r = item / VP, piece = item % VP ^ (VP == 16 ? r & 15 : r >> 1 & 7);
+        const int item = (wave + 4 * n) * 64 + lane, r = item >> 3, piece = (item & 7) ^ (r >> 1 & 7);
         vfrom[n] = (uint32_t)((r < a.vdim ? r : a.vdim - 1) * a.context + piece * 8) * 2;
     }
-    const int kswz = P % 16 == 0 ? r32 & 15 : r32 >> 1 & 7, vswz = VP == 16 ? r32 & 15 : r32 >> 1 & 7;
+    auto fetch = [&](uint32_t stage) {
+#pragma unroll
+        for (int n = 0; n < NK; n++) load_to_lds(keys, kfrom[n], __builtin_amdgcn_readfirstlane(stage + n * 4096));
+#pragma unroll
+        for (int n = 0; n < NV; n++) load_to_lds(values, vfrom[n], __builtin_amdgcn_readfirstlane(stage + kKeyBytes + n * 4096));
+        keys += kKeys * a.ldk * 2;
+        values += kKeys * 2;
+    };
+    u32x4 q[DT];
+    {
+        const uint16_t* qr = p.q + ((b * p.s + (row < p.s ? row : p.s - 1)) * a.heads + h) * a.ldk;
+#pragma unroll
+        for (int k = 0; k < DT; k++) {
+            const int d = k * 16 + hi * 8;
+            q[k] = u32x4{0, 0, 0, 0};
+            if (d < a.ldk) q[k] = *(const u32x4*)(qr + d);
+        }
+    }
+    f32x16 o[VT];
+#pragma unroll
+    for (int t = 0; t < VT; t++)
+#pragma unroll
+        for (int i = 0; i < 16; i++) o[t][i] = 0.f;
+    float m = -__builtin_inff(), l = 0.f;  // the running maximum (in units of log2; not with CAP 1); the sum over the keys this half of the lanes holds
+    const int kswz = P % 16 == 0 ? r32 & 15 : r32 >> 1 & 7, vswz = r32 >> 1 & 7;
 
-    // the last rows first: they see the most keys
-    const int last = p.pair ? (p.s + kPromptRows - 1) / kPromptRows - 1 : gridDim.y - 1;
-    for (int turn = 0; turn < 2; turn++) {
-        const int block = turn == 0 ? last - (int)blockIdx.y : (int)blockIdx.y;
-        if (turn == 1) {
-            if (!p.pair || block >= last - block) break;
-            lds_barrier();  // the rows before have left LDS
-        }
-        const int first = block * kPromptRows;
-        const int row = first + w4 * 32 + r32, pos = p.past + row;  // sees keys 0 .. pos
-        const int seen_wg = p.past + (first + kPromptRows < p.s ? first + kPromptRows : p.s);
-        const int seen_wave = first + w4 * 32 < p.s ? (p.past + (first + w4 * 32 + 32 < p.s ? first + w4 * 32 + 32 : p.s)) : 0;
-        const char* keys = (const char*)((const uint16_t*)a.keys + key_row(a, b, hk, 0));
-        const char* values = (const char*)((const uint16_t*)a.values + value_row(a, b, hk, 0));
-        auto fetch = [&](uint32_t stage) {
-#pragma unroll
-            for (int n = 0; n < NK; n++) load_to_lds(keys, kfrom[n], __builtin_amdgcn_readfirstlane(stage + n * kWaves * 1024));
-#pragma unroll
-            for (int n = 0; n < NV; n++) load_to_lds(values, vfrom[n], __builtin_amdgcn_readfirstlane(stage + kKeyBytes + n * kWaves * 1024));
-            keys += kStep * a.ldk * 2;
-            values += kStep * 2;
-        };
-        fetch(lds0);
-        u32x4 q[DT];
-        {
-            const uint16_t* qr = p.q + ((b * p.s + (row < p.s ? row : p.s - 1)) * a.heads + h) * a.ldk;
-#pragma unroll
-            for (int k = 0; k < DT; k++) {
-                const int d = k * 16 + hi * 8;
-                q[k] = u32x4{0, 0, 0, 0};
-                if (d < a.ldk) q[k] = *(const u32x4*)(qr + d);
-            }
-        }
-        f32x16 o[VT];
-#pragma unroll
-        for (int t = 0; t < VT; t++)
-#pragma unroll
-            for (int i = 0; i < 16; i++) o[t][i] = 0.f;
-        float m = -__builtin_inff(), l = 0.f;  // the running maximum (in units of log2; not with CAP 1); the sum over the keys this half of the lanes holds
-        int stage = 0;
-        for (int s0 = 0; s0 < seen_wg; s0 += kStep, stage ^= 1) {
-            wait_loads();   // this wavefront's part of the stage has landed
-            lds_barrier();  // everyone's has, and everyone has read the other stage
-            if (s0 + kStep < seen_wg) fetch(lds0 + (stage ^ 1) * kStage);
-            const int j0 = s0 + group * kKeys;
-            if (j0 >= seen_wave) continue;
-            const char* ks = lds_prompt + stage * kStage + group * (kKeys * P * 16);
-            const char* vs = lds_prompt + stage * kStage + kKeyBytes;
-            const bool whole = j0 + kKeys - 1 <= p.past + first + w4 * 32;  // every row of the wavefront sees the whole tile
-            f32x16 sc[2];
-            float from = 0.f;
-            u32x4 high[2], low[2];
-            auto key = [&](int c, int k) { return *(const u32x4*)(ks + ((c * 32 + r32) * P + ((2 * k + hi) ^ kswz)) * 16); };
-            // fragments of the keys are requested first (as many as there are registers for), those of the values (a half of the
-            // tile's) before its weights are split
-            constexpr int kAhead = DT == 8 ? 2 : DT == 4 ? 1 : 0;
-            u32x4 kf[2][DT], vf[2][VT];
-#pragma unroll
-            for (int c = 0; c < kAhead; c++)
-#pragma unroll
-                for (int k = 0; k < DT; k++) kf[c][k] = key(c, k);
-            if (kAhead) __builtin_amdgcn_sched_barrier(0);
-            auto multiply_keys = [&](int c, int k) { sc[c] = mfma_bf16(c < kAhead ? kf[c][k] : key(c, k), q[k], sc[c]); };
-            auto hide = [&](int c, float v) {  // what stands for keys that a row does not see
-                if (whole) return;
-#pragma unroll
-                for (int i = 0; i < 16; i++) sc[c][i] = j0 + c * 32 + (i & 3) + 8 * (i >> 2) + 4 * hi > pos ? v : sc[c][i];
-            };
-            auto weight = [&](int c, int i) {  // of a score, in its place
-                if constexpr (CAP == 1) sc[c][i] = __builtin_amdgcn_exp2f(__builtin_amdgcn_rcpf(fmaf(__builtin_amdgcn_exp2f(sc[c][i]), p.inv_cap2, p.inv_cap2)));
-                else sc[c][i] = __builtin_amdgcn_exp2f(sc[c][i] - from);
-            };
-            auto split = [&](int c, int half) {  // eight weights as the sum of two bfloat16
-#pragma unroll
-                for (int i = 0; i < 4; i++) {
-                    const float x = sc[c][half * 8 + 2 * i], y = sc[c][half * 8 + 2 * i + 1];
-                    l += x + y;
-                    high[half][i] = pack_bf16(x, y);
-                    low[half][i] = pack_bf16(x - __uint_as_float(high[half][i] << 16), y - __uint_as_float(high[half][i] & 0xffff0000u));
-                }
-            };
-            auto fetch_values = [&](int c) {
-#pragma unroll
-                for (int half = 0; half < 2; half++)
-#pragma unroll
-                    for (int t = 0; t < VT; t++) vf[half][t] = *(const u32x4*)(vs + (t * 32 + r32) * (VP * 16) + ((group * 8 + c * 4 + half * 2 + hi) ^ vswz) * 16);
-                __builtin_amdgcn_sched_barrier(0);
-            };
+    fetch(lds0);
+    int stage = 0;
+    for (int j0 = 0; j0 < seen_wg; j0 += kKeys, stage ^= 1) {
+        wait_loads();   // this wavefront's part of the tile has landed
+        lds_barrier();  // everyone's has, and everyone has read the other stage
+        if (j0 + kKeys < seen_wg) fetch(lds0 + (stage ^ 1) * kStage);
+        if (j0 >= seen_wave) continue;
+        const char* ks = lds_prompt + stage * kStage;
+        const char* vs = ks + kKeyBytes;
+        const bool whole = j0 + kKeys - 1 <= p.past + first + wave * 32;  // every row of the wavefront sees the whole tile
+        f32x16 sc[2];
+        u32x4 high[2], low[2];
+        auto key = [&](int c, int k) { return *(const u32x4*)(ks + ((c * 32 + r32) * P + ((2 * k + hi) ^ kswz)) * 16); };
+        // all fragments of the keys are requested first, those of the values (a half of the tile's) before its weights are split
+        u32x4 kf[2][DT], vf[2][VT];
+        if constexpr (DT <= 8) {
 #pragma unroll
             for (int c = 0; c < 2; c++)
 #pragma unroll
-                for (int i = 0; i < 16; i++) sc[c][i] = 0.f;
+                for (int k = 0; k < DT; k++) kf[c][k] = key(c, k);
+            __builtin_amdgcn_sched_barrier(0);
+        }
+        auto multiply_keys = [&](int c, int k) { sc[c] = mfma_bf16(DT <= 8 ? kf[c][k] : key(c, k), q[k], sc[c]); };
+        auto hide = [&](int c, float v) {  // what stands for keys that a row does not see
+            if (whole) return;
 #pragma unroll
-            for (int k = 0; k < DT; k++) multiply_keys(0, k);
-            if constexpr (CAP == 1) {
+            for (int i = 0; i < 16; i++) sc[c][i] = j0 + c * 32 + (i & 3) + 8 * (i >> 2) + 4 * hi > pos ? v : sc[c][i];
+        };
+        auto weight = [&](int c, int i) {  // of a score, in its place
+            if constexpr (CAP == 1) sc[c][i] = __builtin_amdgcn_exp2f(__builtin_amdgcn_rcpf(fmaf(__builtin_amdgcn_exp2f(sc[c][i]), p.inv_cap2, p.inv_cap2)));
+            else sc[c][i] = __builtin_amdgcn_exp2f(sc[c][i] - m);
+        };
+        auto split = [&](int c, int half) {  // eight weights as the sum of two bfloat16
 #pragma unroll
-                for (int k = 0; k < DT; k++) {
-                    multiply_keys(1, k);
+            for (int i = 0; i < 4; i++) {
+                const float x = sc[c][half * 8 + 2 * i], y = sc[c][half * 8 + 2 * i + 1];
+                l += x + y;
+                high[half][i] = pack_bf16(x, y);
+                low[half][i] = pack_bf16(x - __uint_as_float(high[half][i] << 16), y - __uint_as_float(high[half][i] & 0xffff0000u));
+            }
+        };
+        auto fetch_values = [&](int c) {
 #pragma unroll
-                    for (int i = 16 * k / DT; i < 16 * (k + 1) / DT; i++) weight(0, i);
-                }
-                hide(0, 0.f);
-            } else {
+            for (int half = 0; half < 2; half++)
 #pragma unroll
-                for (int k = 0; k < DT; k++) multiply_keys(1, k);
-                if constexpr (CAP == 2) {  // capped scores less their cap
+                for (int t = 0; t < VT; t++) vf[half][t] = *(const u32x4*)(vs + (t * 32 + r32) * 128 + ((c * 4 + half * 2 + hi) ^ vswz) * 16);
+            __builtin_amdgcn_sched_barrier(0);
+        };
 #pragma unroll
-                    for (int c = 0; c < 2; c++)
+        for (int c = 0; c < 2; c++)
 #pragma unroll
-                        for (int i = 0; i < 16; i++) sc[c][i] = __builtin_amdgcn_rcpf(fmaf(__builtin_amdgcn_exp2f(sc[c][i]), p.inv_cap2, p.inv_cap2));
-                }
-                hide(0, -__builtin_inff());
-                hide(1, -__builtin_inff());
-                float top = -__builtin_inff();
+            for (int i = 0; i < 16; i++) sc[c][i] = 0.f;
+#pragma unroll
+        for (int k = 0; k < DT; k++) multiply_keys(0, k);
+        if constexpr (CAP == 1) {
+#pragma unroll
+            for (int k = 0; k < DT; k++) {
+                multiply_keys(1, k);
+#pragma unroll
+                for (int i = 16 * k / DT; i < 16 * (k + 1) / DT; i++) weight(0, i);
+            }
+            hide(0, 0.f);
+        } else {
+#pragma unroll
+            for (int k = 0; k < DT; k++) multiply_keys(1, k);
+            if constexpr (CAP == 2) {  // capped scores less their cap
 #pragma unroll
                 for (int c = 0; c < 2; c++)
 #pragma unroll
-                    for (int i = 0; i < 16; i++) top = fmaxf(top, sc[c][i]);
-                top = fmaxf(top, __shfl_xor(top, 32));
-                const float next = fmaxf(m, top);
-                if (__any(next > m)) {
-                    const float back = next > m ? __builtin_amdgcn_exp2f(m - next) : 1.f;
-                    l *= back;
-#pragma unroll
-                    for (int t = 0; t < VT; t++)
-#pragma unroll
-                        for (int i = 0; i < 16; i++) o[t][i] *= back;
-                    m = next;
-                }
-                from = m > -__builtin_inff() ? m : 0.f;  // a row may see no key of the second group's tiles
-#pragma unroll
-                for (int i = 0; i < 16; i++) weight(0, i);
+                    for (int i = 0; i < 16; i++) sc[c][i] = __builtin_amdgcn_rcpf(fmaf(__builtin_amdgcn_exp2f(sc[c][i]), p.inv_cap2, p.inv_cap2));
             }
+            hide(0, -__builtin_inff());
+            hide(1, -__builtin_inff());
+            float top = -__builtin_inff();
 #pragma unroll
-            for (int c = 0; c < 2; c++) {
-                fetch_values(c);
-                split(c, 0);
-                split(c, 1);
+            for (int c = 0; c < 2; c++)
 #pragma unroll
-                for (int half = 0; half < 2; half++) {
-#pragma unroll
-                    for (int part = 0; part < 2; part++)
-#pragma unroll
-                        for (int t = 0; t < VT; t++) {
-                            o[t] = mfma_bf16(vf[half][t], part ? low[half] : high[half], o[t]);
-                            if (c == 0) {  // the other half's weights between these
-                                const int at = (half * 2 + part) * VT + t;
-#pragma unroll
-                                for (int i = 16 * at / (4 * VT); i < 16 * (at + 1) / (4 * VT); i++) weight(1, i);
-                            }
-                        }
-                }
-                if (CAP == 1 && c == 0) hide(1, 0.f);
-            }
-        }
-        float sum = l + __shfl_xor(l, 32);
-        if constexpr (GROUPS > 1) {  // the second group's sums go through LDS, where the stages were
-            float* parts = (float*)lds_prompt + w4 * ((VT * 16 + 2) * 64) + lane;
-            lds_barrier();  // everyone has read the last stage
-            if (group == 1) {
+                for (int i = 0; i < 16; i++) top = fmaxf(top, sc[c][i]);
+            top = fmaxf(top, __shfl_xor(top, 32));
+            const float next = fmaxf(m, top);  // a row past the end sees keys too: finite from the first tile on
+            if (__any(next > m)) {
+                const float back = __builtin_amdgcn_exp2f(m - next);
+                l *= back;
 #pragma unroll
                 for (int t = 0; t < VT; t++)
 #pragma unroll
-                    for (int i = 0; i < 16; i++) parts[(t * 16 + i) * 64] = o[t][i];
-                parts[VT * 16 * 64] = sum;
-                parts[(VT * 16 + 1) * 64] = m;
+                    for (int i = 0; i < 16; i++) o[t][i] *= back;
+                m = next;
             }
-            lds_barrier();
-            if (group == 1) continue;
-            float mine = 1.f, theirs = 1.f;
-            if constexpr (CAP != 1) {
-                const float their = parts[(VT * 16 + 1) * 64], both = fmaxf(m, their);  // the first group's first tile has a key for every row
-                mine = __builtin_amdgcn_exp2f(m - both);
-                theirs = __builtin_amdgcn_exp2f(their - both);
-            }
-            sum = sum * mine + parts[VT * 16 * 64] * theirs;
 #pragma unroll
-            for (int t = 0; t < VT; t++)
-#pragma unroll
-                for (int i = 0; i < 16; i++) o[t][i] = o[t][i] * mine + parts[(t * 16 + i) * 64] * theirs;
+            for (int i = 0; i < 16; i++) weight(0, i);
         }
-        const int64_t at_row = b * p.s + (row < p.s ? row : p.s - 1);
-        const float f = gate_of(a, at_row, h) / sum;
-        uint16_t* out = p.out + at_row * p.ldo + (int64_t)h * a.vdim;
-        const bool wide = a.vdim % 4 == 0 && p.ldo % 4 == 0 && ((uintptr_t)p.out & 7) == 0;
 #pragma unroll
-        for (int t = 0; t < VT; t++)
+        for (int c = 0; c < 2; c++) {
+            fetch_values(c);
+            split(c, 0);
+            split(c, 1);
 #pragma unroll
-            for (int g = 0; g < 4; g++) {
-                const int e = t * 32 + 8 * g + 4 * hi;
-                if (wide) {
-                    if (row < p.s && e < a.vdim) *(u32x2*)(out + e) = u32x2{pack_bf16(o[t][4 * g] * f, o[t][4 * g + 1] * f), pack_bf16(o[t][4 * g + 2] * f, o[t][4 * g + 3] * f)};
-                    continue;
-                }
+            for (int half = 0; half < 2; half++) {
 #pragma unroll
-                for (int i = 0; i < 4; i++)
-                    if (row < p.s && e + i < a.vdim) out[e + i] = round_bf16(o[t][4 * g + i] * f);
+                for (int part = 0; part < 2; part++)
+#pragma unroll
+                    for (int t = 0; t < VT; t++) {
+                        o[t] = mfma_bf16(vf[half][t], part ? low[half] : high[half], o[t]);
+                        if (c == 0) {  // the other half's weights between these
+                            const int at = (half * 2 + part) * VT + t;
+#pragma unroll
+                            for (int i = 16 * at / (4 * VT); i < 16 * (at + 1) / (4 * VT); i++) weight(1, i);
+                        }
+                    }
             }
+            if (CAP == 1 && c == 0) hide(1, 0.f);
+        }
     }
+    const float sum = l + __shfl_xor(l, 32);
+    if (row >= p.s) return;
+    const float f = gate_of(a, b * p.s + row, h) / sum;
+    uint16_t* out = p.out + (b * p.s + row) * p.ldo + (int64_t)h * a.vdim;
+    const bool wide = a.vdim % 4 == 0 && p.ldo % 4 == 0 && ((uintptr_t)p.out & 7) == 0;
+#pragma unroll
+    for (int t = 0; t < VT; t++)
+#pragma unroll
+        for (int g = 0; g < 4; g++) {
+            const int e = t * 32 + 8 * g + 4 * hi;
+            if (wide) {
+                if (e < a.vdim) *(u32x2*)(out + e) = u32x2{pack_bf16(o[t][4 * g] * f, o[t][4 * g + 1] * f), pack_bf16(o[t][4 * g + 2] * f, o[t][4 * g + 3] * f)};
+                continue;
+            }
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+                if (e + i < a.vdim) out[e + i] = round_bf16(o[t][4 * g + i] * f);
+        }
 }
 
 template <int DT, int VT, int CAP>
 hipError_t launch_prompt(PromptArgs p, hipStream_t st) {
-    constexpr size_t lds = 2 * prompt_stage(DT, VT);
+    constexpr size_t lds = 2 * ((size_t)kKeys * DT * 32 + VT * 32 * 128);
     static_assert(lds <= 160 * 1024, "a compute unit's LDS");
-    static_assert(prompt_groups(DT) == 1 || lds >= (size_t)4 * (VT * 16 + 2) * 64 * 4, "the second group's sums");
     hipError_t e = hipFuncSetAttribute((const void*)heads_prompt_kernel<DT, VT, CAP>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return e;
-    const unsigned blocks = (unsigned)((p.s + kPromptRows - 1) / kPromptRows);
-    p.pair = (int64_t)p.a.heads * blocks * p.a.batch >= 512;  // where half as many workgroups still fill the device
-    hipLaunchKernelGGL((heads_prompt_kernel<DT, VT, CAP>), dim3((unsigned)p.a.heads, p.pair ? (blocks + 1) / 2 : blocks, (unsigned)p.a.batch),
-                       dim3(256 * prompt_groups(DT)), lds, st, p);
+    const dim3 grid((unsigned)p.a.heads, (unsigned)((p.s + kPromptRows - 1) / kPromptRows), (unsigned)p.a.batch);
+    p.fold = (int64_t)grid.x * grid.y * grid.z <= 512;
+    hipLaunchKernelGGL((heads_prompt_kernel<DT, VT, CAP>), grid, dim3(256), lds, st, p);
     return hipGetLastError();
 }
 template <int DT, int VT>
@@ -868,7 +827,7 @@ size_t heads_attend_ws_floats(const HeadAttention& a, int64_t rows) {
 hipError_t heads_attend(const HeadAttention& a, float* ws, float* out_f32, uint16_t* out_bf16, int64_t ldo, hipStream_t st) {
     const int64_t rows = (int64_t)a.batch * a.s;
     if (rows == 0) return hipSuccess;
-    if (a.dim > kHeadAttentionMax || a.vdim > kHeadAttentionMax || rows > 65535 || a.ldk % 8 || a.context % kHeadAttentionKeys || a.heads % a.kv_heads) return hipErrorInvalidValue;
+    if (a.dim > kHeadAttentionMax || a.vdim > kHeadAttentionMax || rows > 65535 || a.ldk % 8 || a.context % kKeys || a.heads % a.kv_heads) return hipErrorInvalidValue;
     const int per = a.heads / a.kv_heads;
     Parts parts;
     parts.splits = splits_of(a);
@@ -899,13 +858,13 @@ bool heads_prompt_ok(const HeadAttention& a) {
 
 hipError_t heads_prompt(const HeadAttention& a, uint16_t* q, uint16_t* out, int64_t ldo, hipStream_t st) {
     if (a.batch * a.s == 0) return hipSuccess;
-    if (!heads_prompt_ok(a) || a.ldk % 8 || a.context % kHeadAttentionKeys || a.past + a.s > a.context || a.heads % a.kv_heads) return hipErrorInvalidValue;
+    if (!heads_prompt_ok(a) || a.ldk % 8 || a.context % kKeys || a.past + a.s > a.context || a.heads % a.kv_heads) return hipErrorInvalidValue;
     constexpr float kLog2e = 1.4426950408889634f;
     if (hipError_t e = prepare(a, q, nullptr, a.softcap > 0.f ? 2.f * a.scale / a.softcap * kLog2e : a.scale * kLog2e, st)) return e;
     PromptArgs p;
     p.a = a;
     p.q = q; p.out = out; p.ldo = ldo;
-    p.past = (int)a.past; p.s = (int)a.s;
+    p.past = (int)a.past; p.s = (int)a.s; p.fold = 0;
     p.cap2 = 2.f * a.softcap * kLog2e;
     p.inv_cap2 = -1.f / p.cap2;
     if (a.dim <= 64 && a.vdim <= 64) return launch_prompt<4, 2>(p, st);

@@ -105,7 +105,6 @@ struct Stack : Decoder {
     bool parallel() const { return has(MI355X_STACK_PARALLEL); }
     const Mat& output() const { return has(MI355X_STACK_OUTPUT_MATRIX) ? head_w : embed; }
     int64_t width() const { return c.width; }
-    int64_t positions_of_heads() const { return (context + kHeadAttentionKeys - 1) / kHeadAttentionKeys * kHeadAttentionKeys; }
     void name_tensors();
     Latent latent(const StackLayer& l, int64_t s, const int32_t* pos) const;
     HeadAttention attention(const StackLayer& l, int64_t s, const int32_t* pos) const;
@@ -156,7 +155,7 @@ HeadAttention Stack::attention(const StackLayer& l, int64_t s, const int32_t* po
     a.gated = l.c.head_gate != 0;
     if (l.c.value_mix && l.mixes_first) a.first_out = first_values.as<float>();
     else if (l.c.value_mix) { a.first = first_values.as<float>(); a.mix = l.vmix.p(); }
-    a.keys = l.cache.p; a.values = l.values.p; a.cache_bf16 = half(); a.ldk = l.ldc; a.context = positions_of_heads();
+    a.keys = l.cache.p; a.values = l.values.p; a.cache_bf16 = half(); a.ldk = l.ldc; a.context = pad64(context);
     a.batch = batch; a.s = s;
     a.past = pos ? 0 : cache_len; a.past_dev = pos;
     return a;
@@ -605,7 +604,7 @@ mi355x_status Stack::finalize(int64_t max_tokens) {
         if (mi355x_status st = layer_scales(l)) return st;
         if (l.by_heads()) {
             l.ldc = (l.c.dim + 7) / 8 * 8;
-            const size_t positions = (size_t)batch * l.c.kv_heads * positions_of_heads() * (half() ? 2 : 4);
+            const size_t positions = (size_t)batch * l.c.kv_heads * pad64(context) * (half() ? 2 : 4);
             STACK_BUF(l.cache, positions * l.ldc);
             STACK_BUF(l.values, positions * l.c.vdim);
             if (mi355x_status st = rotation(l)) return st;

@@ -190,14 +190,13 @@ struct HeadAttention {
     void* values = nullptr;  // [batch, kv_heads, vdim, context], positions in the kernels' own order
     bool cache_bf16 = false;
     int64_t ldk = 0;      // a multiple of 8, zeros behind dim
-    int64_t context = 0;  // the capacity, a multiple of kHeadAttentionKeys
+    int64_t context = 0;  // the capacity, a multiple of 64
     int batch = 1;
     int64_t s = 1;     // new positions a sequence
     int64_t past = 0;  // positions before them: past + *past_dev
     const int32_t* past_dev = nullptr;
 };
 constexpr int kHeadAttentionMax = 1024;  // features of a head
-constexpr int kHeadAttentionKeys = 128;
 // Cache entries of the new positions, then attention of few query rows. ws: heads_attend_ws_floats floats. out
 // [rows, heads * vdim] float32 or bfloat16, rows ldo apart.
 size_t heads_attend_ws_floats(const HeadAttention& a, int64_t rows);
