@@ -16,6 +16,7 @@ typedef float f32x16 __attribute__((ext_vector_type(16)));
 
 constexpr int kTile = 64, kStep = 32, kPad = kStep + 1;
 
+template <Out KIND>
 __global__ __launch_bounds__(256) void gemm_f32_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx, int64_t M,
                                                        int64_t N, int64_t K, ProductOut out) {
     __shared__ float xs[2][kTile * kPad], ws[2][kTile * kPad];
@@ -57,7 +58,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const uint16_t* __restric
             part = __builtin_amdgcn_mfma_f32_32x32x2f32(xs[p][(wm + r32) * kPad + k + hi], ws[p][(wn + r32) * kPad + k + hi], part, 0, 0, 0);
 #pragma unroll
         for (int i = 0; i < 16; i++) acc[i] += part[i];
-        if (out.mid && k0 + kStep == out.split) {
+        if (KIND == Out::Scaled && out.mid && k0 + kStep == out.split) {
             const float f = out.mid[n0 + wn + r32 < N ? n0 + wn + r32 : N - 1];
 #pragma unroll
             for (int i = 0; i < 16; i++) acc[i] *= f;
@@ -66,9 +67,9 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const uint16_t* __restric
 #pragma unroll
     for (int i = 0; i < 16; i++) {
         const int64_t m = m0 + wm + (i & 3) + 8 * (i >> 2) + 4 * hi, n = n0 + wn + r32;
-        const float beside = __shfl_xor(acc[i], 1);  // the column beside this one
+        const float beside = KIND == Out::Pairs ? __shfl_xor(acc[i], 1) : 0.f;  // the column beside this one
         if (m >= M || n >= N) continue;
-        if (n < out.pair_from) store_column(out, m, n, acc[i]);
+        if (KIND != Out::Pairs || n < out.pair_from) store_column<KIND>(out, m, n, acc[i]);
         else if ((n & 1) == 0) store_pair(out, m, n, acc[i], beside);
     }
 }
@@ -77,8 +78,7 @@ constexpr int kNarrow = 64;  // rows of W a workgroup
 
 // v_mfma_f32_16x16x4: lane (row, k). A lane brings four neighbouring elements of K of its row, so the four products of a step
 // of sixteen take K in the order 4 k + j, in both operands alike.
-// TWO: the sums below and from out.split on have factors of their own.
-template <bool TWO>
+template <Out KIND>
 __global__ __launch_bounds__(512) void gemm_f32_narrow_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx, int64_t M,
                                                               int64_t N, int64_t K, ProductOut out) {
     __shared__ float red[8][16][kNarrow + 1];
@@ -107,7 +107,7 @@ __global__ __launch_bounds__(512) void gemm_f32_narrow_kernel(const uint16_t* __
         }
     };
     int64_t from = k0;
-    if constexpr (TWO) {  // what of this wavefront's piece lies below split
+    if (KIND == Out::Scaled && out.mid) {  // what of this wavefront's piece lies below split has a factor of its own
         const int64_t to = out.split < k1 ? out.split : k1;
         sum_of(k0, to);
 #pragma unroll
@@ -130,23 +130,29 @@ __global__ __launch_bounds__(512) void gemm_f32_narrow_kernel(const uint16_t* __
             for (int i = 0; i < 8; i++) v += red[i][row][c];
             return v;
         };
-        if (n < out.pair_from) store_column(out, m, n, sum(col));
+        if (KIND != Out::Pairs || n < out.pair_from) store_column<KIND>(out, m, n, sum(col));
         else if ((col & 1) == 0) store_pair(out, m, n, sum(col), sum(col + 1));
     }
+}
+
+template <Out KIND>
+void launch(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st) {
+    if (N <= 2 * kNarrow && ldx % 4 == 0 && ldw % 4 == 0)
+        hipLaunchKernelGGL(gemm_f32_narrow_kernel<KIND>, dim3((unsigned)((N + kNarrow - 1) / kNarrow), (unsigned)((M + 15) / 16)), dim3(512), 0, st, W, ldw, x, ldx,
+                           M, N, K, out);
+    else
+        hipLaunchKernelGGL(gemm_f32_kernel<KIND>, dim3((unsigned)((N + kTile - 1) / kTile), (unsigned)((M + kTile - 1) / kTile)), dim3(256), 0, st, W, ldw, x, ldx,
+                           M, N, K, out);
 }
 
 }  // namespace
 
 hipError_t gemm_f32(const uint16_t* W, int64_t ldw, const float* x, int64_t ldx, int64_t M, int64_t N, int64_t K, const ProductOut& out, hipStream_t st) {
     if (M == 0 || N == 0) return hipSuccess;
-    if (N <= 2 * kNarrow && ldx % 4 == 0 && ldw % 4 == 0) {
-        const dim3 grid((unsigned)((N + kNarrow - 1) / kNarrow), (unsigned)((M + 15) / 16));
-        if (out.mid) hipLaunchKernelGGL(gemm_f32_narrow_kernel<true>, grid, dim3(512), 0, st, W, ldw, x, ldx, M, N, K, out);
-        else hipLaunchKernelGGL(gemm_f32_narrow_kernel<false>, grid, dim3(512), 0, st, W, ldw, x, ldx, M, N, K, out);
-        return hipGetLastError();
-    }
-    hipLaunchKernelGGL(gemm_f32_kernel, dim3((unsigned)((N + kTile - 1) / kTile), (unsigned)((M + kTile - 1) / kTile)), dim3(256), 0, st, W, ldw, x, ldx, M,
-                       N, K, out);
+    const Out kind = out_kind(out, N);
+    if (kind == Out::Plain) launch<Out::Plain>(W, ldw, x, ldx, M, N, K, out, st);
+    else if (kind == Out::Pairs) launch<Out::Pairs>(W, ldw, x, ldx, M, N, K, out, st);
+    else launch<Out::Scaled>(W, ldw, x, ldx, M, N, K, out, st);
     return hipGetLastError();
 }
 

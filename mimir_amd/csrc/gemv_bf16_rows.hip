@@ -8,14 +8,16 @@
 #include "product_store.h"
 #include "stack_ops.h"
 
+#include <type_traits>
+
 namespace mimir {
 
 namespace {
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
-// T: groups of sixteen rows of W a workgroup. TWO: the sums below and from out.split on have factors of their own.
-template <int T, int kWaves, bool TWO>
+// T: groups of sixteen rows of W a workgroup.
+template <int T, int kWaves, Out KIND>
 __global__ __launch_bounds__(64 * kWaves) void gemv_bf16_rows_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx,
                                                                      int M, int N, int K, ProductOut out) {
     __shared__ float red[kWaves][T * 16][17];
@@ -61,7 +63,7 @@ __global__ __launch_bounds__(64 * kWaves) void gemv_bf16_rows_kernel(const uint1
         }
     };
     int from = k0;
-    if constexpr (TWO) {  // what of this wavefront's piece lies below split
+    if (KIND == Out::Scaled && out.mid) {  // what of this wavefront's piece lies below split has a factor of its own
         const int to = out.split < k1 ? (int)out.split : k1;
         sum_of(k0, to);
 #pragma unroll
@@ -89,7 +91,7 @@ __global__ __launch_bounds__(64 * kWaves) void gemv_bf16_rows_kernel(const uint1
             for (int i = 0; i < kWaves; i++) v += red[i][r][col] + red[i][r][col + 8];
             return v;
         };
-        if (n < out.pair_from) store_column(out, col, n, sum(row));
+        if (KIND != Out::Pairs || n < out.pair_from) store_column<KIND>(out, col, n, sum(row));
         else if ((row & 1) == 0) store_pair(out, col, n, sum(row), sum(row + 1));
     }
 }
@@ -103,16 +105,17 @@ hipError_t gemv_bf16_rows(const uint16_t* W, int64_t ldw, const float* x, int64_
     auto launch = [&](auto kernel, int rows, int waves) {
         hipLaunchKernelGGL(kernel, dim3((unsigned)((N + rows - 1) / rows)), dim3(64 * waves), 0, st, W, ldw, x, ldx, (int)M, (int)N, k, out);
     };
-    if (N >= 8192) {
-        if (out.mid) launch(gemv_bf16_rows_kernel<2, 8, true>, 32, 8);
-        else launch(gemv_bf16_rows_kernel<2, 8, false>, 32, 8);
-    } else if (k >= 8192) {
-        if (out.mid) launch(gemv_bf16_rows_kernel<1, 16, true>, 16, 16);
-        else launch(gemv_bf16_rows_kernel<1, 16, false>, 16, 16);
-    } else {
-        if (out.mid) launch(gemv_bf16_rows_kernel<1, 8, true>, 16, 8);
-        else launch(gemv_bf16_rows_kernel<1, 8, false>, 16, 8);
-    }
+    auto by_kind = [&](auto t, auto waves) {
+        constexpr int T = decltype(t)::value, kWaves = decltype(waves)::value;
+        const Out kind = out_kind(out, N);
+        if (kind == Out::Plain) launch(gemv_bf16_rows_kernel<T, kWaves, Out::Plain>, 16 * T, kWaves);
+        else if (kind == Out::Pairs) launch(gemv_bf16_rows_kernel<T, kWaves, Out::Pairs>, 16 * T, kWaves);
+        else launch(gemv_bf16_rows_kernel<T, kWaves, Out::Scaled>, 16 * T, kWaves);
+    };
+    using std::integral_constant;
+    if (N >= 8192) by_kind(integral_constant<int, 2>{}, integral_constant<int, 8>{});
+    else if (k >= 8192) by_kind(integral_constant<int, 1>{}, integral_constant<int, 16>{});
+    else by_kind(integral_constant<int, 1>{}, integral_constant<int, 8>{});
     return hipGetLastError();
 }
 

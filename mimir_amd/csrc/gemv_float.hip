@@ -12,6 +12,8 @@
 #include "product_store.h"
 #include "stack_ops.h"
 
+#include <type_traits>
+
 namespace mimir {
 
 template <typename T>
@@ -53,8 +55,7 @@ hipError_t gemv_float(int dt, const void* W, const float* x, float* y, int64_t M
 
 // M rows of x against R rows of W a wavefront, eight elements of K a lane and step (the rows are padded with zeros to
 // a multiple of 64). The x of a step serves all R rows from registers.
-// TWO: the sums below and from out.split on have factors of their own.
-template <int M, int R, bool TWO>
+template <int M, int R, Out KIND>
 __global__ __launch_bounds__(256) void gemv_bf16_kernel(const uint16_t* __restrict__ W, int64_t ldw, const float* __restrict__ x, int64_t ldx, int N, int K,
                                                         ProductOut out) {
     const int lane = threadIdx.x & 63, n0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * R;
@@ -92,16 +93,17 @@ __global__ __launch_bounds__(256) void gemv_bf16_kernel(const uint16_t* __restri
             }
         }
     };
-    if constexpr (TWO) {
-        sum(0, (int)out.split);
+    const int split = KIND == Out::Scaled && out.mid ? (int)out.split : 0;
+    if constexpr (KIND == Out::Scaled) {  // the sums below split and from there on have factors of their own
+        sum(0, split);
 #pragma unroll
         for (int r = 0; r < R; r++) {
-            const float f = out.mid[n0 + r < N ? n0 + r : N - 1];
+            const float f = out.mid ? out.mid[n0 + r < N ? n0 + r : N - 1] : 1.f;
 #pragma unroll
             for (int m = 0; m < M; m++) acc[m][r] *= f;
         }
     }
-    sum(TWO ? (int)out.split : 0, K);
+    sum(split, K);
 #pragma unroll
     for (int m = 0; m < M; m++) {
         float v[R];
@@ -112,7 +114,7 @@ __global__ __launch_bounds__(256) void gemv_bf16_kernel(const uint16_t* __restri
         for (int r = 0; r < R; r++) {
             const int n = n0 + r;
             if (n >= N) break;
-            if (n < out.pair_from) store_column(out, m0 + m, n, v[r]);
+            if (KIND != Out::Pairs || n < out.pair_from) store_column<KIND>(out, m0 + m, n, v[r]);
             else if (r + 1 < R && (r & 1) == 0) store_pair(out, m0 + m, n, v[r], v[r + 1 < R ? r + 1 : r]);
         }
     }
@@ -127,14 +129,17 @@ void launch_gemv_bf16(const uint16_t* W, int64_t ldw, const float* x, int64_t ld
         hipLaunchKernelGGL(kernel, dim3((unsigned)((N + 4 * rows - 1) / (4 * rows)), (unsigned)groups), dim3(256), 0, st, W, ldw, x, ldx, (int)N, k, out);
     };
     // more rows a wavefront read x less often; fewer give a small matrix enough wavefronts
-    const int rows = N >= 8192 && M <= 4 ? 4 : N >= 2048 || N > out.pair_from ? 2 : 1;
-    if (out.mid) {
-        if (rows == 4) launch(gemv_bf16_kernel<M, (M <= 4 ? 4 : 2), true>, 4);
-        else if (rows == 2) launch(gemv_bf16_kernel<M, 2, true>, 2);
-        else launch(gemv_bf16_kernel<M, 1, true>, 1);
-    } else if (rows == 4) launch(gemv_bf16_kernel<M, (M <= 4 ? 4 : 2), false>, 4);
-    else if (rows == 2) launch(gemv_bf16_kernel<M, 2, false>, 2);
-    else launch(gemv_bf16_kernel<M, 1, false>, 1);
+    const Out kind = out_kind(out, N);
+    const int rows = N >= 8192 && M <= 4 ? 4 : N >= 2048 || kind == Out::Pairs ? 2 : 1;
+    auto by_kind = [&](auto rows_tag) {
+        constexpr int R = decltype(rows_tag)::value;
+        if (kind == Out::Scaled) launch(gemv_bf16_kernel<M, R, Out::Scaled>, R);
+        else if (kind == Out::Plain) launch(gemv_bf16_kernel<M, R, Out::Plain>, R);
+        else if constexpr (R > 1) launch(gemv_bf16_kernel<M, R, Out::Pairs>, R);
+    };
+    if (rows == 4) by_kind(std::integral_constant<int, (M <= 4 ? 4 : 2)>{});
+    else if (rows == 2) by_kind(std::integral_constant<int, 2>{});
+    else by_kind(std::integral_constant<int, 1>{});
 }
 
 }  // namespace

@@ -58,6 +58,7 @@ size_t chain_lds(int width, int groups, int threads) {
 }
 int row_threads(int width) { return width >= 2048 ? 1024 : 256; }
 
+template <bool EMBED>
 __global__ __launch_bounds__(1024) void norm_chain_kernel(NormChain a) {
     extern __shared__ float lds_chain[];
     const int W = a.width, nw = blockDim.x >> 6, gs = W / a.groups;
@@ -65,7 +66,7 @@ __global__ __launch_bounds__(1024) void norm_chain_kernel(NormChain a) {
     float* part = row + W;
     float* scale = part + (a.groups > nw ? a.groups : nw);
     const int64_t r = blockIdx.x;
-    if (a.tokens) {
+    if constexpr (EMBED) {
         const uint16_t* e = a.table + (int64_t)a.tokens[r] * a.table_ld;
         for (int i = threadIdx.x; i < W; i += blockDim.x) row[i] = bf16_bits_to_f32(e[i]);
         if (a.pairs.table) {
@@ -80,7 +81,7 @@ __global__ __launch_bounds__(1024) void norm_chain_kernel(NormChain a) {
     const float own = a.dwa ? a.dwa[a.n_streams] : 1.f;
     for (int i = threadIdx.x; i < W; i += blockDim.x) {
         float z = a.w_post ? row[i] * scale[i / gs] * a.w_post[i] : row[i];
-        if (!a.tokens) z += a.x[r * W + i];
+        if (!EMBED) z += a.x[r * W + i];
         if (a.stream_out) a.stream_out[r * W + i] = z;
         if (a.dwa) {
             float acc = 0.f;
@@ -121,7 +122,7 @@ __global__ __launch_bounds__(1024) void norm_chain_kernel(NormChain a) {
 
 // The same for rows whose groups are whole wavefronts of 256 elements: a thread owns E runs of four neighbouring elements in
 // registers, everything that does not depend on a sum is requested at once, and a norm costs one barrier.
-template <int E>
+template <int E, bool EMBED>
 __global__ __launch_bounds__(1024) void norm_chain_wide_kernel(NormChain a) {
     __shared__ float part[2][64];
     const int W = a.width, gs = W / a.groups, lane = threadIdx.x & 63;
@@ -155,11 +156,11 @@ __global__ __launch_bounds__(1024) void norm_chain_wide_kernel(NormChain a) {
         }
     };
     f32x4 y[E], x[E], wp[E], wn[E], z[E], avg[E];
-    const uint16_t* row = a.tokens ? a.table + (int64_t)a.tokens[r] * a.table_ld : nullptr;
-    const uint16_t* pair = a.tokens && a.pairs.table ? pair_row(a.pairs, a.tokens, r, threadIdx.x == 0) : nullptr;
+    const uint16_t* row = EMBED ? a.table + (int64_t)a.tokens[r] * a.table_ld : nullptr;
+    const uint16_t* pair = EMBED && a.pairs.table ? pair_row(a.pairs, a.tokens, r, threadIdx.x == 0) : nullptr;
 #pragma unroll
     for (int e = 0; e < E; e++) {
-        if (row) {
+        if constexpr (EMBED) {
             u32x2 v = {0, 0};
             if (in[e]) v = *(const u32x2*)(row + at[e]);
             y[e] = f32x4{__uint_as_float(v[0] << 16), __uint_as_float(v[0] & 0xffff0000u), __uint_as_float(v[1] << 16), __uint_as_float(v[1] & 0xffff0000u)};
@@ -373,13 +374,16 @@ hipError_t norm_chain(const NormChain& a, int64_t rows, hipStream_t st) {
     if (a.width / a.groups % 256 == 0 && a.width <= 16384 && whole(a.table, a.table_ld) && whole(a.pairs.table, a.pairs.ld) && whole(a.y, a.ldy) && whole(a.x, 4) && whole(a.h_f32, a.ldh) &&
         whole(a.h_bf16, a.ldh) && whole(a.streams, a.stream_stride) && whole(a.stream_out, 4) && whole(a.x_out, 4) && whole(a.conv_state, 4)) {
         const int threads = a.width < 4096 ? a.width / 4 : 1024;  // a multiple of 64
-        if (a.width <= 4096) hipLaunchKernelGGL(norm_chain_wide_kernel<1>, dim3((unsigned)rows), dim3(threads), 0, st, a);
-        else if (a.width <= 8192) hipLaunchKernelGGL(norm_chain_wide_kernel<2>, dim3((unsigned)rows), dim3(threads), 0, st, a);
-        else hipLaunchKernelGGL(norm_chain_wide_kernel<4>, dim3((unsigned)rows), dim3(threads), 0, st, a);
+        auto launch = [&](auto kernel) { hipLaunchKernelGGL(kernel, dim3((unsigned)rows), dim3(threads), 0, st, a); };
+        if (a.width <= 4096) a.tokens ? launch(norm_chain_wide_kernel<1, true>) : launch(norm_chain_wide_kernel<1, false>);
+        else if (a.width <= 8192) a.tokens ? launch(norm_chain_wide_kernel<2, true>) : launch(norm_chain_wide_kernel<2, false>);
+        else a.tokens ? launch(norm_chain_wide_kernel<4, true>) : launch(norm_chain_wide_kernel<4, false>);
         return hipGetLastError();
     }
     const int threads = row_threads(a.width);
-    hipLaunchKernelGGL(norm_chain_kernel, dim3((unsigned)rows), dim3(threads), chain_lds(a.width, a.groups, threads), st, a);
+    const size_t lds = chain_lds(a.width, a.groups, threads);
+    if (a.tokens) hipLaunchKernelGGL(norm_chain_kernel<true>, dim3((unsigned)rows), dim3(threads), lds, st, a);
+    else hipLaunchKernelGGL(norm_chain_kernel<false>, dim3((unsigned)rows), dim3(threads), lds, st, a);
     return hipGetLastError();
 }
 

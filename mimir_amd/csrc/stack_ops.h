@@ -74,13 +74,14 @@ struct ProductOut {
     int64_t silu_n = 0;
     bool relu2 = false;
     // Columns from pair_from (a multiple of 4) on come in pairs (z, u), side by side, and leave one value silu(z) u a pair, in
-    // one of these, rows pair_ld apart. N is even then.
+    // one of these, rows pair_ld apart. N is even then, and there are no factors.
     int64_t pair_from = INT64_MAX;
     float* pair_f32 = nullptr;
     uint16_t* pair_bf16 = nullptr;
     int64_t pair_ld = 0;
     // y_n = scale[n] (mid[n] (the sum over k < split) + the rest of it), with null pointers for ones: two products of the same
     // row, each with factors of its own (s in front of the first: mid = s / scale), in one. split: a multiple of 64 below K.
+    // Without an activation.
     const float* scale = nullptr;
     const float* mid = nullptr;
     int64_t split = 0;
