@@ -18,7 +18,7 @@ pytestmark = pytest.mark.gpu
 
 DTYPES = ("float32", "bfloat16")
 # of a row's logits, against the spread of all of them (tests.fuvolix.error)
-TOL = {"float32": 2e-5, "bfloat16": 0.05}
+TOL = {"float32": 1e-5, "bfloat16": 0.03}
 off = lambda t: t * 0
 
 
